@@ -43,6 +43,8 @@ _LAZY: dict[str, str] = {
     "miborax": "rapid_llm_amd.models.miborax",
     "Fomunex": "rapid_llm_amd.models.fomunex",
     "fomunex": "rapid_llm_amd.models.fomunex",
+    "Pefulorn": "rapid_llm_amd.models.pefulorn",
+    "pefulorn": "rapid_llm_amd.models.pefulorn",
 }
 
 

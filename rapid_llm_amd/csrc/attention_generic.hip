@@ -8,7 +8,8 @@
 // be d; with `sink` the softmax's denominator has one more term, exp(0) or, with `sink_values`,
 // exp of a number per query head: a key without a value.  With cap > 0 a scaled score s becomes
 // cap * tanh(s / cap); with `slopes` (one number a query head) slope_h * (pos - j) is then taken
-// off it.
+// off it; with `log_r1` and `log_r2` instead r1_h * ln(1 + r2_h * (pos - j)) is.  A token's heads lie
+// side by side in a row of `out` of out_width elements; `out_scale` multiplies the finished outputs.
 //
 // Scores (q . k) / sqrt(d) (rapid_llm/modules/attention.py:62), online softmax over tiles
 // of 256 keys in ascending order (rapid_llm/kernels/ops/attention/flashattention2_nopad.py:
@@ -24,7 +25,8 @@ __global__ __launch_bounds__(ATT_THREADS) void attention_generic_kernel(
     T* __restrict__ out, const int* __restrict__ positions, const int* __restrict__ token_slot,
     const int* __restrict__ block_table, int table_stride, int page_size, int nq, int nkv, int d,
     int window, float scale, int dv, int keep_first, int sink, const float* __restrict__ sink_values,
-    float cap, const float* __restrict__ slopes) {
+    float cap, const float* __restrict__ slopes, const float* __restrict__ log_r1,
+    const float* __restrict__ log_r2, int out_width, float out_scale) {
     __shared__ float qs[256];
     __shared__ float ps[ATT_THREADS];
     __shared__ int key_page[ATT_THREADS];  // page * nkv + kv head of each key of the tile
@@ -63,6 +65,7 @@ __global__ __launch_bounds__(ATT_THREADS) void attention_generic_kernel(
             s = dot * scale;
             if (cap > 0.f) s = cap * tanhf(s / cap);
             if (slopes) s -= slopes[h] * (float)(pos - j);
+            if (log_r1) s -= log_r1[h] * logf(fmaf(log_r2[h], (float)(pos - j), 1.f));
         }
         const float tile_max = block_max(s, scratch);  // finite: the tile holds >= 1 key
         const float m_new = fmaxf(m, tile_max);
@@ -91,7 +94,7 @@ __global__ __launch_bounds__(ATT_THREADS) void attention_generic_kernel(
         l = l * fa + expf(s0 - m_new);
         acc *= fa;
     }
-    if (tid < dv) out[((size_t)t * nq + h) * dv + tid] = from_float<T>(acc / l);
+    if (tid < dv) out[(size_t)t * out_width + h * dv + tid] = from_float<T>(acc / l * out_scale);
 }
 
 extern "C" int rl_attention_generic(const void* q, const void* k_cache, const void* v_cache,
@@ -99,9 +102,10 @@ extern "C" int rl_attention_generic(const void* q, const void* k_cache, const vo
                                     const int* block_table, int table_stride, int page_size,
                                     int tokens, int nq, int nkv, int d, int window, float scale,
                                     int dv, int keep_first, int sink, const float* sink_values, float cap,
-                                    const float* slopes, int act_type, hipStream_t stream) {
+                                    const float* slopes, const float* log_r1, const float* log_r2, int out_width,
+                                    float out_scale, int act_type, hipStream_t stream) {
     if (tokens <= 0) return RL_OK;
-    if (cap < 0.f) return RL_ERR_ARG;
+    if (cap < 0.f || !log_r1 != !log_r2 || out_width < nq * dv) return RL_ERR_ARG;
     if (d < 1 || d > 256 || dv < 1 || dv > 256 || keep_first < 0 || nkv < 1 || nq % nkv || page_size < 1 ||
         nq > 65535)
         return RL_ERR_ARG;
@@ -110,12 +114,14 @@ extern "C" int rl_attention_generic(const void* q, const void* k_cache, const vo
         hipLaunchKernelGGL(attention_generic_kernel<float>, grid, block, 0, stream,
                            (const float*)q, (const float*)k_cache, (const float*)v_cache,
                            (float*)out, positions, token_slot, block_table, table_stride,
-                           page_size, nq, nkv, d, window, scale, dv, keep_first, sink, sink_values, cap, slopes);
+                           page_size, nq, nkv, d, window, scale, dv, keep_first, sink, sink_values, cap, slopes,
+                           log_r1, log_r2, out_width, out_scale);
     else if (act_type == RL_BF16)
         hipLaunchKernelGGL(attention_generic_kernel<bf16_t>, grid, block, 0, stream,
                            (const bf16_t*)q, (const bf16_t*)k_cache, (const bf16_t*)v_cache,
                            (bf16_t*)out, positions, token_slot, block_table, table_stride,
-                           page_size, nq, nkv, d, window, scale, dv, keep_first, sink, sink_values, cap, slopes);
+                           page_size, nq, nkv, d, window, scale, dv, keep_first, sink, sink_values, cap, slopes,
+                           log_r1, log_r2, out_width, out_scale);
     else
         return RL_ERR_ARG;
     return rl_launch_status();

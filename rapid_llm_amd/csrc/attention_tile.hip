@@ -23,7 +23,11 @@
 //
 // Two options change a score s = (q . k) scale before the softmax: with cap > 0 it becomes
 // cap * tanh(s / cap), and with `slopes` (one number a query head) slope_h * (p - j) is taken off
-// it afterwards.  The sink's term has neither.
+// it afterwards.  The sink's term has neither.  With `log_r1` and `log_r2` (one number a query head
+// each) r1_h * ln(1 + r2_h * (p - j)) is taken off instead.
+//
+// A row's heads lie side by side in a row of `out` of out_width elements; `out_scale` multiplies
+// the finished outputs.
 //
 // A row's result does not depend on the tile it falls in, on the other rows there, or on how a
 // prompt was cut into steps: keys are taken in tiles of 16 at absolute positions 0, 16, ..,
@@ -125,6 +129,18 @@ __device__ inline float ftanh<bf16_t>(float x) {
     return 1.f - 2.f * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(2.8853900817779268f * x));
 }
 
+// logarithms: the library's natural one in float32, the hardware's of base 2 in bfloat16
+template <typename T>
+__device__ inline float flog(float x);
+template <>
+__device__ inline float flog<float>(float x) {
+    return logf(x);
+}
+template <>
+__device__ inline float flog<bf16_t>(float x) {
+    return __builtin_amdgcn_logf(x);
+}
+
 // the four lanes (r, g = 0..3) that share a row: the same bits in each of them.  Two lane swaps
 // of gfx950 (the halves of the wave, then neighbouring rows of 16) instead of two trips through
 // the LDS crossbar; maximum and sum are commutative, so both partners of a swap get the same bits.
@@ -155,12 +171,13 @@ __global__ __launch_bounds__(AW* RL_WAVE) void attn_tile_kernel(
     const int* __restrict__ token_slot, const int* __restrict__ block_table, int table_stride,
     int page_size, int nq, int nkv, int window, int keep_first, int sink, float scale,
     float* __restrict__ part, int nsplit, const float* __restrict__ sink_values, float cap,
-    const float* __restrict__ slopes) {
+    const float* __restrict__ slopes, const float* __restrict__ log_r1, const float* __restrict__ log_r2,
+    int out_width, float out_scale) {
     typedef typename Quad<T>::type quad;
     const float in_log2 = sizeof(T) == 2 ? 1.4426950408889634f : 1.f;  // bfloat16: scores in units of log2
     const float cap_in = cap > 0.f ? scale / cap : 0.f;  // a raw product times this is s / cap
     const float cap_out = cap * in_log2;
-    const bool adjusted = cap > 0.f || slopes != nullptr;
+    const bool adjusted = cap > 0.f || slopes != nullptr || log_r1 != nullptr;
     scale *= in_log2;
     const int tile = blockIdx.x;
     const int hk = blockIdx.y;
@@ -189,14 +206,21 @@ __global__ __launch_bounds__(AW* RL_WAVE) void attn_tile_kernel(
         kend[r] = pos + 1;
         kstart[r] = (window > 0 && pos - window + 1 > 0) ? pos - window + 1 : 0;
     }
-    float slope[R];  // what a position of distance costs this lane's row, in the scores' unit
+    // what a position of distance costs this lane's row, in the scores' unit; or the two numbers of
+    // a logarithmic cost (in bfloat16 a logarithm of base 2 in units of log2: the factors cancel)
+    float slope[R], rate[R];
 #pragma unroll
-    for (int r = 0; r < R; ++r) slope[r] = slopes ? slopes[head[r]] * in_log2 : 0.f;
+    for (int r = 0; r < R; ++r) {
+        slope[r] = log_r1 ? log_r1[head[r]] : (slopes ? slopes[head[r]] * in_log2 : 0.f);
+        rate[r] = log_r1 ? log_r2[head[r]] : 0.f;
+    }
     // a raw product of row r and key `key` as the softmax takes it
     auto scored = [&](float raw, int key, int r) -> float {
         if (!adjusted) return raw * scale;
         const float v = cap > 0.f ? cap_out * ftanh<T>(raw * cap_in) : raw * scale;
-        return v - slope[r] * (float)(kend[r] - 1 - key);
+        const float distance = (float)(kend[r] - 1 - key);
+        if (log_r1) return v - slope[r] * flog<T>(fmaf(rate[r], distance, 1.f));
+        return v - slope[r] * distance;
     };
     const int blocks = min(R, (rows - row0 + 15) / 16);  // blocks of the tile that hold rows
     // keys [all_lo, all_hi) are seen by every row of a block (none where the block is not full):
@@ -482,8 +506,8 @@ __global__ __launch_bounds__(AW* RL_WAVE) void attn_tile_kernel(
                 for (int i = 0; i < 4; ++i) acc[r][b][i] *= fa;
         }
         // acc[r][b][i] is channel 16b + 4g + i of the lane's row
-        T* orow = out + ((size_t)(at + tok[r]) * nq + head[r]) * DV + 4 * g;
-        const float inv = 1.f / l[r];
+        T* orow = out + (size_t)(at + tok[r]) * out_width + head[r] * DV + 4 * g;
+        const float inv = out_scale / l[r];
 #pragma unroll
         for (int b = 0; b < VB; ++b)
             store_quad(orow + 16 * b, (f32x4){acc[r][b][0] * inv, acc[r][b][1] * inv, acc[r][b][2] * inv,
@@ -498,7 +522,7 @@ __global__ __launch_bounds__(AW* RL_WAVE) void attn_tile_kernel(
 __global__ __launch_bounds__(256) void attn_tile_merge_kernel(const float* __restrict__ part,
                                                               bf16_t* __restrict__ out, int rows, int nsplit,
                                                               int sink, const float* __restrict__ sink_values,
-                                                              int nq) {
+                                                              int nq, int out_width, float out_scale) {
     const int row = blockIdx.x * 4 + threadIdx.x / RL_WAVE;
     const int lane = threadIdx.x & (RL_WAVE - 1);
     if (row >= rows) return;
@@ -527,7 +551,7 @@ __global__ __launch_bounds__(256) void attn_tile_merge_kernel(const float* __res
 #pragma unroll
             for (int j = 0; j < 8; ++j) sum += __shfl(weight, (s8 + j) & (RL_WAVE - 1)) * v[j];
         }
-        if (live) out[(size_t)row * DV + c] = float_to_bf16(sum / den);
+        if (live) out[(size_t)(row / nq) * out_width + (row % nq) * DV + c] = float_to_bf16(sum * (out_scale / den));
     }
 }
 
@@ -549,9 +573,11 @@ extern "C" int rl_attn_tile(const void* q, const void* k_cache, const void* v_ca
                             const int* token_slot, const int* block_table, int table_stride,
                             int page_size, int nq, int nkv, int window, int keep_first, int sink,
                             float scale, int nsplit, float* part, int tokens, int tile_rows, int act_type,
-                            const float* sink_values, float cap, const float* slopes, hipStream_t stream) {
+                            const float* sink_values, float cap, const float* slopes, const float* log_r1,
+                            const float* log_r2, int out_width, float out_scale, hipStream_t stream) {
     if (num_tiles <= 0) return RL_OK;
-    if (cap < 0.f) return RL_ERR_ARG;
+    if (cap < 0.f || (slopes && log_r1) || !log_r1 != !log_r2) return RL_ERR_ARG;
+    if (out_width < nq * tileattn::DV || out_width % 4) return RL_ERR_ARG;  // (four channels are stored at once)
     if (nkv < 1 || nq % nkv || page_size < 4 || page_size % 4 || nkv > 65535 || window < 0 || keep_first < 0)
         return RL_ERR_ARG;
     constexpr int AW = 4;
@@ -563,7 +589,7 @@ extern "C" int rl_attn_tile(const void* q, const void* k_cache, const void* v_ca
     if (act_type == RL_BF16 && tile_rows == 16 * PB && PB > 1) {
         if (nsplit != 1) return RL_ERR_ARG;
         hipLaunchKernelGGL((tileattn::attn_tile_kernel<bf16_t, AW, PB>), grid, block, 0, stream, RL_TILE_ARGS(bf16_t),
-                           nullptr, 1, sink_values, cap, slopes);
+                           nullptr, 1, sink_values, cap, slopes, log_r1, log_r2, out_width, out_scale);
         return rl_launch_status();
     }
     if (tile_rows != 16) return RL_ERR_ARG;
@@ -573,18 +599,18 @@ extern "C" int rl_attn_tile(const void* q, const void* k_cache, const void* v_ca
     if (nsplit > 1) {
         if (act_type != RL_BF16 || !part || nsplit > 64 || tokens < 1) return RL_ERR_ARG;
         hipLaunchKernelGGL((tileattn::attn_tile_kernel<bf16_t, AW, 1>), dim3(num_tiles, nkv, nsplit), block, 0, stream,
-                           RL_TILE_ARGS(bf16_t), part, nsplit, sink_values, cap, slopes);
+                           RL_TILE_ARGS(bf16_t), part, nsplit, sink_values, cap, slopes, log_r1, log_r2, out_width, out_scale);
         const int rows = tokens * nq;
         hipLaunchKernelGGL(tileattn::attn_tile_merge_kernel, dim3((rows + 3) / 4), dim3(256), 0, stream, part,
-                           (bf16_t*)out, rows, nsplit, sink, sink_values, nq);
+                           (bf16_t*)out, rows, nsplit, sink, sink_values, nq, out_width, out_scale);
         return rl_launch_status();
     }
     if (act_type == RL_F32)
         hipLaunchKernelGGL((tileattn::attn_tile_kernel<float, AW, 1>), grid, block, 0, stream, RL_TILE_ARGS(float),
-                           nullptr, 1, sink_values, cap, slopes);
+                           nullptr, 1, sink_values, cap, slopes, log_r1, log_r2, out_width, out_scale);
     else if (act_type == RL_BF16)
         hipLaunchKernelGGL((tileattn::attn_tile_kernel<bf16_t, AW, 1>), grid, block, 0, stream, RL_TILE_ARGS(bf16_t),
-                           nullptr, 1, sink_values, cap, slopes);
+                           nullptr, 1, sink_values, cap, slopes, log_r1, log_r2, out_width, out_scale);
     else
         return RL_ERR_ARG;
 #undef RL_TILE_ARGS

@@ -99,12 +99,24 @@ __device__ inline float block_max(float v, float* scratch) {
 
 // The gated activation of a feed-forward, act(gate, up).  limit <= 0: silu(gate) * up.
 // limit > 0: the clamped variant, g = min(gate, limit), u = clamp(up, -limit, limit),
-// g * sigmoid(alpha * g) * (u + 1).
-__device__ inline float glu_act(float g, float u, float limit, float alpha) {
-    if (limit > 0.f) {
-        g = fminf(g, limit);
-        u = fminf(fmaxf(u, -limit), limit);
-        return g / (1.f + expf(-alpha * g)) * (u + 1.f);
+// g * sigmoid(alpha * g) * (u + 1).  gelu: gelu(gate) * up with gelu in its tanh form.
+struct Glu {
+    float limit, alpha;
+    int gelu;
+    const float* bias;  // of the two projections, the I gate entries first, or null
+};
+
+// 0.5 z (1 + tanh(y)) with y = sqrt(2/pi) (z + 0.044715 z^3), as z / (1 + exp(-2 y))
+__device__ inline float gelu_tanh(float z) {
+    return z / (1.f + expf(-1.5957691216057308f * (z + 0.044715f * z * z * z)));
+}
+
+__device__ inline float glu_act(float g, float u, const Glu& glu) {
+    if (glu.gelu) return gelu_tanh(g) * u;
+    if (glu.limit > 0.f) {
+        g = fminf(g, glu.limit);
+        u = fminf(fmaxf(u, -glu.limit), glu.limit);
+        return g / (1.f + expf(-glu.alpha * g)) * (u + 1.f);
     }
     return g / (1.f + expf(-g)) * u;
 }

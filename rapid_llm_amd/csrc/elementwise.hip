@@ -94,7 +94,8 @@ extern "C" int rl_embed(const int* ids, const int* fed, int fed_rows, const void
 }
 
 // --------------------------------------------------------------------------- //
-// residual += delta (float32, in place); out = residual * rsqrt(mean(residual^2)+eps) * w
+// residual += delta (+ bias, float32 [hidden]: that of the product that delta is, or null), float32,
+// in place; out = residual * rsqrt(mean(residual^2)+eps) * w
 // One block per produced row; `rows` (optional) selects which residual rows are produced,
 // packed in order.  rapid_llm/kernels/ops/layernorm/skip_rmsnorm.py:51-85: the sum is
 // formed in float32 and the norm reads the unrounded sum.
@@ -102,7 +103,8 @@ extern "C" int rl_embed(const int* ids, const int* fed, int fed_rows, const void
 template <typename T>
 __global__ void add_rmsnorm_kernel(float* __restrict__ residual, const T* __restrict__ delta,
                                    const float* __restrict__ weight, T* __restrict__ out,
-                                   const int* __restrict__ rows, int hidden, float eps) {
+                                   const int* __restrict__ rows, int hidden, float eps,
+                                       const float* __restrict__ bias) {
     __shared__ float scratch[16];
     const int r = blockIdx.x;
     const int row = rows ? rows[r] : r;
@@ -113,6 +115,7 @@ __global__ void add_rmsnorm_kernel(float* __restrict__ residual, const T* __rest
         float v = res[i];
         if (dl) {
             v += to_float(dl[i]);
+            if (bias) v += bias[i];
             res[i] = v;
         }
         ss += v * v;
@@ -136,7 +139,8 @@ struct alignas(sizeof(T) * 4) Vec4 {
 template <typename T, int CHUNKS>
 __global__ void add_rmsnorm_vec_kernel(float* __restrict__ residual, const T* __restrict__ delta,
                                        const float* __restrict__ weight, T* __restrict__ out,
-                                       const int* __restrict__ rows, int hidden, float eps) {
+                                       const int* __restrict__ rows, int hidden, float eps,
+                                       const float* __restrict__ bias) {
     __shared__ float scratch[16];
     const int r = blockIdx.x;
     const int row = rows ? rows[r] : r;
@@ -164,6 +168,10 @@ __global__ void add_rmsnorm_vec_kernel(float* __restrict__ residual, const T* __
                 v.y += to_float(d.v[1]);
                 v.z += to_float(d.v[2]);
                 v.w += to_float(d.v[3]);
+                if (bias) {
+                    const float4 b = reinterpret_cast<const float4*>(bias)[i];
+                    v.x += b.x; v.y += b.y; v.z += b.z; v.w += b.w;
+                }
                 res[i] = v;
             }
             val[c] = v;
@@ -191,7 +199,7 @@ __global__ void add_rmsnorm_vec_kernel(float* __restrict__ residual, const T* __
 template <typename T>
 static void launch_add_rmsnorm(float* residual, const T* delta, const float* weight, T* out,
                                const int* rows, int out_rows, int hidden, float eps,
-                               hipStream_t stream) {
+                               const float* bias, hipStream_t stream) {
     dim3 grid(out_rows);
     if (hidden % 4 == 0 && hidden <= 16 * 1024) {
         const int nvec = hidden / 4;
@@ -199,28 +207,28 @@ static void launch_add_rmsnorm(float* residual, const T* delta, const float* wei
         int threads = ((nvec + RL_WAVE - 1) / RL_WAVE) * RL_WAVE;
         if (threads <= 1024) {
             hipLaunchKernelGGL((add_rmsnorm_vec_kernel<T, 1>), grid, dim3(threads), 0, stream,
-                               residual, delta, weight, out, rows, hidden, eps);
+                               residual, delta, weight, out, rows, hidden, eps, bias);
         } else {
             hipLaunchKernelGGL((add_rmsnorm_vec_kernel<T, 4>), grid, dim3(1024), 0, stream,
-                               residual, delta, weight, out, rows, hidden, eps);
+                               residual, delta, weight, out, rows, hidden, eps, bias);
         }
         return;
     }
     int threads = hidden >= 2048 ? 512 : (hidden >= 512 ? 256 : 64);
     hipLaunchKernelGGL(add_rmsnorm_kernel<T>, grid, dim3(threads), 0, stream, residual, delta,
-                       weight, out, rows, hidden, eps);
+                       weight, out, rows, hidden, eps, bias);
 }
 
 extern "C" int rl_add_rmsnorm(float* residual, const void* delta, const float* weight, void* out,
                               const int* rows, int out_rows, int hidden, float eps, int act_type,
-                              hipStream_t stream) {
+                              const float* bias, hipStream_t stream) {
     if (out_rows <= 0) return RL_OK;
     if (act_type == RL_F32)
         launch_add_rmsnorm<float>(residual, (const float*)delta, weight, (float*)out, rows,
-                                  out_rows, hidden, eps, stream);
+                                  out_rows, hidden, eps, bias, stream);
     else if (act_type == RL_BF16)
         launch_add_rmsnorm<bf16_t>(residual, (const bf16_t*)delta, weight, (bf16_t*)out, rows,
-                                   out_rows, hidden, eps, stream);
+                                   out_rows, hidden, eps, bias, stream);
     else
         return RL_ERR_ARG;
     return rl_launch_status();
@@ -446,12 +454,13 @@ extern "C" int rl_pair_rows(const float* a, const float* b, void* out, int token
 
 // The same norm where the delta arrives as `nparts` float32 runs of a product's K
 // (parts[run][row][hidden], see rl_gemm_mid_parts): the runs are added in order, the sum is
-// rounded to the activation type as a stored product would be, then added to the residual.
+// rounded to the activation type as a stored product would be, then added to the residual (with
+// the product's bias, where it has one).
 template <typename T, int CHUNKS>
 __global__ void add_parts_rmsnorm_kernel(float* __restrict__ residual, const float* __restrict__ parts,
                                          int nparts, size_t part_stride,
                                          const float* __restrict__ weight, T* __restrict__ out,
-                                         int hidden, float eps) {
+                                         int hidden, float eps, const float* __restrict__ bias) {
     __shared__ float scratch[16];
     const int row = blockIdx.x;
     float4* res = reinterpret_cast<float4*>(residual + (size_t)row * hidden);
@@ -483,6 +492,10 @@ __global__ void add_parts_rmsnorm_kernel(float* __restrict__ residual, const flo
             v.y += to_float(from_float<T>(d.y));
             v.z += to_float(from_float<T>(d.z));
             v.w += to_float(from_float<T>(d.w));
+            if (bias) {
+                const float4 b = reinterpret_cast<const float4*>(bias)[i];
+                v.x += b.x; v.y += b.y; v.z += b.z; v.w += b.w;
+            }
             res[i] = v;
             val[c] = v;
             ss += v.x * v.x + v.y * v.y + v.z * v.z + v.w * v.w;
@@ -509,7 +522,7 @@ __global__ void add_parts_rmsnorm_kernel(float* __restrict__ residual, const flo
 // parts [nparts, rows, hidden] float32, contiguous; bfloat16 rows out; hidden a multiple of 4 up to 16 K
 extern "C" int rl_add_rmsnorm_parts(float* residual, const float* parts, int nparts,
                                     const float* weight, void* out, int rows, int hidden, float eps,
-                                    hipStream_t stream) {
+                                    const float* bias, hipStream_t stream) {
     if (rows <= 0) return RL_OK;
     if (nparts < 1 || hidden % 4 || hidden > 16 * 1024) return RL_ERR_ARG;
     const int nvec = hidden / 4;
@@ -517,10 +530,10 @@ extern "C" int rl_add_rmsnorm_parts(float* residual, const float* parts, int npa
     const size_t stride = (size_t)rows * hidden;
     if (threads <= 1024)
         hipLaunchKernelGGL((add_parts_rmsnorm_kernel<bf16_t, 1>), dim3(rows), dim3(threads), 0, stream,
-                           residual, parts, nparts, stride, weight, (bf16_t*)out, hidden, eps);
+                           residual, parts, nparts, stride, weight, (bf16_t*)out, hidden, eps, bias);
     else
         hipLaunchKernelGGL((add_parts_rmsnorm_kernel<bf16_t, 4>), dim3(rows), dim3(1024), 0, stream,
-                           residual, parts, nparts, stride, weight, (bf16_t*)out, hidden, eps);
+                           residual, parts, nparts, stride, weight, (bf16_t*)out, hidden, eps, bias);
     return rl_launch_status();
 }
 
@@ -528,7 +541,8 @@ extern "C" int rl_add_rmsnorm_parts(float* residual, const float* parts, int npa
 // Gated activation on the packed [gate | up] row: out[:, j] = act(x[:, j], x[:, I + j]).
 // limit <= 0: SwiGLU, silu(g) * u (rapid_llm/kernels/ops/activation/swiglu.py:91-121).
 // limit > 0: the clamped variant, g' = min(g, limit), u' = clamp(u, -limit, limit),
-// g' * sigmoid(alpha * g') * (u' + 1).
+// g' * sigmoid(alpha * g') * (u' + 1).  gelu: gelu(g) * u in gelu's tanh form.  `bias` (float32,
+// [2 I]) is added to gate and up values as they are read.
 // With `route` (float32 [tokens, experts]) the first experts * ff hidden units of a row are those
 // of `experts` experts side by side, and expert e's are multiplied by route[t, e]; with
 // `route_input` the gate and up values are multiplied by it instead, before the activation (an
@@ -536,7 +550,7 @@ extern "C" int rl_add_rmsnorm_parts(float* residual, const float* parts, int npa
 // --------------------------------------------------------------------------- //
 template <typename T>
 __global__ void swiglu_kernel(const T* __restrict__ gate_up, T* __restrict__ out, int inter,
-                              size_t total, float limit, float alpha, const float* __restrict__ route,
+                              size_t total, Glu glu, const float* __restrict__ route,
                               int experts, int ff, int route_input) {
     size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
     const size_t step = (size_t)gridDim.x * blockDim.x;
@@ -544,11 +558,15 @@ __global__ void swiglu_kernel(const T* __restrict__ gate_up, T* __restrict__ out
         const size_t t = idx / inter;
         const int j = (int)(idx - t * inter);
         const T* row = gate_up + t * 2 * (size_t)inter;
-        const float g = to_float(row[j]);
-        const float u = to_float(row[inter + j]);
+        float g = to_float(row[j]);
+        float u = to_float(row[inter + j]);
+        if (glu.bias) {
+            g += glu.bias[j];
+            u += glu.bias[inter + j];
+        }
         const float factor = (route && j < experts * ff) ? route[t * experts + j / ff] : 1.f;
-        const float v = route_input ? glu_act(g * factor, u * factor, limit, alpha)
-                                    : glu_act(g, u, limit, alpha) * factor;
+        const float v = route_input ? glu_act(g * factor, u * factor, glu)
+                                    : glu_act(g, u, glu) * factor;
         out[idx] = from_float<T>(v);
     }
 }
@@ -561,7 +579,7 @@ struct alignas(sizeof(T) * 8) Vec8 {
 
 template <typename T>
 __global__ void swiglu_vec_kernel(const T* __restrict__ gate_up, T* __restrict__ out, int inter,
-                                  size_t total_vec, float limit, float alpha, const float* __restrict__ route,
+                                  size_t total_vec, Glu glu, const float* __restrict__ route,
                                   int experts, int ff, int route_input) {
     size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
     const size_t step = (size_t)gridDim.x * blockDim.x;
@@ -577,43 +595,48 @@ __global__ void swiglu_vec_kernel(const T* __restrict__ gate_up, T* __restrict__
         Vec8<T> y;
 #pragma unroll
         for (int i = 0; i < 8; ++i) {
-            y.v[i] = from_float<T>(
-                route_input ? glu_act(to_float(g.v[i]) * factor, to_float(u.v[i]) * factor, limit, alpha)
-                            : glu_act(to_float(g.v[i]), to_float(u.v[i]), limit, alpha) * factor);
+            float gi = to_float(g.v[i]), ui = to_float(u.v[i]);
+            if (glu.bias) {
+                gi += glu.bias[j + i];
+                ui += glu.bias[inter + j + i];
+            }
+            y.v[i] = from_float<T>(route_input ? glu_act(gi * factor, ui * factor, glu) : glu_act(gi, ui, glu) * factor);
         }
         *reinterpret_cast<Vec8<T>*>(out + t * (size_t)inter + j) = y;
     }
 }
 
 template <typename T>
-static void launch_swiglu(const T* gate_up, T* out, int tokens, int inter, float limit, float alpha,
+static void launch_swiglu(const T* gate_up, T* out, int tokens, int inter, const Glu& glu,
                           const float* route, int experts, int ff, int route_input, hipStream_t stream) {
     if (inter % 8 == 0 && (!route || ff % 8 == 0)) {
         const size_t total = (size_t)tokens * (inter / 8);
         size_t blocks = (total + 255) / 256;
         if (blocks > 65536) blocks = 65536;
         hipLaunchKernelGGL(swiglu_vec_kernel<T>, dim3((unsigned)blocks), dim3(256), 0, stream,
-                           gate_up, out, inter, total, limit, alpha, route, experts, ff, route_input);
+                           gate_up, out, inter, total, glu, route, experts, ff, route_input);
         return;
     }
     const size_t total = (size_t)tokens * inter;
     size_t blocks = (total + 255) / 256;
     if (blocks > 65536) blocks = 65536;
     hipLaunchKernelGGL(swiglu_kernel<T>, dim3((unsigned)blocks), dim3(256), 0, stream, gate_up, out,
-                       inter, total, limit, alpha, route, experts, ff, route_input);
+                       inter, total, glu, route, experts, ff, route_input);
 }
 
 extern "C" int rl_swiglu(const void* gate_up, void* out, int tokens, int inter, int act_type,
                          float limit, float alpha, const float* route, int experts, int ff, int route_input,
-                         hipStream_t stream) {
+                         int gelu, const float* bias, hipStream_t stream) {
     if (tokens <= 0) return RL_OK;
+    if (bias && route_input) return RL_ERR_ARG;  // a scaled input does not scale the bias
+    const Glu glu = {limit, alpha, gelu, bias};
     if (route && (experts < 1 || ff < 1 || (long)experts * ff > inter)) return RL_ERR_ARG;
     if (route_input && !route) return RL_ERR_ARG;
     if (act_type == RL_F32)
-        launch_swiglu<float>((const float*)gate_up, (float*)out, tokens, inter, limit, alpha, route, experts, ff,
+        launch_swiglu<float>((const float*)gate_up, (float*)out, tokens, inter, glu, route, experts, ff,
                              route_input, stream);
     else if (act_type == RL_BF16)
-        launch_swiglu<bf16_t>((const bf16_t*)gate_up, (bf16_t*)out, tokens, inter, limit, alpha, route, experts,
+        launch_swiglu<bf16_t>((const bf16_t*)gate_up, (bf16_t*)out, tokens, inter, glu, route, experts,
                               ff, route_input, stream);
     else
         return RL_ERR_ARG;
@@ -915,6 +938,56 @@ extern "C" int rl_add_bias(void* y, const float* bias, int rows, int cols, int a
 }
 
 // --------------------------------------------------------------------------- //
+// residual[r, :] += first[r, :] + row[:] (float32, in place; either may be null): what a pass over
+// a span of layers begins with, the embedding's output once more and a vector of the pass
+// --------------------------------------------------------------------------- //
+__global__ void stream_add_kernel(float* __restrict__ residual, const float* __restrict__ first,
+                                  const float* __restrict__ row, size_t total, int hidden) {
+    size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
+    const size_t step = (size_t)gridDim.x * blockDim.x;
+    for (; idx < total; idx += step) {
+        float v = residual[idx];
+        if (first) v += first[idx];
+        if (row) v += row[idx % hidden];
+        residual[idx] = v;
+    }
+}
+
+__global__ void stream_add_vec_kernel(float4* __restrict__ residual, const float4* __restrict__ first,
+                                      const float4* __restrict__ row, size_t total, int hidden4) {
+    size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
+    const size_t step = (size_t)gridDim.x * blockDim.x;
+    for (; idx < total; idx += step) {
+        float4 v = residual[idx];
+        if (first) {
+            const float4 f = first[idx];
+            v.x += f.x; v.y += f.y; v.z += f.z; v.w += f.w;
+        }
+        if (row) {
+            const float4 w = row[idx % hidden4];
+            v.x += w.x; v.y += w.y; v.z += w.z; v.w += w.w;
+        }
+        residual[idx] = v;
+    }
+}
+
+extern "C" int rl_stream_add(float* residual, const float* first, const float* row, int tokens, int hidden,
+                             hipStream_t stream) {
+    if (tokens <= 0 || hidden <= 0 || (!first && !row)) return RL_OK;
+    const bool vec = hidden % 4 == 0;
+    const size_t total = (size_t)tokens * hidden / (vec ? 4 : 1);
+    size_t blocks = (total + 255) / 256;
+    if (blocks > 65536) blocks = 65536;
+    if (vec)
+        hipLaunchKernelGGL(stream_add_vec_kernel, dim3((unsigned)blocks), dim3(256), 0, stream, (float4*)residual,
+                           (const float4*)first, (const float4*)row, total, hidden / 4);
+    else
+        hipLaunchKernelGGL(stream_add_kernel, dim3((unsigned)blocks), dim3(256), 0, stream, residual, first, row,
+                           total, hidden);
+    return rl_launch_status();
+}
+
+// --------------------------------------------------------------------------- //
 // gate of a head: y[t, h, :] *= sigmoid(packed[t, gate_col + h]), one number a head, read
 // from a column of the row that the mixer's packed projection wrote
 // --------------------------------------------------------------------------- //
@@ -1003,6 +1076,18 @@ extern "C" int rl_rope_table(const float* inv_freq, float* cos_out, float* sin_o
 // A token at position pos of a request lies in page table[slot_of_request][pos / P] at
 // slot_in_page = pos % P.
 // --------------------------------------------------------------------------- //
+// What may happen to the heads besides norm and rotation.
+struct HeadPrep {
+    const float* bias;  // the projection's, one entry a column of the packed row, added as heads are read
+    // temp_coef != 0: finished queries are multiplied by 1 + temp_coef * ln(floor((pos + 1) / temp_every) + 1)
+    float temp_coef, temp_every;
+    int norm_values;  // every value head is divided by its root mean square (eps inside the root, no weight)
+};
+__device__ inline float query_temperature(const HeadPrep& hp, int pos) {
+    // (the division of two integers below 2^24 rounds to an integer only where it is one)
+    return 1.f + hp.temp_coef * logf(floorf((float)(pos + 1) / hp.temp_every) + 1.f);
+}
+
 template <typename T>
 __global__ void qknorm_rope_kvwrite_kernel(
     const T* __restrict__ qkv, T* __restrict__ q_out, T* __restrict__ k_cache,
@@ -1011,12 +1096,12 @@ __global__ void qknorm_rope_kvwrite_kernel(
     const float* __restrict__ sin_tab, const int* __restrict__ positions,
     const int* __restrict__ token_slot, const int* __restrict__ block_table, int table_stride,
     int page_size, int nq, int nkv, int d, int rotary_half, int interleaved, float eps,
-    int write_cache, int write_values, int head0, int row_width, int v_col0, int dv, const float* bias) {
+    int write_cache, int write_values, int head0, int row_width, int v_col0, int dv, HeadPrep hp) {
     const int t = blockIdx.x;
     const int lane = threadIdx.x & (RL_WAVE - 1);
     const int wave = threadIdx.x / RL_WAVE;
     const int nwaves = blockDim.x / RL_WAVE;
-    const int half = d / 2;
+    const int half = (d + 1) / 2;  // of an odd size the last pair holds one channel
     const int pos = positions[t];
     const int total_heads = nq + 2 * nkv;
     const T* row = qkv + (size_t)t * row_width;
@@ -1038,9 +1123,18 @@ __global__ void qknorm_rope_kvwrite_kernel(
             const int h = head - nq - nkv;
             const T* xv = row + v_col0 + (size_t)h * dv;  // where the row keeps this value head
             T* dst = v_cache + ((page * nkv + h) * dv) * page_size + off;
+            const float* vb = hp.bias ? hp.bias + v_col0 + (size_t)h * dv : nullptr;
+            float factor = 1.f;
+            if (hp.norm_values) {
+                float ss = 0.f;
+                for (int i = lane; i < dv; i += RL_WAVE) {
+                    const float v = to_float(xv[i]) + (vb ? vb[i] : 0.f);
+                    ss += v * v;
+                }
+                factor = rsqrtf(wave_sum(ss) / (float)dv + eps);
+            }
             for (int i = lane; i < dv; i += RL_WAVE)
-                dst[(size_t)i * page_size] =
-                    bias ? from_float<T>(to_float(xv[i]) + bias[v_col0 + (size_t)h * dv + i]) : xv[i];
+                dst[(size_t)i * page_size] = from_float<T>((to_float(xv[i]) + (vb ? vb[i] : 0.f)) * factor);
             continue;
         }
         const bool is_q = head < nq;
@@ -1062,10 +1156,10 @@ __global__ void qknorm_rope_kvwrite_kernel(
             x2[r] = 0.f;
             if (p < half) {
                 x1[r] = to_float(x[e1[r]]);
-                x2[r] = to_float(x[e2[r]]);
-                if (bias) {  // the projection's bias, added here instead of by a kernel of its own
-                    x1[r] += bias[(size_t)head * d + e1[r]];
-                    x2[r] += bias[(size_t)head * d + e2[r]];
+                if (e2[r] < d) x2[r] = to_float(x[e2[r]]);
+                if (hp.bias) {  // the projection's bias, added here instead of by a kernel of its own
+                    x1[r] += hp.bias[(size_t)head * d + e1[r]];
+                    if (e2[r] < d) x2[r] += hp.bias[(size_t)head * d + e2[r]];
                 }
                 ss += x1[r] * x1[r] + x2[r] * x2[r];
             }
@@ -1075,6 +1169,7 @@ __global__ void qknorm_rope_kvwrite_kernel(
             ss = wave_sum(ss);
             rrms = rsqrtf(ss / (float)d + eps);
         }
+        const float temp = (is_q && hp.temp_coef != 0.f) ? query_temperature(hp, pos) : 1.f;
         T* dst;
         if (is_q)
             dst = q_out + ((size_t)t * nq + head) * d;
@@ -1087,7 +1182,7 @@ __global__ void qknorm_rope_kvwrite_kernel(
                 float a = x1[r], b = x2[r];
                 if (w) {
                     a = a * rrms * w[e1[r]];
-                    b = b * rrms * w[e2[r]];
+                    if (e2[r] < d) b = b * rrms * w[e2[r]];
                 }
                 if (p < rot) {
                     const float c = cos_tab[(size_t)pos * rotary_half + p];
@@ -1097,8 +1192,8 @@ __global__ void qknorm_rope_kvwrite_kernel(
                     a = ra;
                     b = rb;
                 }
-                dst[e1[r]] = from_float<T>(a);
-                dst[e2[r]] = from_float<T>(b);
+                dst[e1[r]] = from_float<T>(a * temp);
+                if (e2[r] < d) dst[e2[r]] = from_float<T>(b * temp);
             }
         }
     }
@@ -1115,7 +1210,7 @@ __device__ inline void qknorm_rope_kvwrite_vec(
     const float* __restrict__ sin_tab, const int* __restrict__ positions,
     const int* __restrict__ token_slot, const int* __restrict__ block_table, int table_stride,
     int page_size, int nq, int nkv, int d, float eps, int write_cache, int write_values, int head0,
-    int row_width, int v_col0, int dv, const float* bias) {
+    int row_width, int v_col0, int dv, HeadPrep hp) {
     constexpr int HPW = RL_WAVE / LPH;  // heads per wave
     const int lane = threadIdx.x & (RL_WAVE - 1);
     const int wave = threadIdx.x / RL_WAVE;
@@ -1140,9 +1235,20 @@ __device__ inline void qknorm_rope_kvwrite_vec(
         const int h = head - nq - nkv;
         const T* xv = row + v_col0 + (size_t)h * dv;
         T* dst = v_cache + ((page * nkv + h) * dv) * page_size + off;
+        const float* vb = hp.bias ? hp.bias + v_col0 + (size_t)h * dv : nullptr;
+        float factor = 1.f;
+        if (hp.norm_values) {
+            float ss = 0.f;
+            for (int i = li; i < dv; i += LPH) {
+                const float v = to_float(xv[i]) + (vb ? vb[i] : 0.f);
+                ss += v * v;
+            }
+#pragma unroll
+            for (int o = LPH / 2; o > 0; o >>= 1) ss += __shfl_xor(ss, o, RL_WAVE);
+            factor = rsqrtf(ss / (float)dv + eps);
+        }
         for (int i = li; i < dv; i += LPH)
-            dst[(size_t)i * page_size] =
-                bias ? from_float<T>(to_float(xv[i]) + bias[v_col0 + (size_t)h * dv + i]) : xv[i];
+            dst[(size_t)i * page_size] = from_float<T>((to_float(xv[i]) + (vb ? vb[i] : 0.f)) * factor);
         return;
     }
     const bool is_q = head < nq;
@@ -1157,9 +1263,9 @@ __device__ inline void qknorm_rope_kvwrite_vec(
         for (int k = 0; k < 4; ++k) {
             a[k] = to_float(va.v[k]);
             b[k] = to_float(vb.v[k]);
-            if (bias) {
-                a[k] += bias[(size_t)head * d + 4 * li + k];
-                b[k] += bias[(size_t)head * d + half + 4 * li + k];
+            if (hp.bias) {
+                a[k] += hp.bias[(size_t)head * d + 4 * li + k];
+                b[k] += hp.bias[(size_t)head * d + half + 4 * li + k];
             }
             ss += a[k] * a[k] + b[k] * b[k];
         }
@@ -1190,11 +1296,12 @@ __device__ inline void qknorm_rope_kvwrite_vec(
     }
     T* dst = is_q ? q_out + ((size_t)t * nq + head) * d
                   : k_cache + ((page * nkv + (head - nq)) * page_size + off) * d;
+    const float temp = (is_q && hp.temp_coef != 0.f) ? query_temperature(hp, pos) : 1.f;
     Vec4<T> oa, ob;
 #pragma unroll
     for (int k = 0; k < 4; ++k) {
-        oa.v[k] = from_float<T>(a[k]);
-        ob.v[k] = from_float<T>(b[k]);
+        oa.v[k] = from_float<T>(a[k] * temp);
+        ob.v[k] = from_float<T>(b[k] * temp);
     }
     *reinterpret_cast<Vec4<T>*>(dst + 4 * li) = oa;
     *reinterpret_cast<Vec4<T>*>(dst + half + 4 * li) = ob;
@@ -1208,11 +1315,11 @@ __global__ __launch_bounds__(256) void qknorm_rope_kvwrite_vec_kernel(
     const float* __restrict__ sin_tab, const int* __restrict__ positions,
     const int* __restrict__ token_slot, const int* __restrict__ block_table, int table_stride,
     int page_size, int nq, int nkv, int d, float eps, int write_cache, int write_values, int head0,
-    int row_width, int v_col0, int dv, const float* bias) {
+    int row_width, int v_col0, int dv, HeadPrep hp) {
     qknorm_rope_kvwrite_vec<T, LPH>(blockIdx.x, blockIdx.y, qkv, q_out, k_cache, v_cache, q_norm_w, k_norm_w,
                                     cos_tab, sin_tab, positions, token_slot, block_table, table_stride,
                                     page_size, nq, nkv, d, eps, write_cache, write_values, head0, row_width,
-                                    v_col0, dv, bias);
+                                    v_col0, dv, hp);
 }
 
 template <typename T>
@@ -1221,7 +1328,7 @@ static void launch_qknorm(const T* qkv, T* q_out, T* k_cache, T* v_cache, const 
                           const int* positions, const int* token_slot, const int* block_table,
                           int table_stride, int page_size, int tokens, int nq, int nkv, int d,
                           int rotary_half, int interleaved, float eps, int write_cache,
-                          int write_values, int head0, int row_width, int v_col0, int dv, const float* bias, hipStream_t stream) {
+                          int write_values, int head0, int row_width, int v_col0, int dv, HeadPrep hp, hipStream_t stream) {
     const int total_heads = nq + (write_values ? 2 * nkv : nkv) - head0;  // heads to work on
     // the vectorised kernel: head sizes in steps of 8, the half-split rotation of the whole head
     if (d % 8 == 0 && (!cos_tab || (rotary_half == d / 2 && !interleaved))) {
@@ -1233,12 +1340,12 @@ static void launch_qknorm(const T* qkv, T* q_out, T* k_cache, T* v_cache, const 
             hipLaunchKernelGGL((qknorm_rope_kvwrite_vec_kernel<T, 16>), grid, block, 0, stream, qkv,
                                q_out, k_cache, v_cache, q_norm_w, k_norm_w, cos_tab, sin_tab,
                                positions, token_slot, block_table, table_stride, page_size, nq, nkv,
-                               d, eps, write_cache, write_values, head0, row_width, v_col0, dv, bias);
+                               d, eps, write_cache, write_values, head0, row_width, v_col0, dv, hp);
         else
             hipLaunchKernelGGL((qknorm_rope_kvwrite_vec_kernel<T, 32>), grid, block, 0, stream, qkv,
                                q_out, k_cache, v_cache, q_norm_w, k_norm_w, cos_tab, sin_tab,
                                positions, token_slot, block_table, table_stride, page_size, nq, nkv,
-                               d, eps, write_cache, write_values, head0, row_width, v_col0, dv, bias);
+                               d, eps, write_cache, write_values, head0, row_width, v_col0, dv, hp);
         return;
     }
     const int head_groups = (total_heads + 3) / 4;
@@ -1246,7 +1353,7 @@ static void launch_qknorm(const T* qkv, T* q_out, T* k_cache, T* v_cache, const 
     hipLaunchKernelGGL(qknorm_rope_kvwrite_kernel<T>, grid, block, 0, stream, qkv, q_out, k_cache,
                        v_cache, q_norm_w, k_norm_w, cos_tab, sin_tab, positions, token_slot,
                        block_table, table_stride, page_size, nq, nkv, d, rotary_half, interleaved, eps,
-                       write_cache, write_values, head0, row_width, v_col0, dv, bias);
+                       write_cache, write_values, head0, row_width, v_col0, dv, hp);
 }
 
 // Values of 16 consecutive tokens of the batch and one kv head, written by one workgroup.
@@ -1262,10 +1369,11 @@ template <typename T>
 __device__ inline void v_tile_write(
     int tile, int h, const T* __restrict__ qkv, T* __restrict__ v_cache, const int* __restrict__ positions,
     const int* __restrict__ token_slot, const int* __restrict__ block_table, int table_stride,
-    int page_size, int tokens, int nq, int nkv, int d, int row_width, int v_col0, int dv, const float* bias) {
-    __shared__ T vt[VT_TOKENS][256 + 8];
+    int page_size, int tokens, int nq, int nkv, int d, int row_width, int v_col0, int dv, float eps, HeadPrep hp) {
+    __shared__ float vt[VT_TOKENS][256 + 8];
     __shared__ int s_page[VT_TOKENS];
     __shared__ int s_off[VT_TOKENS];
+    __shared__ float s_factor[VT_TOKENS];
     const int t0 = tile * VT_TOKENS;
     if (threadIdx.x < VT_TOKENS) {
         const int t = t0 + threadIdx.x;
@@ -1281,11 +1389,21 @@ __device__ inline void v_tile_write(
     for (int idx = threadIdx.x; idx < VT_TOKENS * dv; idx += 256) {
         const int i = idx / dv, c = idx - i * dv;
         if (t0 + i < tokens) {
-            const T v = qkv[(size_t)(t0 + i) * row_width + v_col0 + (size_t)h * dv + c];
-            vt[i][c] = bias ? from_float<T>(to_float(v) + bias[v_col0 + (size_t)h * dv + c]) : v;
+            const float v = to_float(qkv[(size_t)(t0 + i) * row_width + v_col0 + (size_t)h * dv + c]);
+            vt[i][c] = hp.bias ? v + hp.bias[v_col0 + (size_t)h * dv + c] : v;
         }
     }
     __syncthreads();
+    if (hp.norm_values) {  // sixteen threads a token
+        const int i = threadIdx.x / 16;
+        float ss = 0.f;
+        if (t0 + i < tokens)
+            for (int c = threadIdx.x % 16; c < dv; c += 16) ss += vt[i][c] * vt[i][c];
+#pragma unroll
+        for (int o = 8; o > 0; o >>= 1) ss += __shfl_xor(ss, o, RL_WAVE);
+        if (threadIdx.x % 16 == 0) s_factor[i] = rsqrtf(ss / (float)dv + eps);
+        __syncthreads();
+    }
     for (int idx = threadIdx.x; idx < 4 * dv; idx += 256) {
         const int quarter = idx & 3, c = idx >> 2;
         const int i0 = 4 * quarter;
@@ -1297,14 +1415,16 @@ __device__ inline void v_tile_write(
         if (lined_up) {
             Vec4<T> v;
 #pragma unroll
-            for (int k = 0; k < 4; ++k) v.v[k] = vt[i0 + k][c];
+            for (int k = 0; k < 4; ++k)
+                v.v[k] = from_float<T>(hp.norm_values ? vt[i0 + k][c] * s_factor[i0 + k] : vt[i0 + k][c]);
             *reinterpret_cast<Vec4<T>*>(v_cache + (((size_t)page * nkv + h) * dv + c) * page_size + off) = v;
         } else {
 #pragma unroll
             for (int k = 0; k < 4; ++k) {
                 const int pg = s_page[i0 + k];
                 if (pg >= 0)
-                    v_cache[(((size_t)pg * nkv + h) * dv + c) * page_size + s_off[i0 + k]] = vt[i0 + k][c];
+                    v_cache[(((size_t)pg * nkv + h) * dv + c) * page_size + s_off[i0 + k]] =
+                        from_float<T>(hp.norm_values ? vt[i0 + k][c] * s_factor[i0 + k] : vt[i0 + k][c]);
             }
         }
     }
@@ -1321,17 +1441,17 @@ __global__ __launch_bounds__(256) void qkv_prepare_kernel(
     const float* __restrict__ sin_tab, const int* __restrict__ positions,
     const int* __restrict__ token_slot, const int* __restrict__ block_table, int table_stride,
     int page_size, int tokens, int head_groups, int nq, int nkv, int d, float eps, int head0,
-    int row_width, int v_col0, int dv, const float* bias) {
+    int row_width, int v_col0, int dv, HeadPrep hp) {
     const int qk_blocks = tokens * head_groups;
     if ((int)blockIdx.x < qk_blocks) {
         qknorm_rope_kvwrite_vec<T, LPH>(blockIdx.x / head_groups, blockIdx.x % head_groups, qkv, q_out, k_cache,
                                         v_cache, q_norm_w, k_norm_w, cos_tab, sin_tab, positions, token_slot,
                                         block_table, table_stride, page_size, nq, nkv, d, eps, 1, 0, head0,
-                                        row_width, v_col0, dv, bias);
+                                        row_width, v_col0, dv, hp);
     } else {
         const int b = blockIdx.x - qk_blocks;
         v_tile_write<T>(b / nkv, b % nkv, qkv, v_cache, positions, token_slot, block_table, table_stride,
-                        page_size, tokens, nq, nkv, d, row_width, v_col0, dv, bias);
+                        page_size, tokens, nq, nkv, d, row_width, v_col0, dv, eps, hp);
     }
 }
 
@@ -1339,9 +1459,9 @@ template <typename T>
 __global__ __launch_bounds__(256) void v_tile_write_kernel(
     const T* __restrict__ qkv, T* __restrict__ v_cache, const int* __restrict__ positions,
     const int* __restrict__ token_slot, const int* __restrict__ block_table, int table_stride,
-    int page_size, int tokens, int nq, int nkv, int d, int row_width, int v_col0, int dv, const float* bias) {
+    int page_size, int tokens, int nq, int nkv, int d, int row_width, int v_col0, int dv, float eps, HeadPrep hp) {
     v_tile_write<T>(blockIdx.x, blockIdx.y, qkv, v_cache, positions, token_slot, block_table, table_stride,
-                    page_size, tokens, nq, nkv, d, row_width, v_col0, dv, bias);
+                    page_size, tokens, nq, nkv, d, row_width, v_col0, dv, eps, hp);
 }
 
 // true if it launched: head sizes in steps of 8, and a grid that fits
@@ -1350,7 +1470,7 @@ static bool launch_qkv_prepare(const T* qkv, T* q_out, T* k_cache, T* v_cache, c
                                const float* k_norm_w, const float* cos_tab, const float* sin_tab,
                                const int* positions, const int* token_slot, const int* block_table,
                                int table_stride, int page_size, int tokens, int nq, int nkv, int d,
-                               float eps, int head0, int row_width, int v_col0, int dv, const float* bias, hipStream_t stream) {
+                               float eps, int head0, int row_width, int v_col0, int dv, HeadPrep hp, hipStream_t stream) {
     if (d % 8) return false;
     const int lph = d <= 128 ? 16 : 32;
     const int heads_per_block = 4 * (RL_WAVE / lph);
@@ -1362,12 +1482,12 @@ static bool launch_qkv_prepare(const T* qkv, T* q_out, T* k_cache, T* v_cache, c
         hipLaunchKernelGGL((qkv_prepare_kernel<T, 16>), grid, block, 0, stream, qkv, q_out, k_cache, v_cache,
                            q_norm_w, k_norm_w, cos_tab, sin_tab, positions, token_slot, block_table,
                            table_stride, page_size, tokens, head_groups, nq, nkv, d, eps, head0, row_width,
-                           v_col0, dv, bias);
+                           v_col0, dv, hp);
     else
         hipLaunchKernelGGL((qkv_prepare_kernel<T, 32>), grid, block, 0, stream, qkv, q_out, k_cache, v_cache,
                            q_norm_w, k_norm_w, cos_tab, sin_tab, positions, token_slot, block_table,
                            table_stride, page_size, tokens, head_groups, nq, nkv, d, eps, head0, row_width,
-                           v_col0, dv, bias);
+                           v_col0, dv, hp);
     return true;
 }
 
@@ -1377,9 +1497,13 @@ extern "C" int rl_qknorm_rope_kvwrite(const void* qkv, void* q_out, void* k_cach
                                       const int* positions, const int* token_slot,
                                       const int* block_table, int table_stride, int page_size,
                                       int tokens, int nq, int nkv, int d, int rotary_half,
-                                      int interleaved, float eps, int write_cache, int row_width, int v_col0, int dv, const float* bias, int act_type, hipStream_t stream) {
+                                      int interleaved, float eps, int write_cache, int row_width, int v_col0, int dv,
+                                      const float* bias, float temp_coef, float temp_every, int norm_values,
+                                      int act_type, hipStream_t stream) {
     if (tokens <= 0) return RL_OK;
-    if (d % 2 || d > 256) return RL_ERR_ARG;
+    if (temp_coef != 0.f && !(temp_every > 0.f && q_out)) return RL_ERR_ARG;
+    const HeadPrep hp = {bias, temp_coef, temp_every, norm_values};
+    if (d < 1 || (d % 2 && cos_tab) || d > 256) return RL_ERR_ARG;
     // the packed row: query heads from column 0, key heads behind them, the nkv value heads of dv
     // channels from column v_col0 on ((nq + nkv) * d: behind the keys; nq * d: the values are the
     // unrotated keys)
@@ -1401,34 +1525,34 @@ extern "C" int rl_qknorm_rope_kvwrite(const void* qkv, void* q_out, void* k_cach
     if (tile_values && whole_split && act_type == RL_F32 &&
         launch_qkv_prepare<float>((const float*)qkv, (float*)q_out, (float*)k_cache, (float*)v_cache, q_norm_w,
                                   k_norm_w, cos_tab, sin_tab, positions, token_slot, block_table,
-                                  table_stride, page_size, tokens, nq, nkv, d, eps, head0, row_width, v_col0, dv, bias,
+                                  table_stride, page_size, tokens, nq, nkv, d, eps, head0, row_width, v_col0, dv, hp,
                                   stream))
         return rl_launch_status();
     if (tile_values && whole_split && act_type == RL_BF16 &&
         launch_qkv_prepare<bf16_t>((const bf16_t*)qkv, (bf16_t*)q_out, (bf16_t*)k_cache, (bf16_t*)v_cache,
                                    q_norm_w, k_norm_w, cos_tab, sin_tab, positions, token_slot, block_table,
-                                   table_stride, page_size, tokens, nq, nkv, d, eps, head0, row_width, v_col0, dv, bias,
+                                   table_stride, page_size, tokens, nq, nkv, d, eps, head0, row_width, v_col0, dv, hp,
                                    stream))
         return rl_launch_status();
     if (act_type == RL_F32) {
         launch_qknorm<float>((const float*)qkv, (float*)q_out, (float*)k_cache, (float*)v_cache,
                              q_norm_w, k_norm_w, cos_tab, sin_tab, positions, token_slot,
                              block_table, table_stride, page_size, tokens, nq, nkv, d, rotary_half,
-                             interleaved, eps, write_cache, !tile_values, head0, row_width, v_col0, dv, bias, stream);
+                             interleaved, eps, write_cache, !tile_values, head0, row_width, v_col0, dv, hp, stream);
         if (tile_values)
             hipLaunchKernelGGL(v_tile_write_kernel<float>, vgrid, block, 0, stream,
                                (const float*)qkv, (float*)v_cache, positions, token_slot,
-                               block_table, table_stride, page_size, tokens, nq, nkv, d, row_width, v_col0, dv, bias);
+                               block_table, table_stride, page_size, tokens, nq, nkv, d, row_width, v_col0, dv, eps, hp);
     } else if (act_type == RL_BF16) {
         launch_qknorm<bf16_t>((const bf16_t*)qkv, (bf16_t*)q_out, (bf16_t*)k_cache,
                               (bf16_t*)v_cache, q_norm_w, k_norm_w, cos_tab, sin_tab, positions,
                               token_slot, block_table, table_stride, page_size, tokens, nq, nkv, d,
                               rotary_half, interleaved, eps, write_cache, !tile_values, head0, row_width,
-                              v_col0, dv, bias, stream);
+                              v_col0, dv, hp, stream);
         if (tile_values)
             hipLaunchKernelGGL(v_tile_write_kernel<bf16_t>, vgrid, block, 0, stream,
                                (const bf16_t*)qkv, (bf16_t*)v_cache, positions, token_slot,
-                               block_table, table_stride, page_size, tokens, nq, nkv, d, row_width, v_col0, dv, bias);
+                               block_table, table_stride, page_size, tokens, nq, nkv, d, row_width, v_col0, dv, eps, hp);
     } else {
         return RL_ERR_ARG;
     }

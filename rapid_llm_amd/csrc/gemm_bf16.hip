@@ -97,8 +97,9 @@ struct SkinnyExtra {
     const float* norm_w;  // [N]
     bf16_t* xt;           // [M, N] residual * norm_w
     float* partial;       // [workgroups][16]
-    // the gated activation of the gate/up variants (limit 0: silu(gate) * up)
-    float glu_limit, glu_alpha;
+    const float* bias;    // [N] added to the product in front of the residual, or null
+    // the gated activation of the gate/up variants
+    Glu glu;
 };
 
 // LASTQ: groups of four rows of the last tile that belong to the workgroup: 4, or 2 for
@@ -171,7 +172,7 @@ __global__ __launch_bounds__(GW* RL_WAVE) void gemm_skinny_kernel(
     // (Asking for a scaled input's partial sums this early was measured and lost 1.5 us a
     // product: loads return in order, and the weights then wait behind them.)
     static_assert(NT * 64 <= GW * RL_WAVE, "every result of the workgroup has a thread of its own");
-    float res_in[4] = {0.f, 0.f, 0.f, 0.f}, nw_in[4] = {0.f, 0.f, 0.f, 0.f};
+    float res_in[4] = {0.f, 0.f, 0.f, 0.f}, nw_in[4] = {0.f, 0.f, 0.f, 0.f}, bias_in[4] = {0.f, 0.f, 0.f, 0.f};
     if (!SWIGLU && ex.residual && threadIdx.x < NT * 64) {
         const int ln = threadIdx.x & 63, ot = threadIdx.x >> 6, m = ln & 15;
         const int nbase = blockIdx.x * ROWS + ot * 16 + 4 * (ln >> 4);
@@ -181,6 +182,7 @@ __global__ __launch_bounds__(GW* RL_WAVE) void gemm_skinny_kernel(
             if (m < M && mine && nbase + i < N) {
                 res_in[i] = ex.residual[(size_t)m * N + nbase + i];
                 nw_in[i] = ex.norm_w[nbase + i];
+                if (ex.bias) bias_in[i] = ex.bias[nbase + i];
             }
     }
 
@@ -327,7 +329,11 @@ __global__ __launch_bounds__(GW* RL_WAVE) void gemm_skinny_kernel(
                     // path does where the product's result is stored before the activation
                     gate = bf16_to_float(float_to_bf16(gate * scale));
                     up = bf16_to_float(float_to_bf16(up * scale));
-                    v = glu_act(gate, up, ex.glu_limit, ex.glu_alpha);
+                    if (ex.glu.bias) {
+                        gate += ex.glu.bias[n];
+                        up += ex.glu.bias[N + n];
+                    }
+                    v = glu_act(gate, up, ex.glu);
                 } else {
                     v = 0.f;
 #pragma unroll
@@ -336,7 +342,7 @@ __global__ __launch_bounds__(GW* RL_WAVE) void gemm_skinny_kernel(
                 }
                 if (!SWIGLU && ex.residual) {
                     const size_t at = (size_t)m * N + n;
-                    const float r = res_in[i] + bf16_to_float(float_to_bf16(v));
+                    const float r = res_in[i] + bf16_to_float(float_to_bf16(v)) + bias_in[i];
                     ex.residual[at] = r;
                     ex.xt[at] = float_to_bf16(r * nw_in[i]);
                     sumsq += r * r;
@@ -527,7 +533,11 @@ __global__ __launch_bounds__(GW* RL_WAVE) void gemm_swiglu_stream_kernel(
             // operands rounded to bfloat16, as where the product's result is stored first
             gate = bf16_to_float(float_to_bf16(gate * scale));
             up = bf16_to_float(float_to_bf16(up * scale));
-            out[(size_t)m * ldo + nbase + i] = float_to_bf16(glu_act(gate, up, ex.glu_limit, ex.glu_alpha));
+            if (ex.glu.bias) {
+                gate += ex.glu.bias[nbase + i];
+                up += ex.glu.bias[I + nbase + i];
+            }
+            out[(size_t)m * ldo + nbase + i] = float_to_bf16(glu_act(gate, up, ex.glu));
         }
     }
 }
@@ -619,13 +629,12 @@ extern "C" int rl_gemm_skinny(const void* X, const void* W, void* out, int M, in
 extern "C" int rl_gemm_skinny_swiglu(const void* X, const void* W, void* out, int M, int I, int K,
                                      int ldx, int ldw, int ldo, int nt, int units, const float* x_partial,
                                      int x_parts, int x_size, float x_eps, float glu_limit, float glu_alpha,
-                                     hipStream_t stream) {
+                                     int glu_gelu, const float* glu_bias, hipStream_t stream) {
     if (M <= 0 || I <= 0) return RL_OK;
     if (!skinny_args_ok(M, K, ldx, ldw) || ldo < I || (x_partial && (x_parts < 1 || x_size < 1)))
         return RL_ERR_ARG;
     SkinnyExtra ex = scaled_input(x_partial, x_parts, x_size, x_eps);
-    ex.glu_limit = glu_limit;
-    ex.glu_alpha = glu_alpha;
+    ex.glu = {glu_limit, glu_alpha, glu_gelu, glu_bias};
     int rc = RL_OK;
     if (nt >= 0 && swiglu_stream((const bf16_t*)X, (const bf16_t*)W, (bf16_t*)out, M, I, K, ldx, ldw, ldo, units,
                                  ex, stream, &rc))
@@ -634,7 +643,7 @@ extern "C" int rl_gemm_skinny_swiglu(const void* X, const void* W, void* out, in
                                   ldw, ldo, nt < 0 ? -nt : nt, ex, stream);
 }
 
-// The product with the residual epilogue: residual[M, N] += X W^T (rounded to bfloat16),
+// The product with the residual epilogue: residual[M, N] += X W^T (rounded to bfloat16) + bias (or null),
 // xt[M, N] = residual * norm_w as bfloat16, partial[workgroup][16] = sums of squares of the
 // workgroup's columns per row.  Returns the number of workgroups through *parts (the caller
 // sizes `partial` with rl_gemm_skinny_parts).
@@ -642,7 +651,7 @@ extern "C" int rl_gemm_skinny_parts(int N, int nt) { return (N + nt * 16 - 1) / 
 
 extern "C" int rl_gemm_skinny_residual(const void* X, const void* W, int M, int N, int K, int ldx,
                                        int ldw, int nt, float* residual, const float* norm_w,
-                                       void* xt, float* partial, hipStream_t stream) {
+                                       void* xt, float* partial, const float* bias, hipStream_t stream) {
     if (M <= 0 || N <= 0) return RL_OK;
     if (!skinny_args_ok(M, K, ldx, ldw) || !residual || !norm_w || !xt || !partial) return RL_ERR_ARG;
     SkinnyExtra ex = {};
@@ -650,6 +659,7 @@ extern "C" int rl_gemm_skinny_residual(const void* X, const void* W, int M, int 
     ex.norm_w = norm_w;
     ex.xt = (bf16_t*)xt;
     ex.partial = partial;
+    ex.bias = bias;
     return dispatch<bf16_t, false>((const bf16_t*)X, (const bf16_t*)W, (bf16_t*)nullptr, M, N, K,
                                    ldx, ldw, N, nt, ex, stream);
 }
@@ -816,7 +826,7 @@ extern "C" int rl_gemm_mid_parts(const void* X, const void* W, float* part, int 
 template <int MB, bool SWIGLU>
 __global__ __launch_bounds__(MW* RL_WAVE) void gemm_tile_kernel(
     const bf16_t* __restrict__ X, const bf16_t* __restrict__ W, bf16_t* __restrict__ out, int M,
-    int N, int K, int ldx, int ldw, int ldo, float glu_limit, float glu_alpha) {
+    int N, int K, int ldx, int ldw, int ldo, Glu glu) {
     __shared__ __attribute__((aligned(16))) unsigned char xs[2][MB * 16 * WT_PITCH];
     __shared__ __attribute__((aligned(16))) unsigned char wtile[MW][16 * WT_PITCH];
     const int tid = threadIdx.x, lane = tid & (RL_WAVE - 1), wave = tid / RL_WAVE;
@@ -915,9 +925,14 @@ __global__ __launch_bounds__(MW* RL_WAVE) void gemm_tile_kernel(
         for (int mb = 0; mb < MB; ++mb)
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
-                const float gate = bf16_to_float(float_to_bf16(acc[mb][i]));
-                const float u = bf16_to_float(float_to_bf16(up[((wave * MB + mb) * 4 + i) * RL_WAVE + lane]));
-                acc[mb][i] = glu_act(gate, u, glu_limit, glu_alpha);
+                float gate = bf16_to_float(float_to_bf16(acc[mb][i]));
+                float u = bf16_to_float(float_to_bf16(up[((wave * MB + mb) * 4 + i) * RL_WAVE + lane]));
+                if (glu.bias) {
+                    const int n = min(n0 + 4 * g + i, N - 1);  // (columns beyond are not stored)
+                    gate += glu.bias[n];
+                    u += glu.bias[N + n];
+                }
+                acc[mb][i] = glu_act(gate, u, glu);
             }
     }
 #pragma unroll
@@ -943,7 +958,9 @@ __global__ __launch_bounds__(MW* RL_WAVE) void gemm_tile_kernel(
 // out[M, N] = X W^T as bfloat16 (swiglu == 0), or out[M, N] = silu(X Wg^T) * (X Wu^T) with
 // W = [Wg | Wu] stacked by rows, [2N, K].  K a multiple of 128, ldo a multiple of 4.
 extern "C" int rl_gemm_tile(const void* X, const void* W, void* out, int M, int N, int K, int ldx,
-                            int ldw, int ldo, int swiglu, float glu_limit, float glu_alpha, hipStream_t stream) {
+                            int ldw, int ldo, int swiglu, float glu_limit, float glu_alpha, int glu_gelu,
+                            const float* glu_bias, hipStream_t stream) {
+    const Glu glu = {glu_limit, glu_alpha, glu_gelu, glu_bias};
     if (M <= 0 || N <= 0) return RL_OK;
     if (K < KSTEP || K % KSTEP || ldx % 8 || ldw % 8 || ldx < K || ldw < K || ldo % 4 || ldo < N || !out)
         return RL_ERR_ARG;
@@ -959,10 +976,10 @@ extern "C" int rl_gemm_tile(const void* X, const void* W, void* out, int M, int 
     do {                                                                                          \
         if (swiglu)                                                                               \
             hipLaunchKernelGGL((gemm_tile_kernel<MBV, true>), grid, block, 0, stream, x, w, o, M, \
-                               N, K, ldx, ldw, ldo, glu_limit, glu_alpha);                        \
+                               N, K, ldx, ldw, ldo, glu);                                         \
         else                                                                                      \
             hipLaunchKernelGGL((gemm_tile_kernel<MBV, false>), grid, block, 0, stream, x, w, o,   \
-                               M, N, K, ldx, ldw, ldo, 0.f, 0.f);                                 \
+                               M, N, K, ldx, ldw, ldo, glu);                                      \
     } while (0)
     if (mb == 1)
         RL_TILE(1);

@@ -1,6 +1,7 @@
 // Recurrent mixers with a fixed-size state per request: the token-shift mixes and the per-head
-// scan of an RWKV-style time mixing, and the causal convolution, the scan and the grouped norm of a
-// state-space mixer.  Everything between the projections is float32: mixes of the decay branch,
+// scan of an RWKV-style time mixing; the causal convolution, the scan and the grouped norm of a
+// state-space mixer; the prepared operands and the scan of a gated delta rule with a decay per key
+// channel; and a gated recurrence without a matrix state (minGRU).  Everything between the projections is float32: mixes of the decay branch,
 // decays, step sizes, states, sums, norms; the element type T only says how the projections'
 // results are read and the mixers' outputs written.
 //
@@ -204,7 +205,7 @@ constexpr int SCAN_COLS = 4 * SCAN_WAVES;          // columns of a workgroup: 4 
 // token with r, k, v (d each), the decay w_i = exp(-exp(pre_i + bias_i)), formed as a block of
 // tokens is fetched, and the bonus u_i:
 //   o_j = sum_i r_i (S_ij + u_i k_i v_j)        S_ij <- w_i S_ij + k_i v_j
-// o goes out unfinished (float32); wkv_finish_kernel divides every head by its root mean square
+// o goes out unfinished (float32); head_finish_kernel divides every head by its root mean square
 // and applies the norm's weight and silu(g).
 // --------------------------------------------------------------------------- //
 // one state element's share of a token (the same instructions wherever a token is computed)
@@ -318,24 +319,30 @@ __global__ __launch_bounds__(SCAN_THREADS) __attribute__((amdgpu_waves_per_eu(1,
     state_rows_store<RPL>(Sp, c * RPL, d, live, state);
 }
 
-// out[t, head] = raw / sqrt(mean(raw^2) + eps) * norm_w * silu(g): one wave a (token, head)
+// out[t, head] = raw / sqrt(mean(raw^2) + eps) * norm_w * gate: one wave a (token, head).  The norm's
+// weight has an entry a channel of every head, or (`shared_w`) of one head, for all of them; the gate
+// is silu(g) or (`sigmoid_gate`) sigmoid(g).
 template <typename T>
-__global__ __launch_bounds__(256) void wkv_finish_kernel(const float* __restrict__ raw, const T* __restrict__ g,
-                                                         const float* __restrict__ norm_w, T* __restrict__ out,
-                                                         int rows, int heads, int d, float eps) {
+__global__ __launch_bounds__(256) void head_finish_kernel(const float* __restrict__ raw, const T* __restrict__ g,
+                                                          const float* __restrict__ norm_w, T* __restrict__ out,
+                                                          int rows, int heads, int d, float eps, int shared_w,
+                                                          int sigmoid_gate) {
     const int row = blockIdx.x * 4 + threadIdx.x / RL_WAVE;  // (token, head)
     const int lane = threadIdx.x & (RL_WAVE - 1);
     if (row >= rows) return;  // whole waves leave
     const size_t base = (size_t)row * d;
-    const int h = row % heads;
+    const float* w = norm_w + (shared_w ? 0 : (size_t)(row % heads) * d);
     float ss = 0.f;
     for (int i = lane; i < d; i += RL_WAVE) {
         const float o = raw[base + i];
         ss += o * o;
     }
     const float rr = rsqrtf(wave_sum(ss) / (float)d + eps);
-    for (int i = lane; i < d; i += RL_WAVE)
-        out[base + i] = from_float<T>(raw[base + i] * rr * norm_w[h * d + i] * silu(to_float(g[base + i])));
+    for (int i = lane; i < d; i += RL_WAVE) {
+        const float z = to_float(g[base + i]);
+        const float gate = sigmoid_gate ? 1.f / (1.f + expf(-z)) : silu(z);
+        out[base + i] = from_float<T>(raw[base + i] * rr * w[i] * gate);
+    }
 }
 
 // --------------------------------------------------------------------------- //
@@ -558,6 +565,354 @@ __global__ __launch_bounds__(256) void group_rmsnorm_kernel(const float* __restr
         out[base + i] = from_float<T>(y[base + i] * rr * w[blockIdx.y * size + i]);
 }
 
+// --------------------------------------------------------------------------- //
+// Gated delta rule with a decay per key channel.  The packed rows hold, from column col0 on,
+// [q: kv_heads * d | k: kv_heads * d | v: heads * dv]; every channel passes a causal convolution over
+// time (the state rows before a request's first token, as above) and silu; then every head of q and k
+// is made a unit vector (x / sqrt(sum x^2 + 1e-6)) and q is multiplied by d^(-1/2).  The decays'
+// pre-activations become g = exp(-exp(A_log_h) softplus(pre + dt_bias)) in place.
+//
+// One wave takes one head of q, k, v or of the decays for per_group consecutive tokens of the flat
+// batch, EPL adjacent channels a lane; with TAPS > 0 the inputs of the last TAPS - 1 tokens stay in
+// its registers, so that an input is read once.  In a step of single tokens (`single`) the wave
+// shifts its request's convolution rows itself, otherwise conv_state_kernel does in a second launch.
+// --------------------------------------------------------------------------- //
+constexpr float UNIT_EPS = 1e-6f;
+constexpr int PREPARE_TOKENS = 8;
+
+__device__ inline float softplus(float x) { return x > 20.f ? x : log1pf(expf(x)); }
+
+template <typename T, int TAPS, int EPL>
+__global__ __launch_bounds__(256) void delta_prepare_kernel(
+    const T* __restrict__ packed, int row_width, int col0, const float* __restrict__ w, float* __restrict__ state,
+    float* __restrict__ decay, const float* __restrict__ dt_bias, const float* __restrict__ a_log,
+    float* __restrict__ mixed, const int* __restrict__ cu, const int* __restrict__ seq_slots, int num_seqs, int tokens,
+    int heads, int kv_heads, int d, int dv, int taps, int single, int per_group) {
+    const int head = blockIdx.y * 4 + threadIdx.x / RL_WAVE;
+    const int lane = threadIdx.x & (RL_WAVE - 1);
+    const int convolved = 2 * kv_heads + heads;
+    if (head >= convolved + heads) return;  // whole waves leave; no barrier follows
+    const int first = blockIdx.x * per_group, last = min(tokens, first + per_group);
+    if (head >= convolved) {
+        const int h = head - convolved;
+        const float rate = expf(a_log[h]);
+        for (int t = first; t < last; ++t)
+#pragma unroll
+            for (int e = 0; e < EPL; ++e) {
+                const int i = lane * EPL + e;
+                if (i >= d) continue;
+                float* at = decay + (size_t)t * heads * d + h * d + i;
+                *at = expf(-rate * softplus(*at + dt_bias[h * d + i]));
+            }
+        return;
+    }
+    const bool is_v = head >= 2 * kv_heads, is_q = head < kv_heads;
+    const int size = is_v ? dv : d;
+    const int c0 = is_v ? 2 * kv_heads * d + (head - 2 * kv_heads) * dv : head * d;  // of the convolved channels
+    const int channels = 2 * kv_heads * d + heads * dv;
+    const int reach = TAPS > 0 ? TAPS : taps;
+    const int held = reach - 1;
+    constexpr int WT = TAPS > 0 ? TAPS : 1, WIN = TAPS > 1 ? TAPS - 1 : 1;
+    float wt[EPL][WT], win[EPL][WIN];
+    if constexpr (TAPS > 0) {
+#pragma unroll
+        for (int e = 0; e < EPL; ++e)
+#pragma unroll
+            for (int tap = 0; tap < TAPS; ++tap)
+                wt[e][tap] = lane * EPL + e < size ? w[(size_t)(c0 + lane * EPL + e) * TAPS + tap] : 0.f;
+    }
+    int s = single ? first : request_of(cu, num_seqs, first);
+    const float* st = nullptr;
+    // what the channel at `c` met `back` tokens before token t, the offset-th of its portion
+    auto input = [&](int t, int offset, int back, int c) -> float {
+        return back <= offset ? to_float(packed[(size_t)(t - back) * row_width + col0 + c])
+                              : st[(size_t)(held + offset - back) * channels + c];
+    };
+    bool fresh = true;  // the window does not hold the tokens before this one yet
+    for (int t = first; t < last; ++t) {
+        if (single) {
+            s = t;
+            fresh = true;
+        } else {
+            while (t >= cu[s + 1]) {  // tokens ascend through the requests
+                ++s;
+                fresh = true;
+            }
+        }
+        const int offset = single ? 0 : t - cu[s];
+        if (fresh) st = state + (size_t)seq_slots[s] * max(held, 1) * channels;
+        float y[EPL], now[EPL];
+        float ss = 0.f;
+#pragma unroll
+        for (int e = 0; e < EPL; ++e) {
+            const int i = lane * EPL + e, c = c0 + i;
+            const bool live = i < size;
+            now[e] = live ? to_float(packed[(size_t)t * row_width + col0 + c]) : 0.f;
+            float acc = 0.f;
+            if constexpr (TAPS > 0) {
+                if (fresh) {
+#pragma unroll
+                    for (int q = 0; q < TAPS - 1; ++q) win[e][q] = live ? input(t, offset, TAPS - 1 - q, c) : 0.f;
+                }
+#pragma unroll
+                for (int tap = 0; tap < TAPS - 1; ++tap) acc = fmaf(wt[e][tap], win[e][tap], acc);
+                acc = fmaf(wt[e][TAPS - 1], now[e], acc);
+            } else if (live) {
+                for (int tap = 0; tap < held; ++tap)
+                    acc = fmaf(w[(size_t)c * reach + tap], input(t, offset, held - tap, c), acc);
+                acc = fmaf(w[(size_t)c * reach + held], now[e], acc);
+            }
+            y[e] = live ? silu(acc) : 0.f;
+            ss += y[e] * y[e];
+        }
+        float factor = 1.f;
+        if (!is_v) {
+            factor = rsqrtf(wave_sum(ss) + UNIT_EPS);
+            if (is_q) factor *= rsqrtf((float)d);
+        }
+        float* dst = mixed + (size_t)t * channels + c0;
+#pragma unroll
+        for (int e = 0; e < EPL; ++e) {
+            const int i = lane * EPL + e;
+            if (i < size) dst[i] = y[e] * factor;
+            if (single && held > 0 && i < size) {
+                float* rows = state + (size_t)seq_slots[s] * held * channels + c0 + i;
+                for (int q = 0; q + 1 < held; ++q) rows[(size_t)q * channels] = rows[(size_t)(q + 1) * channels];
+                rows[(size_t)(held - 1) * channels] = now[e];
+            }
+            if constexpr (TAPS > 1) {
+#pragma unroll
+                for (int q = 0; q + 1 < TAPS - 1; ++q) win[e][q] = win[e][q + 1];
+                win[e][TAPS - 2] = now[e];
+            }
+        }
+        fresh = false;
+    }
+}
+
+// The scan.  Per head (head h reads q and k of kv head h / (heads / kv_heads)), state S[key channel i]
+// [value channel j], kept as [j][i]; for a token with q, k, v, the decays g and beta = sigmoid(b):
+//   S_ij <- g_i S_ij      u_j = beta (v_j - sum_i S_ij k_i)      S_ij <- S_ij + k_i u_j      o_j = sum_i S_ij q_i
+// The sum that u needs stands between two tokens and is folded at once; the read-out's sums are folded
+// behind a block of tokens.  o goes out unfinished (float32).
+template <int RPL>
+__global__ __launch_bounds__(SCAN_THREADS) __attribute__((amdgpu_waves_per_eu(1, 2))) void delta_scan_kernel(
+    const float* __restrict__ mixed, const float* __restrict__ decay, const float* __restrict__ beta_pre,
+    int beta_width, float* __restrict__ raw, const int* __restrict__ cu, const int* __restrict__ seq_slots,
+    float* __restrict__ S, int heads, int kv_heads, int d, int dv) {
+    constexpr int DP = 16 * RPL;  // rows, padded
+    constexpr int PER_THREAD = SCAN_TOKENS * DP / SCAN_THREADS;  // = RPL
+    const int s = blockIdx.x, h = blockIdx.y;
+    const int t0 = cu[s], t1 = cu[s + 1];
+    const int channels = 2 * kv_heads * d + heads * dv;
+    const int hk = h / (heads / kv_heads);
+    const int lane = threadIdx.x & (RL_WAVE - 1), wave = threadIdx.x / RL_WAVE;
+    const int c = lane & 15;
+    const int col = wave * 4 + (lane >> 4);
+    const int j = blockIdx.z * SCAN_COLS + col;
+    const bool live = j < dv;
+    __shared__ __attribute__((aligned(16))) float sq[SCAN_TOKENS][DP], sk[SCAN_TOKENS][DP], sg[SCAN_TOKENS][DP];
+    __shared__ float sv[SCAN_TOKENS][SCAN_COLS], sb[SCAN_TOKENS];
+    float* Sp = S + (((size_t)seq_slots[s] * heads + h) * dv + (live ? j : 0)) * d;
+    float state[RPL];
+    state_rows_load<RPL>(Sp, c * RPL, d, live, state);
+    float pq[PER_THREAD], pk[PER_THREAD], pg[PER_THREAD], pv = 0.f, pb = 0.f;
+    auto fetch = [&](int tb) {
+#pragma unroll
+        for (int e = 0; e < PER_THREAD; ++e) {
+            const int idx = e * SCAN_THREADS + threadIdx.x;
+            const int tt = idx / DP, i = idx % DP;
+            const bool ok = tb + tt < t1 && i < d;
+            const float* row = mixed + (size_t)(tb + tt) * channels + hk * d + i;
+            pq[e] = ok ? row[0] : 0.f;
+            pk[e] = ok ? row[kv_heads * d] : 0.f;
+            pg[e] = ok ? decay[(size_t)(tb + tt) * heads * d + h * d + i] : 0.f;
+        }
+        const int tt = threadIdx.x / SCAN_COLS, jj = blockIdx.z * SCAN_COLS + threadIdx.x % SCAN_COLS;
+        const bool ok = tt < SCAN_TOKENS && tb + tt < t1;
+        pv = (ok && jj < dv) ? mixed[(size_t)(tb + tt) * channels + 2 * kv_heads * d + h * dv + jj] : 0.f;
+        const int tk = threadIdx.x;
+        pb = (tk < SCAN_TOKENS && tb + tk < t1) ? beta_pre[(size_t)(tb + tk) * beta_width + h] : 0.f;
+    };
+    auto stage = [&]() {
+#pragma unroll
+        for (int e = 0; e < PER_THREAD; ++e) {
+            const int idx = e * SCAN_THREADS + threadIdx.x;
+            (&sq[0][0])[idx] = pq[e];
+            (&sk[0][0])[idx] = pk[e];
+            (&sg[0][0])[idx] = pg[e];
+        }
+        if (threadIdx.x < SCAN_TOKENS * SCAN_COLS) (&sv[0][0])[threadIdx.x] = pv;
+        if (threadIdx.x < SCAN_TOKENS) sb[threadIdx.x] = 1.f / (1.f + expf(-pb));
+    };
+    fetch(t0);
+    for (int tb = t0; tb < t1; tb += SCAN_TOKENS) {
+        __syncthreads();  // the block before has been read by every wave
+        stage();
+        __syncthreads();
+        if (tb + SCAN_TOKENS < t1) fetch(tb + SCAN_TOKENS);
+        const int nt = min(SCAN_TOKENS, t1 - tb);
+        auto token = [&](int tt) -> float {  // this lane's rows' share of the token's output
+            float even = 0.f, odd = 0.f;
+#pragma unroll
+            for (int ii = 0; ii < RPL; ++ii) {
+                state[ii] *= sg[tt][c * RPL + ii];
+                float& sum = (ii & 1) ? odd : even;
+                sum = fmaf(state[ii], sk[tt][c * RPL + ii], sum);
+            }
+            const float u = sb[tt] * (sv[tt][col] - row16_sum(even + odd));
+            float o = 0.f;
+#pragma unroll
+            for (int ii = 0; ii < RPL; ++ii) {
+                state[ii] = fmaf(sk[tt][c * RPL + ii], u, state[ii]);
+                o = fmaf(state[ii], sq[tt][c * RPL + ii], o);
+            }
+            return o;
+        };
+        float* dst = raw + (size_t)tb * heads * dv + h * dv + j;
+        if (nt == SCAN_TOKENS) {
+            float os[SCAN_TOKENS];
+#pragma unroll
+            for (int tt = 0; tt < SCAN_TOKENS; ++tt) os[tt] = token(tt);
+            row16_sums(os);
+            // every lane of a column holds all sixteen sums: lane c stores token c's
+            float mine = os[0];
+#pragma unroll
+            for (int tt = 1; tt < SCAN_TOKENS; ++tt) mine = c == tt ? os[tt] : mine;
+            if (live) dst[(size_t)c * heads * dv] = mine;
+        } else {
+            for (int tt = 0; tt < nt; ++tt) {
+                const float o = row16_sum(token(tt));
+                if (c == 0 && live) dst[(size_t)tt * heads * dv] = o;
+            }
+        }
+    }
+    state_rows_store<RPL>(Sp, c * RPL, d, live, state);
+}
+
+// --------------------------------------------------------------------------- //
+// Gated recurrence whose gates read the current token alone (minGRU).  With z = sigmoid(zp + bz) and
+// u = xp + bx of the packed row's columns z0 and x0 on, per channel
+//   S <- (1 - z) S + z (u >= 0 ? u + 1/2 : sigmoid(u))        out = scale * S * silu(gp)
+// The chain between tokens is one fused multiply-add, everything else is independent of it: a
+// workgroup takes 8 channels and 64 tokens at a time, all its threads form the two factors, eight
+// lanes walk the chain through LDS, all threads finish the outputs.
+// --------------------------------------------------------------------------- //
+constexpr int GRU_CHANNELS = 8;
+constexpr int GRU_TOKENS = 64;
+
+// float32 keeps the library's exponential and division, bfloat16 takes the hardware's instructions
+template <typename T>
+__device__ inline float sigmoid_of(float x);
+template <>
+__device__ inline float sigmoid_of<float>(float x) {
+    return 1.f / (1.f + expf(-x));
+}
+template <>
+__device__ inline float sigmoid_of<bf16_t>(float x) {
+    return __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(-1.4426950408889634f * x));
+}
+
+// the two factors of the chain
+template <typename T>
+__device__ inline void gru_factors(float zp, float u, float& keep, float& add) {
+    const float z = sigmoid_of<T>(zp);
+    const float candidate = u >= 0.f ? u + 0.5f : sigmoid_of<T>(u);
+    keep = 1.f - z;
+    add = z * candidate;
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void gru_scan_kernel(const T* __restrict__ packed, int row_width, int z0, int x0,
+                                                       int g0, const float* __restrict__ bz,
+                                                       const float* __restrict__ bx, float* __restrict__ S,
+                                                       T* __restrict__ out, int out_width, float scale,
+                                                       const int* __restrict__ cu, const int* __restrict__ seq_slots,
+                                                       int width) {
+    constexpr int PER = GRU_TOKENS * GRU_CHANNELS / 256;
+    const int s = blockIdx.x;
+    const int t0 = cu[s], t1 = cu[s + 1];
+    const int c = blockIdx.y * GRU_CHANNELS + threadIdx.x % GRU_CHANNELS;
+    const int tt0 = threadIdx.x / GRU_CHANNELS;  // and every 32nd token behind it
+    const bool live = c < width;
+    __shared__ float keep[GRU_TOKENS][GRU_CHANNELS], add[GRU_TOKENS][GRU_CHANNELS], sums[GRU_TOKENS][GRU_CHANNELS];
+    const float zb = live ? bz[c] : 0.f, xb = live ? bx[c] : 0.f;
+    float* slot = S + (size_t)seq_slots[s] * width + c;
+    float state = (threadIdx.x < GRU_CHANNELS && live) ? *slot : 0.f;
+    const T zero = from_float<T>(0.f);
+    T pz[PER], px[PER], pg[PER];
+    auto fetch = [&](int tb) {
+#pragma unroll
+        for (int e = 0; e < PER; ++e) {
+            const int t = tb + tt0 + e * (256 / GRU_CHANNELS);
+            const bool ok = live && t < t1;
+            const T* row = packed + (size_t)t * row_width + c;
+            pz[e] = ok ? row[z0] : zero;
+            px[e] = ok ? row[x0] : zero;
+            pg[e] = ok ? row[g0] : zero;
+        }
+    };
+    fetch(t0);
+    for (int tb = t0; tb < t1; tb += GRU_TOKENS) {
+        float gate[PER];
+#pragma unroll
+        for (int e = 0; e < PER; ++e) {
+            const int tt = tt0 + e * (256 / GRU_CHANNELS);
+            gru_factors<T>(to_float(pz[e]) + zb, to_float(px[e]) + xb, keep[tt][threadIdx.x % GRU_CHANNELS],
+                           add[tt][threadIdx.x % GRU_CHANNELS]);
+            const float z = to_float(pg[e]);
+            gate[e] = scale * z * sigmoid_of<T>(z);
+        }
+        __syncthreads();
+        if (tb + GRU_TOKENS < t1) fetch(tb + GRU_TOKENS);
+        const int nt = min(GRU_TOKENS, t1 - tb);
+        if (threadIdx.x < GRU_CHANNELS) {
+            if (nt == GRU_TOKENS) {
+#pragma unroll 16
+                for (int tt = 0; tt < GRU_TOKENS; ++tt) {
+                    state = fmaf(keep[tt][threadIdx.x], state, add[tt][threadIdx.x]);
+                    sums[tt][threadIdx.x] = state;
+                }
+            } else {
+                for (int tt = 0; tt < nt; ++tt) {
+                    state = fmaf(keep[tt][threadIdx.x], state, add[tt][threadIdx.x]);
+                    sums[tt][threadIdx.x] = state;
+                }
+            }
+        }
+        __syncthreads();
+#pragma unroll
+        for (int e = 0; e < PER; ++e) {
+            const int tt = tt0 + e * (256 / GRU_CHANNELS);
+            if (live && tb + tt < t1)
+                out[(size_t)(tb + tt) * out_width + c] = from_float<T>(gate[e] * sums[tt][threadIdx.x % GRU_CHANNELS]);
+        }
+        // (the next round's factors do not touch `sums`, and its chain starts behind a barrier)
+    }
+    if (threadIdx.x < GRU_CHANNELS && live) *slot = state;
+}
+
+// a step of single tokens: one thread a (request, channel)
+template <typename T>
+__global__ __launch_bounds__(256) void gru_single_kernel(const T* __restrict__ packed, int row_width, int z0, int x0,
+                                                         int g0, const float* __restrict__ bz,
+                                                         const float* __restrict__ bx, float* __restrict__ S,
+                                                         T* __restrict__ out, int out_width, float scale,
+                                                         const int* __restrict__ seq_slots, int width) {
+    const int t = blockIdx.x;  // the request's only token
+    const int c = blockIdx.y * 256 + threadIdx.x;
+    if (c >= width) return;
+    const T* row = packed + (size_t)t * row_width + c;
+    float* slot = S + (size_t)seq_slots[t] * width + c;
+    float keep, add;
+    gru_factors<T>(to_float(row[z0]) + bz[c], to_float(row[x0]) + bx[c], keep, add);
+    const float state = fmaf(keep, *slot, add);
+    *slot = state;
+    const float z = to_float(row[g0]);
+    const float gate = scale * z * sigmoid_of<T>(z);
+    out[(size_t)t * out_width + c] = from_float<T>(gate * state);
+}
+
 }  // namespace recurrent
 
 extern "C" int rl_recurrent_max_head_dim() { return 256; }
@@ -610,8 +965,8 @@ static int launch_wkv(const T* r, const T* k, const T* v, const T* g, const floa
         RL_WKV(16);
 #undef RL_WKV
     const int heads_rows = tokens * heads;
-    hipLaunchKernelGGL(recurrent::wkv_finish_kernel<T>, dim3((heads_rows + 3) / 4), dim3(256), 0, stream, raw, g,
-                       norm_w, out, heads_rows, heads, d, eps);
+    hipLaunchKernelGGL(recurrent::head_finish_kernel<T>, dim3((heads_rows + 3) / 4), dim3(256), 0, stream, raw, g,
+                       norm_w, out, heads_rows, heads, d, eps, 0, 0);
     return rl_launch_status();
 }
 
@@ -719,4 +1074,146 @@ extern "C" int rl_group_rmsnorm(const float* y, const float* w, void* out, int t
     else
         return RL_ERR_ARG;
     return rl_launch_status();
+}
+
+template <typename T, int TAPS, int EPL>
+static void launch_delta_prepare(const T* packed, int row_width, int col0, const float* w, float* state, float* decay,
+                                 const float* dt_bias, const float* a_log, float* mixed, const int* cu,
+                                 const int* seq_slots, int num_seqs, int tokens, int heads, int kv_heads, int d, int dv,
+                                 int taps, hipStream_t stream) {
+    const int single = tokens == num_seqs;  // every request brings one token
+    const int per_group = single ? 1 : recurrent::PREPARE_TOKENS;
+    dim3 grid((tokens + per_group - 1) / per_group, (2 * kv_heads + 2 * heads + 3) / 4);
+    hipLaunchKernelGGL((recurrent::delta_prepare_kernel<T, TAPS, EPL>), grid, dim3(256), 0, stream, packed, row_width,
+                       col0, w, state, decay, dt_bias, a_log, mixed, cu, seq_slots, num_seqs, tokens, heads, kv_heads,
+                       d, dv, taps, single, per_group);
+    if (!single && taps > 1) {
+        const int channels = 2 * kv_heads * d + heads * dv;
+        hipLaunchKernelGGL(recurrent::conv_state_kernel<T>, dim3(num_seqs, (channels + 255) / 256), dim3(256), 0, stream,
+                           packed, row_width, col0, state, cu, seq_slots, channels, taps);
+    }
+}
+
+template <typename T>
+static int delta_prepare(const T* packed, int row_width, int col0, const float* w, float* state, float* decay,
+                         const float* dt_bias, const float* a_log, float* mixed, const int* cu, const int* seq_slots,
+                         int num_seqs, int tokens, int heads, int kv_heads, int d, int dv, int taps,
+                         hipStream_t stream) {
+    const int widest = d > dv ? d : dv;
+#define RL_PREPARE(TAPS, EPL)                                                                                        \
+    launch_delta_prepare<T, TAPS, EPL>(packed, row_width, col0, w, state, decay, dt_bias, a_log, mixed, cu, seq_slots, \
+                                       num_seqs, tokens, heads, kv_heads, d, dv, taps, stream)
+#define RL_PREPARE_TAPS(TAPS)         \
+    do {                              \
+        if (widest <= 64)             \
+            RL_PREPARE(TAPS, 1);      \
+        else if (widest <= 128)       \
+            RL_PREPARE(TAPS, 2);      \
+        else                          \
+            RL_PREPARE(TAPS, 4);      \
+    } while (0)
+    if (taps == 4)
+        RL_PREPARE_TAPS(4);
+    else
+        RL_PREPARE_TAPS(0);
+#undef RL_PREPARE_TAPS
+#undef RL_PREPARE
+    return rl_launch_status();
+}
+
+// decay: the decays' pre-activations [tokens, heads * d], replaced by the decays; mixed:
+// [tokens, 2 * kv_heads * d + heads * dv] float32
+extern "C" int rl_delta_prepare(const void* packed, int row_width, int col0, const float* w, float* state,
+                                float* decay, const float* dt_bias, const float* a_log, float* mixed, const int* cu,
+                                const int* seq_slots, int num_seqs, int tokens, int heads, int kv_heads, int d, int dv,
+                                int taps, int act_type, hipStream_t stream) {
+    if (tokens <= 0 || num_seqs <= 0) return RL_OK;
+    if (heads < 1 || kv_heads < 1 || heads % kv_heads || heads > 65535 || d < 1 || d > 256 || dv < 1 || dv > 256 ||
+        taps < 1 || taps > RL_CONV_MAX_TAPS || col0 < 0 || col0 + 2 * kv_heads * d + heads * dv > row_width ||
+        num_seqs > tokens)
+        return RL_ERR_ARG;
+    if (act_type == RL_F32)
+        return delta_prepare<float>((const float*)packed, row_width, col0, w, state, decay, dt_bias, a_log, mixed, cu,
+                                    seq_slots, num_seqs, tokens, heads, kv_heads, d, dv, taps, stream);
+    if (act_type == RL_BF16)
+        return delta_prepare<bf16_t>((const bf16_t*)packed, row_width, col0, w, state, decay, dt_bias, a_log, mixed, cu,
+                                     seq_slots, num_seqs, tokens, heads, kv_heads, d, dv, taps, stream);
+    return RL_ERR_ARG;
+}
+
+// beta_pre: a float32 row of beta_width a token whose first `heads` entries are the pre-activations;
+// raw: [tokens, heads * dv] float32
+extern "C" int rl_delta_scan(const float* mixed, const float* decay, const float* beta_pre, int beta_width, float* raw,
+                             const int* cu, const int* seq_slots, float* S, int num_seqs, int tokens, int heads,
+                             int kv_heads, int d, int dv, hipStream_t stream) {
+    if (tokens <= 0 || num_seqs <= 0) return RL_OK;
+    if (heads < 1 || heads > 65535 || kv_heads < 1 || heads % kv_heads || d < 1 || d > 256 || dv < 1 || dv > 256 ||
+        beta_width < heads || num_seqs > 65535)
+        return RL_ERR_ARG;
+    dim3 grid(num_seqs, heads, (dv + recurrent::SCAN_COLS - 1) / recurrent::SCAN_COLS);
+#define RL_DELTA(RPL)                                                                                               \
+    hipLaunchKernelGGL((recurrent::delta_scan_kernel<RPL>), grid, dim3(recurrent::SCAN_THREADS), 0, stream, mixed, decay, \
+                       beta_pre, beta_width, raw, cu, seq_slots, S, heads, kv_heads, d, dv)
+    const int rows = (d + 15) / 16;
+    if (rows <= 1)
+        RL_DELTA(1);
+    else if (rows <= 2)
+        RL_DELTA(2);
+    else if (rows <= 4)
+        RL_DELTA(4);
+    else if (rows <= 8)
+        RL_DELTA(8);
+    else
+        RL_DELTA(16);
+#undef RL_DELTA
+    return rl_launch_status();
+}
+
+// raw, g and out: [tokens, heads * d]; norm_w: [heads * d], or [d] with shared_w
+extern "C" int rl_head_finish(const float* raw, const void* g, const float* norm_w, void* out, int tokens, int heads,
+                              int d, float eps, int shared_w, int sigmoid_gate, int act_type, hipStream_t stream) {
+    if (tokens <= 0) return RL_OK;
+    if (heads < 1 || d < 1) return RL_ERR_ARG;
+    const int rows = tokens * heads;
+    if (act_type == RL_F32)
+        hipLaunchKernelGGL(recurrent::head_finish_kernel<float>, dim3((rows + 3) / 4), dim3(256), 0, stream, raw,
+                           (const float*)g, norm_w, (float*)out, rows, heads, d, eps, shared_w, sigmoid_gate);
+    else if (act_type == RL_BF16)
+        hipLaunchKernelGGL(recurrent::head_finish_kernel<bf16_t>, dim3((rows + 3) / 4), dim3(256), 0, stream, raw,
+                           (const bf16_t*)g, norm_w, (bf16_t*)out, rows, heads, d, eps, shared_w, sigmoid_gate);
+    else
+        return RL_ERR_ARG;
+    return rl_launch_status();
+}
+
+template <typename T>
+static int launch_gru(const T* packed, int row_width, int z0, int x0, int g0, const float* bz, const float* bx,
+                      float* S, T* out, int out_width, float scale, const int* cu, const int* seq_slots, int num_seqs,
+                      int tokens, int width, hipStream_t stream) {
+    if (tokens == num_seqs)  // every request brings one token
+        hipLaunchKernelGGL(recurrent::gru_single_kernel<T>, dim3(tokens, (width + 255) / 256), dim3(256), 0, stream,
+                           packed, row_width, z0, x0, g0, bz, bx, S, out, out_width, scale, seq_slots, width);
+    else
+        hipLaunchKernelGGL(recurrent::gru_scan_kernel<T>,
+                           dim3(num_seqs, (width + recurrent::GRU_CHANNELS - 1) / recurrent::GRU_CHANNELS), dim3(256), 0,
+                           stream, packed, row_width, z0, x0, g0, bz, bx, S, out, out_width, scale, cu, seq_slots,
+                           width);
+    return rl_launch_status();
+}
+
+// out: the first of `width` columns of rows of out_width elements
+extern "C" int rl_gru_scan(const void* packed, int row_width, int z0, int x0, int g0, const float* bz, const float* bx,
+                           float* S, void* out, int out_width, float scale, const int* cu, const int* seq_slots,
+                           int num_seqs, int tokens, int width, int act_type, hipStream_t stream) {
+    if (tokens <= 0 || num_seqs <= 0) return RL_OK;
+    if (width < 1 || width > 65535 * recurrent::GRU_CHANNELS || out_width < width || num_seqs > tokens) return RL_ERR_ARG;
+    for (int col : {z0, x0, g0})
+        if (col < 0 || col + width > row_width) return RL_ERR_ARG;
+    if (act_type == RL_F32)
+        return launch_gru<float>((const float*)packed, row_width, z0, x0, g0, bz, bx, S, (float*)out, out_width, scale,
+                                 cu, seq_slots, num_seqs, tokens, width, stream);
+    if (act_type == RL_BF16)
+        return launch_gru<bf16_t>((const bf16_t*)packed, row_width, z0, x0, g0, bz, bx, S, (bf16_t*)out, out_width,
+                                  scale, cu, seq_slots, num_seqs, tokens, width, stream);
+    return RL_ERR_ARG;
 }

@@ -216,8 +216,15 @@ def add_rmsnorm(
     out: torch.Tensor,
     eps: float,
     rows: Optional[torch.Tensor] = None,
+    bias: Optional[torch.Tensor] = None,
 ) -> None:
+    """``residual += delta (+ bias)`` in place, ``out = norm(residual) * weight``; ``bias`` (float32
+    ``[hidden]``) is that of the product ``delta`` is."""
     tokens, hidden = residual.shape
+    if bias is not None:
+        if delta is None:
+            raise KernelError("a product's bias comes with the product")
+        _need(bias, "bias", torch.float32, (hidden,))
     _need(residual, "residual", torch.float32)
     _need(weight, "norm weight", torch.float32, (hidden,))
     out_rows = tokens if rows is None else rows.numel()
@@ -229,7 +236,7 @@ def add_rmsnorm(
     _ok(
         core().rl_add_rmsnorm(
             _p(residual), _p(delta), _p(weight), _p(out), _p(rows), out_rows, hidden,
-            ctypes.c_float(eps), _tag(out.dtype), _stream(),
+            ctypes.c_float(eps), _tag(out.dtype), _p(bias), _stream(),
         ),
         "rl_add_rmsnorm",
     )
@@ -275,6 +282,17 @@ def pair_rows(a: torch.Tensor, b: torch.Tensor, out: torch.Tensor) -> None:
     _need(b, "b", torch.float32, (tokens, hidden))
     _need(out, "out", None, (tokens, 2 * hidden))
     _ok(core().rl_pair_rows(_p(a), _p(b), _p(out), tokens, hidden, _tag(out.dtype), _stream()), "rl_pair_rows")
+
+
+def stream_add(residual: torch.Tensor, first: Optional[torch.Tensor], row: Optional[torch.Tensor]) -> None:
+    """``residual[r] += first[r] + row`` in place, all float32; either of the two may be ``None``."""
+    tokens, hidden = residual.shape
+    _need(residual, "residual", torch.float32)
+    if first is not None:
+        _need(first, "first", torch.float32, (tokens, hidden))
+    if row is not None:
+        _need(row, "row", torch.float32, (hidden,))
+    _ok(core().rl_stream_add(_p(residual), _p(first), _p(row), tokens, hidden, _stream()), "rl_stream_add")
 
 
 UNARY_ACTIVATIONS = {"gelu_tanh": 0, "relu_squared": 1, "tanh": 2}
@@ -347,21 +365,34 @@ def router(x: torch.Tensor, w: torch.Tensor, top: int, scale: float, bias: Optio
 
 
 GLU_ALPHA = 1.702  # the sigmoid's slope in the clamped gated activation
+GATE_ACTIVATIONS = {"silu": 0, "gelu_tanh": 1}  # what the gate of a gated feed-forward passes
+
+
+def _gate_kind(activation: str, limit: float) -> int:
+    if activation not in GATE_ACTIVATIONS:
+        raise KernelError(f"gate activation {activation!r} is not one of {sorted(GATE_ACTIVATIONS)}")
+    if limit < 0 or (limit and activation != "silu"):
+        raise KernelError(f"a limit of {limit} does not go with the gate activation {activation!r}")
+    return GATE_ACTIVATIONS[activation]
 
 
 def swiglu(gate_up: torch.Tensor, out: torch.Tensor, limit: float = 0.0, alpha: float = GLU_ALPHA,
-           route: Optional[torch.Tensor] = None, expert_ff: int = 0, route_input: bool = False) -> None:
+           route: Optional[torch.Tensor] = None, expert_ff: int = 0, route_input: bool = False,
+           activation: str = "silu", bias: Optional[torch.Tensor] = None) -> None:
     """The gated activation of a packed ``[gate | up]`` row.  ``limit`` 0: ``silu(g) * u``.
     ``limit > 0``: ``g' * sigmoid(alpha g') * (u' + 1)`` with ``g' = min(g, limit)`` and
     ``u' = clamp(u, -limit, limit)``.  With ``route`` (float32 ``[tokens, experts]``) the first
     ``experts * expert_ff`` hidden units are those of the experts side by side and expert ``e``'s
     are multiplied by ``route[t, e]``; with ``route_input`` its gate and up values are, before the
-    activation (the expert read a scaled input)."""
-    if route_input and route is None:
-        raise KernelError("scaling the experts' inputs needs their weights")
+    activation (the expert read a scaled input).  ``activation`` ``"gelu_tanh"``: the gate passes the
+    tanh form of gelu, ``gelu(g) * u``.  ``bias`` (float32 ``[2 I]``): the projections' biases, added as
+    the values are read."""
+    if route_input and (route is None or bias is not None):
+        raise KernelError("scaling the experts' inputs needs their weights and takes no bias")
     tokens, two_i = gate_up.shape
-    if limit < 0:
-        raise KernelError(f"the gated activation's limit must not be negative, got {limit}")
+    kind = _gate_kind(activation, limit)
+    if bias is not None:
+        _need(bias, "bias of gate and up", torch.float32, (two_i,))
     if two_i % 2:
         raise KernelError(f"the packed [gate | up] row must have even width, has {two_i}")
     _need(gate_up, "gate_up")
@@ -375,7 +406,8 @@ def swiglu(gate_up: torch.Tensor, out: torch.Tensor, limit: float = 0.0, alpha: 
     _ok(
         core().rl_swiglu(
             _p(gate_up), _p(out), tokens, two_i // 2, _tag(out.dtype), ctypes.c_float(limit),
-            ctypes.c_float(alpha), _p(route), experts, int(expert_ff), int(bool(route_input)), _stream(),
+            ctypes.c_float(alpha), _p(route), experts, int(expert_ff), int(bool(route_input)), kind, _p(bias),
+            _stream(),
         ),
         "rl_swiglu",
     )
@@ -475,6 +507,9 @@ def qknorm_rope_kvwrite(
     value_head0: Optional[int] = None,
     bias: Optional[torch.Tensor] = None,
     value_dim: Optional[int] = None,
+    col0: int = 0,
+    query_temperature: Optional[tuple[float, float]] = None,
+    norm_values: bool = False,
 ) -> None:
     """Norm + rotate q and k, write k and v to the cache pages (skipped when the caches
     are ``None``: a layer that reads another layer's cache).  ``q_out`` ``None``: the query
@@ -490,7 +525,12 @@ def qknorm_rope_kvwrite(
     product that another kernel reads).  ``value_dim``: the size of a value head where it is not
     ``d`` (the values then lie behind the keys).  ``bias`` (float32, one entry a column of the packed
     row): the projection's bias, added to the heads as they are read, before norm and rotation,
-    instead of by a kernel of its own after the product."""
+    instead of by a kernel of its own after the product.  ``col0``: the column of the packed row at
+    which all this begins (columns before it, like those behind, belong to other kernels; ``bias``
+    then begins with the entry of column ``col0``).  ``query_temperature`` ``(coef, every)``: a finished
+    query at position p is multiplied by ``1 + coef * ln(floor((p + 1) / every) + 1)``.
+    ``norm_values``: every value head is divided by its root mean square (``eps`` inside the root)
+    on its way into the cache."""
     if pairing not in ROTARY_PAIRINGS:
         raise KernelError(f"rotation pairing {pairing!r} is not one of {sorted(ROTARY_PAIRINGS)}")
     tokens = qkv.shape[0]
@@ -502,8 +542,9 @@ def qknorm_rope_kvwrite(
     value_col0 = value_head0 * d
     _need(qkv, "qkv", None, (tokens, None))
     row_width = qkv.shape[1]
-    if (value_head0 < 0 or not 1 <= dv <= 256 or row_width < max(value_col0 + nkv * dv, (nq + nkv) * d)
-            or (d % 8 == 0 and row_width % 8)):
+    own_width = max(value_col0 + nkv * dv, (nq + nkv) * d)
+    if (value_head0 < 0 or col0 < 0 or not 1 <= dv <= 256 or row_width - col0 < own_width
+            or (d % 8 == 0 and (row_width % 8 or col0 % 8))):
         # (heads in steps of 8 channels are read 8 or 16 bytes at a time, so rows must start aligned)
         raise KernelError(
             f"packed rows of {row_width} columns do not hold {nq} query and {nkv} key heads of {d} and {nkv} "
@@ -539,16 +580,44 @@ def qknorm_rope_kvwrite(
                 f"position {max_position} is beyond the rotation table of {cos.shape[0]} positions"
             )
     if bias is not None:
-        _need(bias, "bias of the packed projection", torch.float32, (row_width,))
+        _need(bias, "bias of the packed projection", torch.float32, (None,))
+        if bias.shape[0] < own_width:
+            raise KernelError(f"a bias of {bias.shape[0]} entries does not cover {own_width} columns")
+    coef, every = query_temperature or (0.0, 1.0)
+    if coef and (not every > 0 or q_out is None):
+        raise KernelError(f"a query temperature needs written queries and a positive step, got {query_temperature}")
     _ok(
         core().rl_qknorm_rope_kvwrite(
-            _p(qkv), _p(q_out), _p(k_cache), _p(v_cache), _p(q_norm_w), _p(k_norm_w), _p(cos),
+            ctypes.c_void_p(qkv.data_ptr() + col0 * qkv.element_size()), _p(q_out), _p(k_cache), _p(v_cache), _p(q_norm_w), _p(k_norm_w), _p(cos),
             _p(sin), _p(positions), _p(token_slot), _p(block_table), block_table.stride(0),
             page_size, tokens, nq, nkv, d, half, ROTARY_PAIRINGS[pairing], ctypes.c_float(eps), int(write),
-            row_width, value_col0, dv, _p(bias), _tag(qkv.dtype), _stream(),
+            row_width, value_col0, dv, _p(bias), ctypes.c_float(coef), ctypes.c_float(every), int(bool(norm_values)),
+            _tag(qkv.dtype), _stream(),
         ),
         "rl_qknorm_rope_kvwrite",
     )
+
+
+def _log_distance(pair, nq: int, slopes) -> tuple:
+    """The two numbers a query head of a logarithmic distance term, checked; ``None``s without one."""
+    if pair is None:
+        return None, None
+    if slopes is not None:
+        raise KernelError("scores take a distance term of one form")
+    for t in pair:
+        _need(t, "distance numbers", torch.float32, (nq,))
+    return pair
+
+
+def _out_columns(out: torch.Tensor, dtype: torch.dtype, tokens: int, width: int, col: int) -> None:
+    """``out`` is a contiguous ``[tokens, at least col + width]`` tensor whose columns from ``col`` on are written."""
+    _need(out, "out", dtype, (tokens, None))
+    if col < 0 or out.shape[1] < col + width:
+        raise KernelError(f"rows of {out.shape[1]} do not hold {width} columns from column {col} on")
+
+
+def _column(t: torch.Tensor, col: int) -> ctypes.c_void_p:
+    return ctypes.c_void_p(t.data_ptr() + col * t.element_size())
 
 
 def attention_generic(
@@ -572,10 +641,14 @@ def attention_generic(
     sink_values: Optional[torch.Tensor] = None,
     score_cap: float = 0.0,
     slopes: Optional[torch.Tensor] = None,
+    log_distance: Optional[tuple[torch.Tensor, torch.Tensor]] = None,
+    out_col: int = 0,
+    out_scale: float = 1.0,
 ) -> None:
     tokens = q.shape[0]
     pages = k_cache.shape[0]
     dv = d if value_dim is None else int(value_dim)
+    r1, r2 = _log_distance(log_distance, nq, slopes)
     if sink_values is not None:
         _need(sink_values, "sink values", torch.float32, (nq,))
     if slopes is not None:
@@ -583,7 +656,7 @@ def attention_generic(
     if score_cap < 0:
         raise KernelError(f"the cap of the scores must not be negative, got {score_cap}")
     _need(q, "q", None, (tokens, nq * d))
-    _need(out, "out", q.dtype, (tokens, nq * dv))
+    _out_columns(out, q.dtype, tokens, nq * dv, out_col)
     _need(k_cache, "k_cache", q.dtype, (pages, nkv, page_size, d))
     _need(v_cache, "v_cache", q.dtype, (pages, nkv, dv, page_size))
     _need(positions, "positions", torch.int32, (tokens,))
@@ -596,10 +669,11 @@ def attention_generic(
         )
     _ok(
         core().rl_attention_generic(
-            _p(q), _p(k_cache), _p(v_cache), _p(out), _p(positions), _p(token_slot),
+            _p(q), _p(k_cache), _p(v_cache), _column(out, out_col), _p(positions), _p(token_slot),
             _p(block_table), block_table.stride(0), page_size, tokens, nq, nkv, d, window,
             ctypes.c_float(scale), dv, int(keep_first), int(bool(sink) or sink_values is not None),
-            _p(sink_values), ctypes.c_float(score_cap), _p(slopes), _tag(q.dtype), _stream(),
+            _p(sink_values), ctypes.c_float(score_cap), _p(slopes), _p(r1), _p(r2),
+            out.shape[1], ctypes.c_float(out_scale), _tag(q.dtype), _stream(),
         ),
         "rl_attention_generic",
     )
@@ -1034,7 +1108,7 @@ def gemm_bf16(x: torch.Tensor, w: torch.Tensor, out_dtype: torch.dtype, scaled=N
         out = torch.empty((m, n), dtype=torch.bfloat16, device=x.device)
         _ok(
             core().rl_gemm_tile(_p(x), _p(w), _p(out), m, n, k, k, k, n, 0, ctypes.c_float(0.0), ctypes.c_float(0.0),
-                                _stream()),
+                                0, None, _stream()),
             "rl_gemm_tile",
         )
         return out
@@ -1044,11 +1118,28 @@ def gemm_bf16(x: torch.Tensor, w: torch.Tensor, out_dtype: torch.dtype, scaled=N
         out = torch.empty((m, n), dtype=wide, device=x.device)
         _ok(
             core().rl_gemm_rows(_p(x), _p(w), _p(out), m, n, k, k, k, n, 0, _tag(wide), *plan, ctypes.c_float(0.0),
-                                ctypes.c_float(0.0), _stream()),
+                                ctypes.c_float(0.0), 0, None, _stream()),
             "rl_gemm_rows",
         )
         return out
     return library_product(x, w)
+
+
+def gemm_bf16_wide(x: torch.Tensor, w: torch.Tensor, scaled=None) -> torch.Tensor:
+    """``x[M,K] @ w[N,K]^T`` with bfloat16 operands as the float32 accumulation leaves it, at every row
+    count (what enters a recurrence in 32-bit).  ``scaled``: as in :func:`gemm_bf16`."""
+    m, k = x.shape
+    if m <= SKINNY_MAX_ROWS and k % 8 == 0:
+        return gemm_bf16(x, w, torch.float32, scaled)
+    if scaled is not None:
+        raise KernelError(f"scaled rows need the few-row product: {m} rows over {k}")
+    if m <= MID_MAX_ROWS and mid_runs(w.shape[0], k) == 1:
+        return gemm_bf16_parts(x, w)[0]
+    _need(x, "x", torch.bfloat16)
+    _need(w, "w", torch.bfloat16, (None, k))
+    global library_products
+    library_products += 1
+    return torch.mm(x, w.t(), out_dtype=torch.float32)
 
 
 # How many products went to the library since the process started.  A step that is recorded into
@@ -1102,9 +1193,10 @@ def rows_plan(m: int, n: int, k: int, swiglu: bool, units: int | None = None) ->
 
 
 def gemm_bf16_residual(
-    x: torch.Tensor, w: torch.Tensor, residual: torch.Tensor, norm_weight: torch.Tensor
+    x: torch.Tensor, w: torch.Tensor, residual: torch.Tensor, norm_weight: torch.Tensor,
+    bias: Optional[torch.Tensor] = None,
 ) -> tuple[torch.Tensor, torch.Tensor]:
-    """The few-row product with the residual epilogue: ``residual += x w^T`` (the product
+    """The few-row product with the residual epilogue: ``residual += x w^T (+ bias)`` (the product
     rounded to bfloat16 first, as a stored result would be) in place; returns
     ``(residual * norm_weight`` as bfloat16, ``partial [workgroups, 16]`` float32``)`` with the
     sums of squares of each workgroup's columns of every row.  A consumer that takes the rows
@@ -1120,13 +1212,15 @@ def gemm_bf16_residual(
         )
     _need(residual, "residual", torch.float32, (m, n))
     _need(norm_weight, "norm weight", torch.float32, (n,))
+    if bias is not None:
+        _need(bias, "bias", torch.float32, (n,))
     lib = core()
     nt = _skinny_tiles(m, n)
     rows = torch.empty((m, n), dtype=torch.bfloat16, device=x.device)
     partial = torch.empty((lib.rl_gemm_skinny_parts(n, nt), 16), dtype=torch.float32, device=x.device)
     _ok(
         lib.rl_gemm_skinny_residual(
-            _p(x), _p(w), m, n, k, k, k, nt, _p(residual), _p(norm_weight), _p(rows), _p(partial), _stream()
+            _p(x), _p(w), m, n, k, k, k, nt, _p(residual), _p(norm_weight), _p(rows), _p(partial), _p(bias), _stream()
         ),
         "rl_gemm_skinny_residual",
     )
@@ -1207,31 +1301,38 @@ def gemm_bf16_parts(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
 
 
 def add_rmsnorm_parts(
-    residual: torch.Tensor, parts: torch.Tensor, weight: torch.Tensor, out: torch.Tensor, eps: float
+    residual: torch.Tensor, parts: torch.Tensor, weight: torch.Tensor, out: torch.Tensor, eps: float,
+    bias: Optional[torch.Tensor] = None,
 ) -> None:
-    """``residual += bfloat16(sum of parts)`` in place, ``out = norm(residual) * weight``."""
+    """``residual += bfloat16(sum of parts) (+ bias)`` in place, ``out = norm(residual) * weight``."""
     runs, tokens, hidden = parts.shape
+    if bias is not None:
+        _need(bias, "bias", torch.float32, (hidden,))
     _need(residual, "residual", torch.float32, (tokens, hidden))
     _need(parts, "parts", torch.float32)
     _need(weight, "norm weight", torch.float32, (hidden,))
     _need(out, "out", torch.bfloat16, (tokens, hidden))
     _ok(
         core().rl_add_rmsnorm_parts(
-            _p(residual), _p(parts), runs, _p(weight), _p(out), tokens, hidden, ctypes.c_float(eps), _stream()
+            _p(residual), _p(parts), runs, _p(weight), _p(out), tokens, hidden, ctypes.c_float(eps), _p(bias), _stream()
         ),
         "rl_add_rmsnorm_parts",
     )
 
 
 def gemm_bf16_swiglu(x: torch.Tensor, w_gate_up: torch.Tensor, scaled=None, limit: float = 0.0,
-                     alpha: float = GLU_ALPHA) -> torch.Tensor | None:
+                     alpha: float = GLU_ALPHA, activation: str = "silu",
+                     bias: Optional[torch.Tensor] = None) -> torch.Tensor | None:
     """``act(x Wg^T, x Wu^T)`` for the packed ``[gate | up]`` matrix in one kernel: for few rows,
     and for up to 512 rows over a small matrix; ``None`` when the shape is not one a fused kernel
-    takes.  ``act`` is ``silu(g) * u``, or with a ``limit`` the clamped variant of :func:`swiglu`.
+    takes.  ``act`` is ``silu(g) * u``, or with a ``limit`` the clamped variant of :func:`swiglu`;
+    ``activation`` and ``bias`` (float32, gate entries first) as there.
     ``scaled``: as in ``gemm_bf16``."""
     m, k = x.shape
-    glu = (ctypes.c_float(limit), ctypes.c_float(alpha))
     two_i = w_gate_up.shape[0]
+    if bias is not None:
+        _need(bias, "bias of gate and up", torch.float32, (two_i,))
+    glu = (ctypes.c_float(limit), ctypes.c_float(alpha), _gate_kind(activation, limit), _p(bias))
     if k % 8 or two_i % 2 or x.dtype != torch.bfloat16 or w_gate_up.dtype != torch.bfloat16:
         return None
     if m > SKINNY_MAX_ROWS:
@@ -1506,15 +1607,21 @@ def attention_tile(
     sink_values: Optional[torch.Tensor] = None,
     score_cap: float = 0.0,
     slopes: Optional[torch.Tensor] = None,
+    log_distance: Optional[tuple[torch.Tensor, torch.Tensor]] = None,
+    out_col: int = 0,
+    out_scale: float = 1.0,
 ) -> None:
     """Attention of every token of the step, in tiles of 16 rows on the matrix cores, for value
     heads of a size of their own, a window that keeps a request's first ``keep_first`` positions
     visible, and (``sink``) a softmax with 1 added to its denominator, or with ``sink_values``
     (float32, one number a query head) ``exp`` of the head's number.  ``score_cap`` c > 0 turns a
     scaled score s into ``c * tanh(s / c)``; ``slopes`` (float32, one number a query head) then take
-    ``slope * (distance between query and key)`` off it.  float32 (bit for bit the same however
+    ``slope * (distance between query and key)`` off it; ``log_distance`` (two of them, r1 and r2)
+    takes ``r1 * ln(1 + r2 * distance)`` off instead.  A token's heads go to the columns of ``out`` from
+    ``out_col`` on, multiplied by ``out_scale``.  float32 (bit for bit the same however
     the step was cut) or bfloat16."""
     tokens = q.shape[0]
+    r1, r2 = _log_distance(log_distance, nq, slopes)
     if sink_values is not None:
         _need(sink_values, "sink values", torch.float32, (nq,))
         sink = True
@@ -1524,7 +1631,9 @@ def attention_tile(
         raise KernelError(f"the cap of the scores must not be negative, got {score_cap}")
     pages = k_cache.shape[0]
     _need(q, "q", None, (tokens, nq * d))
-    _need(out, "out", q.dtype, (tokens, nq * dv))
+    _out_columns(out, q.dtype, tokens, nq * dv, out_col)
+    if out.shape[1] % 4 or out_col % 4:
+        raise KernelError(f"four channels are stored at once: columns from {out_col} on in rows of {out.shape[1]}")
     _need(k_cache, "k_cache", q.dtype, (pages, nkv, page_size, d))
     _need(v_cache, "v_cache", q.dtype, (pages, nkv, dv, page_size))
     _need(ctx.positions, "positions", torch.int32, (tokens,))
@@ -1565,10 +1674,11 @@ def attention_tile(
             part = torch.empty((tokens, nq, nsplit, dv + 2), dtype=torch.float32, device=q.device)
     _ok(
         lib.rl_attn_tile(
-            _p(q), _p(k_cache), _p(v_cache), _p(out), _p(tiles), num_tiles, _p(ctx.positions),
+            _p(q), _p(k_cache), _p(v_cache), _column(out, out_col), _p(tiles), num_tiles, _p(ctx.positions),
             _p(ctx.token_slot), _p(block_table), block_table.stride(0), page_size, nq, nkv, window,
             int(keep_first), int(bool(sink)), ctypes.c_float(scale), nsplit, _p(part), tokens, tile_rows,
-            _tag(q.dtype), _p(sink_values), ctypes.c_float(score_cap), _p(slopes), _stream(),
+            _tag(q.dtype), _p(sink_values), ctypes.c_float(score_cap), _p(slopes), _p(r1), _p(r2),
+            out.shape[1], ctypes.c_float(out_scale), _stream(),
         ),
         "rl_attn_tile",
     )
@@ -1607,6 +1717,9 @@ def paged_attention(
     sink_values: Optional[torch.Tensor] = None,
     score_cap: float = 0.0,
     slopes: Optional[torch.Tensor] = None,
+    log_distance: Optional[tuple[torch.Tensor, torch.Tensor]] = None,
+    out_col: int = 0,
+    out_scale: float = 1.0,
 ) -> None:
     """Attention of every token of the step over its request's cached keys.
 
@@ -1623,23 +1736,28 @@ def paged_attention(
     denominator: a key of score 0 without a value; with ``sink_values`` its score is a number of
     the query head, not scaled), ``score_cap`` (a scaled score s becomes ``cap * tanh(s / cap)``) and
     ``slopes`` (one number a query head, times the distance between query and key, taken off the
-    score) send the step to the kernels that take them:
+    score), ``log_distance`` (two numbers a query head instead: ``r1 * ln(1 + r2 * distance)``), ``out_col``
+    (rows of ``out`` are wider than the heads, which go to the columns from there on) and
+    ``out_scale`` (a factor of the finished outputs) send the step to the kernels that take them:
     tiles of 16 rows on the matrix cores for head sizes in steps of 16, the FMA kernel otherwise."""
     if prepare is not None and not attention_prepares_queries(q.dtype, d, 0 if prepare[1] is None else prepare[1].shape[1]):
         raise KernelError("the attention kernels do not finish the queries of this head size, type or rotation")
     dv = d if value_dim is None else int(value_dim)
     keep_first = int(keep_first) if window > 0 else 0  # without a window every key is seen anyway
-    if dv != d or keep_first or sink or sink_values is not None or score_cap or slopes is not None:
+    if (dv != d or keep_first or sink or sink_values is not None or score_cap or slopes is not None
+            or log_distance is not None or out_col or out_scale != 1.0 or out.shape[1] != nq * dv):
         # value heads of their own size, kept first positions, one more term in the denominator
         if prepare is not None:
             raise KernelError("queries are finished before an attention with these options")
-        if d % 16 == 0 and dv % 16 == 0 and page_size % 4 == 0:
+        if d % 16 == 0 and dv % 16 == 0 and page_size % 4 == 0 and out.shape[1] % 4 == 0 and out_col % 4 == 0:
             attention_tile(q, k_cache, v_cache, out, ctx, block_table, page_size, nq, nkv, d, dv,
-                           window, keep_first, sink, scale, sink_values, score_cap, slopes)
+                           window, keep_first, sink, scale, sink_values, score_cap, slopes, log_distance,
+                           out_col, out_scale)
         else:
             attention_generic(
                 q, k_cache, v_cache, out, ctx.positions, ctx.token_slot, block_table, page_size,
                 nq, nkv, d, window, scale, ctx.max_position, dv, keep_first, sink, sink_values, score_cap, slopes,
+                log_distance, out_col, out_scale,
             )
         return
     if q.dtype == torch.float32 and d % 16 == 0:
@@ -2152,4 +2270,122 @@ def group_rmsnorm(y: torch.Tensor, weight: torch.Tensor, out: torch.Tensor, part
         recurrent_lib().rl_group_rmsnorm(_p(y), _p(weight), _p(out), tokens, width, parts, ctypes.c_float(eps),
                                          _tag(out.dtype), _stream()),
         "rl_group_rmsnorm",
+    )
+
+
+# --------------------------------------------------------------------------- #
+# gated delta rule with a decay per key channel, minGRU
+# --------------------------------------------------------------------------- #
+DELTA_MAX_HEAD_DIM = 256
+
+
+def delta_prepare(packed: torch.Tensor, col0: int, taps: torch.Tensor, conv_state: torch.Tensor, decay: torch.Tensor,
+                  dt_bias: torch.Tensor, decay_log: torch.Tensor, mixed: torch.Tensor, ctx, heads: int, kv_heads: int,
+                  d: int, dv: int) -> None:
+    """What a gated delta rule reads.  ``packed`` holds ``[q: kv_heads * d | k: kv_heads * d | v: heads * dv]``
+    from column ``col0`` on.  Every channel passes a causal convolution (``taps [channels, n]`` float32, the
+    last column meets the current token; ``conv_state`` float32 ``[slots, n - 1, channels]`` as in
+    :func:`causal_conv`) and silu; every head of q and k is then made a unit vector and q multiplied by
+    ``d^(-1/2)``.  ``mixed [T, channels]`` float32.  ``decay [T, heads * d]`` float32 becomes
+    ``exp(-exp(decay_log_h) * softplus(decay + dt_bias))`` in place."""
+    tokens, width = packed.shape
+    channels = 2 * kv_heads * d + heads * dv
+    if heads % kv_heads or not 1 <= d <= DELTA_MAX_HEAD_DIM or not 1 <= dv <= DELTA_MAX_HEAD_DIM:
+        raise KernelError(f"{heads} heads over {kv_heads} key heads of {d} with values of {dv} channels")
+    n = taps.shape[1]
+    _need(packed, "packed rows")
+    _need(taps, "convolution taps", torch.float32, (channels, None))
+    _need(conv_state, "convolution state", torch.float32, (None, max(n - 1, 1), channels))
+    _need(decay, "decays", torch.float32, (tokens, heads * d))
+    _need(dt_bias, "decay bias", torch.float32, (heads * d,))
+    _need(decay_log, "decay rates", torch.float32, (heads,))
+    _need(mixed, "mixed", torch.float32, (tokens, channels))
+    if not 1 <= n <= CONV_MAX_TAPS or col0 < 0 or col0 + channels > width:
+        raise KernelError(f"{n} taps over columns {col0}..{col0 + channels} of rows of {width}")
+    _step_requests(ctx, tokens, conv_state.shape[0])
+    _ok(
+        recurrent_lib().rl_delta_prepare(
+            _p(packed), width, int(col0), _p(taps), _p(conv_state), _p(decay), _p(dt_bias), _p(decay_log), _p(mixed),
+            _p(ctx.cu_seqlens), _p(ctx.seq_slots), ctx.num_seqs, tokens, heads, kv_heads, d, dv, n,
+            _tag(packed.dtype), _stream()),
+        "rl_delta_prepare",
+    )
+
+
+def delta_scan(mixed: torch.Tensor, decay: torch.Tensor, beta_pre: torch.Tensor, raw: torch.Tensor, ctx,
+               S: torch.Tensor, heads: int, kv_heads: int, d: int, dv: int) -> None:
+    """The recurrence over what :func:`delta_prepare` left.  Per head (head h reads q and k of head
+    ``h // (heads // kv_heads)``), ``beta = sigmoid`` of entry h of the row of ``beta_pre`` (float32, at least
+    ``heads`` wide), with the state ``S [slots, heads, dv, d]`` (float32, value channel first) read at the
+    rows ``ctx.seq_slots`` and left after each request's last token::
+
+        S <- diag(decay) S        u = beta (v - S^T k)        S <- S + k u^T        o = S^T q
+
+    ``raw [T, heads * dv]`` float32: ``o``."""
+    tokens = mixed.shape[0]
+    _need(mixed, "mixed", torch.float32, (tokens, 2 * kv_heads * d + heads * dv))
+    _need(decay, "decays", torch.float32, (tokens, heads * d))
+    _need(beta_pre, "beta", torch.float32, (tokens, None))
+    _need(raw, "raw", torch.float32, (tokens, heads * dv))
+    _need(S, "state", torch.float32, (None, heads, dv, d))
+    if heads % kv_heads or not 1 <= d <= DELTA_MAX_HEAD_DIM or not 1 <= dv <= DELTA_MAX_HEAD_DIM or beta_pre.shape[1] < heads:
+        raise KernelError(f"{heads} heads over {kv_heads} key heads of {d} with values of {dv} channels")
+    _step_requests(ctx, tokens, S.shape[0])
+    _ok(
+        recurrent_lib().rl_delta_scan(_p(mixed), _p(decay), _p(beta_pre), beta_pre.shape[1], _p(raw), _p(ctx.cu_seqlens),
+                                      _p(ctx.seq_slots), _p(S), ctx.num_seqs, tokens, heads, kv_heads, d, dv, _stream()),
+        "rl_delta_scan",
+    )
+
+
+HEAD_GATES = {"silu": 0, "sigmoid": 1}
+
+
+def head_finish(raw: torch.Tensor, g: torch.Tensor, norm_weight: torch.Tensor, out: torch.Tensor, heads: int,
+                eps: float, gate: str) -> None:
+    """Every head of ``raw`` (float32 ``[T, heads * d]``) divided by its root mean square (``eps`` inside the
+    root), times ``norm_weight`` (one entry a channel of all heads, or of one head for every head), times
+    ``silu(g)`` or ``sigmoid(g)``."""
+    tokens, inner = raw.shape
+    d = inner // heads
+    if inner != heads * d or gate not in HEAD_GATES:
+        raise KernelError(f"rows of {inner} in {heads} heads behind the gate {gate!r}")
+    _need(raw, "raw", torch.float32)
+    _need(g, "g", out.dtype, (tokens, inner))
+    _need(out, "out", None, (tokens, inner))
+    _need(norm_weight, "head norm weight", torch.float32, (None,))
+    if norm_weight.shape[0] not in (d, inner):
+        raise KernelError(f"a head norm of {norm_weight.shape[0]} entries for {heads} heads of {d}")
+    _ok(
+        recurrent_lib().rl_head_finish(_p(raw), _p(g), _p(norm_weight), _p(out), tokens, heads, d, ctypes.c_float(eps),
+                                       int(norm_weight.shape[0] == d), HEAD_GATES[gate], _tag(out.dtype), _stream()),
+        "rl_head_finish",
+    )
+
+
+def min_gru(packed: torch.Tensor, columns: tuple[int, int, int], z_bias: torch.Tensor, x_bias: torch.Tensor,
+            out: torch.Tensor, ctx, S: torch.Tensor, out_col: int = 0, out_scale: float = 1.0) -> None:
+    """A gated recurrence whose gates read the current token alone.  ``columns``: where the packed row
+    holds ``z``, ``x`` and the output gate ``g``.  Per channel, with ``z' = sigmoid(z + z_bias)``, ``u = x + x_bias``
+    and the state ``S [slots, width]`` (float32) read at the rows ``ctx.seq_slots`` and left after each
+    request's last token::
+
+        S <- (1 - z') S + z' (u + 1/2 where u >= 0, else sigmoid(u))
+
+    The columns of ``out`` from ``out_col`` on get ``out_scale * S * silu(g)``."""
+    tokens, row_width = packed.shape
+    width = S.shape[1]
+    _need(packed, "packed rows")
+    _need(S, "state", torch.float32, (None, width))
+    _need(z_bias, "bias of z", torch.float32, (width,))
+    _need(x_bias, "bias of x", torch.float32, (width,))
+    _out_columns(out, packed.dtype, tokens, width, out_col)
+    if any(c < 0 or c + width > row_width for c in columns):
+        raise KernelError(f"columns {columns} of {width} do not lie in rows of {row_width}")
+    _step_requests(ctx, tokens, S.shape[0])
+    _ok(
+        recurrent_lib().rl_gru_scan(_p(packed), row_width, *(int(c) for c in columns), _p(z_bias), _p(x_bias), _p(S),
+                                    _column(out, out_col), out.shape[1], ctypes.c_float(out_scale), _p(ctx.cu_seqlens),
+                                    _p(ctx.seq_slots), ctx.num_seqs, tokens, width, _tag(packed.dtype), _stream()),
+        "rl_gru_scan",
     )

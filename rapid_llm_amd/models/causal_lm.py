@@ -12,6 +12,7 @@ from dataclasses import replace
 
 import torch
 
+from ..kernels import ops
 from ..parts.base import (
     BLOCKS,
     EMBEDDINGS,
@@ -55,6 +56,12 @@ class CausalLM:
                 if not 0 <= place < len(self.order):
                     raise ValueError(f"a stream mix names place {place} of a run order of {len(self.order)}")
             self.mixes = StreamMix(sm.checkpoint_name, sm.places, spec.hidden_size, name="stream_mix")
+        self.returns: frozenset[int] = frozenset()
+        if spec.stream_returns is not None:
+            self.returns = frozenset(spec.stream_returns.places)
+            for place in self.returns:
+                if not 0 <= place < len(self.order):
+                    raise ValueError(f"the embedding returns at place {place} of a run order of {len(self.order)}")
         self._positions: dict[str, object] = {}
         self.blocks = []
         for i, layer in enumerate(spec.layers):
@@ -156,9 +163,9 @@ class CausalLM:
         """Run the tokens of ``ctx`` through every layer (which writes their keys and values)
         and return float32 logits ``[len(ctx.logit_rows), vocab]``."""
         residual = self.embed.forward(ctx.token_ids, ctx)
-        # the embedding's output, which the stream mixes take in again (the stream itself is
-        # updated in place)
-        first = residual.clone() if self.mixes is not None else None
+        # the embedding's output, which later places take in again (the stream itself is updated
+        # in place)
+        first = residual.clone() if self.mixes is not None or self.returns else None
         delta = None
         for place, li in enumerate(self.order):
             block = self.blocks[li]
@@ -168,8 +175,10 @@ class CausalLM:
                     residual.add_(delta)
                     delta = None
                 residual = self.mixes.forward(residual, first)
-            if self.offsets is not None:
-                self.offsets.add(residual, place)
+            row = self.offsets.at(place) if self.offsets is not None else None
+            again = first if place in self.returns else None
+            if row is not None or again is not None:
+                ops.stream_add(residual, again, row)
             if not getattr(block, "accepts_deferred", False):
                 delta = settle(residual, delta)
             delta = block.forward(residual, delta, ctx, caches[place])

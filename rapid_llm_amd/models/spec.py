@@ -7,7 +7,7 @@ and the order in which layers run.  The order is data too: ``run_order`` may nam
 twice, and a layer may read another layer's cache (``LayerSpec.share_cache_with``).  A layer
 may lack the feed-forward sub-layer, learned vectors may be added to the stream at given
 places of the order (``ModelSpec.stream_offsets``), and the stream may be mixed with the
-embedding's output there (``ModelSpec.stream_mixes``).
+embedding's output there (``ModelSpec.stream_mixes``) or have it added (``ModelSpec.stream_returns``).
 """
 
 from __future__ import annotations
@@ -77,6 +77,14 @@ class StreamOffsets:
 
 
 @dataclass(frozen=True)
+class StreamReturns:
+    """Right before the layer at each of ``places`` of the run order runs (and before a vector of
+    :class:`StreamOffsets` is added there), the embedding's output is added to the stream."""
+
+    places: tuple[int, ...]
+
+
+@dataclass(frozen=True)
 class StreamMixes:
     """Right before the layer at each of ``places`` of the run order runs, the stream becomes
     ``M [x ; x0]``: ``x0`` is the embedding's output, ``M`` the checkpoint tensor
@@ -109,6 +117,7 @@ class ModelSpec:
     max_position: int = 0  # largest position the architecture is defined for (0: unbounded)
     stream_offsets: StreamOffsets | None = None
     stream_mixes: StreamMixes | None = None
+    stream_returns: StreamReturns | None = None
 
     def order(self) -> tuple[int, ...]:
         return self.run_order if self.run_order is not None else tuple(range(len(self.layers)))

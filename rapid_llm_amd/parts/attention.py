@@ -28,6 +28,14 @@ that size, the output projection reads ``num_heads * value_dim`` columns).  ``ke
 a window, a request's first positions stay visible to every later query, and their pages stay
 mapped.  ``sink``: the softmax's denominator is ``1 + sum_j exp(s_j)``, as if one more key of
 score 0 and without a value were always seen.
+
+``log_distance_names``: two learned numbers a query head, ``r1`` and ``r2``; ``r1 * ln(1 + r2 * distance)`` is
+taken off a scaled score.  ``query_temperature`` ``(coef, every)``: a finished query at position p is
+multiplied by ``1 + coef * ln(floor((p + 1) / every) + 1)``.  ``value_norm``: every value head is divided
+by its root mean square before it is cached (the epsilon is that of the query and key norm).
+
+With these options the mixer is a :class:`~rapid_llm_amd.parts.base.PackedMixer`: it can run on columns of
+a product that another mixer shares (``packs``).
 """
 
 from __future__ import annotations
@@ -37,11 +45,11 @@ import math
 import torch
 
 from ..kernels import ops
-from .base import MIXERS, CacheNeed, Mixer, ParamSpec, Source
+from .base import MIXERS, CacheNeed, PackedMixer, ParamSpec, Source
 from .linear import Linear
 
 
-class GQAAttention(Mixer):
+class GQAAttention(PackedMixer):
     replayable = True
 
     def __init__(
@@ -74,13 +82,17 @@ class GQAAttention(Mixer):
         qk_norm_weights: bool = True,
         score_cap: float = 0.0,
         distance_slope_exponent: float | None = None,
+        log_distance_names: tuple[str, str] | None = None,
+        query_temperature: tuple[float, float] | None = None,
+        value_norm: bool = False,
     ) -> None:
         if num_heads % num_kv_heads:
             raise ValueError(f"{num_heads} query heads are not divisible by {num_kv_heads} kv heads")
-        if head_dim % 2 or not 2 <= head_dim <= 256:
-            # multiples of 16 run on the matrix cores, every other even size on the kernel that
-            # takes any size (an architecture's configuration may be stricter)
-            raise ValueError(f"attention kernels take even head sizes up to 256, got {head_dim}")
+        rotates = int(getattr(position, "rotary_dim", 0) or 0) > 0
+        if (head_dim % 2 and rotates) or not 1 <= head_dim <= 256:
+            # multiples of 16 run on the matrix cores, every other size on the kernel that takes
+            # any (an architecture's configuration may be stricter)
+            raise ValueError(f"attention kernels take head sizes up to 256, even where channels rotate, got {head_dim}")
         self.hidden_size = hidden_size
         self.nq, self.nkv, self.d = num_heads, num_kv_heads, head_dim
         self.dv = head_dim if value_dim is None else int(value_dim)
@@ -100,6 +112,19 @@ class GQAAttention(Mixer):
         self.score_cap = float(score_cap)
         self.slope_exponent = None if distance_slope_exponent is None else float(distance_slope_exponent)
         self.slopes = None
+        if log_distance_names is not None and self.slope_exponent is not None:
+            raise ValueError("scores take a distance term of one form")
+        self.log_distance_names = tuple(log_distance_names) if log_distance_names is not None else None
+        self.log_distance = None
+        self.query_temperature = None
+        if query_temperature is not None:
+            coef, every = (float(x) for x in query_temperature)
+            if not every > 0:
+                raise ValueError(f"the query temperature steps every {every} positions")
+            self.query_temperature = (coef, every)
+        self.value_norm = bool(value_norm)
+        if self.value_norm and (qk_norm_eps is None or values == "keys"):
+            raise ValueError("normed values need a value projection and the epsilon of the query and key norm")
         self.prefix = checkpoint_prefix
         self.qk_norm_eps = qk_norm_eps
         self.window = int(window)
@@ -129,10 +154,14 @@ class GQAAttention(Mixer):
         self.gate_pad = -(self.qkv_rows + self.gate_rows) % 8 if self.gate_rows else 0
         # the options that only the tile kernels (or the kernel for any size) take
         self.extended = (self.dv != head_dim or self.keep_first > 0 or self.sink or self.score_cap > 0
-                         or self.slope_exponent is not None)
+                         or self.slope_exponent is not None or self.log_distance_names is not None
+                         or self.query_temperature is not None or self.value_norm)
         self.plain_row = not self.values_are_keys and not self.gate_rows and not self.extended
+        self.packs = self.extended and not self.gate_rows
         self.row_pad = -self.qkv_rows % 8 if (self.extended and not self.gate_rows) else 0
-        self.qkv = Linear(hidden_size, self.qkv_rows + self.gate_rows + self.gate_pad + self.row_pad)
+        self.packed_rows = self.qkv_rows + self.gate_rows + self.gate_pad + self.row_pad
+        self.inner_width = num_heads * self.dv
+        self.qkv = Linear(hidden_size, self.packed_rows)
         self.o = Linear(num_heads * self.dv, hidden_size)
         self.q_norm_w = self.k_norm_w = None
         # Qwen3 has neither (rapid_llm/models/qwen3.py:16-18: qkv_bias=False); architectures of the
@@ -141,24 +170,37 @@ class GQAAttention(Mixer):
         self.qkv_bias, self.o_bias = bool(qkv_bias), bool(o_bias)
 
     # ---- tensors ---------------------------------------------------------------
-    def param_specs(self) -> list[ParamSpec]:
+    def packed_sources(self) -> tuple[Source, ...]:
         p, n = self.prefix, self.names
-        q_rows, kv_rows = self.nq * self.d, self.nkv * self.d
-        v_rows = self.nkv * self.dv
-        packed = [Source(p + n["q"], q_rows), Source(p + n["k"], kv_rows)]
+        packed = [Source(p + n["q"], self.nq * self.d), Source(p + n["k"], self.nkv * self.d)]
         if not self.values_are_keys:
-            packed.append(Source(p + n["v"], v_rows))
+            packed.append(Source(p + n["v"], self.nkv * self.dv))
         if self.gate_rows:
             packed.append(Source(p + n["g"], self.gate_rows))
         if self.gate_pad + self.row_pad:
             packed.append(Source("", self.gate_pad + self.row_pad))  # rows of zeros
+        return tuple(packed)
+
+    def output_source(self) -> str:
+        return self.prefix + self.names["o"]
+
+    def param_specs(self) -> list[ParamSpec]:
         specs = [
-            ParamSpec(self.name + ".qkv", (self.qkv.out_features, self.hidden_size), "matrix", tuple(packed)),
+            ParamSpec(self.name + ".qkv", (self.qkv.out_features, self.hidden_size), "matrix", self.packed_sources()),
             ParamSpec(self.name + ".o", (self.hidden_size, self.nq * self.dv), "matrix",
-                      (Source(p + n["o"], self.hidden_size),)),
+                      (Source(self.output_source(), self.hidden_size),)),
         ]
+        return specs + self.inner_specs()
+
+    def inner_specs(self) -> list[ParamSpec]:
+        p, n = self.prefix, self.names
+        q_rows, kv_rows, v_rows = self.nq * self.d, self.nkv * self.d, self.nkv * self.dv
+        specs = []
         if self.sink_name is not None:
             specs.append(ParamSpec(self.name + ".sink", (self.nq,), "vector", (Source(p + self.sink_name, self.nq),)))
+        if self.log_distance_names is not None:
+            specs += [ParamSpec(f"{self.name}.{which}", (self.nq,), "vector", (Source(p + source, self.nq),))
+                      for which, source in zip(("r1", "r2"), self.log_distance_names)]
         if self.qk_norm_eps is not None and self.qk_norm_weights:
             specs += [
                 ParamSpec(self.name + ".q_norm", (self.d,), "vector", (Source(p + n["qn"], self.d),), init="norm"),
@@ -186,13 +228,18 @@ class GQAAttention(Mixer):
 
     def bind(self, params, runtime) -> None:
         bias = params[self.name + ".qkv_bias"] if self.qkv_bias else None
-        # A plain [q | k | v] row may run through kernels that read the packed row themselves
+        # (bind_inner keeps it where the heads' own kernel adds it.)  A plain [q | k | v] row may run through kernels that read the packed row themselves
         # (the fused decode step, queries finished inside the attention kernels): its bias is
         # added after the product.  Any other row always passes the kernel that norms, rotates
         # and writes the cache, which adds the bias as it reads the heads.
-        self.bias_in_kernel = None if self.plain_row else bias
         self.qkv.bind(params[self.name + ".qkv"], bias if self.plain_row else None)
         self.o.bind(params[self.name + ".o"], params[self.name + ".o_bias"] if self.o_bias else None)
+        self.bind_inner(params, runtime)
+
+    def bind_inner(self, params, runtime) -> None:
+        self.bias_in_kernel = params[self.name + ".qkv_bias"] if self.qkv_bias and not self.plain_row else None
+        if self.log_distance_names is not None:
+            self.log_distance = (params[self.name + ".r1"], params[self.name + ".r2"])
         if self.qk_norm_eps is not None and self.qk_norm_weights:
             self.q_norm_w = params[self.name + ".q_norm"]
             self.k_norm_w = params[self.name + ".k_norm"]
@@ -224,15 +271,45 @@ class GQAAttention(Mixer):
     def accepts_scaled_rows(self) -> bool:
         return self.qkv.takes_scaled_rows()
 
+    def run(self, packed, col0, out, out_col, out_scale, ctx, cache):
+        """The heads between the two products (layers with one of the options beyond plain attention)."""
+        pos_enc = self.position
+        cos = pos_enc.cos if pos_enc is not None else None
+        sin = pos_enc.sin if pos_enc is not None else None
+        pairing = getattr(pos_enc, "pairing", "half_split") if cos is not None else "half_split"
+        eps = self.qk_norm_eps if self.qk_norm_eps is not None else 0.0
+        table = ctx.block_tables[cache.group_id]
+        q = torch.empty((packed.shape[0], self.nq * self.d), dtype=packed.dtype, device=packed.device)
+        ops.qknorm_rope_kvwrite(
+            packed, q,
+            cache.k if cache.owns_pages else None,
+            cache.v if cache.owns_pages else None,
+            self.q_norm_w, self.k_norm_w, cos, sin,
+            ctx.positions, ctx.token_slot, table, cache.page_size,
+            self.nq, self.nkv, self.d, eps, ctx.max_position, pairing, self.value_head0, self.bias_in_kernel,
+            self.dv, col0, self.query_temperature, self.value_norm,
+        )
+        ops.paged_attention(
+            q, cache.k, cache.v, out, ctx, table, cache.page_size, self.nq, self.nkv, self.d, self.window, self.scale,
+            value_dim=self.dv, keep_first=self.keep_first, sink=self.sink, sink_values=self.sink_values,
+            score_cap=self.score_cap, slopes=self.slopes, log_distance=self.log_distance, out_col=out_col,
+            out_scale=out_scale,
+        )
+
     def forward(self, x, ctx, cache):
         tokens = x.shape[0]
         qkv = self.qkv(x)
+        out = torch.empty((tokens, self.inner_width), dtype=qkv.dtype, device=x.device)
+        if self.extended:
+            self.run(qkv, 0, out, 0, 1.0, ctx, cache)
+            if self.gate_rows:
+                ops.head_gate(out, qkv, self.qkv_rows, self.nq, self.d)
+            return self.o.deferred(out, ctx)
         table = ctx.block_tables[cache.group_id]
         pos_enc = self.position
         cos = pos_enc.cos if pos_enc is not None else None
         sin = pos_enc.sin if pos_enc is not None else None
         eps = self.qk_norm_eps if self.qk_norm_eps is not None else 0.0
-        out = torch.empty((tokens, self.nq * self.dv), dtype=qkv.dtype, device=x.device)
         rotary_half = cos.shape[1] if cos is not None else 0
         pairing = getattr(pos_enc, "pairing", "half_split") if cos is not None else "half_split"
         if self.plain_row and ops.decode_attention_fusable(
@@ -255,14 +332,11 @@ class GQAAttention(Mixer):
             self.q_norm_w, self.k_norm_w, cos, sin,
             ctx.positions, ctx.token_slot, table, cache.page_size,
             self.nq, self.nkv, self.d, eps, ctx.max_position, pairing, self.value_head0, self.bias_in_kernel,
-            self.dv,
         )
         ops.paged_attention(
             qkv if in_kernel else q, cache.k, cache.v, out, ctx, table, cache.page_size,
             self.nq, self.nkv, self.d, self.window, self.scale,
             prepare=(self.q_norm_w, cos, sin, eps) if in_kernel else None,
-            value_dim=self.dv, keep_first=self.keep_first, sink=self.sink, sink_values=self.sink_values,
-            score_cap=self.score_cap, slopes=self.slopes,
         )
         if self.gate_rows:
             ops.head_gate(out, qkv, self.qkv_rows, self.nq, self.d)

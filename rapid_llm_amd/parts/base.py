@@ -252,6 +252,38 @@ class Mixer(Part):
         raise NotImplementedError
 
 
+class PackedMixer(Mixer):
+    """A mixer whose work stands between one product of its input and one product into the stream.
+
+    Standing alone it has the two products itself.  A mixer that puts several of these side by
+    side (:mod:`rapid_llm_amd.parts.side_by_side`) packs their input projections into one product
+    and their output projections into another, and has each :meth:`run` on its columns."""
+
+    hidden_size: int
+    packed_rows: int  # columns of the packed input product, ``packed_sources`` in order
+    inner_width: int  # columns the output projection reads
+
+    def packed_sources(self) -> tuple[Source, ...]:
+        raise NotImplementedError
+
+    def output_source(self) -> str:
+        """Checkpoint name of the output projection, ``[hidden_size, inner_width]``."""
+        raise NotImplementedError
+
+    def inner_specs(self) -> list[ParamSpec]:
+        """Every tensor besides the packed input matrix and the output matrix."""
+        return []
+
+    def bind_inner(self, params: dict[str, "torch.Tensor"], runtime: Any) -> None:
+        """Receive the tensors of :meth:`inner_specs`."""
+
+    def run(self, packed: "torch.Tensor", col0: int, out: "torch.Tensor", out_col: int, out_scale: float,
+            ctx: "StepContext", cache: Any) -> None:
+        """From the columns of ``packed`` from ``col0`` on (a multiple of 8) to ``out_scale`` times what the
+        output projection reads, in the columns of ``out`` from ``out_col`` on."""
+        raise NotImplementedError
+
+
 class FeedForward(Part):
     def forward(self, x: "torch.Tensor", ctx: "StepContext") -> "torch.Tensor":
         raise NotImplementedError

@@ -1,6 +1,7 @@
 """``y = x W^T (+ b)`` with ``W [out, in]`` as the checkpoint stores it.  This family has no
-bias; a part of another architecture binds one, which is added by a kernel of its own after
-the product (a product with a bias folds no norm into itself).
+bias; a part of another architecture binds one.  Where the product's result goes into the residual
+(``deferred``) the bias is added there, by the kernel that adds the product; anywhere else by a
+kernel of its own after the product.
 
 Which product runs is decided by the weight's storage type:
 
@@ -49,8 +50,8 @@ class Linear:
 
     def folds(self, x) -> bool:
         """Whether this product may absorb the residual add and norm that follow it: one of the
-        two kernels with that epilogue runs it, and no bias comes between."""
-        return self.bias is None and (self.skinny(x) or self.midsize(x))
+        two kernels with that epilogue runs it."""
+        return self.skinny(x) or self.midsize(x)
 
     def takes_scaled_rows(self) -> bool:
         """Whether this product can finish a norm whose rows arrive unscaled (whatever the
@@ -67,34 +68,45 @@ class Linear:
         )
 
     def partial_sums(self, x: torch.Tensor) -> torch.Tensor:
-        """``[runs, M, out]`` float32 whose sum over the runs is ``x W^T``."""
+        """``[runs, M, out]`` float32 whose sum over the runs is ``x W^T`` (without the bias)."""
         return ops.gemm_bf16_parts(x, self.weight)
 
     def deferred(self, x: torch.Tensor, ctx=None):
         """The product, or a :class:`DeferredProduct` of it where one of this product's kernels
         could fold a neighbouring norm into itself (bfloat16, up to 16 rows, or 17 to 192 rows of a
-        narrow matrix).  Whoever receives it and has no use for that simply materialises it."""
-        if isinstance(x, torch.Tensor) and self.folds(x):
+        narrow matrix), or where it has a bias, which the kernel that adds the product to the
+        residual can add.  Whoever receives it and has no use for that simply materialises it."""
+        if isinstance(x, torch.Tensor) and (self.bias is not None or self.folds(x)):
             return DeferredProduct(self, x)
         return self(x)
 
     def add_to_residual(
         self, x: torch.Tensor, residual: torch.Tensor, norm_weight: torch.Tensor, eps: float
     ) -> ScaledRows:
-        """``residual += x W^T`` in place; returns the new rows times ``norm_weight`` and the
+        """``residual += x W^T (+ bias)`` in place; returns the new rows times ``norm_weight`` and the
         pieces of their sums of squares."""
-        rows, partial = ops.gemm_bf16_residual(x, self.weight, residual, norm_weight)
+        rows, partial = ops.gemm_bf16_residual(x, self.weight, residual, norm_weight, self.bias)
         return ScaledRows(rows, partial, self.out_features, eps)
 
     def __call__(self, x, out_dtype: torch.dtype | None = None) -> torch.Tensor:
+        y = self.product(x, out_dtype)
+        if self.bias is not None:
+            ops.add_bias(y, self.bias)
+        return y
+
+    def wide(self, x) -> torch.Tensor:
+        """``x W^T`` in float32 as the accumulation leaves it, without the bias."""
+        if self.weight.dtype == torch.float32:
+            return self.product(x, torch.float32)
+        return ops.gemm_bf16_wide(x.rows, self.weight, x) if isinstance(x, ScaledRows) else ops.gemm_bf16_wide(x, self.weight)
+
+    def product(self, x, out_dtype: torch.dtype | None = None) -> torch.Tensor:
+        """``x W^T`` without the bias."""
         w = self.weight
         if isinstance(x, ScaledRows):
             if not self.skinny(x):
                 raise ValueError("scaled rows reached a product that cannot apply their factor")
-            y = ops.gemm_bf16(x.rows, w, out_dtype or x.dtype, scaled=x)
-            if self.bias is not None:
-                ops.add_bias(y, self.bias)
-            return y
+            return ops.gemm_bf16(x.rows, w, out_dtype or x.dtype, scaled=x)
         rows = x.shape[0]
         out_dtype = out_dtype or x.dtype
         if w.dtype == torch.float32:
@@ -110,6 +122,4 @@ class Linear:
             narrow = torch.empty(y.shape, dtype=out_dtype, device=y.device)
             ops.cast(y, narrow)
             y = narrow
-        if self.bias is not None:
-            ops.add_bias(y, self.bias)
         return y

@@ -1,6 +1,9 @@
 """Feed-forwards.  Dense gated feed-forward: ``down(act(gate(x), up(x)))`` with ``act(g, u) = silu(g) * u``
-(SwiGLU), or, with a ``limit``, the clamped variant ``g' * sigmoid(alpha * g') * (u' + 1)`` where
-``g' = min(g, limit)`` and ``u' = clamp(u, -limit, limit)``.
+(SwiGLU) or ``gelu(g) * u`` with gelu in its tanh form, or, with a ``limit``, the clamped variant
+``g' * sigmoid(alpha * g') * (u' + 1)`` where ``g' = min(g, limit)`` and ``u' = clamp(u, -limit, limit)``.
+With ``bias`` all three projections have one (the projection's name with ``bias_suffix`` added);
+those of gate and up are added by the activation, that of the down projection by whoever adds
+its result to the residual.
 
 Gate and up are one packed matrix ``[2I, H]`` with rows ``[gate | up]``
 (rapid_llm/models/base.py:401-404, rapid_llm/modules/linear.py:157-172), so one product
@@ -34,10 +37,17 @@ class SwiGLU(FeedForward):
         down_name: str = "down_proj.weight",
         limit: float = 0.0,
         alpha: float = ops.GLU_ALPHA,
+        activation: str = "silu",
+        bias: bool = False,
+        bias_suffix: str = ".b",
     ) -> None:
         if limit < 0:
             raise ValueError(f"the gated activation's limit must not be negative, got {limit}")
-        self.limit, self.alpha = float(limit), float(alpha)
+        if activation not in ops.GATE_ACTIVATIONS or (limit and activation != "silu"):
+            raise ValueError(f"gate activation {activation!r} with a limit of {limit}")
+        self.limit, self.alpha, self.activation = float(limit), float(alpha), activation
+        self.has_bias, self.bias_suffix = bool(bias), bias_suffix
+        self.gate_up_bias: torch.Tensor | None = None
         self.hidden_size = hidden_size
         self.intermediate_size = intermediate_size
         self.prefix = checkpoint_prefix
@@ -49,14 +59,23 @@ class SwiGLU(FeedForward):
     def param_specs(self) -> list[ParamSpec]:
         h, i = self.hidden_size, self.intermediate_size
         g, u, d = (self.prefix + n for n in self.names)
-        return [
+        specs = [
             ParamSpec(self.name + ".gate_up", (2 * i, h), "matrix", (Source(g, i), Source(u, i))),
             ParamSpec(self.name + ".down", (h, i), "matrix", (Source(d, h),)),
         ]
+        if self.has_bias:
+            b = self.bias_suffix
+            specs += [
+                ParamSpec(self.name + ".gate_up_bias", (2 * i,), "vector", (Source(g + b, i), Source(u + b, i))),
+                ParamSpec(self.name + ".down_bias", (h,), "vector", (Source(d + b, h),)),
+            ]
+        return specs
 
     def bind(self, params, runtime) -> None:
         self.gate_up.bind(params[self.name + ".gate_up"])
-        self.down.bind(params[self.name + ".down"])
+        self.down.bind(params[self.name + ".down"], params[self.name + ".down_bias"] if self.has_bias else None)
+        if self.has_bias:
+            self.gate_up_bias = params[self.name + ".gate_up_bias"]
 
     @property
     def accepts_scaled_rows(self) -> bool:
@@ -66,14 +85,14 @@ class SwiGLU(FeedForward):
         w = self.gate_up.weight
         if w.dtype == torch.bfloat16 and x.dtype == torch.bfloat16:
             # few rows: product and activation in one kernel
-            glu = dict(limit=self.limit, alpha=self.alpha)
+            glu = dict(limit=self.limit, alpha=self.alpha, activation=self.activation, bias=self.gate_up_bias)
             act = (ops.gemm_bf16_swiglu(x.rows, w, scaled=x, **glu) if isinstance(x, ScaledRows)
                    else ops.gemm_bf16_swiglu(x, w, **glu))
             if act is not None:
                 return self.down.deferred(act, ctx)
         gu = self.gate_up(x)
         act = torch.empty((x.shape[0], self.intermediate_size), dtype=gu.dtype, device=x.device)
-        ops.swiglu(gu, act, self.limit, self.alpha)
+        ops.swiglu(gu, act, self.limit, self.alpha, activation=self.activation, bias=self.gate_up_bias)
         return self.down.deferred(act, ctx)
 
 

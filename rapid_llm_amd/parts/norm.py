@@ -20,8 +20,10 @@ class RMSNorm(Norm):
     fuses_products = True  # takes a DeferredProduct as delta, may return ScaledRows
 
     def __init__(self, size: int, eps: float, checkpoint_name: str, name: str = "norm",
-                 single_weight: bool = False) -> None:
+                 single_weight: bool = False, weight_offset: float = 0.0) -> None:
         self.size = size
+        # added to the stored weight: 1 where a checkpoint stores weights around zero
+        self.weight_offset = float(weight_offset)
         self.eps = float(eps)
         self.checkpoint_name = checkpoint_name
         self.name = name
@@ -39,12 +41,14 @@ class RMSNorm(Norm):
                 (self.size,),
                 "vector",
                 (Source(self.checkpoint_name, self.size),),
-                init="norm",
+                init="norm" if not self.weight_offset else "zeros",
             )
         ]
 
     def bind(self, params, runtime) -> None:
         self.weight = params[self.name + ".weight"]
+        if self.weight_offset:
+            self.weight = self.weight + self.weight_offset
         if self.single_weight:
             self.weight = self.weight.reshape(1).expand(self.size).contiguous()
         self.dtype = runtime.dtype
@@ -62,27 +66,28 @@ class RMSNorm(Norm):
         if isinstance(delta, SummedDeltas):
             delta.add_to(residual)
             delta = None
+        bias = None
         if isinstance(delta, DeferredProduct):
+            bias = delta.linear.bias
             if (
                 scaled_ok and rows is None and delta.linear.out_features == self.size
-                and self.dtype == torch.bfloat16 and delta.linear.bias is None and delta.linear.skinny(delta.x)
+                and self.dtype == torch.bfloat16 and delta.linear.skinny(delta.x)
             ):
                 # the producer's kernel adds into the residual and leaves what the consumer's
                 # kernel needs to finish the norm: no kernel of this norm's own runs
                 return delta.linear.add_to_residual(delta.x, residual, self.weight, self.eps)
             if (
                 rows is None and delta.linear.out_features == self.size and self.dtype == torch.bfloat16
-                and self.size % 4 == 0 and self.size <= 16 * 1024 and delta.linear.bias is None
-                and delta.linear.midsize(delta.x)
+                and self.size % 4 == 0 and self.size <= 16 * 1024 and delta.linear.midsize(delta.x)
             ):
                 # the product arrives as float32 runs of K, which this norm's kernel adds
                 out = torch.empty((residual.shape[0], self.size), dtype=self.dtype, device=residual.device)
-                ops.add_rmsnorm_parts(residual, delta.linear.partial_sums(delta.x), self.weight, out, self.eps)
+                ops.add_rmsnorm_parts(residual, delta.linear.partial_sums(delta.x), self.weight, out, self.eps, bias)
                 return out
-            delta = delta.materialize()
+            delta = delta.linear.product(delta.x)
         n = residual.shape[0] if rows is None else rows.numel()
         out = torch.empty((n, self.size), dtype=self.dtype, device=residual.device)
-        ops.add_rmsnorm(residual, delta, self.weight, out, self.eps, rows)
+        ops.add_rmsnorm(residual, delta, self.weight, out, self.eps, rows, bias)
         return out
 
 

@@ -10,7 +10,6 @@ from __future__ import annotations
 
 import torch
 
-from ..kernels import ops
 from .base import ParamSpec, Part, Source
 
 
@@ -38,8 +37,6 @@ class StreamOffsetTable(Part):
         table = params[self.name + ".table"]
         self.rows = {place: table[t] for t, place in enumerate(self.places)}
 
-    def add(self, residual: torch.Tensor, place: int) -> None:
-        """``residual[r, :] += row`` (float32, in place) if ``place`` has a row."""
-        row = self.rows.get(place)
-        if row is not None:
-            ops.add_bias(residual, row)
+    def at(self, place: int) -> torch.Tensor | None:
+        """The float32 row added to every token's stream at ``place``, if it has one."""
+        return self.rows.get(place)
