@@ -1088,6 +1088,20 @@ __device__ inline float query_temperature(const HeadPrep& hp, int pos) {
     return 1.f + hp.temp_coef * logf(floorf((float)(pos + 1) / hp.temp_every) + 1.f);
 }
 
+// 1 / (root mean square) of a value head, in every one of (at least) 16 lanes of a wave that read the
+// same head: each row of 16 lanes forms the sum, in the order of the tile kernel below
+template <typename T>
+__device__ inline float value_factor(const T* __restrict__ xv, const float* __restrict__ vb, int dv, float eps) {
+    float ss = 0.f;
+    for (int i = threadIdx.x % 16; i < dv; i += 16) {
+        const float v = to_float(xv[i]) + (vb ? vb[i] : 0.f);
+        ss += v * v;
+    }
+#pragma unroll
+    for (int o = 8; o > 0; o >>= 1) ss += __shfl_xor(ss, o, RL_WAVE);
+    return rsqrtf(ss / (float)dv + eps);
+}
+
 template <typename T>
 __global__ void qknorm_rope_kvwrite_kernel(
     const T* __restrict__ qkv, T* __restrict__ q_out, T* __restrict__ k_cache,
@@ -1124,15 +1138,7 @@ __global__ void qknorm_rope_kvwrite_kernel(
             const T* xv = row + v_col0 + (size_t)h * dv;  // where the row keeps this value head
             T* dst = v_cache + ((page * nkv + h) * dv) * page_size + off;
             const float* vb = hp.bias ? hp.bias + v_col0 + (size_t)h * dv : nullptr;
-            float factor = 1.f;
-            if (hp.norm_values) {
-                float ss = 0.f;
-                for (int i = lane; i < dv; i += RL_WAVE) {
-                    const float v = to_float(xv[i]) + (vb ? vb[i] : 0.f);
-                    ss += v * v;
-                }
-                factor = rsqrtf(wave_sum(ss) / (float)dv + eps);
-            }
+            const float factor = hp.norm_values ? value_factor(xv, vb, dv, eps) : 1.f;
             for (int i = lane; i < dv; i += RL_WAVE)
                 dst[(size_t)i * page_size] = from_float<T>((to_float(xv[i]) + (vb ? vb[i] : 0.f)) * factor);
             continue;
@@ -1236,17 +1242,7 @@ __device__ inline void qknorm_rope_kvwrite_vec(
         const T* xv = row + v_col0 + (size_t)h * dv;
         T* dst = v_cache + ((page * nkv + h) * dv) * page_size + off;
         const float* vb = hp.bias ? hp.bias + v_col0 + (size_t)h * dv : nullptr;
-        float factor = 1.f;
-        if (hp.norm_values) {
-            float ss = 0.f;
-            for (int i = li; i < dv; i += LPH) {
-                const float v = to_float(xv[i]) + (vb ? vb[i] : 0.f);
-                ss += v * v;
-            }
-#pragma unroll
-            for (int o = LPH / 2; o > 0; o >>= 1) ss += __shfl_xor(ss, o, RL_WAVE);
-            factor = rsqrtf(ss / (float)dv + eps);
-        }
+        const float factor = hp.norm_values ? value_factor(xv, vb, dv, eps) : 1.f;
         for (int i = li; i < dv; i += LPH)
             dst[(size_t)i * page_size] = from_float<T>((to_float(xv[i]) + (vb ? vb[i] : 0.f)) * factor);
         return;
