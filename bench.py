@@ -3,7 +3,7 @@
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--layers L] [--dtype bfloat16]
                     [--shape NAME] [--batch B] [--prompt-len T] [--context C]
     python bench.py --workload qwen3-0.6b-256 | qwen3-32b-32
-    python bench.py --design fokulorn|sikevik|miborax|fomunex [--design-size 2b,8b]
+    python bench.py --design fokulorn|sikevik|miborax|fomunex|pefulorn [--design-size 2b,8b]
 
 A "step" is one decode step of the whole batch through the engine's step function and the
 greedy sampling kernel, tokens fed back.  The default run has the layer sizes of
@@ -48,6 +48,12 @@ behind a short convolution, attention again; dense feed-forwards with a polynomi
 the even layers, mixtures of eight clamped gated experts behind a sigmoid router in the odd ones),
 beside the Fokulorn decoder, the engine's closest (recurrent layers with a state per request
 beside windowed attention), and Qwen3 of equal size.
+
+``--design pefulorn`` does the same for the Pefulorn decoder (attention with a logarithmic distance
+term beside a gated recurrence, a token-shift time mixing, a delta rule with a decay per key channel
+behind short convolutions; gated feed-forwards with biases; two of six layers run twice), beside
+the Fomunex decoder, the engine's closest (the same time mixing, a recurrence behind a short
+convolution, attention with a distance term), and Qwen3 of equal size.
 
 Metric definitions follow rapid_llm's docs/benchmark_models.md:141-149: decode tok/s is
 batch / mean step time; prefill tok/s is prompt tokens / prefill latency; both timed
@@ -659,6 +665,38 @@ def _time_miborax_kernels(z: dict, prompt_len: int, batch: int) -> dict:
     return out
 
 
+def _time_attention(z: dict, window: int, seqs, **options) -> float:
+    """Seconds of one attention launch over ``seqs`` = (tokens cached, tokens of the step) per request,
+    heads as the size ``z`` says, with the options of ``ops.paged_attention``."""
+    import types
+
+    import torch
+
+    from rapid_llm_amd.kernels import ops
+
+    dev, bf, page = "cuda", torch.bfloat16, 16
+    nq, nkv, dh = z["heads"], z["kv_heads"], z["head_dim"]
+    tokens = sum(n for _, n in seqs)
+    pages_per = [-(-(a + n) // page) for a, n in seqs]
+    table = torch.zeros((len(seqs), max(pages_per)), dtype=torch.int32)
+    at = 1
+    for i, n in enumerate(pages_per):
+        table[i, :n] = torch.arange(at, at + n, dtype=torch.int32)
+        at += n
+    kc = (torch.randn(at, nkv, page, dh, device=dev) * 0.3).to(bf)
+    vc = (torch.randn(at, nkv, dh, page, device=dev) * 0.3).to(bf)
+    q = (torch.randn(tokens, nq * dh, device=dev) * 0.3).to(bf)
+    o = torch.empty((tokens, nq * dh), dtype=bf, device=dev)
+    positions = torch.cat([torch.arange(a, a + n) for a, n in seqs]).to(torch.int32).to(dev)
+    slot = torch.cat([torch.full((n,), i) for i, (_, n) in enumerate(seqs)]).to(torch.int32).to(dev)
+    ctx = types.SimpleNamespace(positions=positions, token_slot=slot, token_ids=positions,
+                                h_seq_starts=[a for a, _ in seqs], h_seq_lens=[n for _, n in seqs],
+                                max_position=max(a + n for a, n in seqs) - 1, extra={}, static={})
+    table = table.to(dev)
+    return _time_calls(lambda: ops.paged_attention(q, kc, vc, o, ctx, table, page, nq, nkv, dh, window,
+                                                   dh ** -0.5, **options), max(n for _, n in seqs) == 1)
+
+
 def fomunex_body(z: dict) -> dict:
     """Layers in turn attention, time mixing, state-space, attention; the recurrent mixers with
     heads of 64 channels (the time mixing as wide as the model, the state-space mixer twice as
@@ -761,31 +799,13 @@ def _time_fomunex_kernels(z: dict, prompt_len: int, batch: int) -> dict:
     out["polynomial_activation_prefill_us"] = round(sec * 1e6, 1)
     out["polynomial_activation_prefill_frac_hbm"] = round(prompt_len * ff * 4 / sec / 1e9 / HBM_GBPS, 4)
     # ---- attention
-    nq, nkv, dh, window, page = z["heads"], z["kv_heads"], z["head_dim"], z["window"], 16
+    nq, nkv, dh, window = z["heads"], z["kv_heads"], z["head_dim"], z["window"]
     sink = torch.zeros(nq, device=dev)
     slopes = torch.exp2(-8.0 * torch.arange(1, nq + 1, device=dev, dtype=torch.float32) / nq)
 
     def attention(seqs, plain):
-        tokens = sum(n for _, n in seqs)
-        pages_per = [-(-(a + n) // page) for a, n in seqs]
-        table = torch.zeros((len(seqs), max(pages_per)), dtype=torch.int32)
-        at = 1
-        for i, n in enumerate(pages_per):
-            table[i, :n] = torch.arange(at, at + n, dtype=torch.int32)
-            at += n
-        kc = (torch.randn(at, nkv, page, dh, device=dev) * 0.3).to(bf)
-        vc = (torch.randn(at, nkv, dh, page, device=dev) * 0.3).to(bf)
-        q = (torch.randn(tokens, nq * dh, device=dev) * 0.3).to(bf)
-        o = torch.empty((tokens, nq * dh), dtype=bf, device=dev)
-        positions = torch.cat([torch.arange(a, a + n) for a, n in seqs]).to(torch.int32).to(dev)
-        slot = torch.cat([torch.full((n,), i) for i, (_, n) in enumerate(seqs)]).to(torch.int32).to(dev)
-        ctx = types.SimpleNamespace(positions=positions, token_slot=slot, token_ids=positions,
-                                    h_seq_starts=[a for a, _ in seqs], h_seq_lens=[n for _, n in seqs],
-                                    max_position=max(a + n for a, n in seqs) - 1, extra={}, static={})
-        table = table.to(dev)
         more = dict(sink=True) if plain else dict(sink_values=sink, score_cap=50.0, slopes=slopes)
-        return _time_calls(lambda: ops.paged_attention(q, kc, vc, o, ctx, table, page, nq, nkv, dh, window,
-                                                       dh ** -0.5, **more), max(n for _, n in seqs) == 1)
+        return _time_attention(z, window, seqs, **more)
 
     seen = sum(min(p + 1, window) for p in range(prompt_len))
     for label, plain in (("", False), ("_without_cap_and_distance", True)):
@@ -799,6 +819,110 @@ def _time_fomunex_kernels(z: dict, prompt_len: int, batch: int) -> dict:
     return out
 
 
+def pefulorn_body(z: dict) -> dict:
+    """Eight layer runs as six layers, two of them twice: attention beside a gated recurrence as wide
+    as the model, time mixing with heads of 64 channels, a delta rule with heads of 128 channels and
+    low-rank pairs of 128; every layer with a gated feed-forward of Qwen3's width."""
+    w = z["width"]
+    pair = {"left": {"heads": z["heads"], "kv_heads": z["kv_heads"], "dim": z["head_dim"], "vdim": z["head_dim"],
+                     "scale": z["head_dim"] ** -0.5, "q_temp": {"coef": 0.1, "every": 1024}},
+            "right": {"width": w}, "left_scale": 0.5, "right_scale": 0.5}
+    mixing = {"heads": w // 64, "dim": 64, "rank": 64}
+    delta = {"heads": w // 128, "kv_heads": w // 128, "dim": 128, "vdim": 128, "conv": 4, "decay_rank": 128,
+             "gate_rank": 128}
+    kinds = [("parallel", pair), ("wkv", mixing), ("channel_delta", delta), ("parallel", pair)]
+    layers = [{"type": kinds[i % 4][0], "mixer": kinds[i % 4][1], "mlp": {"kind": "dense", "ff": z["ff"]}}
+              for i in range(z["layers"] - 2)]
+    return {"architecture": "Pefulorn", "width": w, "vocab": z["vocab"], "norm": {"eps": 1e-6}, "layers": layers,
+            "loop": {"start": 1, "stop": 3, "times": 2}}
+
+
+def _time_pefulorn_kernels(z: dict, prompt_len: int, batch: int) -> dict:
+    """The design's own kernels alone, microseconds and share of the roofline each, over one prompt and
+    over ``batch`` single tokens: the delta rule's operands (bytes) and scan (float32 operations: seven
+    a state element and token over a prompt; bytes of state for single tokens), the time mixing's scan
+    (four operations), the gated recurrence (bytes), the biased activation (bytes), attention with the
+    distance term and without it."""
+    import types
+
+    import torch
+
+    from rapid_llm_amd.kernels import ops
+
+    dev, width, bf = "cuda", z["width"], torch.bfloat16
+    out: dict = {}
+
+    def rate(name, sec, frac_of, value):
+        out[name + "_us"] = round(sec * 1e6, 1)
+        out[f"{name}_frac_{frac_of}"] = round(value, 4)
+
+    def hbm(count, sec):
+        return count / sec / 1e9 / HBM_GBPS
+
+    def fp32(ops_count, sec):
+        return ops_count / sec / (PEAK_TFLOPS["float32"] * 1e12)
+
+    for what, lens in (("prefill", [prompt_len]), ("decode", [1] * batch)):
+        tokens, single = sum(lens), what == "decode"
+        cu = torch.tensor([0] + list(torch.tensor(lens).cumsum(0)), dtype=torch.int32, device=dev)
+        ctx = types.SimpleNamespace(num_seqs=len(lens), h_seq_lens=list(lens), h_seq_slots=list(range(len(lens))),
+                                    cu_seqlens=cu, seq_slots=torch.arange(len(lens), dtype=torch.int32, device=dev))
+        # ---- delta rule
+        h, d, taps = width // 128, 128, 4
+        channels = 3 * h * d
+        packed = (torch.randn(tokens, channels, device=dev) * 0.5).to(bf)
+        conv_w = torch.randn(channels, taps, device=dev) * 0.5
+        conv_state, S = torch.zeros((batch, taps - 1, channels), device=dev), torch.zeros((batch, h, d, d), device=dev)
+        pre, beta = torch.randn(tokens, h * d, device=dev), torch.randn(tokens, h, device=dev)
+        dt_bias, a_log = torch.full((h * d,), -2.0, device=dev), torch.zeros(h, device=dev)
+        mixed, raw = torch.empty((tokens, channels), device=dev), torch.empty((tokens, h * d), device=dev)
+        sec = _time_calls(lambda: ops.delta_prepare(packed, 0, conv_w, conv_state, pre, dt_bias, a_log, mixed, ctx, h, h, d, d), single)
+        rate(f"delta_operands_{what}", sec, "hbm", hbm(tokens * (channels * (2 + 4) + h * d * 8), sec))
+        decay = torch.full((tokens, h * d), 0.98, device=dev)
+        sec = _time_calls(lambda: ops.delta_scan(mixed, decay, beta, raw, ctx, S, h, h, d, d), single)
+        if single:
+            rate("delta_scan_decode", sec, "hbm", hbm(2.0 * batch * h * d * d * 4, sec))
+        else:
+            rate("delta_scan_prefill", sec, "fp32_matrix", fp32(tokens * h * 7.0 * d * d, sec))
+        g, nw, o = (torch.randn(tokens, h * d, device=dev)).to(bf), torch.ones(d, device=dev), torch.empty((tokens, h * d), dtype=bf, device=dev)
+        sec = _time_calls(lambda: ops.head_finish(raw, g, nw, o, h, 1e-6, "sigmoid"), single)
+        rate(f"head_norm_gate_{what}", sec, "hbm", hbm(tokens * h * d * (4 + 2 + 2), sec))
+        # ---- time mixing
+        hw, dw = width // 64, 64
+        Sw = torch.zeros((batch, hw, dw, dw), device=dev)
+        r, k, v, gw = ((torch.randn(tokens, width, device=dev) * 0.5).to(bf) for _ in range(4))
+        bias, u, nww = torch.full((width,), -2.5, device=dev), torch.zeros((hw, dw), device=dev), torch.ones(width, device=dev)
+        prew = torch.randn(tokens, width, device=dev)
+        ow = torch.empty((tokens, width), dtype=bf, device=dev)
+        sec = _time_calls(lambda: ops.wkv(r, k, v, gw, prew, bias, u, nww, ow, ctx, Sw, hw, dw, 1e-6), single)
+        if single:
+            rate("time_mixing_scan_decode", sec, "hbm", hbm(2.0 * batch * hw * dw * dw * 4, sec))
+        else:
+            rate("time_mixing_scan_prefill", sec, "fp32_matrix", fp32(tokens * hw * 4.0 * dw * dw, sec))
+        # ---- gated recurrence: three projections read, one row written
+        row = (torch.randn(tokens, 3 * width, device=dev)).to(bf)
+        zb, Sg = torch.full((width,), -2.0, device=dev), torch.zeros((batch, width), device=dev)
+        sec = _time_calls(lambda: ops.min_gru(row, (0, width, 2 * width), zb, zb, ow, ctx, Sg), single)
+        rate(f"gated_recurrence_{what}", sec, "hbm", hbm(tokens * width * 2 * 4 + (2 * batch * width * 4 if single else 0), sec))
+        if not single:
+            ff = z["ff"]
+            gate_up = (torch.randn(tokens, 2 * ff, device=dev)).to(bf)
+            act, fb = torch.empty((tokens, ff), dtype=bf, device=dev), torch.zeros(2 * ff, device=dev)
+            for label, more in (("gelu_gate_biased", dict(activation="gelu_tanh", bias=fb)), ("silu_gate", {})):
+                sec = _time_calls(lambda: ops.swiglu(gate_up, act, **more), False)
+                rate(f"{label}_prefill", sec, "hbm", hbm(tokens * ff * 6, sec))
+    # ---- attention
+    nq, nkv, dh = z["heads"], z["kv_heads"], z["head_dim"]
+    numbers = torch.full((nq,), 0.7, device=dev), torch.full((nq,), 0.3, device=dev)
+    seen = prompt_len * (prompt_len + 1) // 2
+    for label, more in (("", dict(log_distance=numbers, out_scale=0.5)), ("_without_distance", dict(out_scale=0.5))):
+        sec = _time_attention(z, 0, [(0, prompt_len)], **more)
+        rate(f"attention_prefill{label}", sec, "bf16_matrix", 4.0 * nq * dh * seen / sec / (PEAK_TFLOPS["bfloat16"] * 1e12))
+        sec = _time_attention(z, 0, [(prompt_len, 1)] * batch, **more)
+        rate(f"attention_decode{label}", sec, "hbm", hbm(batch * (prompt_len + 1) * nkv * dh * 2 * 2, sec))
+    return out
+
+
 # design -> (name, its configuration at a size, its kernels alone, the engine's closest other
 # architecture measured beside it and Qwen3)
 DESIGNS = {
@@ -806,6 +930,7 @@ DESIGNS = {
     "sikevik": ("Sikevik", sikevik_body, _time_sikevik_kernels, None),
     "miborax": ("Miborax", miborax_body, _time_miborax_kernels, ("sikevik", sikevik_body)),
     "fomunex": ("Fomunex", fomunex_body, _time_fomunex_kernels, ("fokulorn", fokulorn_body)),
+    "pefulorn": ("Pefulorn", pefulorn_body, _time_pefulorn_kernels, ("fomunex", fomunex_body)),
 }
 
 
@@ -863,7 +988,7 @@ def main() -> int:
     ap.add_argument("--peaks", action="store_true",
                     help="measure what the device reaches with library kernels (a large read, copy and square products) and exit")
     ap.add_argument("--design", default=None,
-                    help="measure another architecture of the engine beside Qwen3 at equal size (fokulorn, sikevik, miborax, fomunex) and exit")
+                    help="measure another architecture of the engine beside Qwen3 at equal size (fokulorn, sikevik, miborax, fomunex, pefulorn) and exit")
     ap.add_argument("--design-size", default="2b,8b", help=f"sizes for --design: {', '.join(DESIGN_SIZES)}")
     args = ap.parse_args()
     if args.peaks:
