@@ -592,14 +592,15 @@ __global__ void swiglu_vec_kernel(const T* __restrict__ gate_up, T* __restrict__
         const Vec8<T> u = *reinterpret_cast<const Vec8<T>*>(row + inter + j);
         // (with a route, an expert's hidden units are a multiple of 8: one factor a group)
         const float factor = (route && j < experts * ff) ? route[t * experts + j / ff] : 1.f;
+        Vec8<float> gb = {}, ub = {};
+        if (glu.bias) {
+            gb = *reinterpret_cast<const Vec8<float>*>(glu.bias + j);
+            ub = *reinterpret_cast<const Vec8<float>*>(glu.bias + inter + j);
+        }
         Vec8<T> y;
 #pragma unroll
         for (int i = 0; i < 8; ++i) {
-            float gi = to_float(g.v[i]), ui = to_float(u.v[i]);
-            if (glu.bias) {
-                gi += glu.bias[j + i];
-                ui += glu.bias[inter + j + i];
-            }
+            const float gi = to_float(g.v[i]) + gb.v[i], ui = to_float(u.v[i]) + ub.v[i];
             y.v[i] = from_float<T>(route_input ? glu_act(gi * factor, ui * factor, glu) : glu_act(gi, ui, glu) * factor);
         }
         *reinterpret_cast<Vec8<T>*>(out + t * (size_t)inter + j) = y;
@@ -1255,14 +1256,15 @@ __device__ inline void qknorm_rope_kvwrite_vec(
     if (active) {
         const Vec4<T> va = *reinterpret_cast<const Vec4<T>*>(x + 4 * li);
         const Vec4<T> vb = *reinterpret_cast<const Vec4<T>*>(x + half + 4 * li);
+        Vec4<float> ba = {}, bb = {};
+        if (hp.bias) {
+            ba = *reinterpret_cast<const Vec4<float>*>(hp.bias + (size_t)head * d + 4 * li);
+            bb = *reinterpret_cast<const Vec4<float>*>(hp.bias + (size_t)head * d + half + 4 * li);
+        }
 #pragma unroll
         for (int k = 0; k < 4; ++k) {
-            a[k] = to_float(va.v[k]);
-            b[k] = to_float(vb.v[k]);
-            if (hp.bias) {
-                a[k] += hp.bias[(size_t)head * d + 4 * li + k];
-                b[k] += hp.bias[(size_t)head * d + half + 4 * li + k];
-            }
+            a[k] = to_float(va.v[k]) + ba.v[k];
+            b[k] = to_float(vb.v[k]) + bb.v[k];
             ss += a[k] * a[k] + b[k] * b[k];
         }
     }

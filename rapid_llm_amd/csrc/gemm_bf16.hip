@@ -98,6 +98,9 @@ struct SkinnyExtra {
     bf16_t* xt;           // [M, N] residual * norm_w
     float* partial;       // [workgroups][16]
     const float* bias;    // [N] added to the product in front of the residual, or null
+    // plain results: columns from `split` on go to wide [M, N - split] in float32 instead (null: none)
+    float* wide;
+    int split;
     // the gated activation of the gate/up variants
     Glu glu;
 };
@@ -346,6 +349,8 @@ __global__ __launch_bounds__(GW* RL_WAVE) void gemm_skinny_kernel(
                     ex.residual[at] = r;
                     ex.xt[at] = float_to_bf16(r * nw_in[i]);
                     sumsq += r * r;
+                } else if (!SWIGLU && ex.wide && n >= ex.split) {
+                    ex.wide[(size_t)m * (N - ex.split) + n - ex.split] = v;
                 } else {
                     store_out<OutT>(out + (size_t)m * ldo + n, v);
                 }
@@ -604,15 +609,19 @@ static SkinnyExtra scaled_input(const float* x_partial, int x_parts, int x_size,
 }
 
 // out_type: RL_F32 or RL_BF16.  nt: weight-row tiles per workgroup, 1 or 2, or 3 for one and a
-// half (24 rows), see the host wrapper.
+// half (24 rows), see the host wrapper.  wide (optional): the results of columns from `split` on, in
+// float32 and packed; out then has `split` columns.
 extern "C" int rl_gemm_skinny(const void* X, const void* W, void* out, int M, int N, int K,
                               int ldx, int ldw, int ldo, int out_type, int nt,
                               const float* x_partial, int x_parts, int x_size, float x_eps,
-                              hipStream_t stream) {
+                              float* wide, int split, hipStream_t stream) {
     if (M <= 0 || N <= 0) return RL_OK;
-    if (!skinny_args_ok(M, K, ldx, ldw) || ldo < N || (x_partial && (x_parts < 1 || x_size < 1)))
+    if (wide && (split < 0 || split > N)) return RL_ERR_ARG;
+    if (!skinny_args_ok(M, K, ldx, ldw) || ldo < (wide ? split : N) || (x_partial && (x_parts < 1 || x_size < 1)))
         return RL_ERR_ARG;
-    const SkinnyExtra ex = scaled_input(x_partial, x_parts, x_size, x_eps);
+    SkinnyExtra ex = scaled_input(x_partial, x_parts, x_size, x_eps);
+    ex.wide = wide;
+    ex.split = split;
     if (out_type == RL_F32)
         return dispatch<float, false>((const bf16_t*)X, (const bf16_t*)W, (float*)out, M, N, K,
                                       ldx, ldw, ldo, nt, ex, stream);

@@ -690,29 +690,46 @@ __global__ __launch_bounds__(256) void delta_prepare_kernel(
     }
 }
 
+// lane + 16's and lane's value, summed in both (every even row of 16 lanes with the odd one behind it)
+__device__ inline float both_rows(float v) {
+    const unsigned u = __float_as_uint(v);
+    const auto a = __builtin_amdgcn_permlane16_swap(u, u, false, false);
+    return __uint_as_float(a[0]) + __uint_as_float(a[1]);
+}
+// the sum over the 16 or 32 lanes of a column, in every one of them
+template <int LPC>
+__device__ inline float column_sum(float v) {
+    v = row16_sum(v);
+    if constexpr (LPC == 32) v = both_rows(v);
+    return v;
+}
+
 // The scan.  Per head (head h reads q and k of kv head h / (heads / kv_heads)), state S[key channel i]
 // [value channel j], kept as [j][i]; for a token with q, k, v, the decays g and beta = sigmoid(b):
 //   S_ij <- g_i S_ij      u_j = beta (v_j - sum_i S_ij k_i)      S_ij <- S_ij + k_i u_j      o_j = sum_i S_ij q_i
 // The sum that u needs stands between two tokens and is folded at once; the read-out's sums are folded
-// behind a block of tokens.  o goes out unfinished (float32).
-template <int RPL>
+// behind a block of tokens.  o goes out unfinished (float32).  LPC lanes share a column: 16, or 32 where
+// that leaves a lane four rows instead of eight and the workgroups still fill the chip no further.
+template <int LPC, int RPL>
 __global__ __launch_bounds__(SCAN_THREADS) __attribute__((amdgpu_waves_per_eu(1, 2))) void delta_scan_kernel(
     const float* __restrict__ mixed, const float* __restrict__ decay, const float* __restrict__ beta_pre,
     int beta_width, float* __restrict__ raw, const int* __restrict__ cu, const int* __restrict__ seq_slots,
     float* __restrict__ S, int heads, int kv_heads, int d, int dv) {
-    constexpr int DP = 16 * RPL;  // rows, padded
-    constexpr int PER_THREAD = SCAN_TOKENS * DP / SCAN_THREADS;  // = RPL
+    constexpr int DP = LPC * RPL;  // rows, padded
+    constexpr int PER_THREAD = SCAN_TOKENS * DP / SCAN_THREADS;
+    constexpr int CPW = RL_WAVE / LPC;       // columns of a wave
+    constexpr int COLS = CPW * SCAN_WAVES;   // and of a workgroup
     const int s = blockIdx.x, h = blockIdx.y;
     const int t0 = cu[s], t1 = cu[s + 1];
     const int channels = 2 * kv_heads * d + heads * dv;
     const int hk = h / (heads / kv_heads);
     const int lane = threadIdx.x & (RL_WAVE - 1), wave = threadIdx.x / RL_WAVE;
-    const int c = lane & 15;
-    const int col = wave * 4 + (lane >> 4);
-    const int j = blockIdx.z * SCAN_COLS + col;
+    const int c = lane & (LPC - 1);
+    const int col = wave * CPW + lane / LPC;
+    const int j = blockIdx.z * COLS + col;
     const bool live = j < dv;
     __shared__ __attribute__((aligned(16))) float sq[SCAN_TOKENS][DP], sk[SCAN_TOKENS][DP], sg[SCAN_TOKENS][DP];
-    __shared__ float sv[SCAN_TOKENS][SCAN_COLS], sb[SCAN_TOKENS];
+    __shared__ float sv[SCAN_TOKENS][COLS], sb[SCAN_TOKENS];
     float* Sp = S + (((size_t)seq_slots[s] * heads + h) * dv + (live ? j : 0)) * d;
     float state[RPL];
     state_rows_load<RPL>(Sp, c * RPL, d, live, state);
@@ -728,7 +745,7 @@ __global__ __launch_bounds__(SCAN_THREADS) __attribute__((amdgpu_waves_per_eu(1,
             pk[e] = ok ? row[kv_heads * d] : 0.f;
             pg[e] = ok ? decay[(size_t)(tb + tt) * heads * d + h * d + i] : 0.f;
         }
-        const int tt = threadIdx.x / SCAN_COLS, jj = blockIdx.z * SCAN_COLS + threadIdx.x % SCAN_COLS;
+        const int tt = threadIdx.x / COLS, jj = blockIdx.z * COLS + threadIdx.x % COLS;
         const bool ok = tt < SCAN_TOKENS && tb + tt < t1;
         pv = (ok && jj < dv) ? mixed[(size_t)(tb + tt) * channels + 2 * kv_heads * d + h * dv + jj] : 0.f;
         const int tk = threadIdx.x;
@@ -742,7 +759,7 @@ __global__ __launch_bounds__(SCAN_THREADS) __attribute__((amdgpu_waves_per_eu(1,
             (&sk[0][0])[idx] = pk[e];
             (&sg[0][0])[idx] = pg[e];
         }
-        if (threadIdx.x < SCAN_TOKENS * SCAN_COLS) (&sv[0][0])[threadIdx.x] = pv;
+        if (threadIdx.x < SCAN_TOKENS * COLS) (&sv[0][0])[threadIdx.x] = pv;
         if (threadIdx.x < SCAN_TOKENS) sb[threadIdx.x] = 1.f / (1.f + expf(-pb));
     };
     fetch(t0);
@@ -760,7 +777,7 @@ __global__ __launch_bounds__(SCAN_THREADS) __attribute__((amdgpu_waves_per_eu(1,
                 float& sum = (ii & 1) ? odd : even;
                 sum = fmaf(state[ii], sk[tt][c * RPL + ii], sum);
             }
-            const float u = sb[tt] * (sv[tt][col] - row16_sum(even + odd));
+            const float u = sb[tt] * (sv[tt][col] - column_sum<LPC>(even + odd));
             float o = 0.f;
 #pragma unroll
             for (int ii = 0; ii < RPL; ++ii) {
@@ -775,14 +792,16 @@ __global__ __launch_bounds__(SCAN_THREADS) __attribute__((amdgpu_waves_per_eu(1,
 #pragma unroll
             for (int tt = 0; tt < SCAN_TOKENS; ++tt) os[tt] = token(tt);
             row16_sums(os);
-            // every lane of a column holds all sixteen sums: lane c stores token c's
+            // every lane of a row of sixteen holds that row's sums of all tokens: lane c takes
+            // token c's, and where a column is two rows of lanes adds the other row's
             float mine = os[0];
 #pragma unroll
-            for (int tt = 1; tt < SCAN_TOKENS; ++tt) mine = c == tt ? os[tt] : mine;
-            if (live) dst[(size_t)c * heads * dv] = mine;
+            for (int tt = 1; tt < SCAN_TOKENS; ++tt) mine = (c & 15) == tt ? os[tt] : mine;
+            if constexpr (LPC == 32) mine = both_rows(mine);
+            if (live && c < SCAN_TOKENS) dst[(size_t)c * heads * dv] = mine;
         } else {
             for (int tt = 0; tt < nt; ++tt) {
-                const float o = row16_sum(token(tt));
+                const float o = column_sum<LPC>(token(tt));
                 if (c == 0 && live) dst[(size_t)tt * heads * dv] = o;
             }
         }
@@ -794,12 +813,15 @@ __global__ __launch_bounds__(SCAN_THREADS) __attribute__((amdgpu_waves_per_eu(1,
 // Gated recurrence whose gates read the current token alone (minGRU).  With z = sigmoid(zp + bz) and
 // u = xp + bx of the packed row's columns z0 and x0 on, per channel
 //   S <- (1 - z) S + z (u >= 0 ? u + 1/2 : sigmoid(u))        out = scale * S * silu(gp)
-// The chain between tokens is one fused multiply-add, everything else is independent of it: a
-// workgroup takes 8 channels and 64 tokens at a time, all its threads form the two factors, eight
-// lanes walk the chain through LDS, all threads finish the outputs.
+// The chain between tokens is one fused multiply-add, everything else is independent of it.  A
+// workgroup takes 8 channels and 64 tokens at a time in three stages that run side by side: four
+// waves form the two factors of block i and finish the outputs of block i - 2, while lanes of the
+// first wave walk the chain of block i - 1; the stages meet in LDS, one barrier a block.
 // --------------------------------------------------------------------------- //
 constexpr int GRU_CHANNELS = 8;
 constexpr int GRU_TOKENS = 64;
+constexpr int GRU_WORKERS = 256;                   // threads behind the first wave
+constexpr int GRU_PITCH = GRU_TOKENS + 4;          // a channel's tokens side by side
 
 // float32 keeps the library's exponential and division, bfloat16 takes the hardware's instructions
 template <typename T>
@@ -823,28 +845,31 @@ __device__ inline void gru_factors(float zp, float u, float& keep, float& add) {
 }
 
 template <typename T>
-__global__ __launch_bounds__(256) void gru_scan_kernel(const T* __restrict__ packed, int row_width, int z0, int x0,
-                                                       int g0, const float* __restrict__ bz,
-                                                       const float* __restrict__ bx, float* __restrict__ S,
-                                                       T* __restrict__ out, int out_width, float scale,
-                                                       const int* __restrict__ cu, const int* __restrict__ seq_slots,
-                                                       int width) {
-    constexpr int PER = GRU_TOKENS * GRU_CHANNELS / 256;
+__global__ __launch_bounds__(RL_WAVE + GRU_WORKERS) void gru_scan_kernel(
+    const T* __restrict__ packed, int row_width, int z0, int x0, int g0, const float* __restrict__ bz,
+    const float* __restrict__ bx, float* __restrict__ S, T* __restrict__ out, int out_width, float scale,
+    const int* __restrict__ cu, const int* __restrict__ seq_slots, int width) {
+    constexpr int PER = GRU_TOKENS * GRU_CHANNELS / GRU_WORKERS;  // elements of a block a worker takes
+    constexpr int APART = GRU_WORKERS / GRU_CHANNELS;             // tokens between them
     const int s = blockIdx.x;
     const int t0 = cu[s], t1 = cu[s + 1];
-    const int c = blockIdx.y * GRU_CHANNELS + threadIdx.x % GRU_CHANNELS;
-    const int tt0 = threadIdx.x / GRU_CHANNELS;  // and every 32nd token behind it
+    const bool walks = threadIdx.x < RL_WAVE;
+    const int w = walks ? threadIdx.x : threadIdx.x - RL_WAVE;
+    const int ch = w % GRU_CHANNELS, tt0 = w / GRU_CHANNELS;
+    const int c = blockIdx.y * GRU_CHANNELS + ch;
     const bool live = c < width;
-    __shared__ float keep[GRU_TOKENS][GRU_CHANNELS], add[GRU_TOKENS][GRU_CHANNELS], sums[GRU_TOKENS][GRU_CHANNELS];
+    __shared__ __attribute__((aligned(16))) float keep[2][GRU_CHANNELS][GRU_PITCH], add[2][GRU_CHANNELS][GRU_PITCH],
+        sums[2][GRU_CHANNELS][GRU_PITCH];
     const float zb = live ? bz[c] : 0.f, xb = live ? bx[c] : 0.f;
     float* slot = S + (size_t)seq_slots[s] * width + c;
-    float state = (threadIdx.x < GRU_CHANNELS && live) ? *slot : 0.f;
+    const bool chain = walks && w < GRU_CHANNELS && live;
+    float state = chain ? *slot : 0.f;
     const T zero = from_float<T>(0.f);
     T pz[PER], px[PER], pg[PER];
-    auto fetch = [&](int tb) {
+    auto fetch = [&](int block) {
 #pragma unroll
         for (int e = 0; e < PER; ++e) {
-            const int t = tb + tt0 + e * (256 / GRU_CHANNELS);
+            const int t = t0 + block * GRU_TOKENS + tt0 + e * APART;
             const bool ok = live && t < t1;
             const T* row = packed + (size_t)t * row_width + c;
             pz[e] = ok ? row[z0] : zero;
@@ -852,44 +877,58 @@ __global__ __launch_bounds__(256) void gru_scan_kernel(const T* __restrict__ pac
             pg[e] = ok ? row[g0] : zero;
         }
     };
-    fetch(t0);
-    for (int tb = t0; tb < t1; tb += GRU_TOKENS) {
-        float gate[PER];
+    const int blocks = (t1 - t0 + GRU_TOKENS - 1) / GRU_TOKENS;
+    float gate[PER], gate1[PER], gate2[PER];  // of the block at hand and of the two before it
 #pragma unroll
-        for (int e = 0; e < PER; ++e) {
-            const int tt = tt0 + e * (256 / GRU_CHANNELS);
-            gru_factors<T>(to_float(pz[e]) + zb, to_float(px[e]) + xb, keep[tt][threadIdx.x % GRU_CHANNELS],
-                           add[tt][threadIdx.x % GRU_CHANNELS]);
-            const float z = to_float(pg[e]);
-            gate[e] = scale * z * sigmoid_of<T>(z);
-        }
-        __syncthreads();
-        if (tb + GRU_TOKENS < t1) fetch(tb + GRU_TOKENS);
-        const int nt = min(GRU_TOKENS, t1 - tb);
-        if (threadIdx.x < GRU_CHANNELS) {
-            if (nt == GRU_TOKENS) {
-#pragma unroll 16
-                for (int tt = 0; tt < GRU_TOKENS; ++tt) {
-                    state = fmaf(keep[tt][threadIdx.x], state, add[tt][threadIdx.x]);
-                    sums[tt][threadIdx.x] = state;
+    for (int e = 0; e < PER; ++e) gate[e] = gate1[e] = gate2[e] = 0.f;
+    if (!walks) fetch(0);
+    for (int i = 0; i < blocks + 2; ++i) {
+        if (walks) {
+            if (chain && i >= 1 && i <= blocks) {
+                const float4* k4 = reinterpret_cast<const float4*>(keep[(i - 1) & 1][ch]);
+                const float4* a4 = reinterpret_cast<const float4*>(add[(i - 1) & 1][ch]);
+                float4* s4 = reinterpret_cast<float4*>(sums[(i - 1) & 1][ch]);
+#pragma unroll
+                for (int q = 0; q < GRU_TOKENS / 4; ++q) {
+                    const float4 k = k4[q], a = a4[q];
+                    float4 o;
+                    o.x = state = fmaf(k.x, state, a.x);
+                    o.y = state = fmaf(k.y, state, a.y);
+                    o.z = state = fmaf(k.z, state, a.z);
+                    o.w = state = fmaf(k.w, state, a.w);
+                    s4[q] = o;
                 }
-            } else {
-                for (int tt = 0; tt < nt; ++tt) {
-                    state = fmaf(keep[tt][threadIdx.x], state, add[tt][threadIdx.x]);
-                    sums[tt][threadIdx.x] = state;
+            }
+        } else {
+#pragma unroll
+            for (int e = 0; e < PER; ++e) {
+                gate2[e] = gate1[e];
+                gate1[e] = gate[e];
+            }
+            if (i < blocks) {
+#pragma unroll
+                for (int e = 0; e < PER; ++e) {
+                    const int tt = tt0 + e * APART;
+                    float k = 1.f, a = 0.f;  // tokens beyond the portion leave the state as it is
+                    if (t0 + i * GRU_TOKENS + tt < t1) gru_factors<T>(to_float(pz[e]) + zb, to_float(px[e]) + xb, k, a);
+                    keep[i & 1][ch][tt] = k;
+                    add[i & 1][ch][tt] = a;
+                    const float z = to_float(pg[e]);
+                    gate[e] = scale * z * sigmoid_of<T>(z);
+                }
+                if (i + 1 < blocks) fetch(i + 1);
+            }
+            if (i >= 2) {
+#pragma unroll
+                for (int e = 0; e < PER; ++e) {
+                    const int tt = tt0 + e * APART, t = t0 + (i - 2) * GRU_TOKENS + tt;
+                    if (live && t < t1) out[(size_t)t * out_width + c] = from_float<T>(gate2[e] * sums[i & 1][ch][tt]);
                 }
             }
         }
         __syncthreads();
-#pragma unroll
-        for (int e = 0; e < PER; ++e) {
-            const int tt = tt0 + e * (256 / GRU_CHANNELS);
-            if (live && tb + tt < t1)
-                out[(size_t)(tb + tt) * out_width + c] = from_float<T>(gate[e] * sums[tt][threadIdx.x % GRU_CHANNELS]);
-        }
-        // (the next round's factors do not touch `sums`, and its chain starts behind a barrier)
     }
-    if (threadIdx.x < GRU_CHANNELS && live) *slot = state;
+    if (chain) *slot = state;
 }
 
 // a step of single tokens: one thread a (request, channel)
@@ -1150,21 +1189,23 @@ extern "C" int rl_delta_scan(const float* mixed, const float* decay, const float
     if (heads < 1 || heads > 65535 || kv_heads < 1 || heads % kv_heads || d < 1 || d > 256 || dv < 1 || dv > 256 ||
         beta_width < heads || num_seqs > 65535)
         return RL_ERR_ARG;
-    dim3 grid(num_seqs, heads, (dv + recurrent::SCAN_COLS - 1) / recurrent::SCAN_COLS);
-#define RL_DELTA(RPL)                                                                                               \
-    hipLaunchKernelGGL((recurrent::delta_scan_kernel<RPL>), grid, dim3(recurrent::SCAN_THREADS), 0, stream, mixed, decay, \
-                       beta_pre, beta_width, raw, cu, seq_slots, S, heads, kv_heads, d, dv)
-    const int rows = (d + 15) / 16;
-    if (rows <= 1)
-        RL_DELTA(1);
-    else if (rows <= 2)
-        RL_DELTA(2);
-    else if (rows <= 4)
-        RL_DELTA(4);
-    else if (rows <= 8)
-        RL_DELTA(8);
+#define RL_DELTA(LPC, RPL)                                                                                          \
+    do {                                                                                                            \
+        constexpr int cols = RL_WAVE / LPC * recurrent::SCAN_WAVES;                                                 \
+        hipLaunchKernelGGL((recurrent::delta_scan_kernel<LPC, RPL>), dim3(num_seqs, heads, (dv + cols - 1) / cols), \
+                           dim3(recurrent::SCAN_THREADS), 0, stream, mixed, decay, beta_pre, beta_width, raw, cu,   \
+                           seq_slots, S, heads, kv_heads, d, dv);                                                   \
+    } while (0)
+    if (d <= 16)
+        RL_DELTA(16, 1);
+    else if (d <= 32)
+        RL_DELTA(16, 2);
+    else if (d <= 64)
+        RL_DELTA(16, 4);
+    else if (d <= 128)
+        RL_DELTA(32, 4);
     else
-        RL_DELTA(16);
+        RL_DELTA(32, 8);
 #undef RL_DELTA
     return rl_launch_status();
 }
@@ -1195,8 +1236,8 @@ static int launch_gru(const T* packed, int row_width, int z0, int x0, int g0, co
                            packed, row_width, z0, x0, g0, bz, bx, S, out, out_width, scale, seq_slots, width);
     else
         hipLaunchKernelGGL(recurrent::gru_scan_kernel<T>,
-                           dim3(num_seqs, (width + recurrent::GRU_CHANNELS - 1) / recurrent::GRU_CHANNELS), dim3(256), 0,
-                           stream, packed, row_width, z0, x0, g0, bz, bx, S, out, out_width, scale, cu, seq_slots,
+                           dim3(num_seqs, (width + recurrent::GRU_CHANNELS - 1) / recurrent::GRU_CHANNELS),
+                           dim3(RL_WAVE + recurrent::GRU_WORKERS), 0, stream, packed, row_width, z0, x0, g0, bz, bx, S, out, out_width, scale, cu, seq_slots,
                            width);
     return rl_launch_status();
 }

@@ -1074,6 +1074,32 @@ def _scaled_args(scaled, rows: int, k: int) -> tuple:
     return (_p(scaled.partial), scaled.partial.shape[0], scaled.size, ctypes.c_float(scaled.eps))
 
 
+def gemm_bf16_split(x: torch.Tensor, w: torch.Tensor, split: int, scaled=None) -> tuple[torch.Tensor, torch.Tensor]:
+    """``x[M,K] @ w[N,K]^T`` in two types: the first ``split`` columns in bfloat16, the others in float32 as
+    the accumulation leaves them (:func:`gemm_bf16_wide`).  Few rows are one launch.  ``scaled``: as in
+    :func:`gemm_bf16`."""
+    m, k = x.shape
+    n = w.shape[0]
+    if not 0 < split < n:
+        raise KernelError(f"a product of {n} columns does not split at {split}")
+    if m > SKINNY_MAX_ROWS or k % 8:
+        if scaled is not None:
+            raise KernelError(f"scaled rows need the few-row product: {m} rows over {k}")
+        return gemm_bf16(x, w[:split], torch.bfloat16), gemm_bf16_wide(x, w[split:])
+    _need(x, "x", torch.bfloat16)
+    _need(w, "w", torch.bfloat16, (n, k))
+    out = torch.empty((m, split), dtype=torch.bfloat16, device=x.device)
+    wide = torch.empty((m, n - split), dtype=torch.float32, device=x.device)
+    _ok(
+        core().rl_gemm_skinny(
+            _p(x), _p(w), _p(out), m, n, k, k, k, split, BF16, _skinny_tiles(m, n, plain=True),
+            *_scaled_args(scaled, m, k), _p(wide), split, _stream()
+        ),
+        "rl_gemm_skinny",
+    )
+    return out, wide
+
+
 def gemm_bf16(x: torch.Tensor, w: torch.Tensor, out_dtype: torch.dtype, scaled=None) -> torch.Tensor:
     """``x[M,K] @ w[N,K]^T`` with bfloat16 operands and float32 accumulation.  ``scaled``
     (few rows only): the rows of ``x`` still lack their norm's factor, which is applied to
@@ -1083,8 +1109,15 @@ def gemm_bf16(x: torch.Tensor, w: torch.Tensor, out_dtype: torch.dtype, scaled=N
     float32 directly; so does the kernel for 17 to 64 rows over wide matrices.  Small matrices
     run the one-launch tile product up to 512 rows.  Everything else goes to the library
     product, as the reference's dense products do (``F.linear``); a bfloat16 result is returned
-    as is and widened by the caller."""
-    _need(x, "x", torch.bfloat16)
+    as is and widened by the caller.  ``x`` may be columns of a wider row."""
+    if x.dim() == 2 and not x.is_contiguous() and not (
+        x.stride(1) == 1 and x.stride(0) % 8 == 0 and x.data_ptr() % 16 == 0 and x.shape[0] <= SKINNY_MAX_ROWS
+    ):
+        x = x.contiguous()
+    if x.is_contiguous():
+        _need(x, "x", torch.bfloat16)
+    elif not x.is_cuda or x.dtype != torch.bfloat16:
+        raise KernelError(f"x must be bfloat16 on the GPU, is {x.dtype} on {x.device}")
     _need(w, "w", torch.bfloat16)
     m, k = x.shape
     n = w.shape[0]
@@ -1097,11 +1130,13 @@ def gemm_bf16(x: torch.Tensor, w: torch.Tensor, out_dtype: torch.dtype, scaled=N
         nt = _skinny_tiles(m, n, plain=True)
         _ok(
             core().rl_gemm_skinny(
-                _p(x), _p(w), _p(out), m, n, k, k, k, n, _tag(out_dtype), nt, *_scaled_args(scaled, m, k), _stream()
+                _p(x), _p(w), _p(out), m, n, k, k if x.is_contiguous() else x.stride(0), k, n, _tag(out_dtype), nt,
+                *_scaled_args(scaled, m, k), None, 0, _stream()
             ),
             "rl_gemm_skinny",
         )
         return out
+    x = x.contiguous()
     if scaled is not None:
         raise KernelError(f"scaled rows need the few-row product: {m} rows over {k}")
     if _tile_applies(m, n, k, n):

@@ -12,9 +12,8 @@ state ``S [key channel, value channel]``::
 Each head's ``o`` is divided by its root mean square, multiplied by a weight that the heads share and by
 ``sigmoid(W_g2 (W_g1 h))``, and the output projection follows.
 
-``q``, ``k``, ``v`` come from one packed product, with the two products of the output gate in the compute
-type.  ``W_a1`` and ``W_b`` form one product with a float32 result, ``W_a2`` is held in float32; the
-convolution's sums, unit norms, softplus, exponentials, the state and the head norm are float32
+Everything that reads ``h`` is one packed product, ``[q | k | v | g1]`` with a result in the compute type and
+``[b | a1]`` with a float32 one; ``W_a2`` is held in float32.  The convolution's sums, unit norms, softplus, exponentials, the state and the head norm are float32
 (``csrc/recurrent.hip``).  The state and the convolutions' last ``taps - 1`` inputs live in the request's
 slot (``cache.states``).
 """
@@ -77,7 +76,7 @@ class DeltaRule(Mixer):
         self.conv_suffix = conv_suffix
         self.inner = num_heads * value_dim
         self.channels = 2 * num_kv_heads * key_dim + self.inner  # what the convolutions mix
-        self.qkv = Linear(hidden_size, self.channels)
+        self.in_proj = None  # sized when the tensors are bound
         self.o = Linear(self.inner, hidden_size)
 
     # ---- tensors ---------------------------------------------------------------
@@ -110,18 +109,28 @@ class DeltaRule(Mixer):
         def get(which: str) -> torch.Tensor:
             return params[f"{self.name}.{which}"]
 
-        self.qkv.bind(get("qkv"))
         a1, a2, g1, g2 = get("decay_in"), get("decay_out"), get("gate_in"), get("gate_out")
         for first, second, what in ((a1, a2, "decay"), (g1, g2, "gate")):
             if first.shape[0] != second.shape[1]:
                 raise ValueError(f"the {what}'s two matrices do not meet: {tuple(first.shape)} and {tuple(second.shape)}")
-        # one product with a float32 result: beta's rows, then the decay's first matrix
-        low = torch.cat([t.to(torch.promote_types(get("beta").dtype, a1.dtype)) for t in (get("beta"), a1)])
-        self.low = Linear(self.hidden_size, low.shape[0])
-        self.low.bind(low)
+        # The rows of the packed product.  The compute-type part is padded so that both parts are whole
+        # groups of eight rows and the gate's columns begin at one.
+        qkv, beta = get("qkv"), get("beta")
+        pads = (-self.channels % 8, -g1.shape[0] % 8)
+        self.gate_col = self.channels + pads[0]
+        self.split = self.gate_col + g1.shape[0] + pads[1]
+        kept = torch.float32 if any(t.dtype == torch.float32 for t in (qkv, beta, a1, g1)) else qkv.dtype
+        rows = [qkv, qkv.new_zeros(pads[0], self.hidden_size), g1, qkv.new_zeros(pads[1], self.hidden_size), beta, a1]
+        packed = torch.cat([t.to(kept) for t in rows])
+        self.in_proj = Linear(self.hidden_size, packed.shape[0])
+        self.in_proj.bind(packed)
+        # whoever holds the loaded tensors holds these rows from now on, not a second copy
+        at = 0
+        for which, t in zip(("qkv", None, "gate_in", None, "beta", "decay_in"), rows):
+            if which is not None:
+                params[f"{self.name}.{which}"] = packed[at : at + t.shape[0]]
+            at += t.shape[0]
         self.decay_out = a2
-        self.gate_in = Linear(self.hidden_size, g1.shape[0])
-        self.gate_in.bind(g1)
         self.gate_out = Linear(g1.shape[0], self.inner)
         self.gate_out.bind(g2)
         self.conv, self.decay_bias, self.decay_log = get("conv"), get("decay_bias"), get("decay_log")
@@ -139,13 +148,16 @@ class DeltaRule(Mixer):
         )
 
     # ---- step ------------------------------------------------------------------
+    @property
+    def accepts_scaled_rows(self) -> bool:
+        return self.in_proj.takes_scaled_rows()
+
     def forward(self, x, ctx, cache):
         tokens, device = x.shape[0], x.device
-        packed = self.qkv(x)
-        low = self.low.wide(x)
+        packed, low = self.in_proj.split(x, self.split)
         decay = torch.empty((tokens, self.heads * self.d), dtype=torch.float32, device=device)
         ops.gemm_f32(low[:, self.heads :], self.decay_out, decay)
-        gate = self.gate_out(self.gate_in(x))
+        gate = self.gate_out(packed[:, self.gate_col : self.gate_col + self.gate_out.in_features])
         mixed = torch.empty((tokens, self.channels), dtype=torch.float32, device=device)
         ops.delta_prepare(packed, 0, self.conv, cache.states["conv"], decay, self.decay_bias, self.decay_log, mixed, ctx,
                           self.heads, self.kv_heads, self.d, self.dv)

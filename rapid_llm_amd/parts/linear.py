@@ -94,11 +94,18 @@ class Linear:
             ops.add_bias(y, self.bias)
         return y
 
-    def wide(self, x) -> torch.Tensor:
-        """``x W^T`` in float32 as the accumulation leaves it, without the bias."""
-        if self.weight.dtype == torch.float32:
-            return self.product(x, torch.float32)
-        return ops.gemm_bf16_wide(x.rows, self.weight, x) if isinstance(x, ScaledRows) else ops.gemm_bf16_wide(x, self.weight)
+    def split(self, x, split: int) -> tuple[torch.Tensor, torch.Tensor]:
+        """``x W^T`` without the bias in two contiguous parts: the first ``split`` columns in the type of
+        ``x``, the others in float32 as the accumulation leaves them."""
+        w = self.weight
+        if w.dtype == torch.bfloat16:
+            return ops.gemm_bf16_split(x.rows, w, split, x) if isinstance(x, ScaledRows) else ops.gemm_bf16_split(x, w, split)
+        parts = []
+        for rows, dtype in ((w[:split], x.dtype), (w[split:], torch.float32)):
+            part = Linear(self.in_features, rows.shape[0])
+            part.bind(rows)
+            parts.append(part(x, dtype))
+        return parts[0], parts[1]
 
     def product(self, x, out_dtype: torch.dtype | None = None) -> torch.Tensor:
         """``x W^T`` without the bias."""
@@ -112,7 +119,7 @@ class Linear:
         if w.dtype == torch.float32:
             if x.dtype != torch.float32:
                 wide = torch.empty(x.shape, dtype=torch.float32, device=x.device)
-                ops.cast(x, wide)
+                ops.cast(x.contiguous(), wide)
                 x = wide
             y = torch.empty((rows, self.out_features), dtype=torch.float32, device=x.device)
             ops.gemm_f32(x, w, y)

@@ -269,13 +269,20 @@ def test_gelu_gate_with_biases_inside_the_products(rows, width, inter):
     torch.testing.assert_close(got.double().cpu(), pp.gelu_tanh(z[:, :inter]) * z[:, inter:], rtol=2e-2, atol=2e-2)
 
 
-@pytest.mark.parametrize("rows,wide", [(1, 80), (16, 144), (17, 80), (100, 160), (300, 80)])
-def test_product_with_the_float32_result_of_the_accumulation(rows, wide):
+@pytest.mark.parametrize("rows,narrow,wide", [(1, 80, 20), (16, 144, 36), (17, 80, 20), (100, 160, 3), (300, 80, 41), (8, 6272, 144)])
+def test_product_whose_last_columns_stay_float32(rows, narrow, wide):
     ops = _ops()
-    x, w = torch.randn(rows, 256).bfloat16(), torch.randn(wide, 256).bfloat16()
-    got = ops.gemm_bf16_wide(x.to(DEV), w.to(DEV))
-    assert got.dtype == torch.float32
-    torch.testing.assert_close(got.double().cpu(), x.double() @ w.double().T, rtol=1e-5, atol=1e-4)
+    x, w = torch.randn(rows, 256).bfloat16(), torch.randn(narrow + wide, 256).bfloat16()
+    a, b = ops.gemm_bf16_split(x.to(DEV), w.to(DEV), narrow)
+    want = x.double() @ w.double().T
+    assert a.dtype == torch.bfloat16 and b.dtype == torch.float32 and a.is_contiguous() and b.is_contiguous()
+    torch.testing.assert_close(a.double().cpu(), want[:, :narrow], rtol=1e-2, atol=1e-2)
+    torch.testing.assert_close(b.double().cpu(), want[:, narrow:], rtol=1e-5, atol=1e-4)
+    # columns of a wider row as the left operand
+    part = torch.randn(rows, 64 + 40).bfloat16().to(DEV)[:, 40:]
+    v = torch.randn(48, 64).bfloat16().to(DEV)
+    got = ops.gemm_bf16(part, v, torch.bfloat16)
+    torch.testing.assert_close(got.double().cpu(), part.double().cpu() @ v.double().cpu().T, rtol=1e-2, atol=1e-1)
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
