@@ -820,6 +820,7 @@ __global__ __launch_bounds__(SCAN_THREADS) __attribute__((amdgpu_waves_per_eu(1,
 // --------------------------------------------------------------------------- //
 constexpr int GRU_CHANNELS = 8;
 constexpr int GRU_TOKENS = 64;
+constexpr int XCDS = 8;
 constexpr int GRU_WORKERS = 256;                   // threads behind the first wave
 constexpr int GRU_PITCH = GRU_TOKENS + 4;          // a channel's tokens side by side
 
@@ -848,15 +849,20 @@ template <typename T>
 __global__ __launch_bounds__(RL_WAVE + GRU_WORKERS) void gru_scan_kernel(
     const T* __restrict__ packed, int row_width, int z0, int x0, int g0, const float* __restrict__ bz,
     const float* __restrict__ bx, float* __restrict__ S, T* __restrict__ out, int out_width, float scale,
-    const int* __restrict__ cu, const int* __restrict__ seq_slots, int width) {
+    const int* __restrict__ cu, const int* __restrict__ seq_slots, int width, int num_seqs, int channel_blocks) {
     constexpr int PER = GRU_TOKENS * GRU_CHANNELS / GRU_WORKERS;  // elements of a block a worker takes
     constexpr int APART = GRU_WORKERS / GRU_CHANNELS;             // tokens between them
-    const int s = blockIdx.x;
+    // Workgroups go to the chip's XCDs in turn, each with an L2 of its own, and a memory line holds the
+    // channels of several workgroups: neighbouring channels are dealt to the same XCD.
+    const int per_xcd = gridDim.x / XCDS;  // (the launch is a multiple)
+    const int work = (blockIdx.x % XCDS) * per_xcd + blockIdx.x / XCDS;
+    if (work >= num_seqs * channel_blocks) return;  // whole workgroups leave
+    const int s = work / channel_blocks;
     const int t0 = cu[s], t1 = cu[s + 1];
     const bool walks = threadIdx.x < RL_WAVE;
     const int w = walks ? threadIdx.x : threadIdx.x - RL_WAVE;
     const int ch = w % GRU_CHANNELS, tt0 = w / GRU_CHANNELS;
-    const int c = blockIdx.y * GRU_CHANNELS + ch;
+    const int c = (work % channel_blocks) * GRU_CHANNELS + ch;
     const bool live = c < width;
     __shared__ __attribute__((aligned(16))) float keep[2][GRU_CHANNELS][GRU_PITCH], add[2][GRU_CHANNELS][GRU_PITCH],
         sums[2][GRU_CHANNELS][GRU_PITCH];
@@ -864,17 +870,17 @@ __global__ __launch_bounds__(RL_WAVE + GRU_WORKERS) void gru_scan_kernel(
     float* slot = S + (size_t)seq_slots[s] * width + c;
     const bool chain = walks && w < GRU_CHANNELS && live;
     float state = chain ? *slot : 0.f;
-    const T zero = from_float<T>(0.f);
     T pz[PER], px[PER], pg[PER];
+    // (no load stands behind a condition: beyond the portion or the channels a real element is read
+    // and not used)
+    const T* column = packed + min(c, width - 1);
     auto fetch = [&](int block) {
 #pragma unroll
         for (int e = 0; e < PER; ++e) {
-            const int t = t0 + block * GRU_TOKENS + tt0 + e * APART;
-            const bool ok = live && t < t1;
-            const T* row = packed + (size_t)t * row_width + c;
-            pz[e] = ok ? row[z0] : zero;
-            px[e] = ok ? row[x0] : zero;
-            pg[e] = ok ? row[g0] : zero;
+            const T* row = column + (size_t)min(t0 + block * GRU_TOKENS + tt0 + e * APART, t1 - 1) * row_width;
+            pz[e] = row[z0];
+            px[e] = row[x0];
+            pg[e] = row[g0];
         }
     };
     const int blocks = (t1 - t0 + GRU_TOKENS - 1) / GRU_TOKENS;
@@ -888,15 +894,34 @@ __global__ __launch_bounds__(RL_WAVE + GRU_WORKERS) void gru_scan_kernel(
                 const float4* k4 = reinterpret_cast<const float4*>(keep[(i - 1) & 1][ch]);
                 const float4* a4 = reinterpret_cast<const float4*>(add[(i - 1) & 1][ch]);
                 float4* s4 = reinterpret_cast<float4*>(sums[(i - 1) & 1][ch]);
+                // sixteen tokens' factors are asked for while the sixteen before them are walked
+                constexpr int BATCH = 4, BATCHES = GRU_TOKENS / 4 / BATCH;
+                float4 k[2][BATCH], a[2][BATCH];
 #pragma unroll
-                for (int q = 0; q < GRU_TOKENS / 4; ++q) {
-                    const float4 k = k4[q], a = a4[q];
-                    float4 o;
-                    o.x = state = fmaf(k.x, state, a.x);
-                    o.y = state = fmaf(k.y, state, a.y);
-                    o.z = state = fmaf(k.z, state, a.z);
-                    o.w = state = fmaf(k.w, state, a.w);
-                    s4[q] = o;
+                for (int q = 0; q < BATCH; ++q) {
+                    k[0][q] = k4[q];
+                    a[0][q] = a4[q];
+                }
+#pragma unroll
+                for (int n = 0; n < BATCHES; ++n) {
+                    if (n + 1 < BATCHES) {
+#pragma unroll
+                        for (int q = 0; q < BATCH; ++q) {
+                            k[(n + 1) & 1][q] = k4[(n + 1) * BATCH + q];
+                            a[(n + 1) & 1][q] = a4[(n + 1) * BATCH + q];
+                        }
+                    }
+                    __builtin_amdgcn_sched_barrier(0);  // the reads stay in front of the chain
+#pragma unroll
+                    for (int q = 0; q < BATCH; ++q) {
+                        const float4 kk = k[n & 1][q], aa = a[n & 1][q];
+                        float4 o;
+                        o.x = state = fmaf(kk.x, state, aa.x);
+                        o.y = state = fmaf(kk.y, state, aa.y);
+                        o.z = state = fmaf(kk.z, state, aa.z);
+                        o.w = state = fmaf(kk.w, state, aa.w);
+                        s4[n * BATCH + q] = o;
+                    }
                 }
             }
         } else {
@@ -905,18 +930,24 @@ __global__ __launch_bounds__(RL_WAVE + GRU_WORKERS) void gru_scan_kernel(
                 gate2[e] = gate1[e];
                 gate1[e] = gate[e];
             }
-            if (i < blocks) {
+            float zs[PER], xs[PER], gs[PER];
 #pragma unroll
-                for (int e = 0; e < PER; ++e) {
-                    const int tt = tt0 + e * APART;
-                    float k = 1.f, a = 0.f;  // tokens beyond the portion leave the state as it is
-                    if (t0 + i * GRU_TOKENS + tt < t1) gru_factors<T>(to_float(pz[e]) + zb, to_float(px[e]) + xb, k, a);
-                    keep[i & 1][ch][tt] = k;
-                    add[i & 1][ch][tt] = a;
-                    const float z = to_float(pg[e]);
-                    gate[e] = scale * z * sigmoid_of<T>(z);
-                }
-                if (i + 1 < blocks) fetch(i + 1);
+            for (int e = 0; e < PER; ++e) {
+                zs[e] = to_float(pz[e]) + zb;
+                xs[e] = to_float(px[e]) + xb;
+                gs[e] = to_float(pg[e]);
+            }
+            fetch(i + 1);
+            __builtin_amdgcn_sched_barrier(0);  // the next block travels while this one is computed
+#pragma unroll
+            for (int e = 0; e < PER; ++e) {
+                const int tt = tt0 + e * APART;
+                float k, a;
+                gru_factors<T>(zs[e], xs[e], k, a);
+                const bool ok = t0 + i * GRU_TOKENS + tt < t1;  // beyond the portion the state stays as it is
+                keep[i & 1][ch][tt] = ok ? k : 1.f;
+                add[i & 1][ch][tt] = ok ? a : 0.f;
+                gate[e] = scale * gs[e] * sigmoid_of<T>(gs[e]);
             }
             if (i >= 2) {
 #pragma unroll
@@ -1234,11 +1265,14 @@ static int launch_gru(const T* packed, int row_width, int z0, int x0, int g0, co
     if (tokens == num_seqs)  // every request brings one token
         hipLaunchKernelGGL(recurrent::gru_single_kernel<T>, dim3(tokens, (width + 255) / 256), dim3(256), 0, stream,
                            packed, row_width, z0, x0, g0, bz, bx, S, out, out_width, scale, seq_slots, width);
-    else
-        hipLaunchKernelGGL(recurrent::gru_scan_kernel<T>,
-                           dim3(num_seqs, (width + recurrent::GRU_CHANNELS - 1) / recurrent::GRU_CHANNELS),
-                           dim3(RL_WAVE + recurrent::GRU_WORKERS), 0, stream, packed, row_width, z0, x0, g0, bz, bx, S, out, out_width, scale, cu, seq_slots,
-                           width);
+    else {
+        const int blocks = (width + recurrent::GRU_CHANNELS - 1) / recurrent::GRU_CHANNELS;
+        const long groups = ((long)num_seqs * blocks + recurrent::XCDS - 1) / recurrent::XCDS * recurrent::XCDS;
+        if (groups > 0x7fffffffL) return RL_ERR_ARG;
+        hipLaunchKernelGGL(recurrent::gru_scan_kernel<T>, dim3((unsigned)groups),
+                           dim3(RL_WAVE + recurrent::GRU_WORKERS), 0, stream, packed, row_width, z0, x0, g0, bz, bx, S,
+                           out, out_width, scale, cu, seq_slots, width, num_seqs, blocks);
+    }
     return rl_launch_status();
 }
 
