@@ -156,6 +156,33 @@ __device__ inline void row16_sums(float (&v)[N]) {
     for (int i = 0; i < N; ++i) v[i] = ror_add<0x121>(v[i]);
 }
 
+// lane + 16's and lane's value, summed in both (every even row of 16 lanes with the odd one behind it)
+__device__ inline float both_rows(float v) {
+    const unsigned u = __float_as_uint(v);
+    const auto a = __builtin_amdgcn_permlane16_swap(u, u, false, false);
+    return __uint_as_float(a[0]) + __uint_as_float(a[1]);
+}
+// the sum over the 16 or 32 lanes of a column, in every one of them
+template <int LPC>
+__device__ inline float column_sum(float v) {
+    v = row16_sum(v);
+    if constexpr (LPC == 32) v = both_rows(v);
+    return v;
+}
+
+// a block's sixteen sums over the lanes of a column: lane c (of 16 or 32) returns token c % 16's
+template <int LPC>
+__device__ inline float block_sums(float (&os)[16], int c) {
+    row16_sums(os);
+    // every lane of a row of sixteen holds that row's sums of all tokens: lane c takes token c's,
+    // and where a column is two rows of lanes adds the other row's
+    float mine = os[0];
+#pragma unroll
+    for (int tt = 1; tt < 16; ++tt) mine = (c & 15) == tt ? os[tt] : mine;
+    if constexpr (LPC == 32) mine = both_rows(mine);
+    return mine;
+}
+
 // A lane's RPL consecutive state rows from or to memory: sixteen bytes at a time where the rows
 // of a column are a multiple of four (a group of four is then wholly inside the column or wholly
 // beyond it), else one by one.
@@ -195,8 +222,23 @@ __device__ inline void state_rows_store(float* __restrict__ column, int first, i
         if (first + ii < rows) column[first + ii] = state[ii];
 }
 
+// Rows i .. i + 3 of a head of `size` rows: one access where WHOLE (every head starts at a multiple of
+// four elements and has a multiple of four rows), else one by one; a row beyond the head is a real
+// one that is not used.
+template <bool WHOLE, typename T>
+__device__ inline Quad<T> load_quad(const T* __restrict__ head, int i, int size) {
+    if constexpr (WHOLE) return *reinterpret_cast<const Quad<T>*>(head + min(i, size - 4));
+    Quad<T> q;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) q.v[e] = head[min(i + e, size - 1)];
+    return q;
+}
+
 constexpr int SCAN_TOKENS = 16;   // tokens staged at a time
 constexpr int SCAN_WAVES = 4;                      // waves of a workgroup
+// tokens whose operands are read from LDS together, while as many before them are computed (two sets
+// of registers: fewer tokens the more rows a lane holds)
+constexpr int scan_ahead(int rows) { return rows <= 4 ? 4 : (rows <= 8 ? 2 : 1); }
 constexpr int SCAN_THREADS = 64 * SCAN_WAVES;
 constexpr int SCAN_COLS = 4 * SCAN_WAVES;          // columns of a workgroup: 4 a wave
 
@@ -214,26 +256,36 @@ __device__ inline void wkv_row(float r, float k, float w, float u, float vj, flo
     o = fmaf(r, fmaf(u, kv, state), o);
     state = fmaf(w, state, kv);
 }
-__device__ inline float wkv_decay(float pre, float bias) { return expf(-expf(pre + bias)); }
+// the decay exp(-exp(pre + bias)): the library's exponentials in a float32 engine, the hardware's (of base
+// 2, in float32) in a bfloat16 one
+template <typename T>
+__device__ inline float wkv_decay(float pre, float bias) {
+    if constexpr (sizeof(T) == 4) return expf(-expf(pre + bias));
+    constexpr float log2e = 1.4426950408889634f;
+    return __builtin_amdgcn_exp2f(-log2e * __builtin_amdgcn_exp2f(log2e * (pre + bias)));
+}
 
-template <typename T, int RPL>
+template <typename T, int LPC, int RPL, bool WHOLE>
 __global__ __launch_bounds__(SCAN_THREADS) __attribute__((amdgpu_waves_per_eu(1, 2))) void wkv_scan_kernel(
     const T* __restrict__ r, const T* __restrict__ k, const T* __restrict__ v, const float* __restrict__ decay_pre,
     const float* __restrict__ decay_bias, const float* __restrict__ bonus, float* __restrict__ raw,
     const int* __restrict__ cu,
     const int* __restrict__ seq_slots, float* __restrict__ S, int heads, int d) {
-    constexpr int DP = 16 * RPL;  // rows, padded
-    constexpr int PER_THREAD = SCAN_TOKENS * DP / SCAN_THREADS;  // = RPL
+    constexpr int DP = LPC * RPL;  // rows, padded
+    constexpr int QUADS = SCAN_TOKENS * DP / 4;  // of a block, four rows of a token each
+    constexpr int PER_THREAD = (QUADS + SCAN_THREADS - 1) / SCAN_THREADS;
+    constexpr int CPW = RL_WAVE / LPC;      // columns of a wave
+    constexpr int COLS = CPW * SCAN_WAVES;  // and of a workgroup
     const int s = blockIdx.x, h = blockIdx.y;
     const int t0 = cu[s], t1 = cu[s + 1];
     const int inner = heads * d;
     const int lane = threadIdx.x & (RL_WAVE - 1), wave = threadIdx.x / RL_WAVE;
-    const int c = lane & 15;                                  // which share of the rows
-    const int col = wave * 4 + (lane >> 4);                   // column of the workgroup
-    const int j = blockIdx.z * SCAN_COLS + col;
+    const int c = lane & (LPC - 1);                           // which share of the rows
+    const int col = wave * CPW + lane / LPC;                  // column of the workgroup
+    const int j = blockIdx.z * COLS + col;
     const bool live = j < d;
     __shared__ __attribute__((aligned(16))) float sr[SCAN_TOKENS][DP], sk[SCAN_TOKENS][DP], sw[SCAN_TOKENS][DP];
-    __shared__ float sv[SCAN_TOKENS][SCAN_COLS];
+    __shared__ float sv[SCAN_TOKENS][COLS];
     float* Sp = S + (((size_t)seq_slots[s] * heads + h) * d + (live ? j : 0)) * d;
     float state[RPL], u[RPL];
     state_rows_load<RPL>(Sp, c * RPL, d, live, state);
@@ -242,42 +294,98 @@ __global__ __launch_bounds__(SCAN_THREADS) __attribute__((amdgpu_waves_per_eu(1,
         const int i = c * RPL + ii;
         u[ii] = i < d ? bonus[h * d + i] : 0.f;
     }
-    // A block of tokens from memory into registers, as it lies there: element e of the block's
+    // a token's operands from LDS, and this lane's rows' share of its output
+    struct Operands {
+        float r[RPL], k[RPL], w[RPL], v;
+    };
+    auto read = [&](int tt, Operands& x) {
+#pragma unroll
+        for (int ii = 0; ii < RPL; ++ii) {
+            x.r[ii] = sr[tt][c * RPL + ii];
+            x.k[ii] = sk[tt][c * RPL + ii];
+            x.w[ii] = sw[tt][c * RPL + ii];
+        }
+        x.v = sv[tt][col];
+    };
+    auto token = [&](const Operands& x) -> float {
+        float o = 0.f;
+#pragma unroll
+        for (int ii = 0; ii < RPL; ++ii) wkv_row(x.r[ii], x.k[ii], x.w[ii], u[ii], x.v, state[ii], o);
+        return o;
+    };
+    if (t1 - t0 == 1) {
+        // a single token: nothing to stage but itself
+        const int i = threadIdx.x;
+        const size_t at = (size_t)t0 * inner + h * d + i;
+        if (i < DP) {
+            sr[0][i] = i < d ? to_float(r[at]) : 0.f;
+            sk[0][i] = i < d ? to_float(k[at]) : 0.f;
+            sw[0][i] = i < d ? wkv_decay<T>(decay_pre[at], decay_bias[h * d + i]) : 0.f;
+        }
+        const int jj = blockIdx.z * COLS + i;
+        if (i < COLS) sv[0][i] = jj < d ? to_float(v[(size_t)t0 * inner + h * d + jj]) : 0.f;
+        __syncthreads();
+        Operands x;
+        read(0, x);
+        const float o = column_sum<LPC>(token(x));
+        if (c == 0 && live) raw[(size_t)t0 * inner + h * d + j] = o;
+        state_rows_store<RPL>(Sp, c * RPL, d, live, state);
+        return;
+    }
+    // A block of tokens from memory into registers, as it lies there: quad e of the block's
     // [token][row] arrays.  Nothing is computed from what was asked for until the block is staged
     // (a conversion or an exponential here would wait for the loads where they are issued, and
-    // the block before would be computed behind that wait instead of during it).
-    T pr[PER_THREAD], pk[PER_THREAD], pv;
-    float pw[PER_THREAD], pb[PER_THREAD];
+    // the block before would be computed behind that wait instead of during it), and no load stands
+    // behind a condition: beyond the portion or the head a real element is read and not used.
+    Quad<T> pr[PER_THREAD], pk[PER_THREAD];
+    Quad<float> pw[PER_THREAD], pb[PER_THREAD];
+    T pv;
+    auto quad_of = [&](int e, int& tt, int& i) {
+        const int idx = min(e * SCAN_THREADS + (int)threadIdx.x, QUADS - 1);
+        tt = idx / (DP / 4);
+        i = 4 * (idx % (DP / 4));
+    };
 #pragma unroll
     for (int e = 0; e < PER_THREAD; ++e) {
-        const int i = (e * SCAN_THREADS + threadIdx.x) % DP;
-        pb[e] = i < d ? decay_bias[h * d + i] : 0.f;
+        int tt, i;
+        quad_of(e, tt, i);
+        pb[e] = load_quad<WHOLE>(decay_bias + h * d, i, d);
     }
-    const T zero = from_float<T>(0.f);
     auto fetch = [&](int tb) {
 #pragma unroll
         for (int e = 0; e < PER_THREAD; ++e) {
-            const int idx = e * SCAN_THREADS + threadIdx.x;
-            const int tt = idx / DP, i = idx % DP;
-            const bool ok = tb + tt < t1 && i < d;
-            const size_t at = (size_t)(tb + tt) * inner + h * d + i;
-            pr[e] = ok ? r[at] : zero;
-            pk[e] = ok ? k[at] : zero;
-            pw[e] = ok ? decay_pre[at] : INFINITY;  // a decay of exactly 0
+            int tt, i;
+            quad_of(e, tt, i);
+            const size_t row = (size_t)min(tb + tt, t1 - 1) * inner + h * d;
+            pr[e] = load_quad<WHOLE>(r + row, i, d);
+            pk[e] = load_quad<WHOLE>(k + row, i, d);
+            pw[e] = load_quad<WHOLE>(decay_pre + row, i, d);
         }
         // (threads beyond tokens x columns, where a workgroup has more, carry nothing)
-        const int tt = threadIdx.x / SCAN_COLS, jj = blockIdx.z * SCAN_COLS + threadIdx.x % SCAN_COLS;
-        pv = (tt < SCAN_TOKENS && tb + tt < t1 && jj < d) ? v[(size_t)(tb + tt) * inner + h * d + jj] : zero;
+        const int tt = min((int)threadIdx.x / COLS, SCAN_TOKENS - 1), jj = blockIdx.z * COLS + threadIdx.x % COLS;
+        pv = v[(size_t)min(tb + tt, t1 - 1) * inner + h * d + min(jj, d - 1)];
     };
     auto stage = [&]() {
 #pragma unroll
         for (int e = 0; e < PER_THREAD; ++e) {
-            const int idx = e * SCAN_THREADS + threadIdx.x;
-            (&sr[0][0])[idx] = to_float(pr[e]);
-            (&sk[0][0])[idx] = to_float(pk[e]);
-            (&sw[0][0])[idx] = wkv_decay(pw[e], pb[e]);
+            int tt, i;
+            quad_of(e, tt, i);
+            float4 rq, kq, wq;
+            float* ro = &rq.x;
+            float* ko = &kq.x;
+            float* wo = &wq.x;
+#pragma unroll
+            for (int q = 0; q < 4; ++q) {
+                const bool live_row = i + q < d;
+                ro[q] = live_row ? to_float(pr[e].v[q]) : 0.f;
+                ko[q] = live_row ? to_float(pk[e].v[q]) : 0.f;
+                wo[q] = wkv_decay<T>(pw[e].v[q], pb[e].v[q]);
+            }
+            *reinterpret_cast<float4*>(&sr[tt][i]) = rq;
+            *reinterpret_cast<float4*>(&sk[tt][i]) = kq;
+            *reinterpret_cast<float4*>(&sw[tt][i]) = wq;
         }
-        if (threadIdx.x < SCAN_TOKENS * SCAN_COLS) (&sv[0][0])[threadIdx.x] = to_float(pv);
+        if (threadIdx.x < SCAN_TOKENS * COLS) (&sv[0][0])[threadIdx.x] = to_float(pv);
     };
     fetch(t0);
     for (int tb = t0; tb < t1; tb += SCAN_TOKENS) {
@@ -286,32 +394,35 @@ __global__ __launch_bounds__(SCAN_THREADS) __attribute__((amdgpu_waves_per_eu(1,
         __syncthreads();
         if (tb + SCAN_TOKENS < t1) fetch(tb + SCAN_TOKENS);
         const int nt = min(SCAN_TOKENS, t1 - tb);
-        auto token = [&](int tt) -> float {  // this lane's rows' share of the token's output
-            const float vj = sv[tt][col];
-            float o = 0.f;
-#pragma unroll
-            for (int ii = 0; ii < RPL; ++ii)
-                wkv_row(sr[tt][c * RPL + ii], sk[tt][c * RPL + ii], sw[tt][c * RPL + ii], u[ii], vj, state[ii], o);
-            return o;
-        };
         float* dst = raw + (size_t)tb * inner + h * d + j;
         if (nt == SCAN_TOKENS) {
             // a whole block, unrolled and without a branch between its tokens: the reads of later
             // tokens stand in front of the sums of earlier ones, the lane folds of neighbouring
             // tokens interleave, and only the state's own chain orders the tokens; the block's
             // outputs are stored behind it
+            // (operands of the next few tokens are read while these are computed)
+            constexpr int AHEAD = scan_ahead(RPL);
             float os[SCAN_TOKENS];
+            Operands x[2][AHEAD];
 #pragma unroll
-            for (int tt = 0; tt < SCAN_TOKENS; ++tt) os[tt] = token(tt);
-            row16_sums(os);
-            // every lane of a column holds all sixteen sums: lane c stores token c's
-            float mine = os[0];
+            for (int q = 0; q < AHEAD; ++q) read(q, x[0][q]);
 #pragma unroll
-            for (int tt = 1; tt < SCAN_TOKENS; ++tt) mine = c == tt ? os[tt] : mine;
-            if (live) dst[(size_t)c * inner] = mine;
+            for (int n = 0; n < SCAN_TOKENS / AHEAD; ++n) {
+                if (n + 1 < SCAN_TOKENS / AHEAD) {
+#pragma unroll
+                    for (int q = 0; q < AHEAD; ++q) read((n + 1) * AHEAD + q, x[(n + 1) & 1][q]);
+                }
+                __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+                for (int q = 0; q < AHEAD; ++q) os[n * AHEAD + q] = token(x[n & 1][q]);
+            }
+            const float mine = block_sums<LPC>(os, c);
+            if (live && c < SCAN_TOKENS) dst[(size_t)c * inner] = mine;
         } else {
             for (int tt = 0; tt < nt; ++tt) {
-                const float o = row16_sum(token(tt));
+                Operands x;
+                read(tt, x);
+                const float o = column_sum<LPC>(token(x));
                 if (c == 0 && live) dst[(size_t)tt * inner] = o;
             }
         }
@@ -690,33 +801,19 @@ __global__ __launch_bounds__(256) void delta_prepare_kernel(
     }
 }
 
-// lane + 16's and lane's value, summed in both (every even row of 16 lanes with the odd one behind it)
-__device__ inline float both_rows(float v) {
-    const unsigned u = __float_as_uint(v);
-    const auto a = __builtin_amdgcn_permlane16_swap(u, u, false, false);
-    return __uint_as_float(a[0]) + __uint_as_float(a[1]);
-}
-// the sum over the 16 or 32 lanes of a column, in every one of them
-template <int LPC>
-__device__ inline float column_sum(float v) {
-    v = row16_sum(v);
-    if constexpr (LPC == 32) v = both_rows(v);
-    return v;
-}
-
 // The scan.  Per head (head h reads q and k of kv head h / (heads / kv_heads)), state S[key channel i]
 // [value channel j], kept as [j][i]; for a token with q, k, v, the decays g and beta = sigmoid(b):
 //   S_ij <- g_i S_ij      u_j = beta (v_j - sum_i S_ij k_i)      S_ij <- S_ij + k_i u_j      o_j = sum_i S_ij q_i
 // The sum that u needs stands between two tokens and is folded at once; the read-out's sums are folded
-// behind a block of tokens.  o goes out unfinished (float32).  LPC lanes share a column: 16, or 32 where
-// that leaves a lane four rows instead of eight and the workgroups still fill the chip no further.
-template <int LPC, int RPL>
+// behind a block of tokens.  o goes out unfinished (float32).
+template <int LPC, int RPL, bool WHOLE>
 __global__ __launch_bounds__(SCAN_THREADS) __attribute__((amdgpu_waves_per_eu(1, 2))) void delta_scan_kernel(
     const float* __restrict__ mixed, const float* __restrict__ decay, const float* __restrict__ beta_pre,
     int beta_width, float* __restrict__ raw, const int* __restrict__ cu, const int* __restrict__ seq_slots,
     float* __restrict__ S, int heads, int kv_heads, int d, int dv) {
     constexpr int DP = LPC * RPL;  // rows, padded
-    constexpr int PER_THREAD = SCAN_TOKENS * DP / SCAN_THREADS;
+    constexpr int QUADS = SCAN_TOKENS * DP / 4;  // of a block, four rows of a token each
+    constexpr int PER_THREAD = (QUADS + SCAN_THREADS - 1) / SCAN_THREADS;
     constexpr int CPW = RL_WAVE / LPC;       // columns of a wave
     constexpr int COLS = CPW * SCAN_WAVES;   // and of a workgroup
     const int s = blockIdx.x, h = blockIdx.y;
@@ -733,31 +830,95 @@ __global__ __launch_bounds__(SCAN_THREADS) __attribute__((amdgpu_waves_per_eu(1,
     float* Sp = S + (((size_t)seq_slots[s] * heads + h) * dv + (live ? j : 0)) * d;
     float state[RPL];
     state_rows_load<RPL>(Sp, c * RPL, d, live, state);
-    float pq[PER_THREAD], pk[PER_THREAD], pg[PER_THREAD], pv = 0.f, pb = 0.f;
+    // a token's operands from LDS, and this lane's rows' share of its output
+    struct Operands {
+        float q[RPL], k[RPL], g[RPL], v, beta;
+    };
+    auto read = [&](int tt, Operands& x) {
+#pragma unroll
+        for (int ii = 0; ii < RPL; ++ii) {
+            x.q[ii] = sq[tt][c * RPL + ii];
+            x.k[ii] = sk[tt][c * RPL + ii];
+            x.g[ii] = sg[tt][c * RPL + ii];
+        }
+        x.v = sv[tt][col];
+        x.beta = sb[tt];
+    };
+    auto token = [&](const Operands& x) -> float {
+        float even = 0.f, odd = 0.f;
+#pragma unroll
+        for (int ii = 0; ii < RPL; ++ii) {
+            state[ii] *= x.g[ii];
+            float& sum = (ii & 1) ? odd : even;
+            sum = fmaf(state[ii], x.k[ii], sum);
+        }
+        const float u = x.beta * (x.v - column_sum<LPC>(even + odd));
+        float o = 0.f;
+#pragma unroll
+        for (int ii = 0; ii < RPL; ++ii) {
+            state[ii] = fmaf(x.k[ii], u, state[ii]);
+            o = fmaf(state[ii], x.q[ii], o);
+        }
+        return o;
+    };
+    if (t1 - t0 == 1) {
+        // a single token: nothing to stage but itself
+        const int i = threadIdx.x;
+        const float* row = mixed + (size_t)t0 * channels;
+        if (i < DP) {
+            sq[0][i] = i < d ? row[hk * d + i] : 0.f;
+            sk[0][i] = i < d ? row[(kv_heads + hk) * d + i] : 0.f;
+            sg[0][i] = i < d ? decay[(size_t)t0 * heads * d + h * d + i] : 0.f;
+        }
+        const int jj = blockIdx.z * COLS + i;
+        if (i < COLS) sv[0][i] = jj < dv ? row[2 * kv_heads * d + h * dv + jj] : 0.f;
+        if (i == 0) sb[0] = 1.f / (1.f + expf(-beta_pre[(size_t)t0 * beta_width + h]));
+        __syncthreads();
+        Operands x;
+        read(0, x);
+        const float o = column_sum<LPC>(token(x));
+        if (c == 0 && live) raw[(size_t)t0 * heads * dv + h * dv + j] = o;
+        state_rows_store<RPL>(Sp, c * RPL, d, live, state);
+        return;
+    }
+    // a block of tokens from memory into registers, as the time mixing's
+    Quad<float> pq[PER_THREAD], pk[PER_THREAD], pg[PER_THREAD];
+    float pv, pb;
+    auto quad_of = [&](int e, int& tt, int& i) {
+        const int idx = min(e * SCAN_THREADS + (int)threadIdx.x, QUADS - 1);
+        tt = idx / (DP / 4);
+        i = 4 * (idx % (DP / 4));
+    };
     auto fetch = [&](int tb) {
 #pragma unroll
         for (int e = 0; e < PER_THREAD; ++e) {
-            const int idx = e * SCAN_THREADS + threadIdx.x;
-            const int tt = idx / DP, i = idx % DP;
-            const bool ok = tb + tt < t1 && i < d;
-            const float* row = mixed + (size_t)(tb + tt) * channels + hk * d + i;
-            pq[e] = ok ? row[0] : 0.f;
-            pk[e] = ok ? row[kv_heads * d] : 0.f;
-            pg[e] = ok ? decay[(size_t)(tb + tt) * heads * d + h * d + i] : 0.f;
+            int tt, i;
+            quad_of(e, tt, i);
+            const size_t t = min(tb + tt, t1 - 1);
+            pq[e] = load_quad<WHOLE>(mixed + t * channels + hk * d, i, d);
+            pk[e] = load_quad<WHOLE>(mixed + t * channels + (kv_heads + hk) * d, i, d);
+            pg[e] = load_quad<WHOLE>(decay + (t * heads + h) * d, i, d);
         }
-        const int tt = threadIdx.x / COLS, jj = blockIdx.z * COLS + threadIdx.x % COLS;
-        const bool ok = tt < SCAN_TOKENS && tb + tt < t1;
-        pv = (ok && jj < dv) ? mixed[(size_t)(tb + tt) * channels + 2 * kv_heads * d + h * dv + jj] : 0.f;
-        const int tk = threadIdx.x;
-        pb = (tk < SCAN_TOKENS && tb + tk < t1) ? beta_pre[(size_t)(tb + tk) * beta_width + h] : 0.f;
+        const int tt = min((int)threadIdx.x / COLS, SCAN_TOKENS - 1), jj = blockIdx.z * COLS + threadIdx.x % COLS;
+        pv = mixed[(size_t)min(tb + tt, t1 - 1) * channels + 2 * kv_heads * d + h * dv + min(jj, dv - 1)];
+        pb = beta_pre[(size_t)min(tb + ((int)threadIdx.x & (SCAN_TOKENS - 1)), t1 - 1) * beta_width + h];
     };
     auto stage = [&]() {
 #pragma unroll
         for (int e = 0; e < PER_THREAD; ++e) {
-            const int idx = e * SCAN_THREADS + threadIdx.x;
-            (&sq[0][0])[idx] = pq[e];
-            (&sk[0][0])[idx] = pk[e];
-            (&sg[0][0])[idx] = pg[e];
+            int tt, i;
+            quad_of(e, tt, i);
+            float4 qq, kq;
+            float* qo = &qq.x;
+            float* ko = &kq.x;
+#pragma unroll
+            for (int q = 0; q < 4; ++q) {
+                qo[q] = i + q < d ? pq[e].v[q] : 0.f;
+                ko[q] = i + q < d ? pk[e].v[q] : 0.f;
+            }
+            *reinterpret_cast<float4*>(&sq[tt][i]) = qq;
+            *reinterpret_cast<float4*>(&sk[tt][i]) = kq;
+            *reinterpret_cast<Quad<float>*>(&sg[tt][i]) = pg[e];
         }
         if (threadIdx.x < SCAN_TOKENS * COLS) (&sv[0][0])[threadIdx.x] = pv;
         if (threadIdx.x < SCAN_TOKENS) sb[threadIdx.x] = 1.f / (1.f + expf(-pb));
@@ -769,39 +930,30 @@ __global__ __launch_bounds__(SCAN_THREADS) __attribute__((amdgpu_waves_per_eu(1,
         __syncthreads();
         if (tb + SCAN_TOKENS < t1) fetch(tb + SCAN_TOKENS);
         const int nt = min(SCAN_TOKENS, t1 - tb);
-        auto token = [&](int tt) -> float {  // this lane's rows' share of the token's output
-            float even = 0.f, odd = 0.f;
-#pragma unroll
-            for (int ii = 0; ii < RPL; ++ii) {
-                state[ii] *= sg[tt][c * RPL + ii];
-                float& sum = (ii & 1) ? odd : even;
-                sum = fmaf(state[ii], sk[tt][c * RPL + ii], sum);
-            }
-            const float u = sb[tt] * (sv[tt][col] - column_sum<LPC>(even + odd));
-            float o = 0.f;
-#pragma unroll
-            for (int ii = 0; ii < RPL; ++ii) {
-                state[ii] = fmaf(sk[tt][c * RPL + ii], u, state[ii]);
-                o = fmaf(state[ii], sq[tt][c * RPL + ii], o);
-            }
-            return o;
-        };
         float* dst = raw + (size_t)tb * heads * dv + h * dv + j;
         if (nt == SCAN_TOKENS) {
+            constexpr int AHEAD = scan_ahead(RPL);
             float os[SCAN_TOKENS];
+            Operands x[2][AHEAD];
 #pragma unroll
-            for (int tt = 0; tt < SCAN_TOKENS; ++tt) os[tt] = token(tt);
-            row16_sums(os);
-            // every lane of a row of sixteen holds that row's sums of all tokens: lane c takes
-            // token c's, and where a column is two rows of lanes adds the other row's
-            float mine = os[0];
+            for (int q = 0; q < AHEAD; ++q) read(q, x[0][q]);
 #pragma unroll
-            for (int tt = 1; tt < SCAN_TOKENS; ++tt) mine = (c & 15) == tt ? os[tt] : mine;
-            if constexpr (LPC == 32) mine = both_rows(mine);
+            for (int n = 0; n < SCAN_TOKENS / AHEAD; ++n) {
+                if (n + 1 < SCAN_TOKENS / AHEAD) {
+#pragma unroll
+                    for (int q = 0; q < AHEAD; ++q) read((n + 1) * AHEAD + q, x[(n + 1) & 1][q]);
+                }
+                __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+                for (int q = 0; q < AHEAD; ++q) os[n * AHEAD + q] = token(x[n & 1][q]);
+            }
+            const float mine = block_sums<LPC>(os, c);
             if (live && c < SCAN_TOKENS) dst[(size_t)c * heads * dv] = mine;
         } else {
             for (int tt = 0; tt < nt; ++tt) {
-                const float o = column_sum<LPC>(token(tt));
+                Operands x;
+                read(tt, x);
+                const float o = column_sum<LPC>(token(x));
                 if (c == 0 && live) dst[(size_t)tt * heads * dv] = o;
             }
         }
@@ -1018,22 +1170,41 @@ static int launch_wkv(const T* r, const T* k, const T* v, const T* g, const floa
                       const float* bonus, const float* norm_w, T* out, float* raw, const int* cu,
                       const int* seq_slots, float* S, int num_seqs, int tokens, int heads, int d, float eps,
                       hipStream_t stream) {
-    dim3 grid(num_seqs, heads, (d + recurrent::SCAN_COLS - 1) / recurrent::SCAN_COLS);
-#define RL_WKV(RPL)                                                                                              \
-    hipLaunchKernelGGL((recurrent::wkv_scan_kernel<T, RPL>), grid, dim3(recurrent::SCAN_THREADS), 0, stream, r, k, v, \
-                       decay, decay_bias, bonus, raw, cu, seq_slots, S, heads, d)
-    const int rows = (d + 15) / 16;
-    if (rows <= 1)
-        RL_WKV(1);
-    else if (rows <= 2)
-        RL_WKV(2);
-    else if (rows <= 4)
-        RL_WKV(4);
-    else if (rows <= 8)
-        RL_WKV(8);
+#define RL_WKV_AS(LPC, RPL, WHOLE)                                                                                  \
+    hipLaunchKernelGGL((recurrent::wkv_scan_kernel<T, LPC, RPL, WHOLE>), dim3(num_seqs, heads, (d + cols - 1) / cols), \
+                       dim3(recurrent::SCAN_THREADS), 0, stream, r, k, v, decay, decay_bias, bonus, raw, cu,        \
+                       seq_slots, S, heads, d)
+#define RL_WKV(LPC, RPL)                                           \
+    do {                                                           \
+        constexpr int cols = RL_WAVE / LPC * recurrent::SCAN_WAVES; \
+        if (d % 4 == 0)                                            \
+            RL_WKV_AS(LPC, RPL, true);                             \
+        else                                                       \
+            RL_WKV_AS(LPC, RPL, false);                            \
+    } while (0)
+    // Two rows of lanes a column where one row's workgroups of one request leave half the chip or more
+    // without one.  (A property of the model, not of the step: a token's sums keep one order.)
+    const bool wide = heads * ((d + 15) / 16) <= 128;
+    if (d <= 16)
+        RL_WKV(16, 1);
+    else if (d <= 32)
+        RL_WKV(16, 2);
+    else if (d <= 64) {
+        if (wide)
+            RL_WKV(32, 2);
+        else
+            RL_WKV(16, 4);
+    } else if (d <= 128) {
+        if (wide)
+            RL_WKV(32, 4);
+        else
+            RL_WKV(16, 8);
+    } else if (wide)
+        RL_WKV(32, 8);
     else
-        RL_WKV(16);
+        RL_WKV(16, 16);
 #undef RL_WKV
+#undef RL_WKV_AS
     const int heads_rows = tokens * heads;
     hipLaunchKernelGGL(recurrent::head_finish_kernel<T>, dim3((heads_rows + 3) / 4), dim3(256), 0, stream, raw, g,
                        norm_w, out, heads_rows, heads, d, eps, 0, 0);
@@ -1220,24 +1391,39 @@ extern "C" int rl_delta_scan(const float* mixed, const float* decay, const float
     if (heads < 1 || heads > 65535 || kv_heads < 1 || heads % kv_heads || d < 1 || d > 256 || dv < 1 || dv > 256 ||
         beta_width < heads || num_seqs > 65535)
         return RL_ERR_ARG;
-#define RL_DELTA(LPC, RPL)                                                                                          \
-    do {                                                                                                            \
-        constexpr int cols = RL_WAVE / LPC * recurrent::SCAN_WAVES;                                                 \
-        hipLaunchKernelGGL((recurrent::delta_scan_kernel<LPC, RPL>), dim3(num_seqs, heads, (dv + cols - 1) / cols), \
-                           dim3(recurrent::SCAN_THREADS), 0, stream, mixed, decay, beta_pre, beta_width, raw, cu,   \
-                           seq_slots, S, heads, kv_heads, d, dv);                                                   \
+#define RL_DELTA_AS(LPC, RPL, WHOLE)                                                                                  \
+    hipLaunchKernelGGL((recurrent::delta_scan_kernel<LPC, RPL, WHOLE>), dim3(num_seqs, heads, (dv + cols - 1) / cols), \
+                       dim3(recurrent::SCAN_THREADS), 0, stream, mixed, decay, beta_pre, beta_width, raw, cu,         \
+                       seq_slots, S, heads, kv_heads, d, dv)
+#define RL_DELTA(LPC, RPL)                                         \
+    do {                                                           \
+        constexpr int cols = RL_WAVE / LPC * recurrent::SCAN_WAVES; \
+        if (d % 4 == 0 && dv % 4 == 0)                             \
+            RL_DELTA_AS(LPC, RPL, true);                           \
+        else                                                       \
+            RL_DELTA_AS(LPC, RPL, false);                          \
     } while (0)
+    const bool wide = heads * ((dv + 15) / 16) <= 256;  // as for the time mixing
     if (d <= 16)
         RL_DELTA(16, 1);
     else if (d <= 32)
         RL_DELTA(16, 2);
-    else if (d <= 64)
-        RL_DELTA(16, 4);
-    else if (d <= 128)
-        RL_DELTA(32, 4);
-    else
+    else if (d <= 64) {
+        if (wide)
+            RL_DELTA(32, 2);
+        else
+            RL_DELTA(16, 4);
+    } else if (d <= 128) {
+        if (wide)
+            RL_DELTA(32, 4);
+        else
+            RL_DELTA(16, 8);
+    } else if (wide)
         RL_DELTA(32, 8);
+    else
+        RL_DELTA(16, 16);
 #undef RL_DELTA
+#undef RL_DELTA_AS
     return rl_launch_status();
 }
 
