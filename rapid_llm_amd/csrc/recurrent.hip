@@ -236,6 +236,8 @@ __device__ inline Quad<T> load_quad(const T* __restrict__ head, int i, int size)
 
 constexpr int SCAN_TOKENS = 16;   // tokens staged at a time
 constexpr int SCAN_WAVES = 4;                      // waves of a workgroup
+// blocks of tokens in LDS at a time: two where three operands of so many rows fit 64 KB twice
+constexpr int scan_buffers(int rows) { return rows <= 128 ? 2 : 1; }
 // tokens whose operands are read from LDS together, while as many before them are computed (two sets
 // of registers: fewer tokens the more rows a lane holds)
 constexpr int scan_ahead(int rows) { return rows <= 4 ? 4 : (rows <= 8 ? 2 : 1); }
@@ -272,6 +274,7 @@ __global__ __launch_bounds__(SCAN_THREADS) __attribute__((amdgpu_waves_per_eu(1,
     const int* __restrict__ cu,
     const int* __restrict__ seq_slots, float* __restrict__ S, int heads, int d) {
     constexpr int DP = LPC * RPL;  // rows, padded
+    constexpr int BUFS = scan_buffers(DP);
     constexpr int QUADS = SCAN_TOKENS * DP / 4;  // of a block, four rows of a token each
     constexpr int PER_THREAD = (QUADS + SCAN_THREADS - 1) / SCAN_THREADS;
     constexpr int CPW = RL_WAVE / LPC;      // columns of a wave
@@ -284,8 +287,9 @@ __global__ __launch_bounds__(SCAN_THREADS) __attribute__((amdgpu_waves_per_eu(1,
     const int col = wave * CPW + lane / LPC;                  // column of the workgroup
     const int j = blockIdx.z * COLS + col;
     const bool live = j < d;
-    __shared__ __attribute__((aligned(16))) float sr[SCAN_TOKENS][DP], sk[SCAN_TOKENS][DP], sw[SCAN_TOKENS][DP];
-    __shared__ float sv[SCAN_TOKENS][COLS];
+    __shared__ __attribute__((aligned(16))) float sr[BUFS][SCAN_TOKENS][DP], sk[BUFS][SCAN_TOKENS][DP],
+        sw[BUFS][SCAN_TOKENS][DP];
+    __shared__ float sv[BUFS][SCAN_TOKENS][COLS];
     float* Sp = S + (((size_t)seq_slots[s] * heads + h) * d + (live ? j : 0)) * d;
     float state[RPL], u[RPL];
     state_rows_load<RPL>(Sp, c * RPL, d, live, state);
@@ -298,14 +302,14 @@ __global__ __launch_bounds__(SCAN_THREADS) __attribute__((amdgpu_waves_per_eu(1,
     struct Operands {
         float r[RPL], k[RPL], w[RPL], v;
     };
-    auto read = [&](int tt, Operands& x) {
+    auto read = [&](int buf, int tt, Operands& x) {
 #pragma unroll
         for (int ii = 0; ii < RPL; ++ii) {
-            x.r[ii] = sr[tt][c * RPL + ii];
-            x.k[ii] = sk[tt][c * RPL + ii];
-            x.w[ii] = sw[tt][c * RPL + ii];
+            x.r[ii] = sr[buf][tt][c * RPL + ii];
+            x.k[ii] = sk[buf][tt][c * RPL + ii];
+            x.w[ii] = sw[buf][tt][c * RPL + ii];
         }
-        x.v = sv[tt][col];
+        x.v = sv[buf][tt][col];
     };
     auto token = [&](const Operands& x) -> float {
         float o = 0.f;
@@ -318,15 +322,15 @@ __global__ __launch_bounds__(SCAN_THREADS) __attribute__((amdgpu_waves_per_eu(1,
         const int i = threadIdx.x;
         const size_t at = (size_t)t0 * inner + h * d + i;
         if (i < DP) {
-            sr[0][i] = i < d ? to_float(r[at]) : 0.f;
-            sk[0][i] = i < d ? to_float(k[at]) : 0.f;
-            sw[0][i] = i < d ? wkv_decay<T>(decay_pre[at], decay_bias[h * d + i]) : 0.f;
+            sr[0][0][i] = i < d ? to_float(r[at]) : 0.f;
+            sk[0][0][i] = i < d ? to_float(k[at]) : 0.f;
+            sw[0][0][i] = i < d ? wkv_decay<T>(decay_pre[at], decay_bias[h * d + i]) : 0.f;
         }
         const int jj = blockIdx.z * COLS + i;
-        if (i < COLS) sv[0][i] = jj < d ? to_float(v[(size_t)t0 * inner + h * d + jj]) : 0.f;
+        if (i < COLS) sv[0][0][i] = jj < d ? to_float(v[(size_t)t0 * inner + h * d + jj]) : 0.f;
         __syncthreads();
         Operands x;
-        read(0, x);
+        read(0, 0, x);
         const float o = column_sum<LPC>(token(x));
         if (c == 0 && live) raw[(size_t)t0 * inner + h * d + j] = o;
         state_rows_store<RPL>(Sp, c * RPL, d, live, state);
@@ -365,7 +369,7 @@ __global__ __launch_bounds__(SCAN_THREADS) __attribute__((amdgpu_waves_per_eu(1,
         const int tt = min((int)threadIdx.x / COLS, SCAN_TOKENS - 1), jj = blockIdx.z * COLS + threadIdx.x % COLS;
         pv = v[(size_t)min(tb + tt, t1 - 1) * inner + h * d + min(jj, d - 1)];
     };
-    auto stage = [&]() {
+    auto stage = [&](int buf) {
 #pragma unroll
         for (int e = 0; e < PER_THREAD; ++e) {
             int tt, i;
@@ -381,18 +385,32 @@ __global__ __launch_bounds__(SCAN_THREADS) __attribute__((amdgpu_waves_per_eu(1,
                 ko[q] = live_row ? to_float(pk[e].v[q]) : 0.f;
                 wo[q] = wkv_decay<T>(pw[e].v[q], pb[e].v[q]);
             }
-            *reinterpret_cast<float4*>(&sr[tt][i]) = rq;
-            *reinterpret_cast<float4*>(&sk[tt][i]) = kq;
-            *reinterpret_cast<float4*>(&sw[tt][i]) = wq;
+            *reinterpret_cast<float4*>(&sr[buf][tt][i]) = rq;
+            *reinterpret_cast<float4*>(&sk[buf][tt][i]) = kq;
+            *reinterpret_cast<float4*>(&sw[buf][tt][i]) = wq;
         }
-        if (threadIdx.x < SCAN_TOKENS * COLS) (&sv[0][0])[threadIdx.x] = to_float(pv);
+        if (threadIdx.x < SCAN_TOKENS * COLS) (&sv[buf][0][0])[threadIdx.x] = to_float(pv);
     };
+    // With two buffers in LDS the next block is staged, and the one after it asked for, in front of the
+    // block at hand: one barrier a block.  With one buffer the waves meet before and after staging.
+    // (Beyond the portion real elements are fetched and staged, and not used.)
+    int buf = 0;
     fetch(t0);
-    for (int tb = t0; tb < t1; tb += SCAN_TOKENS) {
-        __syncthreads();  // the block before has been read by every wave
-        stage();
+    if constexpr (BUFS == 2) {
+        stage(0);
+        fetch(t0 + SCAN_TOKENS);
         __syncthreads();
-        if (tb + SCAN_TOKENS < t1) fetch(tb + SCAN_TOKENS);
+    }
+    for (int tb = t0; tb < t1; tb += SCAN_TOKENS) {
+        if constexpr (BUFS == 2) {
+            stage(buf ^ 1);
+            fetch(tb + 2 * SCAN_TOKENS);
+        } else {
+            __syncthreads();  // the block before has been read by every wave
+            stage(0);
+            __syncthreads();
+            fetch(tb + SCAN_TOKENS);
+        }
         const int nt = min(SCAN_TOKENS, t1 - tb);
         float* dst = raw + (size_t)tb * inner + h * d + j;
         if (nt == SCAN_TOKENS) {
@@ -405,12 +423,12 @@ __global__ __launch_bounds__(SCAN_THREADS) __attribute__((amdgpu_waves_per_eu(1,
             float os[SCAN_TOKENS];
             Operands x[2][AHEAD];
 #pragma unroll
-            for (int q = 0; q < AHEAD; ++q) read(q, x[0][q]);
+            for (int q = 0; q < AHEAD; ++q) read(buf, q, x[0][q]);
 #pragma unroll
             for (int n = 0; n < SCAN_TOKENS / AHEAD; ++n) {
                 if (n + 1 < SCAN_TOKENS / AHEAD) {
 #pragma unroll
-                    for (int q = 0; q < AHEAD; ++q) read((n + 1) * AHEAD + q, x[(n + 1) & 1][q]);
+                    for (int q = 0; q < AHEAD; ++q) read(buf, (n + 1) * AHEAD + q, x[(n + 1) & 1][q]);
                 }
                 __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
@@ -421,10 +439,14 @@ __global__ __launch_bounds__(SCAN_THREADS) __attribute__((amdgpu_waves_per_eu(1,
         } else {
             for (int tt = 0; tt < nt; ++tt) {
                 Operands x;
-                read(tt, x);
+                read(buf, tt, x);
                 const float o = column_sum<LPC>(token(x));
                 if (c == 0 && live) dst[(size_t)tt * inner] = o;
             }
+        }
+        if constexpr (BUFS == 2) {
+            buf ^= 1;
+            __syncthreads();  // the next block is staged, and this one has been read
         }
     }
     state_rows_store<RPL>(Sp, c * RPL, d, live, state);
@@ -812,6 +834,7 @@ __global__ __launch_bounds__(SCAN_THREADS) __attribute__((amdgpu_waves_per_eu(1,
     int beta_width, float* __restrict__ raw, const int* __restrict__ cu, const int* __restrict__ seq_slots,
     float* __restrict__ S, int heads, int kv_heads, int d, int dv) {
     constexpr int DP = LPC * RPL;  // rows, padded
+    constexpr int BUFS = scan_buffers(DP);
     constexpr int QUADS = SCAN_TOKENS * DP / 4;  // of a block, four rows of a token each
     constexpr int PER_THREAD = (QUADS + SCAN_THREADS - 1) / SCAN_THREADS;
     constexpr int CPW = RL_WAVE / LPC;       // columns of a wave
@@ -825,8 +848,9 @@ __global__ __launch_bounds__(SCAN_THREADS) __attribute__((amdgpu_waves_per_eu(1,
     const int col = wave * CPW + lane / LPC;
     const int j = blockIdx.z * COLS + col;
     const bool live = j < dv;
-    __shared__ __attribute__((aligned(16))) float sq[SCAN_TOKENS][DP], sk[SCAN_TOKENS][DP], sg[SCAN_TOKENS][DP];
-    __shared__ float sv[SCAN_TOKENS][COLS], sb[SCAN_TOKENS];
+    __shared__ __attribute__((aligned(16))) float sq[BUFS][SCAN_TOKENS][DP], sk[BUFS][SCAN_TOKENS][DP],
+        sg[BUFS][SCAN_TOKENS][DP];
+    __shared__ float sv[BUFS][SCAN_TOKENS][COLS], sb[BUFS][SCAN_TOKENS];
     float* Sp = S + (((size_t)seq_slots[s] * heads + h) * dv + (live ? j : 0)) * d;
     float state[RPL];
     state_rows_load<RPL>(Sp, c * RPL, d, live, state);
@@ -834,15 +858,15 @@ __global__ __launch_bounds__(SCAN_THREADS) __attribute__((amdgpu_waves_per_eu(1,
     struct Operands {
         float q[RPL], k[RPL], g[RPL], v, beta;
     };
-    auto read = [&](int tt, Operands& x) {
+    auto read = [&](int buf, int tt, Operands& x) {
 #pragma unroll
         for (int ii = 0; ii < RPL; ++ii) {
-            x.q[ii] = sq[tt][c * RPL + ii];
-            x.k[ii] = sk[tt][c * RPL + ii];
-            x.g[ii] = sg[tt][c * RPL + ii];
+            x.q[ii] = sq[buf][tt][c * RPL + ii];
+            x.k[ii] = sk[buf][tt][c * RPL + ii];
+            x.g[ii] = sg[buf][tt][c * RPL + ii];
         }
-        x.v = sv[tt][col];
-        x.beta = sb[tt];
+        x.v = sv[buf][tt][col];
+        x.beta = sb[buf][tt];
     };
     auto token = [&](const Operands& x) -> float {
         float even = 0.f, odd = 0.f;
@@ -866,16 +890,16 @@ __global__ __launch_bounds__(SCAN_THREADS) __attribute__((amdgpu_waves_per_eu(1,
         const int i = threadIdx.x;
         const float* row = mixed + (size_t)t0 * channels;
         if (i < DP) {
-            sq[0][i] = i < d ? row[hk * d + i] : 0.f;
-            sk[0][i] = i < d ? row[(kv_heads + hk) * d + i] : 0.f;
-            sg[0][i] = i < d ? decay[(size_t)t0 * heads * d + h * d + i] : 0.f;
+            sq[0][0][i] = i < d ? row[hk * d + i] : 0.f;
+            sk[0][0][i] = i < d ? row[(kv_heads + hk) * d + i] : 0.f;
+            sg[0][0][i] = i < d ? decay[(size_t)t0 * heads * d + h * d + i] : 0.f;
         }
         const int jj = blockIdx.z * COLS + i;
-        if (i < COLS) sv[0][i] = jj < dv ? row[2 * kv_heads * d + h * dv + jj] : 0.f;
-        if (i == 0) sb[0] = 1.f / (1.f + expf(-beta_pre[(size_t)t0 * beta_width + h]));
+        if (i < COLS) sv[0][0][i] = jj < dv ? row[2 * kv_heads * d + h * dv + jj] : 0.f;
+        if (i == 0) sb[0][0] = 1.f / (1.f + expf(-beta_pre[(size_t)t0 * beta_width + h]));
         __syncthreads();
         Operands x;
-        read(0, x);
+        read(0, 0, x);
         const float o = column_sum<LPC>(token(x));
         if (c == 0 && live) raw[(size_t)t0 * heads * dv + h * dv + j] = o;
         state_rows_store<RPL>(Sp, c * RPL, d, live, state);
@@ -903,7 +927,7 @@ __global__ __launch_bounds__(SCAN_THREADS) __attribute__((amdgpu_waves_per_eu(1,
         pv = mixed[(size_t)min(tb + tt, t1 - 1) * channels + 2 * kv_heads * d + h * dv + min(jj, dv - 1)];
         pb = beta_pre[(size_t)min(tb + ((int)threadIdx.x & (SCAN_TOKENS - 1)), t1 - 1) * beta_width + h];
     };
-    auto stage = [&]() {
+    auto stage = [&](int buf) {
 #pragma unroll
         for (int e = 0; e < PER_THREAD; ++e) {
             int tt, i;
@@ -916,19 +940,33 @@ __global__ __launch_bounds__(SCAN_THREADS) __attribute__((amdgpu_waves_per_eu(1,
                 qo[q] = i + q < d ? pq[e].v[q] : 0.f;
                 ko[q] = i + q < d ? pk[e].v[q] : 0.f;
             }
-            *reinterpret_cast<float4*>(&sq[tt][i]) = qq;
-            *reinterpret_cast<float4*>(&sk[tt][i]) = kq;
-            *reinterpret_cast<Quad<float>*>(&sg[tt][i]) = pg[e];
+            *reinterpret_cast<float4*>(&sq[buf][tt][i]) = qq;
+            *reinterpret_cast<float4*>(&sk[buf][tt][i]) = kq;
+            *reinterpret_cast<Quad<float>*>(&sg[buf][tt][i]) = pg[e];
         }
-        if (threadIdx.x < SCAN_TOKENS * COLS) (&sv[0][0])[threadIdx.x] = pv;
-        if (threadIdx.x < SCAN_TOKENS) sb[threadIdx.x] = 1.f / (1.f + expf(-pb));
+        if (threadIdx.x < SCAN_TOKENS * COLS) (&sv[buf][0][0])[threadIdx.x] = pv;
+        if (threadIdx.x < SCAN_TOKENS) sb[buf][threadIdx.x] = 1.f / (1.f + expf(-pb));
     };
+    // With two buffers in LDS the next block is staged, and the one after it asked for, in front of the
+    // block at hand: one barrier a block.  With one buffer the waves meet before and after staging.
+    // (Beyond the portion real elements are fetched and staged, and not used.)
+    int buf = 0;
     fetch(t0);
-    for (int tb = t0; tb < t1; tb += SCAN_TOKENS) {
-        __syncthreads();  // the block before has been read by every wave
-        stage();
+    if constexpr (BUFS == 2) {
+        stage(0);
+        fetch(t0 + SCAN_TOKENS);
         __syncthreads();
-        if (tb + SCAN_TOKENS < t1) fetch(tb + SCAN_TOKENS);
+    }
+    for (int tb = t0; tb < t1; tb += SCAN_TOKENS) {
+        if constexpr (BUFS == 2) {
+            stage(buf ^ 1);
+            fetch(tb + 2 * SCAN_TOKENS);
+        } else {
+            __syncthreads();  // the block before has been read by every wave
+            stage(0);
+            __syncthreads();
+            fetch(tb + SCAN_TOKENS);
+        }
         const int nt = min(SCAN_TOKENS, t1 - tb);
         float* dst = raw + (size_t)tb * heads * dv + h * dv + j;
         if (nt == SCAN_TOKENS) {
@@ -936,12 +974,12 @@ __global__ __launch_bounds__(SCAN_THREADS) __attribute__((amdgpu_waves_per_eu(1,
             float os[SCAN_TOKENS];
             Operands x[2][AHEAD];
 #pragma unroll
-            for (int q = 0; q < AHEAD; ++q) read(q, x[0][q]);
+            for (int q = 0; q < AHEAD; ++q) read(buf, q, x[0][q]);
 #pragma unroll
             for (int n = 0; n < SCAN_TOKENS / AHEAD; ++n) {
                 if (n + 1 < SCAN_TOKENS / AHEAD) {
 #pragma unroll
-                    for (int q = 0; q < AHEAD; ++q) read((n + 1) * AHEAD + q, x[(n + 1) & 1][q]);
+                    for (int q = 0; q < AHEAD; ++q) read(buf, (n + 1) * AHEAD + q, x[(n + 1) & 1][q]);
                 }
                 __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
@@ -952,10 +990,14 @@ __global__ __launch_bounds__(SCAN_THREADS) __attribute__((amdgpu_waves_per_eu(1,
         } else {
             for (int tt = 0; tt < nt; ++tt) {
                 Operands x;
-                read(tt, x);
+                read(buf, tt, x);
                 const float o = column_sum<LPC>(token(x));
                 if (c == 0 && live) dst[(size_t)tt * heads * dv] = o;
             }
+        }
+        if constexpr (BUFS == 2) {
+            buf ^= 1;
+            __syncthreads();  // the next block is staged, and this one has been read
         }
     }
     state_rows_store<RPL>(Sp, c * RPL, d, live, state);
