@@ -90,7 +90,20 @@ PEFU_D = {
 }
 PAGE_D = 16
 
-PEFU = {"A": (PEFU_A, PAGE_A, 701), "B": (PEFU_B, PAGE_B, 702), "C": (PEFU_C, PAGE_C, 703), "D": (PEFU_D, PAGE_D, 704)}
+# E: recurrent layers alone, so that no request has pages: a delta rule of 48 key channels, time
+# mixing with heads of 24, passes over the last layer only; pages of 8 that nobody asks for
+PEFU_E = {
+    "architecture": "Pefulorn", "width": 80, "vocab": 141, "norm": {"eps": 1e-5},
+    "layers": [
+        _layer("channel_delta", _delta(4, 4, 48, 20, 5, 7, 9), 40),
+        _layer("wkv", _wkv(2, 24, 5), 56),
+    ],
+    "loop": {"start": 1, "stop": 2, "times": 4},
+}
+PAGE_E = 8
+
+PEFU = {"A": (PEFU_A, PAGE_A, 701), "B": (PEFU_B, PAGE_B, 702), "C": (PEFU_C, PAGE_C, 703), "D": (PEFU_D, PAGE_D, 704),
+        "E": (PEFU_E, PAGE_E, 705)}
 
 
 def tensor_shapes(cfg) -> dict[str, tuple[int, ...]]:

@@ -492,6 +492,7 @@ LENGTHS = {
     "B": [1, 2, 4, 5, 9, 33, 80],
     "C": [1, 2, 8, 9, 10, 34, 90],
     "D": [2, 15, 16, 17, 20, 70, 150],
+    "E": [1, 2, 16, 17, 40],
 }
 
 
@@ -541,7 +542,7 @@ def _check(got, want, dtype, label, rounding=None):
         parity.record(label, worst, worst)
 
 
-@pytest.mark.parametrize("which", ["A", "B", "C", "D"])
+@pytest.mark.parametrize("which", ["A", "B", "C", "D", "E"])
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
 def test_every_cut_matches_plain(tmp_path, which, dtype):
     cfg, page, seed = PEFU[which]
@@ -651,7 +652,7 @@ def test_trace_program(tmp_path):
 
 
 @pytest.mark.parametrize("use_graph", [False, True])
-@pytest.mark.parametrize("which,dtype", [("A", "float32"), ("C", "float32"), ("D", "bfloat16")])
+@pytest.mark.parametrize("which,dtype", [("A", "float32"), ("C", "float32"), ("D", "bfloat16"), ("E", "float32")])
 def test_greedy_generation_through_the_entry_point(tmp_path, which, dtype, use_graph):
     """``LLM.generate``: scheduler, chunked prompts beside decoding requests, sampling kernels;
     decode steps eagerly and replayed from graphs.  The plain implementation re-runs the whole
