@@ -185,8 +185,12 @@ __global__ __launch_bounds__(GW* RL_WAVE) void gemm_skinny_kernel(
             if (m < M && mine && nbase + i < N) {
                 res_in[i] = ex.residual[(size_t)m * N + nbase + i];
                 nw_in[i] = ex.norm_w[nbase + i];
-                if (ex.bias) bias_in[i] = ex.bias[nbase + i];
             }
+        if (ex.bias) {
+#pragma unroll
+            for (int i = 0; i < 4; ++i)
+                if (mine && nbase + i < N) bias_in[i] = ex.bias[nbase + i];
+        }
     }
 
     // whole chunks of 128: no predicates.  The bound is the same for every lane of a wave.
