@@ -12,8 +12,8 @@ Two kinds of library exist:
 * ``attn_d<D>``: the matrix-core attention kernels, compiled for one head size ``D``.
   A model compiles only the head sizes it has.
 * ``mlstm``: the matrix-memory recurrence, compiled when a model has such a mixer.
-* ``recurrent``: the token-shift time mixing and the state-space mixer (scans, short convolution,
-  grouped norm), compiled when a model has such a mixer.
+* ``recurrent``: the token-shift time mixing, the state-space mixer, the gated delta rule and minGRU
+  (scans, short convolutions, head and grouped norms), compiled when a model has such a mixer.
 * ``attn_tile_d<D>_v<DV>``: the tile attention for key heads of ``D`` and value heads of ``DV``
   channels, compiled when a model has a mixer that needs it.
 
