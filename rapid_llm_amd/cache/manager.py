@@ -76,12 +76,14 @@ class PagePool:
 @dataclass(frozen=True)
 class GroupSpec:
     """Layers that share page ids.  ``window`` 0: every position is kept.  With a window,
-    the pages of the first ``keep_first`` positions are never given back before the request ends."""
+    the pages of the first ``keep_first`` positions are never given back before the request ends.
+    ``chunked``: the window does not slide; a position reads its own chunk of ``window`` positions."""
 
     group_id: int
     window: int
     layers: tuple[int, ...]
     keep_first: int = 0
+    chunked: bool = False
 
 
 @dataclass
@@ -173,6 +175,8 @@ class CacheManager:
         """Index of the first page a query at ``next_position`` or later can still read."""
         if group.window <= 0:
             return 0
+        if group.chunked:
+            return next_position // group.window * group.window // self.page_size
         first_pos = max(0, next_position - group.window + 1)
         return first_pos // self.page_size
 

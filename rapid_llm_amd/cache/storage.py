@@ -60,16 +60,16 @@ class LayerCache:
 
 
 def plan_groups(needs: list[CacheNeed]) -> tuple[list[GroupSpec], list[int | None]]:
-    """Group layers by what they keep (all keys / a window of w, with k kept first positions).  Returns the groups and,
+    """Group layers by what they keep (all keys / a sliding window or a chunk of w, with k kept first positions).  Returns the groups and,
     per layer, its group id (``None`` for layers without paged cache).  A layer that shares
     another layer's cache joins that layer's group."""
-    keys: dict[tuple[int, int], int] = {}  # (window, kept first positions) -> group id
+    keys: dict[tuple[int, int, bool], int] = {}  # (window, kept first positions, chunked) -> group id
     layers_of: dict[int, list[int]] = {}
     group_of: list[int | None] = [None] * len(needs)
     for i, need in enumerate(needs):
         if need.kind != "paged" or need.share_with is not None:
             continue
-        gid = keys.setdefault((need.window, need.keep_first if need.window else 0), len(keys))
+        gid = keys.setdefault((need.window, need.keep_first if need.window else 0, need.chunked), len(keys))
         layers_of.setdefault(gid, []).append(i)
         group_of[i] = gid
     for i, need in enumerate(needs):
@@ -82,7 +82,7 @@ def plan_groups(needs: list[CacheNeed]) -> tuple[list[GroupSpec], list[int | Non
                     f"layer {i} shares the cache of layer {src} but names other paged tensors: "
                     f"{need.paged} against {needs[src].paged}"
                 )
-            if (needs[src].window, needs[src].keep_first) != (need.window, need.keep_first):
+            if (needs[src].window, needs[src].keep_first, needs[src].chunked) != (need.window, need.keep_first, need.chunked):
                 raise ValueError(
                     f"layer {i} (window {need.window}, {need.keep_first} kept) shares the cache of layer {src} "
                     f"(window {needs[src].window}, {needs[src].keep_first} kept): a shared cache must keep the "
@@ -91,7 +91,7 @@ def plan_groups(needs: list[CacheNeed]) -> tuple[list[GroupSpec], list[int | Non
             group_of[i] = group_of[src]
             layers_of[group_of[i]].append(i)
     windows = {gid: w for w, gid in keys.items()}
-    groups = [GroupSpec(gid, windows[gid][0], tuple(layers_of[gid]), windows[gid][1]) for gid in sorted(windows)]
+    groups = [GroupSpec(gid, windows[gid][0], tuple(layers_of[gid]), *windows[gid][1:]) for gid in sorted(windows)]
     return groups, group_of
 
 

@@ -45,6 +45,8 @@ _LAZY: dict[str, str] = {
     "fomunex": "rapid_llm_amd.models.fomunex",
     "Pefulorn": "rapid_llm_amd.models.pefulorn",
     "pefulorn": "rapid_llm_amd.models.pefulorn",
+    "Renitar": "rapid_llm_amd.models.renitar",
+    "renitar": "rapid_llm_amd.models.renitar",
 }
 
 

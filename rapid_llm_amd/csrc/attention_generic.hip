@@ -9,7 +9,9 @@
 // exp of a number per query head: a key without a value.  With cap > 0 a scaled score s becomes
 // cap * tanh(s / cap); with `slopes` (one number a query head) slope_h * (pos - j) is then taken
 // off it; with `log_r1` and `log_r2` instead r1_h * ln(1 + r2_h * (pos - j)) is.  A token's heads lie
-// side by side in a row of `out` of out_width elements; `out_scale` multiplies the finished outputs.
+// side by side in a row of `out` of out_width elements; `out_scale` multiplies the finished outputs, and
+// with `gate` the sigmoid of gate[t * gate_width + h * dv + c] channel c of head h.  With `chunked` a token
+// sees the keys of its own chunk of `window` positions, counted from the request's first.
 //
 // Scores (q . k) / sqrt(d) (rapid_llm/modules/attention.py:62), online softmax over tiles
 // of 256 keys in ascending order (rapid_llm/kernels/ops/attention/flashattention2_nopad.py:
@@ -26,7 +28,8 @@ __global__ __launch_bounds__(ATT_THREADS) void attention_generic_kernel(
     const int* __restrict__ block_table, int table_stride, int page_size, int nq, int nkv, int d,
     int window, float scale, int dv, int keep_first, int sink, const float* __restrict__ sink_values,
     float cap, const float* __restrict__ slopes, const float* __restrict__ log_r1,
-    const float* __restrict__ log_r2, int out_width, float out_scale) {
+    const float* __restrict__ log_r2, int out_width, float out_scale, int chunked,
+    const T* __restrict__ gate, int gate_width) {
     __shared__ float qs[256];
     __shared__ float ps[ATT_THREADS];
     __shared__ int key_page[ATT_THREADS];  // page * nkv + kv head of each key of the tile
@@ -40,7 +43,7 @@ __global__ __launch_bounds__(ATT_THREADS) void attention_generic_kernel(
     const int pos = positions[t];
     const int* table = block_table + (size_t)token_slot[t] * table_stride;
     const int kend = pos + 1;
-    const int kstart = (window > 0 && pos - window + 1 > 0) ? pos - window + 1 : 0;
+    const int kstart = window <= 0 ? 0 : (chunked ? pos / window * window : max(pos - window + 1, 0));
     // the keys read, in ascending order: the kept first ones below the window, then the window's
     const int kept = window > 0 ? min(keep_first, kstart) : 0;
     const int nkeys = kept + (kend - kstart);
@@ -94,7 +97,11 @@ __global__ __launch_bounds__(ATT_THREADS) void attention_generic_kernel(
         l = l * fa + expf(s0 - m_new);
         acc *= fa;
     }
-    if (tid < dv) out[(size_t)t * out_width + h * dv + tid] = from_float<T>(acc / l * out_scale);
+    if (tid < dv) {
+        float y = acc / l * out_scale;
+        if (gate) y /= 1.f + expf(-to_float(gate[(size_t)t * gate_width + h * dv + tid]));
+        out[(size_t)t * out_width + h * dv + tid] = from_float<T>(y);
+    }
 }
 
 extern "C" int rl_attention_generic(const void* q, const void* k_cache, const void* v_cache,
@@ -103,9 +110,11 @@ extern "C" int rl_attention_generic(const void* q, const void* k_cache, const vo
                                     int tokens, int nq, int nkv, int d, int window, float scale,
                                     int dv, int keep_first, int sink, const float* sink_values, float cap,
                                     const float* slopes, const float* log_r1, const float* log_r2, int out_width,
-                                    float out_scale, int act_type, hipStream_t stream) {
+                                    float out_scale, int chunked, const void* gate, int gate_width, int act_type,
+                                    hipStream_t stream) {
     if (tokens <= 0) return RL_OK;
     if (cap < 0.f || !log_r1 != !log_r2 || out_width < nq * dv) return RL_ERR_ARG;
+    if ((chunked && (window < 1 || keep_first)) || (gate && gate_width < nq * dv)) return RL_ERR_ARG;
     if (d < 1 || d > 256 || dv < 1 || dv > 256 || keep_first < 0 || nkv < 1 || nq % nkv || page_size < 1 ||
         nq > 65535)
         return RL_ERR_ARG;
@@ -115,13 +124,13 @@ extern "C" int rl_attention_generic(const void* q, const void* k_cache, const vo
                            (const float*)q, (const float*)k_cache, (const float*)v_cache,
                            (float*)out, positions, token_slot, block_table, table_stride,
                            page_size, nq, nkv, d, window, scale, dv, keep_first, sink, sink_values, cap, slopes,
-                           log_r1, log_r2, out_width, out_scale);
+                           log_r1, log_r2, out_width, out_scale, chunked, (const float*)gate, gate_width);
     else if (act_type == RL_BF16)
         hipLaunchKernelGGL(attention_generic_kernel<bf16_t>, grid, block, 0, stream,
                            (const bf16_t*)q, (const bf16_t*)k_cache, (const bf16_t*)v_cache,
                            (bf16_t*)out, positions, token_slot, block_table, table_stride,
                            page_size, nq, nkv, d, window, scale, dv, keep_first, sink, sink_values, cap, slopes,
-                           log_r1, log_r2, out_width, out_scale);
+                           log_r1, log_r2, out_width, out_scale, chunked, (const bf16_t*)gate, gate_width);
     else
         return RL_ERR_ARG;
     return rl_launch_status();

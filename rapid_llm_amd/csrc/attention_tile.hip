@@ -26,8 +26,12 @@
 // it afterwards.  The sink's term has neither.  With `log_r1` and `log_r2` (one number a query head
 // each) r1_h * ln(1 + r2_h * (p - j)) is taken off instead.
 //
+// With `chunked` the window is not a sliding one: positions are cut into chunks of `window` from a
+// request's first position on, and a row sees the keys of its own chunk (no kept first ones).
+//
 // A row's heads lie side by side in a row of `out` of out_width elements; `out_scale` multiplies
-// the finished outputs.
+// the finished outputs.  With `gate` every channel is also multiplied by the sigmoid of a number:
+// that of head h and channel c of token t is gate[t * gate_width + h * DV + c].
 //
 // A row's result does not depend on the tile it falls in, on the other rows there, or on how a
 // prompt was cut into steps: keys are taken in tiles of 16 at absolute positions 0, 16, ..,
@@ -97,6 +101,23 @@ __device__ inline void to_quad(const f32x4& p, s16x4& out) {
     out = __builtin_bit_cast(s16x4, b);
 }
 __device__ inline float quad_elem(const f32x4& q, int i) { return q[i]; }
+template <typename T>
+__device__ inline float gate_float(const T* p, int i);
+template <>
+__device__ inline float gate_float<float>(const float* p, int i) {
+    return p[i];
+}
+template <>
+__device__ inline float gate_float<bf16_t>(const bf16_t* p, int i) {
+    return bf16_to_float(p[i]);
+}
+__device__ inline float sigmoid(float z) { return 1.f / (1.f + expf(-z)); }
+// the first position that a query at `pos` sees (kept first ones aside)
+__device__ inline int first_seen(int pos, int window, int chunked) {
+    if (window <= 0) return 0;
+    if (chunked) return pos / window * window;
+    return max(pos - window + 1, 0);
+}
 __device__ inline void store_quad(float* p, f32x4 v) { *reinterpret_cast<f32x4*>(p) = v; }
 __device__ inline void store_quad(bf16_t* p, f32x4 v) {
     s16x4 o;
@@ -172,7 +193,7 @@ __global__ __launch_bounds__(AW* RL_WAVE) void attn_tile_kernel(
     int page_size, int nq, int nkv, int window, int keep_first, int sink, float scale,
     float* __restrict__ part, int nsplit, const float* __restrict__ sink_values, float cap,
     const float* __restrict__ slopes, const float* __restrict__ log_r1, const float* __restrict__ log_r2,
-    int out_width, float out_scale) {
+    int out_width, float out_scale, int chunked, const T* __restrict__ gate, int gate_width) {
     typedef typename Quad<T>::type quad;
     const float in_log2 = sizeof(T) == 2 ? 1.4426950408889634f : 1.f;  // bfloat16: scores in units of log2
     const float cap_in = cap > 0.f ? scale / cap : 0.f;  // a raw product times this is s / cap
@@ -204,7 +225,7 @@ __global__ __launch_bounds__(AW* RL_WAVE) void attn_tile_kernel(
         head[r] = hk * G + (row_ok[r] ? row : rows - 1) % G;
         const int pos = start + tok[r];
         kend[r] = pos + 1;
-        kstart[r] = (window > 0 && pos - window + 1 > 0) ? pos - window + 1 : 0;
+        kstart[r] = first_seen(pos, window, chunked);
     }
     // what a position of distance costs this lane's row, in the scores' unit; or the two numbers of
     // a logarithmic cost (in bfloat16 a logarithm of base 2 in units of log2: the factors cancel)
@@ -234,7 +255,7 @@ __global__ __launch_bounds__(AW* RL_WAVE) void attn_tile_kernel(
         if (rl < rows) {
             const int pl = start + rl / G;
             all_hi[r] = start + rf / G + 1;
-            all_lo[r] = (window > 0 && pl - window + 1 > 0) ? pl - window + 1 : 0;
+            all_lo[r] = first_seen(pl, window, chunked);
         }
     }
 
@@ -242,7 +263,7 @@ __global__ __launch_bounds__(AW* RL_WAVE) void attn_tile_kernel(
     // (rows ascend with the tokens), in whole tiles of 16, up to the last row's own position
     const int first_pos = start + row0 / G;
     const int last_pos = start + (min(rows, row0 + 16 * R) - 1) / G;
-    const int first_key = (window > 0 && first_pos - window + 1 > 0) ? first_pos - window + 1 : 0;
+    const int first_key = first_seen(first_pos, window, chunked);
     const int lo = first_key & ~15;
     const int hi = last_pos + 1;                     // keys below hi are in the cache
     const int kept_end = min((keep + 15) & ~15, lo);  // tiles [0, kept_end) come before those of [lo, hi)
@@ -508,6 +529,16 @@ __global__ __launch_bounds__(AW* RL_WAVE) void attn_tile_kernel(
         // acc[r][b][i] is channel 16b + 4g + i of the lane's row
         T* orow = out + (size_t)(at + tok[r]) * out_width + head[r] * DV + 4 * g;
         const float inv = out_scale / l[r];
+        if (gate) {
+            const T* grow = gate + (size_t)(at + tok[r]) * gate_width + head[r] * DV + 4 * g;
+#pragma unroll
+            for (int b = 0; b < VB; ++b) {
+                const quad z = ld_quad<T>(grow + 16 * b);
+                const T* zt = reinterpret_cast<const T*>(&z);
+#pragma unroll
+                for (int i = 0; i < 4; ++i) acc[r][b][i] *= sigmoid(gate_float<T>(zt, i));
+            }
+        }
 #pragma unroll
         for (int b = 0; b < VB; ++b)
             store_quad(orow + 16 * b, (f32x4){acc[r][b][0] * inv, acc[r][b][1] * inv, acc[r][b][2] * inv,
@@ -522,7 +553,8 @@ __global__ __launch_bounds__(AW* RL_WAVE) void attn_tile_kernel(
 __global__ __launch_bounds__(256) void attn_tile_merge_kernel(const float* __restrict__ part,
                                                               bf16_t* __restrict__ out, int rows, int nsplit,
                                                               int sink, const float* __restrict__ sink_values,
-                                                              int nq, int out_width, float out_scale) {
+                                                              int nq, int out_width, float out_scale,
+                                                              const bf16_t* __restrict__ gate, int gate_width) {
     const int row = blockIdx.x * 4 + threadIdx.x / RL_WAVE;
     const int lane = threadIdx.x & (RL_WAVE - 1);
     if (row >= rows) return;
@@ -551,7 +583,10 @@ __global__ __launch_bounds__(256) void attn_tile_merge_kernel(const float* __res
 #pragma unroll
             for (int j = 0; j < 8; ++j) sum += __shfl(weight, (s8 + j) & (RL_WAVE - 1)) * v[j];
         }
-        if (live) out[(size_t)(row / nq) * out_width + (row % nq) * DV + c] = float_to_bf16(sum * (out_scale / den));
+        if (!live) continue;
+        float y = sum * (out_scale / den);
+        if (gate) y *= sigmoid(bf16_to_float(gate[(size_t)(row / nq) * gate_width + (row % nq) * DV + c]));
+        out[(size_t)(row / nq) * out_width + (row % nq) * DV + c] = float_to_bf16(y);
     }
 }
 
@@ -574,10 +609,13 @@ extern "C" int rl_attn_tile(const void* q, const void* k_cache, const void* v_ca
                             int page_size, int nq, int nkv, int window, int keep_first, int sink,
                             float scale, int nsplit, float* part, int tokens, int tile_rows, int act_type,
                             const float* sink_values, float cap, const float* slopes, const float* log_r1,
-                            const float* log_r2, int out_width, float out_scale, hipStream_t stream) {
+                            const float* log_r2, int out_width, float out_scale, int chunked, const void* gate,
+                            int gate_width, hipStream_t stream) {
     if (num_tiles <= 0) return RL_OK;
     if (cap < 0.f || (slopes && log_r1) || !log_r1 != !log_r2) return RL_ERR_ARG;
     if (out_width < nq * tileattn::DV || out_width % 4) return RL_ERR_ARG;  // (four channels are stored at once)
+    if (chunked && (window < 1 || keep_first)) return RL_ERR_ARG;
+    if (gate && (gate_width < nq * tileattn::DV || gate_width % 4)) return RL_ERR_ARG;
     if (nkv < 1 || nq % nkv || page_size < 4 || page_size % 4 || nkv > 65535 || window < 0 || keep_first < 0)
         return RL_ERR_ARG;
     constexpr int AW = 4;
@@ -589,7 +627,8 @@ extern "C" int rl_attn_tile(const void* q, const void* k_cache, const void* v_ca
     if (act_type == RL_BF16 && tile_rows == 16 * PB && PB > 1) {
         if (nsplit != 1) return RL_ERR_ARG;
         hipLaunchKernelGGL((tileattn::attn_tile_kernel<bf16_t, AW, PB>), grid, block, 0, stream, RL_TILE_ARGS(bf16_t),
-                           nullptr, 1, sink_values, cap, slopes, log_r1, log_r2, out_width, out_scale);
+                           nullptr, 1, sink_values, cap, slopes, log_r1, log_r2, out_width, out_scale, chunked, (const bf16_t*)gate,
+                           gate_width);
         return rl_launch_status();
     }
     if (tile_rows != 16) return RL_ERR_ARG;
@@ -599,18 +638,22 @@ extern "C" int rl_attn_tile(const void* q, const void* k_cache, const void* v_ca
     if (nsplit > 1) {
         if (act_type != RL_BF16 || !part || nsplit > 64 || tokens < 1) return RL_ERR_ARG;
         hipLaunchKernelGGL((tileattn::attn_tile_kernel<bf16_t, AW, 1>), dim3(num_tiles, nkv, nsplit), block, 0, stream,
-                           RL_TILE_ARGS(bf16_t), part, nsplit, sink_values, cap, slopes, log_r1, log_r2, out_width, out_scale);
+                           RL_TILE_ARGS(bf16_t), part, nsplit, sink_values, cap, slopes, log_r1, log_r2, out_width, out_scale,
+                           chunked, nullptr, 0);
         const int rows = tokens * nq;
         hipLaunchKernelGGL(tileattn::attn_tile_merge_kernel, dim3((rows + 3) / 4), dim3(256), 0, stream, part,
-                           (bf16_t*)out, rows, nsplit, sink, sink_values, nq, out_width, out_scale);
+                           (bf16_t*)out, rows, nsplit, sink, sink_values, nq, out_width, out_scale, (const bf16_t*)gate,
+                           gate_width);
         return rl_launch_status();
     }
     if (act_type == RL_F32)
         hipLaunchKernelGGL((tileattn::attn_tile_kernel<float, AW, 1>), grid, block, 0, stream, RL_TILE_ARGS(float),
-                           nullptr, 1, sink_values, cap, slopes, log_r1, log_r2, out_width, out_scale);
+                           nullptr, 1, sink_values, cap, slopes, log_r1, log_r2, out_width, out_scale, chunked, (const float*)gate,
+                           gate_width);
     else if (act_type == RL_BF16)
         hipLaunchKernelGGL((tileattn::attn_tile_kernel<bf16_t, AW, 1>), grid, block, 0, stream, RL_TILE_ARGS(bf16_t),
-                           nullptr, 1, sink_values, cap, slopes, log_r1, log_r2, out_width, out_scale);
+                           nullptr, 1, sink_values, cap, slopes, log_r1, log_r2, out_width, out_scale, chunked, (const bf16_t*)gate,
+                           gate_width);
     else
         return RL_ERR_ARG;
 #undef RL_TILE_ARGS

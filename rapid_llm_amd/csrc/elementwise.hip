@@ -649,10 +649,12 @@ extern "C" int rl_swiglu(const void* gate_up, void* out, int tokens, int inter, 
 //   kind 0: gelu in its tanh form, 0.5 z (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3)))
 //   kind 1: relu(z)^2
 //   kind 2: tanh(z)
+//   kind 3: gelu in its exact form, 0.5 z (1 + erf(z / sqrt(2)))
 // With `route` (float32 [tokens, experts]) the first experts * ff columns of a row are the
 // hidden units of `experts` experts side by side, and expert e's units are multiplied by
 // route[t, e] (0 for an expert the token does not use); columns beyond (a shared expert's)
-// pass with the activation alone.
+// pass with the activation alone, or with `route_shared` are multiplied by entry `experts` of the
+// token's row of `route`, whose rows have route_width entries.
 // --------------------------------------------------------------------------- //
 __device__ inline float unary_act(float z, int kind) {
     if (kind == 1) {
@@ -660,12 +662,14 @@ __device__ inline float unary_act(float z, int kind) {
         return r * r;
     }
     if (kind == 2) return tanhf(z);
+    if (kind == 3) return 0.5f * z * (1.f + erff(0.7071067811865476f * z));
     return 0.5f * z * (1.f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
 }
 
 template <typename T>
 __global__ void unary_act_kernel(const T* __restrict__ x, T* __restrict__ out, size_t total, int cols,
-                                 int kind, const float* __restrict__ route, int experts, int ff) {
+                                 int kind, const float* __restrict__ route, int experts, int ff, int route_width,
+                                 int route_shared) {
     size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
     const size_t step = (size_t)gridDim.x * blockDim.x;
     for (; idx < total; idx += step) {
@@ -673,7 +677,7 @@ __global__ void unary_act_kernel(const T* __restrict__ x, T* __restrict__ out, s
         if (route) {
             const size_t t = idx / cols;
             const int c = (int)(idx - t * cols);
-            if (c < experts * ff) v *= route[t * experts + c / ff];
+            if (c < experts * ff || route_shared) v *= route[t * route_width + min(c / ff, experts)];
         }
         out[idx] = from_float<T>(v);
     }
@@ -683,7 +687,8 @@ __global__ void unary_act_kernel(const T* __restrict__ x, T* __restrict__ out, s
 // units, so that a group of eight belongs to one expert; `total` counts groups
 template <typename T>
 __global__ void unary_act_vec_kernel(const T* __restrict__ x, T* __restrict__ out, size_t total, int cols8,
-                                     int kind, const float* __restrict__ route, int experts, int ff8) {
+                                     int kind, const float* __restrict__ route, int experts, int ff8, int route_width,
+                                     int route_shared) {
     struct alignas(sizeof(T) * 8) Pack {
         T v[8];
     };
@@ -695,7 +700,7 @@ __global__ void unary_act_vec_kernel(const T* __restrict__ x, T* __restrict__ ou
         if (route) {
             const size_t t = idx / cols8;
             const int c = (int)(idx - t * cols8);
-            if (c < experts * ff8) factor = route[t * experts + c / ff8];
+            if (c < experts * ff8 || route_shared) factor = route[t * route_width + min(c / ff8, experts)];
         }
         Pack o;
 #pragma unroll
@@ -705,10 +710,12 @@ __global__ void unary_act_vec_kernel(const T* __restrict__ x, T* __restrict__ ou
 }
 
 extern "C" int rl_unary_act(const void* x, void* out, int tokens, int cols, int kind, const float* route,
-                            int experts, int ff, int act_type, hipStream_t stream) {
+                            int experts, int ff, int route_width, int route_shared, int act_type,
+                            hipStream_t stream) {
     if (tokens <= 0 || cols <= 0) return RL_OK;
-    if (kind < 0 || kind > 2) return RL_ERR_ARG;
-    if (route && (experts < 1 || ff < 1 || (long)experts * ff > cols)) return RL_ERR_ARG;
+    if (kind < 0 || kind > 3) return RL_ERR_ARG;
+    if (route && (experts < 1 || ff < 1 || (long)experts * ff > cols || route_width < experts + (route_shared ? 1 : 0)))
+        return RL_ERR_ARG;
     if (act_type != RL_F32 && act_type != RL_BF16) return RL_ERR_ARG;
     const bool vec = cols % 8 == 0 && (!route || ff % 8 == 0);
     const size_t total = (size_t)tokens * cols / (vec ? 8 : 1);
@@ -717,16 +724,16 @@ extern "C" int rl_unary_act(const void* x, void* out, int tokens, int cols, int 
     dim3 grid((unsigned)blocks), block(256);
     if (vec && act_type == RL_F32)
         hipLaunchKernelGGL(unary_act_vec_kernel<float>, grid, block, 0, stream, (const float*)x, (float*)out, total,
-                           cols / 8, kind, route, experts, ff / 8);
+                           cols / 8, kind, route, experts, ff / 8, route_width, route_shared);
     else if (vec)
         hipLaunchKernelGGL(unary_act_vec_kernel<bf16_t>, grid, block, 0, stream, (const bf16_t*)x, (bf16_t*)out,
-                           total, cols / 8, kind, route, experts, ff / 8);
+                           total, cols / 8, kind, route, experts, ff / 8, route_width, route_shared);
     else if (act_type == RL_F32)
         hipLaunchKernelGGL(unary_act_kernel<float>, grid, block, 0, stream, (const float*)x, (float*)out, total,
-                           cols, kind, route, experts, ff);
+                           cols, kind, route, experts, ff, route_width, route_shared);
     else
         hipLaunchKernelGGL(unary_act_kernel<bf16_t>, grid, block, 0, stream, (const bf16_t*)x, (bf16_t*)out,
-                           total, cols, kind, route, experts, ff);
+                           total, cols, kind, route, experts, ff, route_width, route_shared);
     return rl_launch_status();
 }
 

@@ -14,6 +14,8 @@ Two kinds of library exist:
 * ``mlstm``: the matrix-memory recurrence, compiled when a model has such a mixer.
 * ``recurrent``: the token-shift time mixing, the state-space mixer, the gated delta rule and minGRU
   (scans, short convolutions, head and grouped norms), compiled when a model has such a mixer.
+* ``linear_attention``: linear attention with decays a channel or a head (chunked walk, single tokens,
+  gated norm of its outputs), compiled when a model has such a mixer.
 * ``attn_tile_d<D>_v<DV>``: the tile attention for key heads of ``D`` and value heads of ``DV``
   channels, compiled when a model has a mixer that needs it.
 
@@ -46,10 +48,14 @@ CORE_SOURCES = (
     "gemm_bf16.hip",
     "gemm_rows.hip",
     "latent.hip",
+    "router.hip",
+    "sublayer_sum.hip",
+    "conv_heads.hip",
 )
 ATTENTION_SOURCES = ("attention_mfma.hip", "attention_f32.hip")
 MLSTM_SOURCES = ("mlstm.hip",)
 RECURRENT_SOURCES = ("recurrent.hip",)
+LINEAR_ATTENTION_SOURCES = ("linear_attention.hip",)
 ATTENTION_TILE_SOURCES = ("attention_tile.hip",)
 HEADERS = ("common.h", "static_entry.h")
 
@@ -233,6 +239,10 @@ def recurrent_library(force: bool = False) -> Path:
     return compile_library("recurrent", RECURRENT_SOURCES, force=force)
 
 
+def linear_attention_library(force: bool = False) -> Path:
+    return compile_library("linear_attention", LINEAR_ATTENTION_SOURCES, force=force)
+
+
 def attention_tile_library(head_dim: int, value_dim: int, force: bool = False) -> Path:
     # beyond 320 / 256 channels a lane's operands no longer fit its registers: the compiler
     # parks some in scratch memory, which is slower and as exact
@@ -245,7 +255,8 @@ def attention_tile_library(head_dim: int, value_dim: int, force: bool = False) -
 
 def build_all(head_dims: tuple[int, ...] = DEFAULT_HEAD_DIMS, force: bool = True) -> list[Path]:
     """Compile every library (what ``__graft_entry__.build`` calls)."""
-    out = [core_library(force=force), mlstm_library(force=force), recurrent_library(force=force)]
+    out = [core_library(force=force), mlstm_library(force=force), recurrent_library(force=force),
+           linear_attention_library(force=force)]
     with ThreadPoolExecutor(8) as pool:
         out += list(pool.map(lambda pair: attention_tile_library(*pair, force=force), DEFAULT_TILE_HEAD_DIMS))
     if not all((CSRC / s).is_file() for s in ATTENTION_SOURCES):

@@ -119,6 +119,20 @@ def recurrent_lib() -> ctypes.CDLL:
     return _recurrent
 
 
+_linear_attention: ctypes.CDLL | None = None
+
+
+def linear_attention_lib() -> ctypes.CDLL:
+    global _linear_attention
+    if _linear_attention is None:
+        lib = build.load(build.linear_attention_library())
+        limits = (lib.rl_linear_attention_max_key_dim(), lib.rl_linear_attention_max_value_dim(), lib.rl_linear_attention_chunk())
+        if limits != (LINEAR_MAX_KEY_DIM, LINEAR_MAX_VALUE_DIM, LINEAR_CHUNK):
+            raise KernelError(f"the linear attention library's limits {limits} are not the launch rules'")
+        _linear_attention = lib
+    return _linear_attention
+
+
 def _stream() -> ctypes.c_void_p:
     # the raw handle of the current stream of the current device, without the stream object
     # that ``torch.cuda.current_stream()`` builds (2.8 against 0.2 us a call, on every launch)
@@ -295,28 +309,32 @@ def stream_add(residual: torch.Tensor, first: Optional[torch.Tensor], row: Optio
     _ok(core().rl_stream_add(_p(residual), _p(first), _p(row), tokens, hidden, _stream()), "rl_stream_add")
 
 
-UNARY_ACTIVATIONS = {"gelu_tanh": 0, "relu_squared": 1, "tanh": 2}
+UNARY_ACTIVATIONS = {"gelu_tanh": 0, "relu_squared": 1, "tanh": 2, "gelu": 3}
 
 
 def unary_act(x: torch.Tensor, out: torch.Tensor, kind: str, route: Optional[torch.Tensor] = None,
-              expert_ff: int = 0) -> None:
+              expert_ff: int = 0, experts: Optional[int] = None) -> None:
     """``out = act(x)`` for a one-operand activation (:data:`UNARY_ACTIVATIONS`).  With ``route``
     (float32 ``[tokens, experts]``) the first ``experts * expert_ff`` columns are the hidden units
-    of the experts side by side and expert ``e``'s are multiplied by ``route[t, e]``."""
+    of the experts side by side and expert ``e``'s are multiplied by ``route[t, e]``.  With ``experts``
+    given, the rows of ``route`` are wider than that and the columns beyond (a shared expert's) are
+    multiplied by ``route[t, experts]``."""
     if kind not in UNARY_ACTIVATIONS:
         raise KernelError(f"activation {kind!r} is not one of {sorted(UNARY_ACTIVATIONS)}")
     tokens, cols = x.shape
     _need(x, "x")
     _need(out, "out", x.dtype, (tokens, cols))
-    experts = 0
+    shared = route is not None and experts is not None
+    width = 0
     if route is not None:
-        experts = route.shape[1]
-        _need(route, "route", torch.float32, (tokens, experts))
-        if expert_ff < 1 or experts * expert_ff > cols:
-            raise KernelError(f"{experts} experts of {expert_ff} hidden units do not fit rows of {cols}")
+        width = route.shape[1]
+        experts = width if experts is None else int(experts)
+        _need(route, "route", torch.float32, (tokens, width))
+        if expert_ff < 1 or experts < 1 or experts * expert_ff > cols or (shared and width <= experts):
+            raise KernelError(f"{experts} experts of {expert_ff} hidden units do not fit rows of {cols}, weighed by {width} numbers")
     _ok(
-        core().rl_unary_act(_p(x), _p(out), tokens, cols, UNARY_ACTIVATIONS[kind], _p(route), experts, expert_ff,
-                            _tag(x.dtype), _stream()),
+        core().rl_unary_act(_p(x), _p(out), tokens, cols, UNARY_ACTIVATIONS[kind], _p(route), experts or 0, expert_ff,
+                            width, int(shared), _tag(x.dtype), _stream()),
         "rl_unary_act",
     )
 
@@ -362,6 +380,87 @@ def router(x: torch.Tensor, w: torch.Tensor, top: int, scale: float, bias: Optio
                          ROUTER_SCORES[scores], _tag(x.dtype), _stream()),
         "rl_router")
     return out
+
+
+def choose_experts(x: torch.Tensor, w: torch.Tensor, experts: int, identity: int, top: int, scale: float,
+                   correction: Optional[torch.Tensor] = None, gate: bool = False) -> torch.Tensor:
+    """The weights ``[tokens, experts + 2]`` (float32) of a mixture whose experts are chosen by corrected
+    scores.  ``w`` (float32) has a row for each of ``experts`` experts and ``identity`` experts that return their
+    input, and with ``gate`` one more.  Scores are the softmax over all experts; the ``top`` largest scores plus
+    ``correction`` are chosen (the lower index wins a tie), and a chosen expert's weight is its score times
+    ``scale``, not divided by anything.  A row holds the experts' weights (0 for those not chosen), the
+    sigmoid of the gate's row (1 without one), and the sum of the chosen identity experts' weights."""
+    tokens, k = x.shape
+    choices = experts + identity
+    _need(x, "x")
+    _need(w, "router matrix", torch.float32, (choices + int(bool(gate)), k))
+    if experts < 1 or identity < 0 or not 1 <= top <= choices <= ROUTE_MAX_EXPERTS:
+        raise KernelError(f"the router kernel chooses 1 to {choices} of at most {ROUTE_MAX_EXPERTS} experts, not {top}")
+    if correction is not None:
+        _need(correction, "correction of the scores", torch.float32, (choices,))
+    out = torch.empty((tokens, experts + 2), dtype=torch.float32, device=x.device)
+    _ok(core().rl_choose_experts(_p(x), _p(w), _p(correction), _p(out), tokens, k, experts, identity, int(bool(gate)), top,
+                                 ctypes.c_float(scale), _tag(x.dtype), _stream()),
+        "rl_choose_experts")
+    return out
+
+
+SUM_TERMS = 3  # rows that the kernel below adds at most
+
+
+def sublayer_sum_norm(residual: torch.Tensor, terms, factor: float, term_eps: float = 0.0,
+                      returned: Optional[tuple[torch.Tensor, torch.Tensor, int]] = None,
+                      weight: Optional[torch.Tensor] = None, out: Optional[torch.Tensor] = None, eps: float = 0.0,
+                      rows: Optional[torch.Tensor] = None) -> None:
+    """``residual += factor * (sum of terms + c x)`` (float32, in place), then, unless ``out`` is ``None``,
+    ``out = rmsnorm(residual) * weight``.  ``terms``: up to three of ``(y, bias, weight)``: the rows ``y`` plus
+    ``bias`` (float32 ``[hidden]`` or ``None``), with a ``weight`` (float32 ``[hidden]``) divided by their root mean
+    square (``term_eps`` inside the root) and multiplied by it.  ``returned`` ``(x, numbers, column)``: the rows ``x``
+    times one number a token, ``numbers[t, column]`` (float32).  ``rows`` as in :func:`add_rmsnorm`; the
+    stream is then left as it was."""
+    tokens, hidden = residual.shape
+    _need(residual, "residual", torch.float32)
+    if not 1 <= len(terms) <= SUM_TERMS:
+        raise KernelError(f"{len(terms)} terms; the kernel adds 1 to {SUM_TERMS}")
+    dtype = terms[0][0].dtype
+    args = []
+    for y, bias, w in terms:
+        _need(y, "term", dtype, (tokens, hidden))
+        if bias is not None:
+            _need(bias, "bias of a term", torch.float32, (hidden,))
+        if w is not None:
+            _need(w, "norm weight of a term", torch.float32, (hidden,))
+            if not term_eps > 0:
+                raise KernelError("a normed term needs an epsilon")
+        args += [_p(y), _p(bias), _p(w)]
+    args += [None] * (3 * (SUM_TERMS - len(terms)))
+    x = c = None
+    stride = 0
+    if returned is not None:
+        x, numbers, column = returned
+        _need(x, "returned rows", dtype, (tokens, hidden))
+        _need(numbers, "numbers of the returned rows", torch.float32, (tokens, None))
+        stride = numbers.shape[1]
+        if not 0 <= column < stride:
+            raise KernelError(f"column {column} of {stride} numbers a row")
+        c = _column(numbers, column)
+    out_rows = tokens
+    if out is not None:
+        out_rows = tokens if rows is None else rows.numel()
+        _need(out, "out", dtype, (out_rows, hidden))
+        _need(weight, "norm weight", torch.float32, (hidden,))
+        if rows is not None:
+            _need(rows, "rows", torch.int32)
+    elif rows is not None:
+        raise KernelError("rows are selected for the norm only")
+    _ok(
+        core().rl_sublayer_sum_norm(
+            _p(residual), *args, _p(x), c, stride, ctypes.c_float(term_eps), ctypes.c_float(factor),
+            _p(weight if out is not None else None), _p(out), _p(rows), out_rows, hidden, ctypes.c_float(eps),
+            _tag(dtype), _stream(),
+        ),
+        "rl_sublayer_sum_norm",
+    )
 
 
 GLU_ALPHA = 1.702  # the sigmoid's slope in the clamped gated activation
@@ -609,6 +708,17 @@ def _log_distance(pair, nq: int, slopes) -> tuple:
     return pair
 
 
+def _gate_columns(gate, dtype: torch.dtype, tokens: int, width: int) -> tuple:
+    """``gate`` ``(rows, first column)`` or ``None`` as the kernels' arguments (pointer, row width), checked."""
+    if gate is None:
+        return None, 0
+    rows, col = gate
+    _need(rows, "gate rows", dtype, (tokens, None))
+    if col < 0 or col + width > rows.shape[1]:
+        raise KernelError(f"gates of {width} columns from column {col} lie outside rows of {rows.shape[1]}")
+    return _column(rows, col), rows.shape[1]
+
+
 def _out_columns(out: torch.Tensor, dtype: torch.dtype, tokens: int, width: int, col: int) -> None:
     """``out`` is a contiguous ``[tokens, at least col + width]`` tensor whose columns from ``col`` on are written."""
     _need(out, "out", dtype, (tokens, None))
@@ -644,6 +754,8 @@ def attention_generic(
     log_distance: Optional[tuple[torch.Tensor, torch.Tensor]] = None,
     out_col: int = 0,
     out_scale: float = 1.0,
+    chunked: bool = False,
+    gate: Optional[tuple[torch.Tensor, int]] = None,
 ) -> None:
     tokens = q.shape[0]
     pages = k_cache.shape[0]
@@ -673,7 +785,8 @@ def attention_generic(
             _p(block_table), block_table.stride(0), page_size, tokens, nq, nkv, d, window,
             ctypes.c_float(scale), dv, int(keep_first), int(bool(sink) or sink_values is not None),
             _p(sink_values), ctypes.c_float(score_cap), _p(slopes), _p(r1), _p(r2),
-            out.shape[1], ctypes.c_float(out_scale), _tag(q.dtype), _stream(),
+            out.shape[1], ctypes.c_float(out_scale), int(bool(chunked)), *_gate_columns(gate, q.dtype, tokens, nq * dv),
+            _tag(q.dtype), _stream(),
         ),
         "rl_attention_generic",
     )
@@ -1645,6 +1758,8 @@ def attention_tile(
     log_distance: Optional[tuple[torch.Tensor, torch.Tensor]] = None,
     out_col: int = 0,
     out_scale: float = 1.0,
+    chunked: bool = False,
+    gate: Optional[tuple[torch.Tensor, int]] = None,
 ) -> None:
     """Attention of every token of the step, in tiles of 16 rows on the matrix cores, for value
     heads of a size of their own, a window that keeps a request's first ``keep_first`` positions
@@ -1653,7 +1768,9 @@ def attention_tile(
     scaled score s into ``c * tanh(s / c)``; ``slopes`` (float32, one number a query head) then take
     ``slope * (distance between query and key)`` off it; ``log_distance`` (two of them, r1 and r2)
     takes ``r1 * ln(1 + r2 * distance)`` off instead.  A token's heads go to the columns of ``out`` from
-    ``out_col`` on, multiplied by ``out_scale``.  float32 (bit for bit the same however
+    ``out_col`` on, multiplied by ``out_scale`` and, with ``gate`` ``(rows, column)``, by the sigmoid of the same
+    number of columns of ``rows`` from ``column`` on.  ``chunked``: positions are cut into chunks of ``window``
+    from a request's first on, and a token sees its own chunk.  float32 (bit for bit the same however
     the step was cut) or bfloat16."""
     tokens = q.shape[0]
     r1, r2 = _log_distance(log_distance, nq, slopes)
@@ -1667,6 +1784,10 @@ def attention_tile(
     pages = k_cache.shape[0]
     _need(q, "q", None, (tokens, nq * d))
     _out_columns(out, q.dtype, tokens, nq * dv, out_col)
+    if chunked and (window < 1 or keep_first):
+        raise KernelError(f"chunks of {window} positions with {keep_first} kept first ones")
+    if gate is not None and (gate[0].shape[1] % 4 or gate[1] % 4):
+        raise KernelError(f"four gates are read at once: columns from {gate[1]} on in rows of {gate[0].shape[1]}")
     if out.shape[1] % 4 or out_col % 4:
         raise KernelError(f"four channels are stored at once: columns from {out_col} on in rows of {out.shape[1]}")
     _need(k_cache, "k_cache", q.dtype, (pages, nkv, page_size, d))
@@ -1713,7 +1834,8 @@ def attention_tile(
             _p(ctx.token_slot), _p(block_table), block_table.stride(0), page_size, nq, nkv, window,
             int(keep_first), int(bool(sink)), ctypes.c_float(scale), nsplit, _p(part), tokens, tile_rows,
             _tag(q.dtype), _p(sink_values), ctypes.c_float(score_cap), _p(slopes), _p(r1), _p(r2),
-            out.shape[1], ctypes.c_float(out_scale), _stream(),
+            out.shape[1], ctypes.c_float(out_scale), int(bool(chunked)), *_gate_columns(gate, q.dtype, tokens, nq * dv),
+            _stream(),
         ),
         "rl_attn_tile",
     )
@@ -1755,6 +1877,8 @@ def paged_attention(
     log_distance: Optional[tuple[torch.Tensor, torch.Tensor]] = None,
     out_col: int = 0,
     out_scale: float = 1.0,
+    chunked: bool = False,
+    gate: Optional[tuple[torch.Tensor, int]] = None,
 ) -> None:
     """Attention of every token of the step over its request's cached keys.
 
@@ -1773,26 +1897,32 @@ def paged_attention(
     ``slopes`` (one number a query head, times the distance between query and key, taken off the
     score), ``log_distance`` (two numbers a query head instead: ``r1 * ln(1 + r2 * distance)``), ``out_col``
     (rows of ``out`` are wider than the heads, which go to the columns from there on) and
-    ``out_scale`` (a factor of the finished outputs) send the step to the kernels that take them:
+    ``out_scale`` (a factor of the finished outputs), ``chunked`` (the window is not a sliding one: a token sees
+    its own chunk of ``window`` positions, counted from the request's first) and ``gate`` (``(rows, column)``: the
+    outputs are multiplied by the sigmoid of as many columns of ``rows``) send the step to the kernels that take them:
     tiles of 16 rows on the matrix cores for head sizes in steps of 16, the FMA kernel otherwise."""
     if prepare is not None and not attention_prepares_queries(q.dtype, d, 0 if prepare[1] is None else prepare[1].shape[1]):
         raise KernelError("the attention kernels do not finish the queries of this head size, type or rotation")
     dv = d if value_dim is None else int(value_dim)
     keep_first = int(keep_first) if window > 0 else 0  # without a window every key is seen anyway
     if (dv != d or keep_first or sink or sink_values is not None or score_cap or slopes is not None
-            or log_distance is not None or out_col or out_scale != 1.0 or out.shape[1] != nq * dv):
+            or log_distance is not None or out_col or out_scale != 1.0 or out.shape[1] != nq * dv
+            or chunked or gate is not None):
         # value heads of their own size, kept first positions, one more term in the denominator
         if prepare is not None:
             raise KernelError("queries are finished before an attention with these options")
-        if d % 16 == 0 and dv % 16 == 0 and page_size % 4 == 0 and out.shape[1] % 4 == 0 and out_col % 4 == 0:
+        aligned = out.shape[1] % 4 == 0 and out_col % 4 == 0
+        if gate is not None:
+            aligned = aligned and gate[0].shape[1] % 4 == 0 and gate[1] % 4 == 0
+        if d % 16 == 0 and dv % 16 == 0 and page_size % 4 == 0 and aligned:
             attention_tile(q, k_cache, v_cache, out, ctx, block_table, page_size, nq, nkv, d, dv,
                            window, keep_first, sink, scale, sink_values, score_cap, slopes, log_distance,
-                           out_col, out_scale)
+                           out_col, out_scale, chunked, gate)
         else:
             attention_generic(
                 q, k_cache, v_cache, out, ctx.positions, ctx.token_slot, block_table, page_size,
                 nq, nkv, d, window, scale, ctx.max_position, dv, keep_first, sink, sink_values, score_cap, slopes,
-                log_distance, out_col, out_scale,
+                log_distance, out_col, out_scale, chunked, gate,
             )
         return
     if q.dtype == torch.float32 and d % 16 == 0:
@@ -2423,4 +2553,216 @@ def min_gru(packed: torch.Tensor, columns: tuple[int, int, int], z_bias: torch.T
                                     _column(out, out_col), out.shape[1], ctypes.c_float(out_scale), _p(ctx.cu_seqlens),
                                     _p(ctx.seq_slots), ctx.num_seqs, tokens, width, _tag(packed.dtype), _stream()),
         "rl_gru_scan",
+    )
+
+
+# --------------------------------------------------------------------------- #
+# linear attention with decays; attention heads behind short convolutions
+# --------------------------------------------------------------------------- #
+LINEAR_MAX_KEY_DIM = 256
+LINEAR_MAX_VALUE_DIM = 512
+LINEAR_CHUNK = 16  # tokens that the walk over a portion takes at a time
+LINEAR_MAX_RANK = 1024  # of the decays' low-rank pair
+
+
+def _linear_chunks(ctx):
+    """The step's chunk tables, made once a step and shared by its layers: per chunk (request,
+    first token, tokens, 0), per request (first chunk, chunks)."""
+    key = "linear_chunks"
+    found = ctx.extra.get(key) if hasattr(ctx, "extra") else None
+    if found is None:
+        chunks, per_seq, at = [], [], 0
+        for i, n in enumerate(ctx.h_seq_lens):
+            per_seq += [len(chunks) // 4, -(-n // LINEAR_CHUNK)]
+            for lo in range(0, n, LINEAR_CHUNK):
+                chunks += [i, at + lo, min(LINEAR_CHUNK, n - lo), 0]
+            at += n
+        dev = ctx.seq_slots.device
+        found = (upload_ints(chunks, dev), len(chunks) // 4, upload_ints(per_seq, dev))
+        if hasattr(ctx, "extra"):
+            ctx.extra[key] = found
+    return found
+
+
+class ChannelDecay:
+    """Decays of every key channel that depend on the token: ``sigmoid(z)^(1 / tau)`` with ``z = low W^T + bias``.
+    ``low`` (float32 ``[T, at least rank]``) are a token's inner values, ``out_t`` (float32 ``[rank, heads * d]``) is
+    ``W`` transposed, ``bias`` float32 ``[heads * d]``."""
+
+    def __init__(self, low: torch.Tensor, out_t: torch.Tensor, bias: torch.Tensor, tau: float) -> None:
+        self.low, self.out_t, self.bias, self.tau = low, out_t, bias, float(tau)
+
+    def args(self, tokens: int, heads: int, d: int) -> tuple:
+        rank = self.out_t.shape[0]
+        low = self.low
+        if not low.is_cuda or low.dtype != torch.float32 or low.dim() != 2 or low.shape[0] != tokens or low.stride(1) != 1:
+            raise KernelError(f"inner values of the decays must be float32 rows on the GPU, one a token, are {tuple(low.shape)}")
+        if low.shape[1] < rank or not 1 <= rank <= LINEAR_MAX_RANK:
+            raise KernelError(f"rows of {low.shape[1]} inner values for decays of rank {rank} (at most {LINEAR_MAX_RANK})")
+        _need(self.out_t, "decay matrix", torch.float32, (rank, heads * d))
+        _need(self.bias, "decay bias", torch.float32, (heads * d,))
+        if not self.tau > 0:
+            raise KernelError(f"decays are taken to the power 1 / {self.tau}")
+        return (_p(low), low.stride(0), rank, _p(self.out_t), _p(self.bias), ctypes.c_float(1.0 / self.tau), None)
+
+
+class FixedDecay:
+    """One decay a head, given as its logarithm (float32 ``[heads]``)."""
+
+    def __init__(self, log_decay: torch.Tensor) -> None:
+        self.log_decay = log_decay
+
+    def args(self, tokens: int, heads: int, d: int) -> tuple:
+        _need(self.log_decay, "logarithms of the decays", torch.float32, (heads,))
+        return (None, 0, 0, None, None, ctypes.c_float(0.0), _p(self.log_decay))
+
+
+def linear_attention(packed: torch.Tensor, columns: tuple[int, int, int, int], decay, norm_weight: torch.Tensor,
+                     out: torch.Tensor, ctx, S: torch.Tensor, heads: int, d: int, dv: int, q_scale: float, silu: bool,
+                     norm_parts: int, gate: str, eps: float, out_col: int = 0) -> None:
+    """Linear attention between its input projections and its output projection.  ``columns``: where the packed
+    rows hold ``q``, ``k`` (``heads * d`` each), ``v`` and the output gate (``heads * dv`` each); with ``silu`` q, k and v
+    pass it; q is multiplied by ``q_scale``.  ``decay`` (:class:`ChannelDecay` or :class:`FixedDecay`) gives ``a``.  Per
+    head, with the memory ``S [slots, heads, d, dv]`` (float32) read at the rows ``ctx.seq_slots`` and left after each
+    request's last token::
+
+        S <- diag(a) S + k v^T        o = S^T q
+
+    The columns of ``out`` from ``out_col`` on get ``o`` in ``norm_parts`` equal parts (``heads``, or 1 for the whole
+    row), each divided by its root mean square (``eps`` inside the root), times ``norm_weight`` (an entry a channel
+    of every head, or of one part for all), times ``silu`` or ``sigmoid`` of the gate.  A step of single tokens streams the memory
+    through once; portions are walked in chunks of 16 tokens (the two differ by rounding)."""
+    tokens, width = packed.shape
+    inner = heads * dv
+    if not 1 <= d <= LINEAR_MAX_KEY_DIM or not 1 <= dv <= LINEAR_MAX_VALUE_DIM:
+        raise KernelError(f"heads of {d} key and {dv} value channels (at most {LINEAR_MAX_KEY_DIM} and {LINEAR_MAX_VALUE_DIM})")
+    if norm_parts not in (1, heads) or gate not in HEAD_GATES:
+        raise KernelError(f"{norm_parts} normed parts of {heads} heads behind the gate {gate!r}")
+    _need(packed, "packed rows")
+    sizes = (heads * d, heads * d, inner, inner)
+    for name, col, size in zip(("q", "k", "v", "gate"), columns, sizes):
+        if col < 0 or col + size > width:
+            raise KernelError(f"columns {col}..{col + size} of {name} lie outside packed rows of {width}")
+    _need(S, "memory", torch.float32, (None, heads, d, dv))
+    part = inner // norm_parts
+    _need(norm_weight, "norm weight", torch.float32, (None,))
+    if norm_weight.shape[0] not in (part, inner):
+        raise KernelError(f"a norm of {norm_weight.shape[0]} entries for {norm_parts} parts of {part}")
+    shared = int(norm_weight.shape[0] == part)
+    _out_columns(out, packed.dtype, tokens, inner, out_col)
+    _step_requests(ctx, tokens, S.shape[0])
+    lib = linear_attention_lib()
+    q_col, k_col, v_col, g_col = (int(c) for c in columns)
+    decays = decay.args(tokens, heads, d)
+    source = (_p(packed), width, q_col, k_col, v_col, int(bool(silu)), ctypes.c_float(q_scale), *decays)
+    single = tokens == ctx.num_seqs
+    finish = single and norm_parts == heads
+    raw = None
+    if not finish:
+        raw = torch.empty((tokens, inner), dtype=torch.float32, device=packed.device)
+    if single:
+        _ok(
+            lib.rl_linear_step(
+                *source, _p(ctx.seq_slots), _p(S), _p(raw), int(finish), _p(norm_weight), shared, g_col,
+                HEAD_GATES[gate], ctypes.c_float(eps), _column(out, out_col), out.shape[1], tokens, heads, d, dv,
+                _tag(packed.dtype), _stream(),
+            ),
+            "rl_linear_step",
+        )
+        if finish:
+            return
+    else:
+        chunks, nchunks, seq_chunks = _linear_chunks(ctx)
+        rows = -(-d // 16) * 16
+        dev = packed.device
+        Q = torch.empty((nchunks, heads, LINEAR_CHUNK, rows), dtype=torch.float32, device=dev)
+        KT = torch.empty((nchunks, heads, rows, LINEAR_CHUNK), dtype=torch.float32, device=dev)
+        G = torch.empty((nchunks, heads, rows), dtype=torch.float32, device=dev)
+        A = torch.empty((nchunks, heads, LINEAR_CHUNK, LINEAR_CHUNK), dtype=torch.float32, device=dev)
+        _ok(
+            lib.rl_linear_scan(
+                *source, _p(chunks), nchunks, _p(ctx.cu_seqlens), _p(ctx.seq_slots), _p(seq_chunks), _p(Q), _p(KT), _p(G),
+                _p(A), _p(S), _p(raw), ctx.num_seqs, heads, d, dv, _tag(packed.dtype), _stream(),
+            ),
+            "rl_linear_scan",
+        )
+    _ok(
+        lib.rl_gated_norm(
+            _p(raw), _p(packed), width, g_col, _p(norm_weight), shared, HEAD_GATES[gate], ctypes.c_float(eps),
+            _column(out, out_col), out.shape[1], tokens, norm_parts, part, _tag(packed.dtype), _stream(),
+        ),
+        "rl_gated_norm",
+    )
+
+
+def conv_heads(packed: torch.Tensor, col0: int, bias: Optional[torch.Tensor], taps_t: Optional[torch.Tensor],
+               state: Optional[torch.Tensor], q_norm_w: Optional[torch.Tensor], k_norm_w: Optional[torch.Tensor], eps: float,
+               cos: Optional[torch.Tensor], sin: Optional[torch.Tensor], pairing: str, q_out: Optional[torch.Tensor],
+               k_cache: Optional[torch.Tensor], v_cache: Optional[torch.Tensor], ctx, block_table: torch.Tensor,
+               page_size: int, nq: int, nkv: int, d: int, dv: int) -> None:
+    """What attention behind short convolutions reads.  ``packed`` holds ``[q: nq * d | k: nkv * d | v: nkv * dv]`` from
+    column ``col0`` on; ``bias`` (float32, at least that many entries) is added.  With ``taps_t`` (float32 ``[taps, channels]``,
+    the last row meets the current token) every channel passes a causal convolution; inputs before a request's first
+    token of the step are its ``state`` rows (float32 ``[slots, max(taps - 1, 1), channels]``, oldest first), left holding
+    the last ``taps - 1`` (projected values with their bias).  With norm weights (float32 ``[nq * d]`` and ``[nkv * d]``) the whole
+    of q and the whole of k are divided by their root mean square (``eps`` inside the root) and multiplied by
+    them.  The first ``2 * cos.shape[1]`` channels of every head then rotate by the token's position.  ``q_out [T, nq * d]``
+    and the pages get the results (``None``: not written)."""
+    tokens, width = packed.shape
+    qk = (nq + nkv) * d
+    channels = qk + nkv * dv
+    if pairing not in ROTARY_PAIRINGS:
+        raise KernelError(f"rotation pairing {pairing!r} is not one of {sorted(ROTARY_PAIRINGS)}")
+    _need(packed, "packed rows")
+    if col0 < 0 or col0 + channels > width:
+        raise KernelError(f"{channels} columns from column {col0} lie outside rows of {width}")
+    if bias is not None:
+        _need(bias, "bias", torch.float32, (None,))
+        if bias.shape[0] < channels:
+            raise KernelError(f"a bias of {bias.shape[0]} entries does not cover {channels} columns")
+    taps = 0
+    if taps_t is not None:
+        taps = taps_t.shape[0]
+        _need(taps_t, "convolution taps", torch.float32, (taps, channels))
+        if not 1 <= taps <= CONV_MAX_TAPS:
+            raise KernelError(f"the convolution takes up to {CONV_MAX_TAPS} taps, got {taps}")
+        _need(state, "convolution state", torch.float32, (None, max(taps - 1, 1), channels))
+        _step_requests(ctx, tokens, state.shape[0])
+    if (q_norm_w is None) != (k_norm_w is None):
+        raise KernelError("queries and keys are normed alike")
+    if q_norm_w is not None:
+        _need(q_norm_w, "query norm weight", torch.float32, (nq * d,))
+        _need(k_norm_w, "key norm weight", torch.float32, (nkv * d,))
+    _need(ctx.positions, "positions", torch.int32, (tokens,))
+    _need(ctx.token_slot, "token_slot", torch.int32, (tokens,))
+    _need(block_table, "block_table", torch.int32)
+    if q_out is not None:
+        _need(q_out, "q_out", packed.dtype, (tokens, nq * d))
+    if k_cache is not None:
+        pages = k_cache.shape[0]
+        _need(k_cache, "k_cache", packed.dtype, (pages, nkv, page_size, d))
+        _need(v_cache, "v_cache", packed.dtype, (pages, nkv, dv, page_size))
+        if ctx.max_position // page_size >= block_table.shape[1]:
+            raise KernelError(
+                f"position {ctx.max_position} needs page {ctx.max_position // page_size} of a block table "
+                f"with {block_table.shape[1]} columns"
+            )
+    half = 0
+    if cos is not None:
+        half = cos.shape[1]
+        _need(cos, "cos table", torch.float32, (None, half))
+        _need(sin, "sin table", torch.float32, tuple(cos.shape))
+        if not 1 <= half <= d // 2 or ctx.max_position >= cos.shape[0]:
+            raise KernelError(
+                f"rotation tables of {half} pairs and {cos.shape[0]} positions for heads of {d} channels at "
+                f"position {ctx.max_position}"
+            )
+    _ok(
+        core().rl_conv_heads(
+            _column(packed, col0), width, _p(bias), _p(taps_t), _p(state), taps, _p(q_norm_w), _p(k_norm_w),
+            ctypes.c_float(eps), _p(cos), _p(sin), half, ROTARY_PAIRINGS[pairing], _p(q_out), _p(k_cache), _p(v_cache),
+            _p(ctx.positions), _p(ctx.token_slot), _p(block_table), block_table.stride(0), page_size, _p(ctx.cu_seqlens),
+            _p(ctx.seq_slots), ctx.num_seqs, tokens, nq, nkv, d, dv, _tag(packed.dtype), _stream(),
+        ),
+        "rl_conv_heads",
     )

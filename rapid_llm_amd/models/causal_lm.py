@@ -73,13 +73,15 @@ class CausalLM:
             mixer = MIXERS.create(
                 layer.mixer.kind, **layer.mixer.params, position=position, name=f"layers.{i}.mixer"
             )
-            if (layer.feed_forward is None) != (layer.feed_forward_norm is None):
+            alone = layer.shared_norm or layer.feed_forward is None
+            if alone != (layer.feed_forward_norm is None):
                 raise ValueError(f"layer {i}: a feed-forward and its norm come together or not at all")
             ff = n2 = None
             if layer.feed_forward is not None:
                 ff = FEED_FORWARDS.create(
                     layer.feed_forward.kind, **layer.feed_forward.params, name=f"layers.{i}.ff"
                 )
+            if layer.feed_forward_norm is not None:
                 n2 = NORMS.create(
                     layer.feed_forward_norm.kind, **layer.feed_forward_norm.params, name=f"layers.{i}.ff_norm"
                 )

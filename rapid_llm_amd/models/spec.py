@@ -43,6 +43,7 @@ class LayerSpec:
     position: PartSpec = PartSpec("none")
     checkpoint_prefix: str = ""
     share_cache_with: int | None = None  # index of the layer whose cache this one reads
+    shared_norm: bool = False  # both sub-layers read the mixer's norm (block kind "shared_norm")
     # norms behind the sub-layers, applied to their outputs before the add (a block kind that
     # has them, "sandwich", receives them; None: the block has none)
     mixer_post_norm: PartSpec | None = None

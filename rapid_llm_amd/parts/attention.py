@@ -34,6 +34,13 @@ taken off a scaled score.  ``query_temperature`` ``(coef, every)``: a finished q
 multiplied by ``1 + coef * ln(floor((p + 1) / every) + 1)``.  ``value_norm``: every value head is divided
 by its root mean square before it is cached (the epsilon is that of the query and key norm).
 
+``chunked``: the window does not slide; positions are cut into chunks of ``window`` from a request's first
+on, and a query sees the keys of its own chunk.  ``conv_taps``: every channel of q, k and v passes a short
+causal convolution behind the projection (with its bias), before norm and rotation; its last inputs are
+state of the request.  ``qk_norm_scope="projection"``: the norm of q and of k is one over all heads, with a
+weight a channel, instead of one a head.  ``gate_name``: the heads' outputs are multiplied, channel by
+channel, by the sigmoid of a projection of the mixer's input, which rides in the packed product.
+
 With these options the mixer is a :class:`~rapid_llm_amd.parts.base.PackedMixer`: it can run on columns of
 a product that another mixer shares (``packs``).
 """
@@ -45,7 +52,7 @@ import math
 import torch
 
 from ..kernels import ops
-from .base import MIXERS, CacheNeed, PackedMixer, ParamSpec, Source
+from .base import MIXERS, CacheNeed, PackedMixer, ParamSpec, Source, StateSpec
 from .linear import Linear
 
 
@@ -85,6 +92,11 @@ class GQAAttention(PackedMixer):
         log_distance_names: tuple[str, str] | None = None,
         query_temperature: tuple[float, float] | None = None,
         value_norm: bool = False,
+        chunked: bool = False,
+        conv_taps: int = 0,
+        conv_suffix: str = ".conv",
+        qk_norm_scope: str = "head",
+        gate_name: str | None = None,
     ) -> None:
         if num_heads % num_kv_heads:
             raise ValueError(f"{num_heads} query heads are not divisible by {num_kv_heads} kv heads")
@@ -125,6 +137,23 @@ class GQAAttention(PackedMixer):
         self.value_norm = bool(value_norm)
         if self.value_norm and (qk_norm_eps is None or values == "keys"):
             raise ValueError("normed values need a value projection and the epsilon of the query and key norm")
+        if qk_norm_scope not in ("head", "projection"):
+            raise ValueError(f"queries and keys are normed by 'head' or 'projection', not by {qk_norm_scope!r}")
+        self.chunked = bool(chunked)
+        if self.chunked and (window < 1 or self.keep_first):
+            raise ValueError(f"chunks of {window} positions with {keep_first} kept first positions")
+        if not 0 <= conv_taps <= ops.CONV_MAX_TAPS:
+            raise ValueError(f"the convolution's kernel takes up to {ops.CONV_MAX_TAPS} taps, got {conv_taps}")
+        self.taps, self.conv_suffix = int(conv_taps), conv_suffix
+        self.whole_norm = qk_norm_scope == "projection" and qk_norm_eps is not None
+        # the kernel that works on whole rows: convolution, norms over all heads
+        self.row_prepare = self.taps > 0 or self.whole_norm
+        if self.row_prepare and (values == "keys" or self.query_temperature or self.value_norm
+                                 or (qk_norm_eps is not None and not self.whole_norm)):
+            raise ValueError("short convolutions and norms over all heads come with values of their own, without norms a "
+                             "head, query temperature and normed values")
+        if gate_name is not None and head_gate_name:
+            raise ValueError("outputs pass one gate, of a head or of a channel")
         self.prefix = checkpoint_prefix
         self.qk_norm_eps = qk_norm_eps
         self.window = int(window)
@@ -143,7 +172,7 @@ class GQAAttention(PackedMixer):
         self.scale = float(softmax_scale) if softmax_scale is not None else 1.0 / math.sqrt(head_dim)
         self.name = name
         self.names = dict(q=q_name, k=k_name, v=v_name, o=o_name, qn=q_norm_name, kn=k_norm_name,
-                          g=head_gate_name)
+                          g=head_gate_name, og=gate_name)
         self.bias_names = dict(bias_names or {})
         self.values_are_keys = values == "keys"
         # the packed row: query heads, key heads, value heads unless they are the keys, then
@@ -151,15 +180,17 @@ class GQAAttention(PackedMixer):
         self.value_head0 = num_heads if self.values_are_keys else num_heads + num_kv_heads
         self.qkv_rows = (num_heads + num_kv_heads) * head_dim + (0 if self.values_are_keys else num_kv_heads * self.dv)
         self.gate_rows = num_heads if head_gate_name else 0
+        self.out_gate_rows = num_heads * self.dv if gate_name is not None else 0
         self.gate_pad = -(self.qkv_rows + self.gate_rows) % 8 if self.gate_rows else 0
         # the options that only the tile kernels (or the kernel for any size) take
         self.extended = (self.dv != head_dim or self.keep_first > 0 or self.sink or self.score_cap > 0
                          or self.slope_exponent is not None or self.log_distance_names is not None
-                         or self.query_temperature is not None or self.value_norm)
+                         or self.query_temperature is not None or self.value_norm or self.chunked or self.row_prepare
+                         or gate_name is not None)
         self.plain_row = not self.values_are_keys and not self.gate_rows and not self.extended
         self.packs = self.extended and not self.gate_rows
-        self.row_pad = -self.qkv_rows % 8 if (self.extended and not self.gate_rows) else 0
-        self.packed_rows = self.qkv_rows + self.gate_rows + self.gate_pad + self.row_pad
+        self.row_pad = -(self.qkv_rows + self.out_gate_rows) % 8 if (self.extended and not self.gate_rows) else 0
+        self.packed_rows = self.qkv_rows + self.out_gate_rows + self.gate_rows + self.gate_pad + self.row_pad
         self.inner_width = num_heads * self.dv
         self.qkv = Linear(hidden_size, self.packed_rows)
         self.o = Linear(num_heads * self.dv, hidden_size)
@@ -175,6 +206,8 @@ class GQAAttention(PackedMixer):
         packed = [Source(p + n["q"], self.nq * self.d), Source(p + n["k"], self.nkv * self.d)]
         if not self.values_are_keys:
             packed.append(Source(p + n["v"], self.nkv * self.dv))
+        if self.out_gate_rows:
+            packed.append(Source(p + n["og"], self.out_gate_rows))
         if self.gate_rows:
             packed.append(Source(p + n["g"], self.gate_rows))
         if self.gate_pad + self.row_pad:
@@ -201,11 +234,14 @@ class GQAAttention(PackedMixer):
         if self.log_distance_names is not None:
             specs += [ParamSpec(f"{self.name}.{which}", (self.nq,), "vector", (Source(p + source, self.nq),))
                       for which, source in zip(("r1", "r2"), self.log_distance_names)]
+        if self.taps:
+            channels = q_rows + kv_rows + v_rows
+            convolved = tuple(Source(p + n[s] + self.conv_suffix, rows) for s, rows in (("q", q_rows), ("k", kv_rows), ("v", v_rows)))
+            specs.append(ParamSpec(self.name + ".conv", (channels, self.taps), "vector", convolved))
         if self.qk_norm_eps is not None and self.qk_norm_weights:
-            specs += [
-                ParamSpec(self.name + ".q_norm", (self.d,), "vector", (Source(p + n["qn"], self.d),), init="norm"),
-                ParamSpec(self.name + ".k_norm", (self.d,), "vector", (Source(p + n["kn"], self.d),), init="norm"),
-            ]
+            for which, rows in (("q", q_rows), ("k", kv_rows)):
+                size = rows if self.whole_norm else self.d
+                specs.append(ParamSpec(f"{self.name}.{which}_norm", (size,), "vector", (Source(p + n[which + "n"], size),), init="norm"))
 
         def bias_of(which: str) -> str:
             if which in self.bias_names:
@@ -217,8 +253,9 @@ class GQAAttention(PackedMixer):
             biases = [Source(p + bias_of("q"), q_rows), Source(p + bias_of("k"), kv_rows)]
             if not self.values_are_keys:
                 biases.append(Source(p + bias_of("v"), v_rows))
-            if self.gate_rows + self.gate_pad + self.row_pad:
-                biases.append(Source("", self.gate_rows + self.gate_pad + self.row_pad))  # the gates have none
+            rest = self.out_gate_rows + self.gate_rows + self.gate_pad + self.row_pad
+            if rest:
+                biases.append(Source("", rest))  # the gates have none
             specs.append(ParamSpec(self.name + ".qkv_bias", (self.qkv.out_features,), "vector", tuple(biases)))
         if self.o_bias:
             specs.append(ParamSpec(
@@ -243,9 +280,13 @@ class GQAAttention(PackedMixer):
         if self.qk_norm_eps is not None and self.qk_norm_weights:
             self.q_norm_w = params[self.name + ".q_norm"]
             self.k_norm_w = params[self.name + ".k_norm"]
+        elif self.whole_norm:
+            self.q_norm_w, self.k_norm_w = (torch.ones(n * self.d, dtype=torch.float32, device=runtime.device) for n in (self.nq, self.nkv))
         elif self.qk_norm_eps is not None:
             # a norm without a learned weight: the kernels get a weight of ones
             self.q_norm_w = self.k_norm_w = torch.ones(self.d, dtype=torch.float32, device=runtime.device)
+        if self.taps:
+            self.conv_t = params[self.name + ".conv"].t().contiguous()  # neighbouring channels side by side
         if self.sink_name is not None:
             self.sink_values = params[self.name + ".sink"]
         if self.slope_exponent is not None:
@@ -255,8 +296,13 @@ class GQAAttention(PackedMixer):
 
     # ---- cache -----------------------------------------------------------------
     def cache_need(self) -> CacheNeed:
+        states = ()
+        if self.taps:
+            channels = (self.nq + self.nkv) * self.d + self.nkv * self.dv
+            states = (StateSpec("conv", (max(self.taps - 1, 1), channels), "float32"),)
         return CacheNeed.keys_and_values(
-            self.nkv, self.d, window=self.window, value_dim=self.dv, keep_first=self.keep_first
+            self.nkv, self.d, window=self.window, value_dim=self.dv, keep_first=self.keep_first, chunked=self.chunked,
+            states=states,
         )
 
     def recorded_step_bytes(self, rows: int, context_bound: int, page_size: int) -> int:
@@ -280,20 +326,26 @@ class GQAAttention(PackedMixer):
         eps = self.qk_norm_eps if self.qk_norm_eps is not None else 0.0
         table = ctx.block_tables[cache.group_id]
         q = torch.empty((packed.shape[0], self.nq * self.d), dtype=packed.dtype, device=packed.device)
-        ops.qknorm_rope_kvwrite(
-            packed, q,
-            cache.k if cache.owns_pages else None,
-            cache.v if cache.owns_pages else None,
-            self.q_norm_w, self.k_norm_w, cos, sin,
-            ctx.positions, ctx.token_slot, table, cache.page_size,
-            self.nq, self.nkv, self.d, eps, ctx.max_position, pairing, self.value_head0, self.bias_in_kernel,
-            self.dv, col0, self.query_temperature, self.value_norm,
-        )
+        pages = (cache.k, cache.v) if cache.owns_pages else (None, None)
+        if self.row_prepare:
+            ops.conv_heads(
+                packed, col0, self.bias_in_kernel, self.conv_t if self.taps else None, cache.states.get("conv"),
+                self.q_norm_w, self.k_norm_w, eps, cos, sin, pairing, q, *pages, ctx, table, cache.page_size,
+                self.nq, self.nkv, self.d, self.dv,
+            )
+        else:
+            ops.qknorm_rope_kvwrite(
+                packed, q, *pages, self.q_norm_w, self.k_norm_w, cos, sin,
+                ctx.positions, ctx.token_slot, table, cache.page_size,
+                self.nq, self.nkv, self.d, eps, ctx.max_position, pairing, self.value_head0, self.bias_in_kernel,
+                self.dv, col0, self.query_temperature, self.value_norm,
+            )
         ops.paged_attention(
             q, cache.k, cache.v, out, ctx, table, cache.page_size, self.nq, self.nkv, self.d, self.window, self.scale,
             value_dim=self.dv, keep_first=self.keep_first, sink=self.sink, sink_values=self.sink_values,
             score_cap=self.score_cap, slopes=self.slopes, log_distance=self.log_distance, out_col=out_col,
-            out_scale=out_scale,
+            out_scale=out_scale, chunked=self.chunked,
+            gate=(packed, col0 + self.qkv_rows) if self.out_gate_rows else None,
         )
 
     def forward(self, x, ctx, cache):

@@ -142,7 +142,9 @@ class CacheNeed:
     by a :class:`PagedSpec` (keys and values here; a mixer may name one latent row, or keys and
     values of different widths).  ``window`` 0 keeps every position, otherwise only the last
     ``window`` positions of a request are kept and older pages are given back, except the pages
-    of the first ``keep_first`` positions, which every later query still reads.
+    of the first ``keep_first`` positions, which every later query still reads.  ``chunked``: the window
+    does not slide; positions are cut into chunks of ``window`` from a request's first on, a query reads
+    its own chunk, and a chunk's pages are given back once it is complete.
     ``kind == "state"``: nothing paged.  Fixed-size per-request tensors the mixer owns, zeroed
     when a request takes the slot, may accompany either kind: one as ``state_shape`` (and
     ``state_dtype``), or several, each under a name, as ``states`` (a mixer with a short
@@ -159,8 +161,11 @@ class CacheNeed:
     state_dtype: str | None = None  # torch dtype name; None: the engine's compute type
     share_with: int | None = None
     states: tuple[StateSpec, ...] = ()
+    chunked: bool = False
 
     def __post_init__(self) -> None:
+        if self.chunked and (self.window < 1 or self.keep_first):
+            raise ValueError(f"chunks of {self.window} positions with {self.keep_first} kept first positions")
         if self.kind not in ("paged", "state", "none"):
             raise ValueError(f"a cache need is 'paged', 'state' or 'none', not {self.kind!r}")
         if self.keep_first < 0 or self.window < 0:

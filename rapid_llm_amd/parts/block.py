@@ -1,6 +1,8 @@
 """Pre-norm arrangement: ``r += mixer(norm(r)); r += feed_forward(norm(r))``; a layer
 without a feed-forward has the first sub-layer only.  The sandwich arrangement has a second
-norm behind each sub-layer, applied to its output before the add.
+norm behind each sub-layer, applied to its output before the add.  In the parallel and the
+shared-norm arrangement both sub-layers read the same stream, through norms of their own or
+through one.
 
 The add of each sub-layer's output is carried forward as ``delta`` and happens inside the
 next norm kernel, as the reference threads ``(hidden, residual)`` through its layers
@@ -10,7 +12,7 @@ next norm kernel, as the reference threads ``(hidden, residual)`` through its la
 from __future__ import annotations
 
 from .base import BLOCKS, Block
-from .lazy import NormedDelta, SummedDeltas, plain, run_norm
+from .lazy import LayerSum, NormedDelta, SummedDeltas, plain, run_norm
 
 
 class PreNormBlock(Block):
@@ -111,6 +113,37 @@ class ParallelBlock(Block):
         return SummedDeltas(a, b)
 
 
+class SharedNormBlock(Block):
+    """One norm, whose output both sub-layers read: with ``h = norm(r)``,
+    ``r += factor * (mixer(h) + feed_forward(h))``.  What the two return travels on as one pending
+    :class:`~rapid_llm_amd.parts.lazy.LayerSum`, which the norm that runs next adds in its own kernel."""
+
+    replayable = True
+    accepts_deferred = True
+    shares_norm = True  # there is no norm in front of the feed-forward
+
+    def __init__(self, mixer, feed_forward, mixer_norm, feed_forward_norm=None, factor: float = 1.0) -> None:
+        if feed_forward_norm is not None:
+            raise ValueError("both sub-layers read the output of one norm")
+        self.mixer = mixer
+        self.feed_forward = feed_forward
+        self.mixer_norm = mixer_norm
+        self.factor = float(factor)
+
+    def parts(self):
+        if self.feed_forward is None:
+            return (self.mixer_norm, self.mixer)
+        return (self.mixer_norm, self.mixer, self.feed_forward)
+
+    def forward(self, residual, delta, ctx, cache):
+        h = plain(run_norm(self.mixer_norm, residual, delta, ctx))
+        outputs = [self.mixer.forward(h, ctx, cache)]
+        if self.feed_forward is not None:
+            outputs.append(self.feed_forward.forward(h, ctx))
+        return LayerSum.of(outputs, self.factor)
+
+
 BLOCKS.register("parallel", ParallelBlock)
 BLOCKS.register("prenorm", PreNormBlock)
 BLOCKS.register("sandwich", SandwichBlock)
+BLOCKS.register("shared_norm", SharedNormBlock)

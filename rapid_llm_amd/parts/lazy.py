@@ -24,6 +24,12 @@ products on either side absorb it, without any part knowing its neighbours:
   type adds both into the stream in the kernel that computes its own rows; anything else gets
   their sum joined to the stream first (``add_to``) or as a tensor (``materialize``).
 
+* :class:`LayerSum`: what a block whose two sub-layers read the same rows returns where their outputs are
+  more than two tensors: some pass a norm of their own first, some are the input times a number a token,
+  and the sum has a factor.  Sub-layers contribute a tensor, a :class:`DeferredProduct` or their own
+  :class:`LayerSum`.  A norm that declares ``fuses_products`` and knows the type adds everything in the
+  kernel that computes its own rows; anything else gets the sum joined to the stream first.
+
 Blocks and models route these only between parts that declare them (``fuses_products`` on
 a norm, ``accepts_scaled_rows`` on a mixer or feed-forward, ``accepts_deferred`` on a
 block); everything else sees plain tensors.
@@ -48,6 +54,10 @@ class DeferredProduct:
 
     def materialize(self, out_dtype: torch.dtype | None = None) -> torch.Tensor:
         return self.linear(self.x, out_dtype)
+
+    def term(self, weight: torch.Tensor | None = None) -> "Term":
+        """The product as a term of a :class:`LayerSum`, which adds its bias."""
+        return Term(self.linear.product(self.x), self.linear.bias, weight)
 
 
 class NormedDelta:
@@ -104,6 +114,74 @@ class SummedDeltas:
         return out
 
 
+@dataclass(frozen=True)
+class Term:
+    """A sub-layer's output on its way into the stream: ``y (+ bias)``, with ``weight`` normed by its root mean
+    square and multiplied by that weight."""
+
+    y: Any  # [T, hidden] tensor
+    bias: torch.Tensor | None = None
+    weight: torch.Tensor | None = None
+
+
+@dataclass(frozen=True)
+class Returned:
+    """The sub-layer's input ``x`` times one number a token, ``numbers[t, column]``."""
+
+    x: Any
+    numbers: torch.Tensor
+    column: int
+
+
+class LayerSum:
+    """``factor * (sum of terms + returned)``, not yet added; ``eps`` is that of the normed terms."""
+
+    def __init__(self, terms, returned: Returned | None = None, factor: float = 1.0, eps: float = 0.0) -> None:
+        self.terms, self.returned = list(terms), returned
+        self.factor, self.eps = float(factor), float(eps)
+
+    @classmethod
+    def of(cls, parts, factor: float) -> "LayerSum":
+        """The sum of what several sub-layers return, times ``factor``."""
+        terms, returned, eps = [], None, 0.0
+        for part in parts:
+            if isinstance(part, LayerSum):
+                if part.factor != 1.0 or (part.returned is not None and returned is not None):
+                    raise ValueError("sums of sub-layers nest once, with one returned input")
+                normed = any(t.weight is not None for t in part.terms)
+                if normed and eps and part.eps != eps:
+                    raise ValueError("normed terms of one sum share an epsilon")
+                terms += part.terms
+                returned = part.returned or returned
+                eps = part.eps if normed else eps
+            elif isinstance(part, DeferredProduct):
+                terms.append(part.term())
+            else:
+                terms.append(Term(plain(part)))
+        return cls(terms, returned, factor, eps)
+
+    @property
+    def shape(self):
+        return self.terms[0].y.shape
+
+    def run(self, residual: torch.Tensor, **norm) -> None:
+        """``residual += the sum`` in place (float32), and the norm behind it where one is given
+        (``weight``, ``out``, ``eps``, ``rows`` of :func:`~rapid_llm_amd.kernels.ops.sublayer_sum_norm`)."""
+        from ..kernels import ops
+
+        returned = self.returned and (self.returned.x, self.returned.numbers, self.returned.column)
+        ops.sublayer_sum_norm(residual, [(t.y, t.bias, t.weight) for t in self.terms], self.factor, self.eps, returned, **norm)
+
+    add_to = run
+
+    def materialize(self, out_dtype: torch.dtype | None = None) -> torch.Tensor:
+        """The sum as a float32 tensor."""
+        y = self.terms[0].y
+        out = torch.zeros(y.shape, dtype=torch.float32, device=y.device)
+        self.run(out)
+        return out
+
+
 @dataclass
 class ScaledRows:
     rows: torch.Tensor  # [M, size], the residual rows times the norm's weight
@@ -126,13 +204,13 @@ class ScaledRows:
 
 def plain(value):
     """A tensor, whatever lazy value it still was."""
-    return value.materialize() if isinstance(value, (DeferredProduct, NormedDelta, SummedDeltas)) else value
+    return value.materialize() if isinstance(value, (DeferredProduct, NormedDelta, SummedDeltas, LayerSum)) else value
 
 
 def settle(residual, delta):
     """What is left to add once lazy values are settled: a pending normed delta joins the stream
     now, a deferred product becomes a tensor."""
-    if isinstance(delta, (NormedDelta, SummedDeltas)):
+    if isinstance(delta, (NormedDelta, SummedDeltas, LayerSum)):
         delta.add_to(residual)
         return None
     return plain(delta)
@@ -144,7 +222,7 @@ def run_norm(norm, residual, delta, ctx, consumer=None, rows=None):
         return norm.forward(
             residual, delta, ctx, rows, scaled_ok=bool(getattr(consumer, "accepts_scaled_rows", False))
         )
-    if isinstance(delta, (NormedDelta, SummedDeltas)):
+    if isinstance(delta, (NormedDelta, SummedDeltas, LayerSum)):
         # a norm that knows nothing of it: the stream takes it first
         delta.add_to(residual)
         delta = None

@@ -19,7 +19,7 @@ import torch
 
 from ..kernels import ops
 from .base import FEED_FORWARDS, FeedForward, ParamSpec, Source
-from .lazy import ScaledRows
+from .lazy import LayerSum, Returned, ScaledRows, Term, plain
 from .linear import Linear
 
 
@@ -172,6 +172,12 @@ class RoutedExperts(FeedForward):
     weight multiplies what the expert reads, not what it returns; its first products being linear,
     the gate and up values are multiplied by it before they are clamped.
 
+    ``scores="softmax_raw"``: the chosen experts' weights are their softmax scores over all experts as they
+    are (times ``route_scale``).  With it, ``correction_name``: a number an expert, added to the scores for the
+    choice alone; ``identity`` more experts, behind the others in the router, have no tensors and return
+    their input; ``shared_gate_name``: the shared expert's output is multiplied by the sigmoid of a product of
+    one row, which rides in the router's matrix.
+
     The router's product and scores are float32 in every engine (its matrix is held in
     float32).  The experts' up projections are one packed matrix ``[experts * expert_size +
     shared_size, hidden]`` and their down projections one matrix side by side over the same
@@ -206,10 +212,22 @@ class RoutedExperts(FeedForward):
         alpha: float = ops.GLU_ALPHA,
         scores: str = "softmax",
         weights_scale: str = "output",
+        identity: int = 0,
+        correction_name: str | None = None,
+        shared_gate_name: str | None = None,
     ) -> None:
         self.gated = bool(gated)
-        if scores not in ops.ROUTER_SCORES:
-            raise ValueError(f"router scores are one of {sorted(ops.ROUTER_SCORES)}, not {scores!r}")
+        self.raw_scores = scores == "softmax_raw"
+        if scores not in ops.ROUTER_SCORES and not self.raw_scores:
+            raise ValueError(f"router scores are one of {sorted(ops.ROUTER_SCORES)} or 'softmax_raw', not {scores!r}")
+        if self.raw_scores and (gated or router_bias_name):
+            raise ValueError("raw scores come with experts that have no gate and a router without a bias")
+        if (identity or correction_name or shared_gate_name) and not self.raw_scores:
+            raise ValueError("identity experts, a correction and a shared expert's gate come with raw scores")
+        if identity < 0 or (shared_gate_name and not shared_size):
+            raise ValueError(f"{identity} identity experts, a gate {shared_gate_name!r} of a shared expert of {shared_size} units")
+        self.identity, self.correction_name, self.shared_gate_name = int(identity), correction_name, shared_gate_name
+        self.correction = None
         if weights_scale not in ("output", "input") or (weights_scale == "input" and not gated):
             raise ValueError(f"an expert's weight scales its 'output', or the 'input' of a gated expert, not {weights_scale!r}")
         if limit < 0 or (limit and not gated):
@@ -223,15 +241,16 @@ class RoutedExperts(FeedForward):
             raise ValueError(f"activation {activation!r} is not one of {sorted(ops.UNARY_ACTIVATIONS)}")
         self.gate_name, self.router_bias_name = gate_name, router_bias_name
         self.router_bias = None
-        if not 1 <= top <= num_experts <= ops.ROUTE_MAX_EXPERTS:
-            raise ValueError(f"a token uses 1 to {num_experts} of at most {ops.ROUTE_MAX_EXPERTS} experts, not {top}")
+        choices = num_experts + self.identity
+        if num_experts < 1 or not 1 <= top <= choices <= ops.ROUTE_MAX_EXPERTS:
+            raise ValueError(f"a token uses 1 to {choices} of at most {ops.ROUTE_MAX_EXPERTS} experts, not {top}")
         self.hidden_size, self.num_experts, self.top = hidden_size, num_experts, top
         self.expert_size, self.shared_size = expert_size, shared_size
         self.route_scale = float(route_scale)
         self.prefix, self.activation, self.name = checkpoint_prefix, activation, name
         self.names = (router_name, expert_prefix, shared_prefix, up_name, down_name)
         self.inner = num_experts * expert_size + shared_size
-        self.router = Linear(hidden_size, num_experts)
+        self.router = Linear(hidden_size, choices + (1 if shared_gate_name else 0))
         self.up = Linear(hidden_size, (2 if self.gated else 1) * self.inner)
         self.down = Linear(self.inner, hidden_size)
 
@@ -248,9 +267,12 @@ class RoutedExperts(FeedForward):
         first = self._sources(up, self.expert_size, self.shared_size)
         if self.gated:  # [every gate | every up]
             first = self._sources(self.gate_name, self.expert_size, self.shared_size) + first
+        choices = self.num_experts + self.identity
+        routed = [Source(self.prefix + router, choices)]
+        if self.shared_gate_name:
+            routed.append(Source(self.prefix + self.shared_gate_name, 1))
         specs = [
-            ParamSpec(self.name + ".router", (self.num_experts, h), "matrix_f32",
-                      (Source(self.prefix + router, self.num_experts),)),
+            ParamSpec(self.name + ".router", (self.router.out_features, h), "matrix_f32", tuple(routed)),
             ParamSpec(self.name + ".up", (self.up.out_features, h), "matrix", first),
             ParamSpec(self.name + ".down", (h, self.inner), "matrix",
                       self._sources(down, self.expert_size, self.shared_size), axis=1),
@@ -258,9 +280,14 @@ class RoutedExperts(FeedForward):
         if self.router_bias_name:
             specs.append(ParamSpec(self.name + ".router_bias", (self.num_experts,), "vector",
                                    (Source(self.prefix + self.router_bias_name, self.num_experts),)))
+        if self.correction_name:
+            specs.append(ParamSpec(self.name + ".correction", (choices,), "vector",
+                                   (Source(self.prefix + self.correction_name, choices),)))
         return specs
 
     def bind(self, params, runtime) -> None:
+        if self.correction_name:
+            self.correction = params[self.name + ".correction"]
         if self.router_bias_name:
             self.router_bias = params[self.name + ".router_bias"]
         self.router.bind(params[self.name + ".router"])
@@ -268,6 +295,16 @@ class RoutedExperts(FeedForward):
         self.down.bind(params[self.name + ".down"])
 
     def forward(self, x, ctx):
+        if self.raw_scores:
+            weights = ops.choose_experts(x, self.router.weight, self.num_experts, self.identity, self.top, self.route_scale,
+                                         self.correction, self.shared_gate_name is not None)
+            hidden = self.up(x)
+            ops.unary_act(hidden, hidden, self.activation, weights, self.expert_size, self.num_experts)
+            y = self.down.deferred(hidden, ctx)
+            if not self.identity:
+                return y
+            # the identity experts' output, the input times their weights, joins the stream where y does
+            return LayerSum([Term(plain(y))], Returned(x, weights, self.num_experts + 1))
         # float32 throughout
         weights = ops.router(x, self.router.weight, self.top, self.route_scale, self.router_bias, self.scores)
         hidden = self.up(x)

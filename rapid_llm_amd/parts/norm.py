@@ -12,7 +12,7 @@ import torch
 
 from ..kernels import ops
 from .base import NORMS, Norm, ParamSpec, Source
-from .lazy import DeferredProduct, NormedDelta, SummedDeltas, plain
+from .lazy import DeferredProduct, LayerSum, NormedDelta, SummedDeltas, plain
 
 
 class RMSNorm(Norm):
@@ -62,6 +62,11 @@ class RMSNorm(Norm):
             if y.dtype != self.dtype:
                 y = y.to(self.dtype)
             ops.normed_add_rmsnorm(residual, y, delta.weight, delta.eps, self.weight, out, self.eps, rows)
+            return out
+        if isinstance(delta, LayerSum):
+            n = residual.shape[0] if rows is None else rows.numel()
+            out = torch.empty((n, self.size), dtype=self.dtype, device=residual.device)
+            delta.run(residual, weight=self.weight, out=out, eps=self.eps, rows=rows)
             return out
         if isinstance(delta, SummedDeltas):
             delta.add_to(residual)
@@ -131,7 +136,7 @@ class LayerNorm(Norm):
         d1 = d2 = None
         if isinstance(delta, SummedDeltas):
             d1, d2 = delta.tensors()
-        elif isinstance(delta, NormedDelta):
+        elif isinstance(delta, (NormedDelta, LayerSum)):
             delta.add_to(residual)
         else:
             d1 = plain(delta)
