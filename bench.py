@@ -3,7 +3,7 @@
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--layers L] [--dtype bfloat16]
                     [--shape NAME] [--batch B] [--prompt-len T] [--context C]
     python bench.py --workload qwen3-0.6b-256 | qwen3-32b-32
-    python bench.py --design fokulorn|sikevik|miborax|fomunex|pefulorn [--design-size 2b,8b]
+    python bench.py --design fokulorn|sikevik|miborax|fomunex|pefulorn|renitar [--design-size 2b,8b]
 
 A "step" is one decode step of the whole batch through the engine's step function and the
 greedy sampling kernel, tokens fed back.  The default run has the layer sizes of
@@ -54,6 +54,13 @@ term beside a gated recurrence, a token-shift time mixing, a delta rule with a d
 behind short convolutions; gated feed-forwards with biases; two of six layers run twice), beside
 the Fomunex decoder, the engine's closest (the same time mixing, a recurrence behind a short
 convolution, attention with a distance term), and Qwen3 of equal size.
+
+``--design renitar`` does the same for the Renitar decoder (gated linear attention with a decay per
+key channel; attention in chunks behind short convolutions beside lightning attention, each normed
+before half of their sum is taken; mixtures of sixteen ungated experts, four that return their input
+and a gated shared one; one norm a layer), beside the Pefulorn decoder, the engine's closest (two
+mixers side by side, a recurrence with a decay per key channel behind short convolutions), and
+Qwen3 of equal size.
 
 Metric definitions follow rapid_llm's docs/benchmark_models.md:141-149: decode tok/s is
 batch / mean step time; prefill tok/s is prompt tokens / prefill latency; both timed
@@ -923,6 +930,132 @@ def _time_pefulorn_kernels(z: dict, prompt_len: int, batch: int) -> dict:
     return out
 
 
+def renitar_body(z: dict) -> dict:
+    """Gated linear attention and the pair in turn, all heads of 128 channels, the lightning attention as wide as
+    the model; sixteen experts of a sixteenth of Qwen3's feed-forward width and a shared one of half of it, so
+    that a layer's feed-forward matrices hold what Qwen3's three do."""
+    w, ff, heads = z["width"], z["ff"], z["width"] // 128
+    gla = {"heads": heads, "dim": 128, "vdim": 128, "tau": 16.0, "rank": 16}
+    left = {"heads": z["heads"], "kv_heads": z["kv_heads"], "dim": z["head_dim"], "vdim": z["head_dim"], "conv": 4,
+            "scale": z["head_dim"] ** -0.5, "softcap": 20.0, "mask": {"size": z["window"] * 3 // 2},
+            "rot": {"base": 500000.0, "dims": z["head_dim"] // 4}}
+    right = {"heads": heads, "dim": 128, "vdim": 128, "decay": [1.0 - 2.0 ** -(1 + 8 * h / heads) for h in range(heads)]}
+    mlp = {"kind": "moe", "expert": {"ff": ff // 16}, "router": {"experts": 16, "identity": 4, "top": 3, "scale": 2.0},
+           "shared": {"ff": ff // 2}}
+    kinds = [("gla", gla), ("parallel", {"left": left, "right": right})]
+    layers = [{"type": kinds[i % 2][0], "mixer": kinds[i % 2][1], "mlp": mlp} for i in range(z["layers"])]
+    return {"architecture": "Renitar", "width": w, "vocab": z["vocab"], "norm": {"eps": 1e-6}, "residual_mult": 0.5,
+            "layers": layers}
+
+
+def _time_renitar_kernels(z: dict, prompt_len: int, batch: int) -> dict:
+    """The design's own kernels alone, microseconds and share of the roofline each, over one prompt and over
+    ``batch`` single tokens, beside the like kernels of the engine's other designs on the same operands:
+    linear attention with its norm and gate, decays a channel and fixed (float32 operations: four a memory
+    element and token over a prompt; bytes of memory for single tokens); the heads behind short
+    convolutions, the router, the weighed exact gelu, the norm that adds a layer's outputs (bytes); and
+    attention in chunks with cap and gate, and without them (matrix rate over the keys every query
+    sees; bytes of keys and values for single tokens in the middle of a chunk)."""
+    import types
+
+    import torch
+
+    from rapid_llm_amd.kernels import ops
+
+    dev, width, bf, ff = "cuda", z["width"], torch.bfloat16, z["ff"]
+    nq, nkv, dh, chunk = z["heads"], z["kv_heads"], z["head_dim"], z["window"] * 3 // 2
+    out: dict = {}
+
+    def rate(name, sec, frac_of, value):
+        out[name + "_us"] = round(sec * 1e6, 1)
+        out[f"{name}_frac_{frac_of}"] = round(value, 4)
+
+    def hbm(count, sec):
+        return count / sec / 1e9 / HBM_GBPS
+
+    def fp32(ops_count, sec):
+        return ops_count / sec / (PEAK_TFLOPS["float32"] * 1e12)
+
+    def rows(*shape, scale=1.0):
+        return (torch.randn(*shape, device=dev) * scale).to(bf)
+
+    for what, lens in (("prefill", [prompt_len]), ("decode", [1] * batch)):
+        tokens, single = sum(lens), what == "decode"
+        n = len(lens)
+        cu = torch.tensor([0] + list(torch.tensor(lens).cumsum(0)), dtype=torch.int32, device=dev)
+        slots = torch.arange(n, dtype=torch.int32, device=dev)
+        positions = torch.full((n,), prompt_len, dtype=torch.int32, device=dev) if single else torch.arange(tokens, dtype=torch.int32, device=dev)
+        ctx = types.SimpleNamespace(num_seqs=n, h_seq_lens=list(lens), h_seq_slots=list(range(n)), cu_seqlens=cu, seq_slots=slots,
+                                    positions=positions, token_slot=slots if single else torch.zeros(tokens, dtype=torch.int32, device=dev),
+                                    max_position=prompt_len, extra={}, static={})
+        # ---- linear attention
+        h, d = width // 128, 128
+        inner = h * d
+        packed = rows(tokens, 4 * inner, scale=0.5)
+        S, nw_head, nw_row = torch.zeros((batch, h, d, d), device=dev), torch.ones(d, device=dev), torch.ones(inner, device=dev)
+        o = torch.empty((tokens, inner), dtype=bf, device=dev)
+        channel = ops.ChannelDecay(torch.randn(tokens, 16, device=dev), torch.randn(16, inner, device=dev) * 0.25,
+                                   torch.randn(inner, device=dev), 16.0)
+        fixed = ops.FixedDecay(torch.full((h,), -0.02, device=dev))
+        cols = (0, inner, 2 * inner, 3 * inner)
+        for label, decay, norm, more in (("linear_attention_channel_decay", channel, nw_head, (128 ** -0.5, False, h, "silu")),
+                                         ("linear_attention_fixed_decay", fixed, nw_row, (1.0, True, 1, "sigmoid"))):
+            sec = _time_calls(lambda: ops.linear_attention(packed, cols, decay, norm, o, ctx, S, h, d, d, *more, 1e-6), single)
+            if single:
+                rate(f"{label}_decode", sec, "hbm", hbm(2.0 * batch * h * d * d * 4, sec))
+            else:
+                rate(f"{label}_prefill", sec, "fp32_matrix", fp32(tokens * h * 4.0 * d * d, sec))
+        # ---- heads behind short convolutions
+        own = (nq + 2 * nkv) * dh
+        pk = rows(tokens, own + nq * dh)
+        page, pages = 16, -(-(prompt_len + 1) // 16)
+        table = torch.arange(1, 1 + batch * pages, dtype=torch.int32, device=dev).view(batch, pages)
+        kc, vc = (torch.zeros(s, dtype=bf, device=dev) for s in ((1 + batch * pages, nkv, page, dh), (1 + batch * pages, nkv, dh, page)))
+        taps, conv_state, bias = torch.randn(4, own, device=dev), torch.zeros((batch, 3, own), device=dev), torch.zeros(own, device=dev)
+        qn, kn = torch.ones(nq * dh, device=dev), torch.ones(nkv * dh, device=dev)
+        angles = torch.randn(prompt_len + 1, dh // 8, device=dev)
+        qo = torch.empty((tokens, nq * dh), dtype=bf, device=dev)
+        sec = _time_calls(lambda: ops.conv_heads(pk, 0, bias, taps, conv_state, qn, kn, 1e-6, angles.cos(), angles.sin(), "half_split",
+                                                 qo, kc, vc, ctx, table, page, nq, nkv, dh, dh), single)
+        rate(f"convolved_heads_{what}", sec, "hbm", hbm(tokens * own * (2 + 2) + (2 * n * 3 * own * 4 if single else 0), sec))
+        # ---- router, experts' activation, the norm that adds a layer
+        x = rows(tokens, width)
+        rw, corr = torch.randn(21, width, device=dev) * 0.02, torch.zeros(20, device=dev)
+        rwb = rw.to(bf)
+        sec = _time_calls(lambda: ops.choose_experts(x, rwb, 16, 4, 3, 2.0, corr, True), single)
+        rate(f"router_{what}", sec, "hbm", hbm(tokens * (width * 2 + 18 * 4) + 21 * width * 4, sec))
+        rw8 = rw[:8].contiguous()
+        sec = _time_calls(lambda: ops.router(x, rw8, 2, 1.0), single)
+        rate(f"router_of_8_other_designs_{what}", sec, "hbm", hbm(tokens * (width * 2 + 8 * 4) + 8 * width * 4, sec))
+        weights = ops.choose_experts(x, rwb, 16, 4, 3, 2.0, corr, True)
+        hidden = rows(tokens, ff + ff // 2)
+        sec = _time_calls(lambda: ops.unary_act(hidden, hidden, "gelu", weights, ff // 16, 16), single)
+        rate(f"weighed_gelu_{what}", sec, "hbm", hbm(tokens * (ff + ff // 2) * 4, sec))
+        weights16 = weights[:, :16].contiguous()
+        sec = _time_calls(lambda: ops.unary_act(hidden, hidden, "gelu_tanh", weights16, ff // 16), single)
+        rate(f"weighed_gelu_tanh_other_designs_{what}", sec, "hbm", hbm(tokens * (ff + ff // 2) * 4, sec))
+        stream, wn, y = torch.randn(tokens, width, device=dev), torch.ones(width, device=dev), [rows(tokens, width) for _ in range(3)]
+        ob = torch.empty((tokens, width), dtype=bf, device=dev)
+        for label, terms in (("pair", [(y[0], wn, wn), (y[1], None, wn), (y[2], None, None)]), ("one", [(y[0], None, None), (y[2], None, None)])):
+            sec = _time_calls(lambda: ops.sublayer_sum_norm(stream, terms, 0.5, 1e-6, (x, weights, 17), wn, ob, 1e-6), single)
+            rate(f"layer_sum_norm_{label}_{what}", sec, "hbm", hbm(tokens * width * (8 + 2 * len(terms) + 2 + 2), sec))
+        sec = _time_calls(lambda: ops.add_rmsnorm(stream, y[0], wn, ob, 1e-6), single)
+        rate(f"add_norm_other_designs_{what}", sec, "hbm", hbm(tokens * width * (8 + 2 + 2), sec))
+    # ---- attention
+    seen = sum(p % chunk + 1 for p in range(prompt_len))
+    middle = prompt_len + chunk // 2
+    gates = {True: rows(prompt_len, nq * dh), False: rows(batch, nq * dh)}
+    for label, own in (("", True), ("_sliding_without_cap_and_gate", False)):
+        def more(prompt):
+            return dict(chunked=True, score_cap=20.0, gate=(gates[prompt], 0)) if own else dict(sink=True)
+        sec = _time_attention(z, chunk, [(0, prompt_len)], **more(True))
+        pairs = seen if own else sum(min(p + 1, chunk) for p in range(prompt_len))
+        rate(f"attention_prefill{label}", sec, "bf16_matrix", 4.0 * nq * dh * pairs / sec / (PEAK_TFLOPS["bfloat16"] * 1e12))
+        sec = _time_attention(z, chunk, [(middle, 1)] * batch, **more(False))
+        rate(f"attention_decode{label}", sec, "hbm", hbm(batch * (middle % chunk + 1 if own else chunk) * nkv * dh * 2 * 2, sec))
+    return out
+
+
 # design -> (name, its configuration at a size, its kernels alone, the engine's closest other
 # architecture measured beside it and Qwen3)
 DESIGNS = {
@@ -931,6 +1064,7 @@ DESIGNS = {
     "miborax": ("Miborax", miborax_body, _time_miborax_kernels, ("sikevik", sikevik_body)),
     "fomunex": ("Fomunex", fomunex_body, _time_fomunex_kernels, ("fokulorn", fokulorn_body)),
     "pefulorn": ("Pefulorn", pefulorn_body, _time_pefulorn_kernels, ("fomunex", fomunex_body)),
+    "renitar": ("Renitar", renitar_body, _time_renitar_kernels, ("pefulorn", pefulorn_body)),
 }
 
 
@@ -988,7 +1122,7 @@ def main() -> int:
     ap.add_argument("--peaks", action="store_true",
                     help="measure what the device reaches with library kernels (a large read, copy and square products) and exit")
     ap.add_argument("--design", default=None,
-                    help="measure another architecture of the engine beside Qwen3 at equal size (fokulorn, sikevik, miborax, fomunex, pefulorn) and exit")
+                    help="measure another architecture of the engine beside Qwen3 at equal size (fokulorn, sikevik, miborax, fomunex, pefulorn, renitar) and exit")
     ap.add_argument("--design-size", default="2b,8b", help=f"sizes for --design: {', '.join(DESIGN_SIZES)}")
     args = ap.parse_args()
     if args.peaks:

@@ -11,10 +11,13 @@
 // oldest first, zeros when the request begins; they are left holding the last taps - 1 inputs
 // (by a second launch, after every read; in a step of single tokens by the token's own workgroup).
 //
-// A workgroup takes TT consecutive tokens of the flat batch, VEC adjacent channels a thread at a
-// time.  With TAPS > 0 the inputs that the next token needs again stay in registers.  The convolved
-// q and k wait in LDS for their norms.  Cache layout: keys [page][nkv][P][d], values
-// [page][nkv][dv][P].
+// A workgroup takes the queries and keys of TT consecutive tokens of the flat batch, VEC adjacent
+// channels a thread at a time; with TAPS > 0 the inputs that the next token needs again stay in
+// registers, and the convolved q and k wait in LDS for their norms.  The values have neither norm
+// nor rotation.  In a step of portions (TT = 4) they are further workgroups of the same launch, of 16
+// tokens each: four neighbouring threads take four tokens each of the same channels, so that the
+// sixteen places of a channel in a page (which are contiguous) are written together.  Cache layout:
+// keys [page][nkv][P][d], values [page][nkv][dv][P].
 #include "common.h"
 
 namespace conv_heads {
@@ -44,6 +47,8 @@ __device__ inline int request_of(const int* __restrict__ cu, int num_seqs, int t
     return lo;
 }
 
+constexpr int VALUE_TOKENS = 16;  // of a workgroup of values
+
 template <typename T, int VEC, int TT, int TAPS>
 __global__ __launch_bounds__(1024) void prepare_kernel(
     const T* __restrict__ packed, const float* __restrict__ bias, const float* __restrict__ taps_t,
@@ -51,81 +56,97 @@ __global__ __launch_bounds__(1024) void prepare_kernel(
     const float* __restrict__ cos_tab, const float* __restrict__ sin_tab, T* __restrict__ q_out,
     T* __restrict__ k_cache, T* __restrict__ v_cache, const int* __restrict__ positions,
     const int* __restrict__ token_slot, const int* __restrict__ block_table, const int* __restrict__ cu, int num_seqs,
-    int tokens, int single, Sizes z) {
+    int tokens, int single, int qk_groups, Sizes z) {
     extern __shared__ __attribute__((aligned(16))) float conv[];  // [TT][q and k channels]
-    __shared__ int s_offset[TT], s_slot[TT], s_pos[TT], s_page[TT], s_request[TT];
+    constexpr int HELD = TT == 1 ? 1 : VALUE_TOKENS;
+    __shared__ int s_offset[HELD], s_slot[HELD], s_pos[HELD], s_page[HELD], s_request[HELD];
     __shared__ float s_sum[2 * TT][16], s_factor[2 * TT];
     const int nqd = z.nq * z.d, qk = nqd + z.nkv * z.d, channels = qk + z.nkv * z.dv;
     const int tid = threadIdx.x, lane = tid & (RL_WAVE - 1), wave = tid / RL_WAVE;
-    const int first = blockIdx.x * TT;
-    const int nt = min(TT, tokens - first);
-    if (tid < TT) {
-        const int t = min(first + tid, tokens - 1);
-        const int s = single ? t : request_of(cu, num_seqs, t);
-        const int pos = positions[t], slot = token_slot[t];
-        s_request[tid] = s;
-        s_offset[tid] = single ? 0 : t - cu[s];
-        s_slot[tid] = slot;
-        s_pos[tid] = pos;
-        s_page[tid] = k_cache ? block_table[(size_t)slot * z.table_stride + pos / z.page_size] : 0;
+    const bool of_values = TT > 1 && (int)blockIdx.x >= qk_groups;  // (the whole workgroup)
+    const int first = of_values ? ((int)blockIdx.x - qk_groups) * VALUE_TOKENS : (int)blockIdx.x * TT;
+    const int nt = min(of_values ? VALUE_TOKENS : TT, tokens - first);
+    // what is known of each token; of one token alone in registers
+    int offset1 = 0, slot1 = 0, pos1 = 0, page1 = 0;
+    if constexpr (TT == 1) {
+        const int s = single ? first : request_of(cu, num_seqs, first);
+        offset1 = single ? 0 : first - cu[s];
+        slot1 = token_slot[first];
+        pos1 = positions[first];
+        page1 = k_cache ? block_table[(size_t)slot1 * z.table_stride + pos1 / z.page_size] : 0;
+    } else {
+        if (tid < HELD) {
+            const int t = min(first + tid, tokens - 1);
+            const int s = request_of(cu, num_seqs, t);
+            const int pos = positions[t], slot = token_slot[t];
+            s_request[tid] = s;
+            s_offset[tid] = t - cu[s];
+            s_slot[tid] = slot;
+            s_pos[tid] = pos;
+            s_page[tid] = k_cache ? block_table[(size_t)slot * z.table_stride + pos / z.page_size] : 0;
+        }
+        __syncthreads();
     }
-    __syncthreads();
+    auto offset_of = [&](int tt) -> int { return TT == 1 ? offset1 : s_offset[tt]; };
+    auto slot_of = [&](int tt) -> int { return TT == 1 ? slot1 : s_slot[tt]; };
+    auto pos_of = [&](int tt) -> int { return TT == 1 ? pos1 : s_pos[tt]; };
+    auto page_of = [&](int tt) -> int { return TT == 1 ? page1 : s_page[tt]; };
     const int reach = TAPS > 0 ? TAPS : z.taps, held = reach - 1;
 
     typedef Pack<T, VEC> TP;
     typedef Pack<float, VEC> FP;
     // the projected values (with bias) of token t
-    auto projected = [&](int t, int c, float (&u)[VEC]) {
+    auto projected = [&](int t, int c, const FP& b, float (&u)[VEC]) {
         const TP q = *reinterpret_cast<const TP*>(packed + (size_t)t * z.width + c);
 #pragma unroll
-        for (int e = 0; e < VEC; ++e) u[e] = to_float(q.v[e]);
-        if (bias) {
-            const FP b = *reinterpret_cast<const FP*>(bias + c);
-#pragma unroll
-            for (int e = 0; e < VEC; ++e) u[e] += b.v[e];
-        }
+        for (int e = 0; e < VEC; ++e) u[e] = to_float(q.v[e]) + b.v[e];
     };
-    // and `back` tokens before the step's token tt
-    auto before = [&](int tt, int back, int c, float (&u)[VEC]) {
-        const int offset = s_offset[tt];
+    // and `back` tokens before the workgroup's token tt
+    auto before = [&](int tt, int back, int c, const FP& b, float (&u)[VEC]) {
+        const int offset = offset_of(tt);
         if (back <= offset) {
-            projected(first + tt - back, c, u);
+            projected(first + tt - back, c, b, u);
         } else {
-            const FP q = *reinterpret_cast<const FP*>(state + ((size_t)s_slot[tt] * held + held + offset - back) * channels + c);
+            const FP q = *reinterpret_cast<const FP*>(state + ((size_t)slot_of(tt) * held + held + offset - back) * channels + c);
 #pragma unroll
             for (int e = 0; e < VEC; ++e) u[e] = q.v[e];
         }
     };
-    // the convolved values of channels c .. c + VEC - 1 of every token of the workgroup
-    auto convolve = [&](int c, float (&y)[TT][VEC]) {
+    // the convolved values of channels c .. c + VEC - 1 of the workgroup's tokens tt0 .. tt0 + TT - 1
+    auto convolve = [&](int tt0, int c, float (&y)[TT][VEC]) {
         constexpr int WT = TAPS > 0 ? TAPS : 1, WIN = TAPS > 1 ? TAPS - 1 : 1;
-        FP wt[WT];
+        FP wt[WT], b;
         float win[WIN][VEC];
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) b.v[e] = 0.f;
+        if (bias) b = *reinterpret_cast<const FP*>(bias + c);
         if constexpr (TAPS > 0) {
 #pragma unroll
             for (int tap = 0; tap < TAPS; ++tap) wt[tap] = *reinterpret_cast<const FP*>(taps_t + (size_t)tap * channels + c);
         }
 #pragma unroll
-        for (int tt = 0; tt < TT; ++tt) {
+        for (int n = 0; n < TT; ++n) {
+            const int tt = tt0 + n;
             if (tt >= nt) {
 #pragma unroll
-                for (int e = 0; e < VEC; ++e) y[tt][e] = 0.f;
+                for (int e = 0; e < VEC; ++e) y[n][e] = 0.f;
                 continue;
             }
             float now[VEC];
-            projected(first + tt, c, now);
+            projected(first + tt, c, b, now);
             if (!taps_t) {
 #pragma unroll
-                for (int e = 0; e < VEC; ++e) y[tt][e] = now[e];
+                for (int e = 0; e < VEC; ++e) y[n][e] = now[e];
                 continue;
             }
             float acc[VEC];
 #pragma unroll
             for (int e = 0; e < VEC; ++e) acc[e] = 0.f;
+            float* rows = state + (size_t)slot_of(tt) * max(held, 1) * channels + c;
             if constexpr (TAPS > 0) {
-                if (tt == 0 || s_request[tt] != s_request[tt - 1]) {
+                if (n == 0 || s_request[TT == 1 ? 0 : tt] != s_request[TT == 1 ? 0 : tt - 1]) {
 #pragma unroll
-                    for (int q = 0; q < TAPS - 1; ++q) before(tt, TAPS - 1 - q, c, win[q]);
+                    for (int q = 0; q < TAPS - 1; ++q) before(tt, TAPS - 1 - q, c, b, win[q]);
                 }
 #pragma unroll
                 for (int tap = 0; tap < TAPS - 1; ++tap)
@@ -140,38 +161,92 @@ __global__ __launch_bounds__(1024) void prepare_kernel(
                 if constexpr (TAPS > 1) {
 #pragma unroll
                     for (int e = 0; e < VEC; ++e) win[TAPS - 2][e] = now[e];
+                    if (single) {
+                        // (this thread alone reads these channels of the request's rows)
+#pragma unroll
+                        for (int q = 0; q < TAPS - 1; ++q) {
+                            FP row;
+#pragma unroll
+                            for (int e = 0; e < VEC; ++e) row.v[e] = win[q][e];
+                            *reinterpret_cast<FP*>(rows + (size_t)q * channels) = row;
+                        }
+                    }
                 }
             } else {
                 for (int tap = 0; tap < reach; ++tap) {
                     const FP w = *reinterpret_cast<const FP*>(taps_t + (size_t)tap * channels + c);
                     float u[VEC];
-                    before(tt, held - tap, c, u);
+                    before(tt, held - tap, c, b, u);
 #pragma unroll
                     for (int e = 0; e < VEC; ++e) acc[e] = fmaf(w.v[e], u[e], acc[e]);
                 }
+                if (single && held > 0) {
+                    for (int q = 0; q + 1 < held; ++q)
+                        *reinterpret_cast<FP*>(rows + (size_t)q * channels) =
+                            *reinterpret_cast<const FP*>(rows + (size_t)(q + 1) * channels);
+                    FP last;
+#pragma unroll
+                    for (int e = 0; e < VEC; ++e) last.v[e] = now[e];
+                    *reinterpret_cast<FP*>(rows + (size_t)(held - 1) * channels) = last;
+                }
             }
 #pragma unroll
-            for (int e = 0; e < VEC; ++e) y[tt][e] = acc[e];
-            if (single && held > 0) {
-                // this thread alone reads these channels of the request's rows
-                float* rows = state + (size_t)s_slot[tt] * held * channels + c;
-                for (int q = 0; q + 1 < held; ++q)
-                    *reinterpret_cast<FP*>(rows + (size_t)q * channels) =
-                        *reinterpret_cast<const FP*>(rows + (size_t)(q + 1) * channels);
-                FP last;
+            for (int e = 0; e < VEC; ++e) y[n][e] = acc[e];
+        }
+    };
+    // channels c .. of the values of tokens tt0 .. into their pages
+    auto write_values = [&](int tt0, int c, const float (&y)[TT][VEC]) {
+        const int head = c / z.dv, ch = c - head * z.dv;
+        auto place = [&](int tt) -> T* {
+            return v_cache + (((size_t)page_of(tt) * z.nkv + head) * z.dv + ch) * z.page_size + pos_of(tt) % z.page_size;
+        };
+        // consecutive places of a page, from a multiple of TT on
+        if (TT > 1 && tt0 + TT <= nt && z.page_size % TT == 0 && pos_of(tt0) % TT == 0 &&
+            s_request[TT == 1 ? 0 : tt0] == s_request[TT == 1 ? 0 : tt0 + TT - 1]) {
+            T* dst = place(tt0);
 #pragma unroll
-                for (int e = 0; e < VEC; ++e) last.v[e] = now[e];
-                *reinterpret_cast<FP*>(rows + (size_t)(held - 1) * channels) = last;
+            for (int e = 0; e < VEC; ++e) {
+                Pack<T, TT> o;
+#pragma unroll
+                for (int n = 0; n < TT; ++n) o.v[n] = from_float<T>(y[n][e]);
+                *reinterpret_cast<Pack<T, TT>*>(dst + (size_t)e * z.page_size) = o;
             }
+            return;
+        }
+#pragma unroll
+        for (int n = 0; n < TT; ++n) {
+            if (tt0 + n >= nt) continue;
+            T* dst = place(tt0 + n);
+#pragma unroll
+            for (int e = 0; e < VEC; ++e) dst[(size_t)e * z.page_size] = from_float<T>(y[n][e]);
         }
     };
 
+    if constexpr (TT > 1) {
+        if (of_values) {
+            constexpr int PARTS = VALUE_TOKENS / TT;
+            for (int item = tid; item < z.nkv * z.dv / VEC * PARTS; item += blockDim.x) {
+                const int tt0 = item % PARTS * TT, c = item / PARTS * VEC;
+                if (tt0 >= nt) continue;
+                float y[TT][VEC];
+                convolve(tt0, qk + c, y);
+                write_values(tt0, c, y);
+            }
+            return;
+        }
+    }
+
+    // q and k to LDS, with the sums of their squares
     float ss[2][TT];
 #pragma unroll
     for (int tt = 0; tt < TT; ++tt) ss[0][tt] = ss[1][tt] = 0.f;
-    for (int c = VEC * tid; c < qk; c += VEC * blockDim.x) {
+    for (int c = VEC * tid; c < (TT == 1 ? channels : qk); c += VEC * blockDim.x) {
         float y[TT][VEC];
-        convolve(c, y);
+        convolve(0, c, y);
+        if (TT == 1 && c >= qk) {
+            if (v_cache) write_values(0, c - qk, y);
+            continue;
+        }
         const bool is_k = c >= nqd;
 #pragma unroll
         for (int tt = 0; tt < TT; ++tt) {
@@ -187,36 +262,6 @@ __global__ __launch_bounds__(1024) void prepare_kernel(
             ss[1][tt] += is_k ? sq : 0.f;
         }
     }
-    // the values have neither norm nor rotation: they are written at once
-    bool lined_up = TT == 4 && nt == TT && z.page_size % TT == 0 && (s_pos[0] % z.page_size) % TT == 0;
-#pragma unroll
-    for (int tt = 1; tt < TT; ++tt)
-        lined_up = lined_up && s_request[tt] == s_request[0];
-    if (v_cache || single)
-        for (int c = VEC * tid; c < z.nkv * z.dv; c += VEC * blockDim.x) {
-            float y[TT][VEC];
-            convolve(qk + c, y);
-            if (!v_cache) continue;
-            const int head = c / z.dv, ch = c - head * z.dv;
-            if (lined_up) {
-                T* dst = v_cache + (((size_t)s_page[0] * z.nkv + head) * z.dv + ch) * z.page_size + s_pos[0] % z.page_size;
-#pragma unroll
-                for (int e = 0; e < VEC; ++e) {
-                    Pack<T, TT> o;
-#pragma unroll
-                    for (int tt = 0; tt < TT; ++tt) o.v[tt] = from_float<T>(y[tt][e]);
-                    *reinterpret_cast<Pack<T, TT>*>(dst + (size_t)e * z.page_size) = o;
-                }
-            } else {
-#pragma unroll
-                for (int tt = 0; tt < TT; ++tt) {
-                    if (tt >= nt) continue;
-                    T* dst = v_cache + (((size_t)s_page[tt] * z.nkv + head) * z.dv + ch) * z.page_size + s_pos[tt] % z.page_size;
-#pragma unroll
-                    for (int e = 0; e < VEC; ++e) dst[(size_t)e * z.page_size] = from_float<T>(y[tt][e]);
-                }
-            }
-        }
     // the norms' sums over the workgroup
 #pragma unroll
     for (int n = 0; n < 2 * TT; ++n) {
@@ -236,32 +281,55 @@ __global__ __launch_bounds__(1024) void prepare_kernel(
         const int local = is_k ? c - nqd : c;
         const int head = local / z.d, i = local - head * z.d;
         const float* w = is_k ? k_norm_w : q_norm_w;
+        const bool turns = cos_tab && i < 2 * z.rotary_half;
+        // whole quads turn with whole quads
+        const bool quads = turns && !z.interleaved && z.rotary_half % VEC == 0;
+        const bool second = i >= z.rotary_half;
+        const int there = second ? -z.rotary_half : z.rotary_half;
+        FP weight, weight2;
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) weight.v[e] = weight2.v[e] = 1.f;
+        if (w) {
+            weight = *reinterpret_cast<const FP*>(w + local);
+            if (quads) weight2 = *reinterpret_cast<const FP*>(w + local + there);
+        }
 #pragma unroll
         for (int tt = 0; tt < TT; ++tt) {
             if (tt >= nt) continue;
-            const float factor = s_factor[is_k ? TT + tt : tt];
-            // channel i + o of this head, normed
-            auto normed = [&](int o) -> float {
-                const float v = conv[(size_t)tt * qk + c + o];
-                return w ? v * factor * w[local + o] : v;
-            };
-            const float* cs = cos_tab ? cos_tab + (size_t)s_pos[tt] * z.rotary_half : nullptr;
-            const float* sn = cos_tab ? sin_tab + (size_t)s_pos[tt] * z.rotary_half : nullptr;
+            const float factor = w ? s_factor[is_k ? TT + tt : tt] : 1.f;
+            const float* row = conv + (size_t)tt * qk + c;
+            const FP own = *reinterpret_cast<const FP*>(row);
+            const float* cs = cos_tab + (size_t)pos_of(tt) * z.rotary_half;
+            const float* sn = sin_tab + (size_t)pos_of(tt) * z.rotary_half;
+            float v[VEC];
+#pragma unroll
+            for (int e = 0; e < VEC; ++e) v[e] = own.v[e] * factor * weight.v[e];
+            if (quads) {
+                const FP other = *reinterpret_cast<const FP*>(row + there);
+                const int pair = second ? i - z.rotary_half : i;
+                const FP cq = *reinterpret_cast<const FP*>(cs + pair), sq = *reinterpret_cast<const FP*>(sn + pair);
+#pragma unroll
+                for (int e = 0; e < VEC; ++e) {
+                    const float o = other.v[e] * factor * weight2.v[e];
+                    v[e] = second ? v[e] * cq.v[e] + o * sq.v[e] : v[e] * cq.v[e] - o * sq.v[e];
+                }
+            } else if (turns) {
+#pragma unroll
+                for (int e = 0; e < VEC; ++e) {
+                    const int ch = i + e;
+                    if (ch >= 2 * z.rotary_half) continue;
+                    const bool sec = z.interleaved ? (ch & 1) : ch >= z.rotary_half;
+                    const int by = z.interleaved ? 1 : z.rotary_half;
+                    const int pair = z.interleaved ? ch >> 1 : (sec ? ch - z.rotary_half : ch);
+                    const int at = e + (sec ? -by : by);
+                    const float o = row[at] * factor * (w ? w[local + at] : 1.f);
+                    v[e] = sec ? v[e] * cs[pair] + o * sn[pair] : v[e] * cs[pair] - o * sn[pair];
+                }
+            }
             TP out;
 #pragma unroll
-            for (int e = 0; e < VEC; ++e) {
-                const int ch = i + e;
-                float v = normed(e);
-                if (cs && ch < 2 * z.rotary_half) {
-                    const bool second = z.interleaved ? (ch & 1) : ch >= z.rotary_half;
-                    const int pair = z.interleaved ? ch >> 1 : (second ? ch - z.rotary_half : ch);
-                    const int reach_to = z.interleaved ? 1 : z.rotary_half;
-                    const float other = normed(e + (second ? -reach_to : reach_to));
-                    v = second ? v * cs[pair] + other * sn[pair] : v * cs[pair] - other * sn[pair];
-                }
-                out.v[e] = from_float<T>(v);
-            }
-            T* dst = is_k ? k_cache + (((size_t)s_page[tt] * z.nkv + head) * z.page_size + s_pos[tt] % z.page_size) * z.d + i
+            for (int e = 0; e < VEC; ++e) out.v[e] = from_float<T>(v[e]);
+            T* dst = is_k ? k_cache + (((size_t)page_of(tt) * z.nkv + head) * z.page_size + pos_of(tt) % z.page_size) * z.d + i
                           : q_out + (size_t)(first + tt) * nqd + local;
             *reinterpret_cast<TP*>(dst) = out;
         }
@@ -295,11 +363,15 @@ static int launch(const T* packed, const float* bias, const float* taps_t, float
                   const int* seq_slots, int num_seqs, int tokens, const Sizes& z, hipStream_t stream) {
     const int single = tokens == num_seqs;  // every request brings one token
     const int qk = (z.nq + z.nkv) * z.d, channels = qk + z.nkv * z.dv;
+    // (the rotation tables' rows are read four entries at a time where whole quads turn)
     const bool vec = z.d % 4 == 0 && z.dv % 4 == 0 && z.width % 4 == 0 && (uintptr_t)packed % (4 * sizeof(T)) == 0;
     const int tt = !single && (size_t)qk * 4 * sizeof(float) <= 80 * 1024 ? 4 : 1;
     const size_t lds = (size_t)tt * qk * sizeof(float);
     if (lds > 156 * 1024) return RL_ERR_ARG;
-    dim3 grid((tokens + tt - 1) / tt), block(single ? 1024 : 256);
+    const int qk_groups = (tokens + tt - 1) / tt;
+    const int value_groups = tt > 1 && v_cache ? (tokens + VALUE_TOKENS - 1) / VALUE_TOKENS : 0;
+    const int items = (tt > 1 ? qk : channels) / (vec ? 4 : 1);  // a thread each, where they fit
+    dim3 grid(qk_groups + value_groups), block(items >= 1024 ? 1024 : (items + 255) / 256 * 256);
 #define RL_HEADS(VEC, TT, TAPS)                                                                                        \
     do {                                                                                                               \
         auto kernel = prepare_kernel<T, VEC, TT, TAPS>;                                                                \
@@ -308,7 +380,7 @@ static int launch(const T* packed, const float* bias, const float* taps_t, float
             return RL_ERR_LAUNCH;                                                                                      \
         hipLaunchKernelGGL(kernel, grid, block, lds, stream, packed, bias, taps_t, state, q_norm_w, k_norm_w, cos_tab, \
                            sin_tab, q_out, k_cache, v_cache, positions, token_slot, block_table, cu, num_seqs, tokens,  \
-                           single, z);                                                                                 \
+                           single, qk_groups, z);                                                                      \
     } while (0)
 #define RL_HEADS_TAPS(VEC, TT)                      \
     do {                                            \

@@ -49,7 +49,21 @@ __device__ inline float fexp<bf16_t>(float x) {
     return __builtin_amdgcn_exp2f(1.4426950408889634f * x);
 }
 
-__device__ inline float silu(float z) { return z / (1.f + expf(-z)); }
+// (the division likewise)
+template <typename T>
+__device__ inline float fsigmoid(float z);
+template <>
+__device__ inline float fsigmoid<float>(float z) {
+    return 1.f / (1.f + expf(-z));
+}
+template <>
+__device__ inline float fsigmoid<bf16_t>(float z) {
+    return __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(-1.4426950408889634f * z));
+}
+template <typename T>
+__device__ inline float silu(float z) {
+    return z * fsigmoid<T>(z);
+}
 __device__ inline float log_sigmoid(float z) { return fminf(z, 0.f) - log1pf(expf(-fabsf(z))); }
 
 // what the kernels read of a token
@@ -63,7 +77,7 @@ struct Rows {
 template <typename T>
 __device__ inline float input(const Rows<T>& in, int t, int col) {
     const float x = to_float(in.packed[(size_t)t * in.width + col]);
-    return in.silu ? linattn::silu(x) : x;
+    return in.silu ? silu<T>(x) : x;
 }
 
 // where a token's decays come from
@@ -78,61 +92,88 @@ struct Decays {
 
 // --------------------------------------------------------------------------- //
 // The factors of a chunk: Q [16][DP] = q e^(b_t), KT [DP][16] = k e^(b_last - b_t), G [DP] =
-// e^(b_last), A [16][16] (0 above the diagonal), where DP is d rounded up to whole blocks of 16
-// rows and what lies beyond d or the chunk's tokens is zero.
+// e^(b_last), A [16][16] (0 above the diagonal), where DP is d rounded up to whole blocks of 64
+// rows (16 for each of the four waves that walk) and what lies beyond d or the chunk's tokens is zero.
+// Q, KT and A lie in the order in which the lanes of the walk hold them as operands, so that a wave
+// reads a block of 16 rows as one run of memory: with lane = 16 g + r, Q[block][lane][4] holds channels
+// 4g .. 4g + 3 of the block for token r, KT[block][lane][4] tokens 4g .. for channel r, and A[w][lane]
+// token r with token 4g + w.
 // chunks: [n][4] = request, first token, tokens, unused.
 // --------------------------------------------------------------------------- //
-template <typename T, bool CHANNEL>
+template <typename T, bool CHANNEL, int DP>
 __global__ __launch_bounds__(256) void chunk_factors_kernel(Rows<T> in, Decays dec, const int* __restrict__ chunks,
                                                             float* __restrict__ Q, float* __restrict__ KT,
                                                             float* __restrict__ G, float* __restrict__ A, int heads,
-                                                            int d, int DP) {
+                                                            int d) {
     extern __shared__ __attribute__((aligned(16))) float lds[];
+    constexpr int P = DP + 4;  // pitch of a token's channels
     const int chunk = blockIdx.x, h = blockIdx.y;
     const int t0 = chunks[4 * chunk + 1], n = chunks[4 * chunk + 2];
-    const int P = DP + 4;  // pitch of a token's channels
     float* sq = lds;
     float* sk = sq + CT * P;
-    float* sb = sk + CT * P;                       // CHANNEL: the sums of ln a
-    float* red = CHANNEL ? sb + CT * P : sb;       // [4][16][16]
-    float* slow = red + 4 * CT * CT;               // CHANNEL: [16][rank]
+    float* sb = sk + CT * P;                       // CHANNEL: the sums of ln a, and a itself
+    float* sa = sb + CT * P;
+    float* red = CHANNEL ? sa + CT * P : sb;       // [4][16][16]
+    float* slow = red + 4 * CT * CT;               // CHANNEL: [16][rank up to a multiple of 4]
     const int tid = threadIdx.x, lane = tid & (RL_WAVE - 1), wave = tid / RL_WAVE;
-    for (int idx = tid; idx < CT * DP; idx += 256) {
-        const int t = idx / DP, i = idx - t * DP;
-        const bool ok = t < n && i < d;
-        sq[t * P + i] = ok ? input(in, t0 + t, in.q_col + h * d + i) * in.q_scale : 0.f;
-        sk[t * P + i] = ok ? input(in, t0 + t, in.k_col + h * d + i) : 0.f;
+    // every thread's elements are asked for together, without a condition (a real element where there is none)
+    constexpr int PER = CT * DP / 256;
+    T pq[PER], pk[PER];
+#pragma unroll
+    for (int e = 0; e < PER; ++e) {
+        const int idx = e * 256 + tid, t = min(idx / DP, n - 1), i = min(idx % DP, d - 1);
+        const T* row = in.packed + (size_t)(t0 + t) * in.width + h * d + i;
+        pq[e] = row[in.q_col];
+        pk[e] = row[in.k_col];
     }
     const float fixed = CHANNEL ? 0.f : dec.fixed[h];
+    const int pitch = (dec.rank + 3) & ~3;
     if constexpr (CHANNEL) {
-        for (int idx = tid; idx < CT * dec.rank; idx += 256) {
-            const int t = idx / dec.rank, r = idx - t * dec.rank;
-            slow[idx] = t < n ? dec.low[(size_t)(t0 + t) * dec.low_stride + r] : 0.f;
+        for (int idx = tid; idx < CT * pitch; idx += 256) {
+            const int t = idx / pitch, r = idx - t * pitch;
+            slow[idx] = t < n && r < dec.rank ? dec.low[(size_t)(t0 + t) * dec.low_stride + r] : 0.f;
         }
+    }
+#pragma unroll
+    for (int e = 0; e < PER; ++e) {
+        const int idx = e * 256 + tid, t = idx / DP, i = idx % DP;
+        const bool ok = t < n && i < d;
+        float q = to_float(pq[e]), k = to_float(pk[e]);
+        if (in.silu) {
+            q = silu<T>(q);
+            k = silu<T>(k);
+        }
+        sq[t * P + i] = ok ? q * in.q_scale : 0.f;
+        sk[t * P + i] = ok ? k : 0.f;
+    }
+    if constexpr (CHANNEL) {
         __syncthreads();
-        // a thread takes a channel of eight tokens, so that an entry of W_out serves eight sums
-        for (int item = tid; item < 2 * DP; item += 256) {
-            const int half = item / DP, i = item - half * DP;
-            if (i >= d) {
-                for (int t = 0; t < CT / 2; ++t) sb[(half * (CT / 2) + t) * P + i] = 0.f;
-                continue;
+        // a thread takes a channel of TPT tokens, so that an entry of W_out serves as many sums
+        constexpr int PARTS = DP >= 256 ? 1 : 256 / DP, TPT = CT / PARTS;
+        for (int item = tid; item < PARTS * DP; item += 256) {
+            const int part = item / DP, i = item % DP, ic = min(i, d - 1);
+            float z[TPT];
+            const float b = dec.bias[h * d + ic];
+#pragma unroll
+            for (int t = 0; t < TPT; ++t) z[t] = 0.f;
+            const float* col = dec.out_t + h * d + ic;
+            const float* lrow = slow + part * TPT * pitch;
+            for (int r = 0; r < dec.rank; r += 4) {
+                float w[4];
+#pragma unroll
+                for (int e = 0; e < 4; ++e) w[e] = col[(size_t)min(r + e, dec.rank - 1) * heads * d];  // (beyond: times 0)
+#pragma unroll
+                for (int t = 0; t < TPT; ++t) {
+                    const f32x4 l = *reinterpret_cast<const f32x4*>(lrow + t * pitch + r);
+                    z[t] = fmaf(w[3], l[3], fmaf(w[2], l[2], fmaf(w[1], l[1], fmaf(w[0], l[0], z[t]))));
+                }
             }
-            float z[CT / 2];
-            const float b = dec.bias[h * d + i];
 #pragma unroll
-            for (int t = 0; t < CT / 2; ++t) z[t] = 0.f;
-            const float* col = dec.out_t + h * d + i;
-            const float* lrow = slow + half * (CT / 2) * dec.rank;
-#pragma unroll 4
-            for (int r = 0; r < dec.rank; ++r) {
-                const float w = col[(size_t)r * heads * d];
-#pragma unroll
-                for (int t = 0; t < CT / 2; ++t) z[t] = fmaf(w, lrow[t * dec.rank + r], z[t]);
-            }
-#pragma unroll
-            for (int t = 0; t < CT / 2; ++t) {
-                const int tt = half * (CT / 2) + t;
-                sb[tt * P + i] = tt < n ? log_sigmoid(z[t] + b) * dec.inv_tau : 0.f;
+            for (int t = 0; t < TPT; ++t) {
+                const int tt = part * TPT + t;
+                const float la = tt < n && i < d ? log_sigmoid(z[t] + b) * dec.inv_tau : 0.f;
+                sb[tt * P + i] = la;
+                sa[tt * P + i] = fexp<T>(la);
             }
         }
         __syncthreads();
@@ -147,52 +188,81 @@ __global__ __launch_bounds__(256) void chunk_factors_kernel(Rows<T> in, Decays d
     }
     __syncthreads();
     const size_t cb = (size_t)chunk * heads + h;
-    for (int idx = tid; idx < CT * DP; idx += 256) {
-        const int t = idx / DP, i = idx - t * DP;
-        const float b = CHANNEL ? sb[t * P + i] : fixed * (float)(t + 1);
-        Q[cb * CT * DP + idx] = sq[t * P + i] * fexp<T>(b);
+    const int r16 = lane & 15, g = lane >> 4;
+#pragma unroll
+    for (int e = 0; e < PER / 4; ++e) {
+        const int block = e * 4 + wave, t = r16, i = 16 * block + 4 * g;
+        const f32x4 q = *reinterpret_cast<const f32x4*>(sq + t * P + i);
+        f32x4 o;
+        if constexpr (CHANNEL) {
+            const f32x4 b = *reinterpret_cast<const f32x4*>(sb + t * P + i);
+#pragma unroll
+            for (int c = 0; c < 4; ++c) o[c] = q[c] * fexp<T>(b[c]);
+        } else {
+            o = q * fexp<T>(fixed * (float)(t + 1));
+        }
+        *reinterpret_cast<f32x4*>(Q + cb * CT * DP + 4 * (block * RL_WAVE + lane)) = o;
     }
-    for (int idx = tid; idx < CT * DP; idx += 256) {
-        const int i = idx / CT, t = idx & (CT - 1);
-        // (t beyond the chunk's tokens: its key is zero, and the exponent is kept from growing)
-        const float b = CHANNEL ? sb[(CT - 1) * P + i] - sb[t * P + i] : fixed * (float)max(n - 1 - t, 0);
-        KT[cb * CT * DP + idx] = sk[t * P + i] * fexp<T>(b);
+#pragma unroll
+    for (int e = 0; e < PER / 4; ++e) {
+        const int block = e * 4 + wave, t = 4 * g, i = 16 * block + r16;
+        const float last = CHANNEL ? sb[(CT - 1) * P + i] : 0.f;
+        f32x4 o;
+#pragma unroll
+        for (int c = 0; c < 4; ++c) {
+            // (t beyond the chunk's tokens: its key is zero, and the exponent is kept from growing)
+            const float b = CHANNEL ? last - sb[(t + c) * P + i] : fixed * (float)max(n - 1 - t - c, 0);
+            o[c] = sk[(t + c) * P + i] * fexp<T>(b);
+        }
+        *reinterpret_cast<f32x4*>(KT + cb * CT * DP + 4 * (block * RL_WAVE + lane)) = o;
     }
     for (int i = tid; i < DP; i += 256) G[cb * DP + i] = fexp<T>(CHANNEL ? sb[(CT - 1) * P + i] : fixed * (float)n);
-    // A: a lane takes two by two tokens, a wave a quarter of the channels
-    const int ta = 2 * (lane >> 3), sa = 2 * (lane & 7);
+    // A: a lane takes two by two tokens (t, t + 1 with s, s + 1), a wave a quarter of the channels.  One
+    // exponential serves the four pairs: with E = e^(b_t - b_(s+1)), the others are E a_(s+1), E a_(t+1)
+    // and E a_(s+1) a_(t+1); on the diagonal they are 1 and a_(t+1).
+    const int ta = 2 * (lane >> 3), s0 = 2 * (lane & 7);
+    const bool diagonal = s0 == ta;
     float acc[2][2] = {{0.f, 0.f}, {0.f, 0.f}};
-    if (sa <= ta) {
+    if (s0 <= ta) {
+#pragma unroll 2
         for (int i = wave * (DP / 4); i < (wave + 1) * (DP / 4); i += 4) {
-            f32x4 q[2], k[2], bt[2], bs[2];
+            f32x4 q[2], k[2];
 #pragma unroll
             for (int e = 0; e < 2; ++e) {
                 q[e] = *reinterpret_cast<const f32x4*>(sq + (ta + e) * P + i);
-                k[e] = *reinterpret_cast<const f32x4*>(sk + (sa + e) * P + i);
-                if constexpr (CHANNEL) {
-                    bt[e] = *reinterpret_cast<const f32x4*>(sb + (ta + e) * P + i);
-                    bs[e] = *reinterpret_cast<const f32x4*>(sb + (sa + e) * P + i);
-                }
+                k[e] = *reinterpret_cast<const f32x4*>(sk + (s0 + e) * P + i);
             }
+            if constexpr (CHANNEL) {
+                const f32x4 bt = *reinterpret_cast<const f32x4*>(sb + ta * P + i);
+                const f32x4 bs = *reinterpret_cast<const f32x4*>(sb + (s0 + 1) * P + i);
+                const f32x4 at = *reinterpret_cast<const f32x4*>(sa + (ta + 1) * P + i);
+                const f32x4 as = *reinterpret_cast<const f32x4*>(sa + (s0 + 1) * P + i);
 #pragma unroll
-            for (int a = 0; a < 2; ++a)
+                for (int c = 0; c < 4; ++c) {
+                    const float e01 = fexp<T>(fminf(bt[c] - bs[c], 0.f));
+                    const float e00 = diagonal ? 1.f : e01 * as[c];
+                    const float e11 = diagonal ? 1.f : e01 * at[c];
+                    acc[0][0] = fmaf(q[0][c] * k[0][c], e00, acc[0][0]);
+                    acc[0][1] = fmaf(q[0][c] * k[1][c], e01, acc[0][1]);  // (not used on the diagonal)
+                    acc[1][0] = fmaf(q[1][c] * k[0][c], e00 * at[c], acc[1][0]);
+                    acc[1][1] = fmaf(q[1][c] * k[1][c], e11, acc[1][1]);
+                }
+            } else {
 #pragma unroll
-                for (int s = 0; s < 2; ++s)
+                for (int c = 0; c < 4; ++c)
 #pragma unroll
-                    for (int c = 0; c < 4; ++c) {
-                        float x = q[a][c] * k[s][c];
-                        // (a pair above the diagonal is not used; its exponent would be positive)
-                        if constexpr (CHANNEL) x *= fexp<T>(fminf(bt[a][c] - bs[s][c], 0.f));
-                        acc[a][s] += x;
-                    }
+                    for (int a = 0; a < 2; ++a)
+#pragma unroll
+                        for (int s = 0; s < 2; ++s) acc[a][s] = fmaf(q[a][c], k[s][c], acc[a][s]);
+            }
         }
     }
 #pragma unroll
     for (int a = 0; a < 2; ++a)
 #pragma unroll
-        for (int s = 0; s < 2; ++s) red[(wave * CT + ta + a) * CT + sa + s] = acc[a][s];
+        for (int s = 0; s < 2; ++s) red[(wave * CT + ta + a) * CT + s0 + s] = acc[a][s];
     __syncthreads();
-    const int t = tid / CT, s = tid % CT;
+    const int t = r16, s = 4 * g + wave;
     float sum = 0.f;
 #pragma unroll
     for (int w = 0; w < 4; ++w) sum += red[(w * CT + t) * CT + s];
@@ -203,30 +273,52 @@ __global__ __launch_bounds__(256) void chunk_factors_kernel(Rows<T> in, Decays d
 // --------------------------------------------------------------------------- //
 // The walk over a request's chunks.  A workgroup of four waves takes 16 columns of a head; the
 // blocks of 16 rows are dealt to the waves, RB at most each, so that a wave's own chain of matrix
-// instructions is short.  The read-outs' shares of the waves are added through LDS behind the
-// update, which does not wait for them.  Operands of the next two chunks travel meanwhile.
+// instructions is short.  The read-outs' shares of the waves meet in LDS and are added and stored while
+// the next chunk is multiplied.  Operands of the next chunks travel meanwhile.  A wave is alone on
+// its SIMD, so what is not a matrix instruction is to fit between two of them: everything is read
+// through buffer resources, whose loads take a constant lane offset and a uniform one, and whose bounds
+// stand for the ends of the portion and of the head (reads beyond give zeros, writes are dropped).
 // seq_chunks: [requests][2] = first chunk, chunks.
 // --------------------------------------------------------------------------- //
-template <typename T, int RB>
+constexpr int walk_buffers(int rb) { return rb <= 2 ? 6 : 4; }  // as the registers hold
+
+__device__ inline __amdgpu_buffer_rsrc_t buffer_of(const void* p, size_t bytes) {
+    return __builtin_amdgcn_make_buffer_rsrc(const_cast<void*>(p), 0, (int)(unsigned)min(bytes, (size_t)0xfffffffcu), 0x00027000);
+}
+__device__ inline f32x4 load4(__amdgpu_buffer_rsrc_t r, int lane_bytes, int bytes) {
+    return __builtin_bit_cast(f32x4, __builtin_amdgcn_raw_buffer_load_b128(r, lane_bytes, bytes, 0));
+}
+template <typename T>
+__device__ inline T load1(__amdgpu_buffer_rsrc_t r, int lane_bytes, int bytes);
+template <>
+__device__ inline float load1<float>(__amdgpu_buffer_rsrc_t r, int lane_bytes, int bytes) {
+    return __uint_as_float(__builtin_amdgcn_raw_buffer_load_b32(r, lane_bytes, bytes, 0));
+}
+template <>
+__device__ inline bf16_t load1<bf16_t>(__amdgpu_buffer_rsrc_t r, int lane_bytes, int bytes) {
+    return bf16_t{__builtin_amdgcn_raw_buffer_load_b16(r, lane_bytes, bytes, 0)};
+}
+
+template <typename T, int RB, bool SILU>
 __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 2))) void chunk_walk_kernel(
     Rows<T> in, const float* __restrict__ Q, const float* __restrict__ KT, const float* __restrict__ G,
     const float* __restrict__ A, const int* __restrict__ cu, const int* __restrict__ seq_slots,
     const int* __restrict__ seq_chunks, float* __restrict__ S, float* __restrict__ raw, int num_seqs, int heads, int d,
-    int DP, int dv, int col_groups) {
+    int dv, int col_groups) {
+    constexpr int DP = 64 * RB;
     // the column groups of a (request, head) read the same factors: they go to one XCD, whose L2 holds them
     const int per_xcd = gridDim.x / XCDS;  // (the launch is a multiple)
     const int work = (blockIdx.x % XCDS) * per_xcd + blockIdx.x / XCDS;
     if (work >= num_seqs * heads * col_groups) return;  // whole workgroups leave
     const int pair = work / col_groups;
     const int s = pair / heads, h = pair - s * heads;
-    const int lane = threadIdx.x & (RL_WAVE - 1), wave = threadIdx.x / RL_WAVE;
+    const int lane = threadIdx.x & (RL_WAVE - 1), wave = __builtin_amdgcn_readfirstlane(threadIdx.x / RL_WAVE);
     const int r16 = lane & 15, g = lane >> 4;
     const int j0 = (work - pair * col_groups) * 16;
     const int j = min(j0 + r16, dv - 1);
     const int t0 = cu[s], t1 = cu[s + 1];
     const int c0 = seq_chunks[2 * s], nc = seq_chunks[2 * s + 1];
-    const int NB = DP / 16;
-    __shared__ float red[2][4][CT][CT + 1];
+    __shared__ float red[2][4][CT][CT + 1], sv[2][CT][CT + 1];
 
     f32x4 st[RB];
     float* Sp = S + ((size_t)seq_slots[s] * heads + h) * d * dv;
@@ -241,48 +333,65 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 2))) voi
     struct Operands {
         f32x4 q[RB], k[RB], decay[RB];
         float a;
-        T v[4];
+        T v;  // the value that this thread brings to LDS: token threadIdx.x / 16, column threadIdx.x % 16
     };
+    // the request's first factors of this head; those of its other chunks follow at equal distances
+    const size_t first = (size_t)c0 * heads + h;
+    const size_t spread = (size_t)nc * heads;
+    const auto qb = buffer_of(Q + first * CT * DP, spread * CT * DP * 4), kb = buffer_of(KT + first * CT * DP, spread * CT * DP * 4);
+    const auto gb = buffer_of(G + first * DP, spread * DP * 4), ab = buffer_of(A + first * CT * CT, spread * CT * CT * 4);
+    const int at = 16 * (wave * RL_WAVE + lane), a_at = 4 * (wave * RL_WAVE + lane), decay_at = 4 * (16 * wave + 4 * g);
+    // values: the portion's rows from this head's first column on; the last row ends the resource
+    const int row_bytes = in.width * (int)sizeof(T);
+    const auto vb = buffer_of(in.packed + (size_t)t0 * in.width + in.v_col + h * dv,
+                              (size_t)(t1 - t0 - 1) * row_bytes + (size_t)dv * sizeof(T));
+    const int tt = threadIdx.x / 16, jj = threadIdx.x % 16;
+    const bool column = j0 + jj < dv;
+    const int v_at = tt * row_bytes + (j0 + jj) * (int)sizeof(T);
     auto load = [&](int c, Operands& x) {
-        const size_t cb = (size_t)(c0 + c) * heads + h;
+        const int qc = c * heads * (CT * DP * 4), gc = c * heads * (DP * 4), ac = c * heads * (CT * CT * 4);
 #pragma unroll
         for (int m = 0; m < RB; ++m) {
-            const int rb = min(wave + 4 * m, NB - 1);
-            x.q[m] = *reinterpret_cast<const f32x4*>(Q + (cb * CT + r16) * DP + 16 * rb + 4 * g);
-            x.k[m] = *reinterpret_cast<const f32x4*>(KT + (cb * DP + 16 * rb + r16) * CT + 4 * g);
-            x.decay[m] = *reinterpret_cast<const f32x4*>(G + cb * DP + 16 * rb + 4 * g);
+            x.q[m] = load4(qb, at + 4096 * m, qc);
+            x.k[m] = load4(kb, at + 4096 * m, qc);
+            x.decay[m] = load4(gb, decay_at + 256 * m, gc);
         }
-        x.a = A[cb * CT * CT + r16 * CT + 4 * g + wave];
-#pragma unroll
-        for (int r = 0; r < 4; ++r) {
-            // (beyond the portion a real row, which meets zeros)
-            const int t = min(t0 + c * CT + 4 * g + r, t1 - 1);
-            x.v[r] = in.packed[(size_t)t * in.width + in.v_col + h * dv + j];
-        }
+        x.a = load1<float>(ab, a_at, ac);
+        x.v = load1<T>(vb, column ? v_at + c * CT * row_bytes : -4, 0);
     };
-    auto walk = [&](int c, const Operands& x) {
+    // a chunk's values, read by every wave
+    auto stage = [&](int c, T raw_value) {
+        const float v = to_float(raw_value);
+        sv[c & 1][tt][jj] = SILU ? silu<T>(v) : v;
+    };
+    // the outputs of a chunk: thread (token, column); a column beyond the head is beyond the resource
+    const int out_row = heads * dv * 4;
+    const auto ob = buffer_of(raw + (size_t)t0 * heads * dv + h * dv, (size_t)(t1 - t0 - 1) * out_row + (size_t)dv * 4);
+    const int out_at = tt * out_row + 4 * (j0 + jj);
+    auto store = [&](int c) {
+        float(*buf)[CT][CT + 1] = red[c & 1];
+        const float o = (buf[0][tt][jj] + buf[1][tt][jj]) + (buf[2][tt][jj] + buf[3][tt][jj]);
+        __builtin_amdgcn_raw_buffer_store_b32(__float_as_uint(o), ob, column ? out_at + c * CT * out_row : -4, 0, 0);
+    };
+    auto walk = [&](int c, const Operands& x, T next_value, int next, Operands& y, bool more) {
         float v[4];
 #pragma unroll
-        for (int r = 0; r < 4; ++r) {
-            v[r] = to_float(x.v[r]);
-            if (in.silu) v[r] = linattn::silu(v[r]);
-        }
-        // the chunk's own pairs: wave w takes tokens 4g + w
-        const float mine = wave == 0 ? v[0] : (wave == 1 ? v[1] : (wave == 2 ? v[2] : v[3]));
+        for (int r = 0; r < 4; ++r) v[r] = sv[c & 1][4 * g + r][r16];
         f32x4 o = (f32x4){0.f, 0.f, 0.f, 0.f};
-        f32x4 o2 = __builtin_amdgcn_mfma_f32_16x16x4f32(x.a, mine, o, 0, 0, 0);
+        // the chunk's own pairs: wave w takes tokens 4g + w
+        f32x4 o2 = __builtin_amdgcn_mfma_f32_16x16x4f32(x.a, sv[c & 1][4 * g + wave][r16], o, 0, 0, 0);
 #pragma unroll
-        for (int m = 0; m < RB; ++m) {
-            if (wave + 4 * m < NB) {
+        for (int m = 0; m < RB; ++m)
 #pragma unroll
-                for (int r = 0; r < 4; ++r) {
-                    if (r & 1)
-                        o2 = __builtin_amdgcn_mfma_f32_16x16x4f32(x.q[m][r], st[m][r], o2, 0, 0, 0);
-                    else
-                        o = __builtin_amdgcn_mfma_f32_16x16x4f32(x.q[m][r], st[m][r], o, 0, 0, 0);
-                }
+            for (int r = 0; r < 4; ++r) {
+                if (r & 1)
+                    o2 = __builtin_amdgcn_mfma_f32_16x16x4f32(x.q[m][r], st[m][r], o2, 0, 0, 0);
+                else
+                    o = __builtin_amdgcn_mfma_f32_16x16x4f32(x.q[m][r], st[m][r], o, 0, 0, 0);
             }
-        }
+        if (c > 0) store(c - 1);  // its shares were complete at the last barrier
+        if (more) load(next, y);
+        stage(c + 1, next_value);
 #pragma unroll
         for (int m = 0; m < RB; ++m)
 #pragma unroll
@@ -290,33 +399,35 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 2))) voi
 #pragma unroll
         for (int r = 0; r < 4; ++r)
 #pragma unroll
-            for (int m = 0; m < RB; ++m)
-                if (wave + 4 * m < NB) st[m] = __builtin_amdgcn_mfma_f32_16x16x4f32(x.k[m][r], v[r], st[m], 0, 0, 0);
+            for (int m = 0; m < RB; ++m) st[m] = __builtin_amdgcn_mfma_f32_16x16x4f32(x.k[m][r], v[r], st[m], 0, 0, 0);
         float(*buf)[CT][CT + 1] = red[c & 1];
 #pragma unroll
         for (int r = 0; r < 4; ++r) buf[wave][4 * g + r][r16] = o[r] + o2[r];
         // one barrier a chunk: the other buffer is written next, and this one again only after
-        // every wave has passed the next barrier
+        // every wave has passed the next barrier, before which it was read
         __syncthreads();
-        const int tt = threadIdx.x / 16, jj = threadIdx.x % 16;
-        const int t = t0 + c * CT + tt;
-        if (t < t1 && j0 + jj < dv)
-            raw[(size_t)t * heads * dv + h * dv + j0 + jj] =
-                (buf[0][tt][jj] + buf[1][tt][jj]) + (buf[2][tt][jj] + buf[3][tt][jj]);
+        __builtin_amdgcn_sched_barrier(0);  // the loads of a chunk stay as far ahead as they are written
     };
-    Operands x[3];
-    load(0, x[0]);
-    load(min(1, nc - 1), x[1]);
-    for (int c = 0; c < nc; c += 3) {
+    // the operands of the next AHEAD chunks are on their way (they come from memory: the factors were
+    // written by workgroups on other XCDs)
+    constexpr int BUFS = walk_buffers(RB), AHEAD = BUFS - 1;
+    Operands x[BUFS];
 #pragma unroll
-        for (int u = 0; u < 3; ++u) {
-            if (c + u < nc) {
-                load(min(c + u + 2, nc - 1), x[(u + 2) % 3]);
-                __builtin_amdgcn_sched_barrier(0);
-                walk(c + u, x[u]);
-            }
-        }
+    for (int u = 0; u < AHEAD; ++u) load(min(u, nc - 1), x[u]);
+    // Nothing is on its way when the loop is entered: the compiler's waits inside it then stand for the
+    // loop's own loads alone.
+    __builtin_amdgcn_s_waitcnt(0x0f70);  // vmcnt(0)
+    stage(0, x[0].v);
+    __syncthreads();
+    int c = 0;
+    for (; c + BUFS <= nc; c += BUFS) {
+#pragma unroll
+        for (int u = 0; u < BUFS; ++u) walk(c + u, x[u], x[(u + 1) % BUFS].v, min(c + u + AHEAD, nc - 1), x[(u + AHEAD) % BUFS], true);
     }
+#pragma unroll
+    for (int u = 0; u < AHEAD; ++u)
+        if (c + u < nc) walk(c + u, x[u], x[u + 1 < AHEAD ? u + 1 : u].v, 0, x[AHEAD], false);
+    store(nc - 1);
 #pragma unroll
     for (int m = 0; m < RB; ++m)
 #pragma unroll
@@ -343,7 +454,7 @@ struct Finish {
 template <typename T>
 __device__ inline float gate_of(const Finish<T>& f, int t, int col) {
     const float z = to_float(f.gate[(size_t)t * f.gate_width + col]);
-    return f.sigmoid_gate ? 1.f / (1.f + expf(-z)) : silu(z);
+    return f.sigmoid_gate ? fsigmoid<T>(z) : silu<T>(z);
 }
 
 // parts of up to 1024 channels: LPP lanes of a wave a part, four channels a lane at a time
@@ -379,7 +490,7 @@ __global__ __launch_bounds__(256) void gated_norm_kernel(const float* __restrict
 #pragma unroll
             for (int e = 0; e < 4; ++e) {
                 const float z = to_float(gq.v[e]);
-                y.v[e] = from_float<T>(x[e] * rr * (f.sigmoid_gate ? 1.f / (1.f + expf(-z)) : silu(z)));
+                y.v[e] = from_float<T>(x[e] * rr * (f.sigmoid_gate ? fsigmoid<T>(z) : silu<T>(z)));
             }
             *reinterpret_cast<Quad<T>*>(f.out + (size_t)t * f.out_width + part * size + i) = y;
         }
@@ -417,7 +528,7 @@ __global__ __launch_bounds__(512) void gated_norm_row_kernel(const float* __rest
 #pragma unroll
             for (int e = 0; e < 4; ++e) {
                 const float z = to_float(gq.v[e]);
-                y.v[e] = from_float<T>(x[e] * rr * (f.sigmoid_gate ? 1.f / (1.f + expf(-z)) : silu(z)));
+                y.v[e] = from_float<T>(x[e] * rr * (f.sigmoid_gate ? fsigmoid<T>(z) : silu<T>(z)));
             }
             *reinterpret_cast<Quad<T>*>(f.out + (size_t)t * f.out_width + part * size + i) = y;
         }
@@ -557,28 +668,60 @@ template <typename T>
 static int launch_scan(const Rows<T>& in, const Decays& dec, const int* chunks, int nchunks, const int* cu,
                        const int* seq_slots, const int* seq_chunks, float* Q, float* KT, float* G, float* A, float* S,
                        float* raw, int num_seqs, int heads, int d, int dv, hipStream_t stream) {
-    const int DP = (d + 15) / 16 * 16;
     const bool channel = dec.out_t != nullptr;
-    const size_t lds = sizeof(float) * ((size_t)(channel ? 3 : 2) * CT * (DP + 4) + 4 * CT * CT +
-                                        (channel ? (size_t)CT * dec.rank : 0));
-    if (lds > 156 * 1024) return RL_ERR_ARG;
-    auto factors = channel ? chunk_factors_kernel<T, true> : chunk_factors_kernel<T, false>;
-    if (lds > 60 * 1024 &&
-        hipFuncSetAttribute((const void*)factors, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess)
-        return RL_ERR_LAUNCH;
-    hipLaunchKernelGGL(factors, dim3(nchunks, heads), dim3(256), lds, stream, in, dec, chunks, Q, KT, G, A, heads, d, DP);
+#define RL_FACTORS(CHANNEL, DP)                                                                                      \
+    do {                                                                                                             \
+        const size_t lds = sizeof(float) * ((size_t)(CHANNEL ? 4 : 2) * CT * (DP + 4) + 4 * CT * CT +                \
+                                            (CHANNEL ? (size_t)CT * ((dec.rank + 3) & ~3) : 0));                     \
+        if (lds > 156 * 1024) return RL_ERR_ARG;                                                                     \
+        auto kernel = chunk_factors_kernel<T, CHANNEL, DP>;                                                          \
+        if (lds > 60 * 1024 &&                                                                                       \
+            hipFuncSetAttribute((const void*)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess) \
+            return RL_ERR_LAUNCH;                                                                                    \
+        hipLaunchKernelGGL(kernel, dim3(nchunks, heads), dim3(256), lds, stream, in, dec, chunks, Q, KT, G, A, heads, d); \
+    } while (0)
+#define RL_FACTORS_OF(DP)           \
+    do {                            \
+        if (channel)                \
+            RL_FACTORS(true, DP);   \
+        else                        \
+            RL_FACTORS(false, DP);  \
+    } while (0)
+    if (d <= 64)
+        RL_FACTORS_OF(64);
+    else if (d <= 128)
+        RL_FACTORS_OF(128);
+    else if (d <= 192)
+        RL_FACTORS_OF(192);
+    else
+        RL_FACTORS_OF(256);
+#undef RL_FACTORS_OF
+#undef RL_FACTORS
     const int col_groups = (dv + 15) / 16;
     const long groups = ((long)num_seqs * heads * col_groups + XCDS - 1) / XCDS * XCDS;
     if (groups > 0x7fffffffL) return RL_ERR_ARG;
-#define RL_WALK(RB)                                                                                                  \
-    hipLaunchKernelGGL((chunk_walk_kernel<T, RB>), dim3((unsigned)groups), dim3(256), 0, stream, in, Q, KT, G, A, cu, \
-                       seq_slots, seq_chunks, S, raw, num_seqs, heads, d, DP, dv, col_groups)
-    if (DP <= 64)
+    // a request's factors, values and outputs are addressed by 32-bit offsets (nchunks bounds its chunks)
+    const long span = (long)nchunks * CT * ((d + 63) / 64 * 64 > dv ? (d + 63) / 64 * 64 : dv) * heads * 4;
+    if (span > 0x7fffff00L || (long)nchunks * CT * in.width * (long)sizeof(T) > 0x7fffff00L) return RL_ERR_ARG;
+#define RL_WALK_AS(RB, SILU)                                                                                         \
+    hipLaunchKernelGGL((chunk_walk_kernel<T, RB, SILU>), dim3((unsigned)groups), dim3(256), 0, stream, in, Q, KT, G, A, \
+                       cu, seq_slots, seq_chunks, S, raw, num_seqs, heads, d, dv, col_groups)
+#define RL_WALK(RB)                 \
+    do {                            \
+        if (in.silu)                \
+            RL_WALK_AS(RB, true);   \
+        else                        \
+            RL_WALK_AS(RB, false);  \
+    } while (0)
+    if (d <= 64)
         RL_WALK(1);
-    else if (DP <= 128)
+    else if (d <= 128)
         RL_WALK(2);
+    else if (d <= 192)
+        RL_WALK(3);
     else
         RL_WALK(4);
+#undef RL_WALK_AS
 #undef RL_WALK
     return rl_launch_status();
 }
@@ -621,7 +764,7 @@ extern "C" int rl_linear_attention_max_value_dim() { return linattn::MAX_DV; }
 extern "C" int rl_linear_attention_chunk() { return linattn::CT; }
 
 // Portions: raw [tokens, heads * dv] float32 gets o.  Q, KT [chunks, heads, 16 * DP], G [chunks, heads, DP]
-// and A [chunks, heads, 256] are scratch.
+// (DP: d up to a multiple of 64) and A [chunks, heads, 256] are scratch.
 extern "C" int rl_linear_scan(const void* packed, int width, int q_col, int k_col, int v_col, int silu, float q_scale,
                               const float* low, int low_stride, int rank, const float* out_t, const float* bias,
                               float inv_tau, const float* fixed, const int* chunks, int nchunks, const int* cu,

@@ -240,7 +240,9 @@ def recurrent_library(force: bool = False) -> Path:
 
 
 def linear_attention_library(force: bool = False) -> Path:
-    return compile_library("linear_attention", LINEAR_ATTENTION_SOURCES, force=force)
+    # (matrix instructions accumulate in ordinary vector registers: the memory is multiplied by the decays
+    # between two of them)
+    return compile_library("linear_attention", LINEAR_ATTENTION_SOURCES, ("-mllvm", "-amdgpu-mfma-vgpr-form=1"), force=force)
 
 
 def attention_tile_library(head_dim: int, value_dim: int, force: bool = False) -> Path:

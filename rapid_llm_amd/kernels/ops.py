@@ -385,7 +385,7 @@ def router(x: torch.Tensor, w: torch.Tensor, top: int, scale: float, bias: Optio
 def choose_experts(x: torch.Tensor, w: torch.Tensor, experts: int, identity: int, top: int, scale: float,
                    correction: Optional[torch.Tensor] = None, gate: bool = False) -> torch.Tensor:
     """The weights ``[tokens, experts + 2]`` (float32) of a mixture whose experts are chosen by corrected
-    scores.  ``w`` (float32) has a row for each of ``experts`` experts and ``identity`` experts that return their
+    scores.  ``w`` (float32, or bfloat16 where ``x`` is: the products are exact and summed in float32) has a row for each of ``experts`` experts and ``identity`` experts that return their
     input, and with ``gate`` one more.  Scores are the softmax over all experts; the ``top`` largest scores plus
     ``correction`` are chosen (the lower index wins a tie), and a chosen expert's weight is its score times
     ``scale``, not divided by anything.  A row holds the experts' weights (0 for those not chosen), the
@@ -393,14 +393,16 @@ def choose_experts(x: torch.Tensor, w: torch.Tensor, experts: int, identity: int
     tokens, k = x.shape
     choices = experts + identity
     _need(x, "x")
-    _need(w, "router matrix", torch.float32, (choices + int(bool(gate)), k))
+    _need(w, "router matrix", None, (choices + int(bool(gate)), k))
+    if w.dtype != torch.float32 and (w.dtype != torch.bfloat16 or x.dtype != torch.bfloat16):
+        raise KernelError(f"a router matrix of {w.dtype} for rows of {x.dtype}")
     if experts < 1 or identity < 0 or not 1 <= top <= choices <= ROUTE_MAX_EXPERTS:
         raise KernelError(f"the router kernel chooses 1 to {choices} of at most {ROUTE_MAX_EXPERTS} experts, not {top}")
     if correction is not None:
         _need(correction, "correction of the scores", torch.float32, (choices,))
     out = torch.empty((tokens, experts + 2), dtype=torch.float32, device=x.device)
     _ok(core().rl_choose_experts(_p(x), _p(w), _p(correction), _p(out), tokens, k, experts, identity, int(bool(gate)), top,
-                                 ctypes.c_float(scale), _tag(x.dtype), _stream()),
+                                 ctypes.c_float(scale), _tag(x.dtype), _tag(w.dtype), _stream()),
         "rl_choose_experts")
     return out
 
@@ -1672,20 +1674,28 @@ def _static(ctx) -> dict:
     return ctx.extra if static is None else static
 
 
-def _f32_tiles(ctx, group: int, tile_rows: int = 16) -> tuple[torch.Tensor, int]:
+def _f32_tiles(ctx, group: int, tile_rows: int = 16, chunk: int = 0) -> tuple[torch.Tensor, int]:
     """Tiles of ``tile_rows`` (token, head of the group) rows, request by request: ``[tiles, 3]``
     int32 (first token of the request in the step, its tokens, first row of the tile).  A function
-    of the requests' token counts alone."""
+    of the requests' token counts alone, except that with ``chunk`` (attention within chunks of so many
+    positions) the tiles of a step with portions are listed by the keys they read, most first: the last
+    to start are then the short ones."""
     key = ("f32_tiles", group) if tile_rows == 16 else ("row_tiles", group, tile_rows)
     store = _static(ctx)
+    if chunk and max(ctx.h_seq_lens, default=1) > 1:
+        key, store = (*key, chunk), ctx.extra
     made = store.get(key)
     if made is None:
-        tiles: list[int] = []
+        rows: list[tuple[int, int, int, int]] = []  # (keys with the sign turned, the tile)
         at = 0
-        for n in ctx.h_seq_lens:
+        for start, n in zip(ctx.h_seq_starts, ctx.h_seq_lens):
             for row0 in range(0, n * group, tile_rows):
-                tiles += [at, n, row0]
+                first, last = start + row0 // group, start + (min(row0 + tile_rows, n * group) - 1) // group
+                rows.append((first // chunk * chunk - last if chunk else 0, at, n, row0))
             at += n
+        if len(key) > 2 and key[-1] == chunk and chunk:
+            rows.sort(key=lambda r: r[0])
+        tiles = [v for r in rows for v in r[1:]]
         made = (upload_ints(tiles, ctx.token_ids.device), len(tiles) // 3)
         store[key] = made
     return made
@@ -1820,7 +1830,7 @@ def attention_tile(
             bound = _static(ctx).get("context_bound", ctx.max_position + 1)
             if tile_splits(blocks, bound, window, keep_first) > 1:
                 tile_rows = 16
-    tiles, num_tiles = _f32_tiles(ctx, group, tile_rows)
+    tiles, num_tiles = _f32_tiles(ctx, group, tile_rows, window if chunked else 0)
     # few tiles over many keys (a step of single tokens, mostly): a tile's keys are dealt to
     # several workgroups, on compute units of their own, and their shares merged
     nsplit, part = 1, None
@@ -2673,7 +2683,7 @@ def linear_attention(packed: torch.Tensor, columns: tuple[int, int, int, int], d
             return
     else:
         chunks, nchunks, seq_chunks = _linear_chunks(ctx)
-        rows = -(-d // 16) * 16
+        rows = -(-d // 64) * 64
         dev = packed.device
         Q = torch.empty((nchunks, heads, LINEAR_CHUNK, rows), dtype=torch.float32, device=dev)
         KT = torch.empty((nchunks, heads, rows, LINEAR_CHUNK), dtype=torch.float32, device=dev)

@@ -291,12 +291,18 @@ class RoutedExperts(FeedForward):
         if self.router_bias_name:
             self.router_bias = params[self.name + ".router_bias"]
         self.router.bind(params[self.name + ".router"])
+        # the same weights as bfloat16 where they are exactly that and meet rows of that type
+        self.router_narrow = None
+        if self.raw_scores and runtime.dtype == torch.bfloat16:
+            narrow = self.router.weight.to(torch.bfloat16)
+            if torch.equal(narrow.to(torch.float32), self.router.weight):
+                self.router_narrow = narrow
         self.up.bind(params[self.name + ".up"])
         self.down.bind(params[self.name + ".down"])
 
     def forward(self, x, ctx):
         if self.raw_scores:
-            weights = ops.choose_experts(x, self.router.weight, self.num_experts, self.identity, self.top, self.route_scale,
+            weights = ops.choose_experts(x, self.router.weight if self.router_narrow is None else self.router_narrow, self.num_experts, self.identity, self.top, self.route_scale,
                                          self.correction, self.shared_gate_name is not None)
             hidden = self.up(x)
             ops.unary_act(hidden, hidden, self.activation, weights, self.expert_size, self.num_experts)
