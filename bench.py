@@ -1014,8 +1014,9 @@ def _time_renitar_kernels(z: dict, prompt_len: int, batch: int) -> dict:
         taps, conv_state, bias = torch.randn(4, own, device=dev), torch.zeros((batch, 3, own), device=dev), torch.zeros(own, device=dev)
         qn, kn = torch.ones(nq * dh, device=dev), torch.ones(nkv * dh, device=dev)
         angles = torch.randn(prompt_len + 1, dh // 8, device=dev)
+        cos, sin = angles.cos(), angles.sin()
         qo = torch.empty((tokens, nq * dh), dtype=bf, device=dev)
-        sec = _time_calls(lambda: ops.conv_heads(pk, 0, bias, taps, conv_state, qn, kn, 1e-6, angles.cos(), angles.sin(), "half_split",
+        sec = _time_calls(lambda: ops.conv_heads(pk, 0, bias, taps, conv_state, qn, kn, 1e-6, cos, sin, "half_split",
                                                  qo, kc, vc, ctx, table, page, nq, nkv, dh, dh), single)
         rate(f"convolved_heads_{what}", sec, "hbm", hbm(tokens * own * (2 + 2) + (2 * n * 3 * own * 4 if single else 0), sec))
         # ---- router, experts' activation, the norm that adds a layer
